@@ -158,6 +158,17 @@ int retro_engine_debug_attention_timeline_read(retro_engine * engine, uint64_t *
  * reference's tests hold (tests/engine_runtime.rs:713-722). */
 int retro_engine_debug_single_token_matvec(retro_engine * engine, int32_t enable);
 
+/* A step whose rows sample nothing (row fields as in retro_engine_step_v2, sample = false), returning the logits of
+ * chosen tokens instead: place i is token want_index[i] of row want_row[i], its logits are out_logits[i * n_vocab ..).
+ * n_want may be 0. Errors as retro_engine_step_v2. */
+int retro_engine_step_logits(retro_engine * engine, const retro_step_row_v2 * rows, size_t n_rows,
+                             const uint32_t * want_row, const uint32_t * want_index, size_t n_want, float * out_logits);
+
+/* Layer-stack models: while on, every step keeps the residual stream after each layer; read copies the last step's,
+ * [layer][token][width] (out = NULL: only the number of tokens). */
+int retro_engine_debug_keep_residual(retro_engine * engine, bool on);
+int retro_engine_debug_read_residual(retro_engine * engine, float * out, size_t n_floats, size_t * out_tokens);
+
 #ifdef __cplusplus
 }
 #endif

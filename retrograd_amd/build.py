@@ -15,7 +15,8 @@ PKG = Path(__file__).resolve().parent
 CSRC = PKG / "csrc"
 LIB_DIR = PKG / "lib"
 LIB_PATH = LIB_DIR / "libretro_hip.so"
-SOURCES = ["kernels.hip", "mm_lds.hip", "gemv.hip", "moe.hip", "mxfp4_scaled.hip", "engine.cpp", "generate.cpp", "capi.cpp", "capi_trainer.cpp", "capi_test.cpp"]
+SOURCES = ["kernels.hip", "mm_lds.hip", "gemv.hip", "moe.hip", "mxfp4_scaled.hip", "dense.hip", "norms.hip",
+           "latent_attention.hip", "mamba2.hip", "engine.cpp", "engine_stack.cpp", "generate.cpp", "capi.cpp", "capi_trainer.cpp", "capi_test.cpp"]
 # host-only sources (the step scheduler): plain C++, no device pass
 HOST_SOURCES = ["sched/prefix_tree.cpp", "sched/scheduler.cpp", "sched/fake_backend.cpp", "sched/engine_backend.cpp",
                 "sched/capi_sched.cpp"]
@@ -47,9 +48,10 @@ def _compile(cmd, src, verbose):
         print(err, file=sys.stderr)
 
 
-def build(verbose: bool = False, incremental: bool = False) -> Path:
+def build(verbose: bool = False, incremental: bool = False, library_only: bool = False) -> Path:
     """Compiles every source (several at a time) and links the library. `incremental` skips a source whose object
-    is newer than it and than every header; the default recompiles everything."""
+    is newer than it and than every header; the default recompiles everything. `library_only` leaves the stand-alone
+    micro-benchmark out."""
     from concurrent.futures import ThreadPoolExecutor
 
     LIB_DIR.mkdir(exist_ok=True)
@@ -76,6 +78,8 @@ def build(verbose: bool = False, incremental: bool = False) -> Path:
     res = subprocess.run(cmd, capture_output=True, text=True)
     if res.returncode != 0:
         raise RuntimeError("link failed:\n" + res.stderr)
+    if library_only:
+        return LIB_PATH
     # the stand-alone micro-benchmark of the compute unit's issue and LDS rates (no part of the library)
     ub_src, ub_bin = CSRC / "ubench" / "issue_model.hip", LIB_DIR / "ubench_issue_model"
     if not (incremental and ub_bin.exists() and ub_bin.stat().st_mtime > ub_src.stat().st_mtime):

@@ -3,6 +3,7 @@
 // boundary(), which clears the thread's error string and turns any C++
 // exception into -1 (reference retro_runtime.hpp:1255-1267).
 #include "engine.hpp"
+#include "../../include/retro_kernels.h"
 #include "json_grammar.hpp"
 #include "json_schema.hpp"
 
@@ -92,10 +93,6 @@ bool validate_config(const retro_engine_config & c, bool * invalid_placement) {
     }
     if (c.device == RETRO_DEVICE_CPU) {
         set_error("device=cpu requested, but this library only executes on an MI355X GPU");
-        return false;
-    }
-    if (c.kv_dtype == RETRO_ENGINE_KV_DTYPE_F32) {
-        set_error("the f32 KV cache is not implemented by this library (f16, q8_0 and q4_0 are)");
         return false;
     }
     if (c.expert_placement == RETRO_EXPERT_PLACEMENT_HOST || c.expert_device_cache_bytes != 0) {
@@ -193,6 +190,34 @@ int retro_engine_step_v2(retro_engine * engine, const retro_step_row_v2 * rows, 
         }
         e->forget_generation_bookkeeping();
         return e->step(rows, nullptr, n_rows, out_rows, nullptr, out_top_ids, out_top_logprobs, n_top_stride);
+    });
+}
+
+int retro_engine_step_logits(retro_engine * engine, const retro_step_row_v2 * rows, size_t n_rows,
+                             const uint32_t * want_row, const uint32_t * want_index, size_t n_want, float * out_logits) {
+    return boundary([&]() -> int {
+        Engine * e = checked(engine);
+        if (!e) return -1;
+        if (!rows || n_rows == 0) {
+            set_error("step rows are required");
+            return -3;
+        }
+        e->forget_generation_bookkeeping();
+        return e->step_logits(rows, n_rows, Engine::WantLogits{want_row, want_index, n_want, out_logits});
+    });
+}
+
+int retro_engine_debug_keep_residual(retro_engine * engine, bool on) {
+    return boundary([&]() -> int {
+        Engine * e = checked(engine);
+        return e ? e->debug_keep_residual(on) : -1;
+    });
+}
+
+int retro_engine_debug_read_residual(retro_engine * engine, float * out, size_t n_floats, size_t * out_tokens) {
+    return boundary([&]() -> int {
+        Engine * e = checked(engine);
+        return e ? e->debug_read_residual(out, n_floats, out_tokens) : -1;
     });
 }
 
@@ -335,7 +360,7 @@ int retro_engine_is_hybrid(retro_engine * engine, bool * out_is_hybrid) {
             if (e) set_error("out_is_hybrid is required");
             return -1;
         }
-        *out_is_hybrid = false;   // attention-only architectures
+        *out_is_hybrid = e->is_hybrid();
         return 0;
     });
 }

@@ -90,7 +90,8 @@ Engine::Engine(const std::string & path, const retro_engine_config & config) : c
         if (mode == "ggml") ggml_activations_ = true;
         else if (mode != "exact" && !mode.empty()) throw std::runtime_error("RETRO_ACTIVATIONS must be \"exact\" or \"ggml\"");
     }
-    load_model(path);
+    if (StackConfig::is_folder(path)) load_stack(path);
+    else load_model(path);
 
     // Per-sequence context: the whole pool when unified, an equal share otherwise.
     n_ctx_seq_ = cfg_.kv_unified ? (int)cfg_.n_ctx : (int)(cfg_.n_ctx / cfg_.n_seq_max);
@@ -101,26 +102,34 @@ Engine::Engine(const std::string & path, const retro_engine_config & config) : c
     // page repeats up to PAGE - 1 shared cells). Two spare pages per slot cover both, so a step that fits
     // n_ctx distinct cells always finds its pages.
     n_pages_ = (int)((cfg_.n_ctx + rk::PAGE - 1) / rk::PAGE + 2 * cfg_.n_seq_max);
-    // [page][kv head]: the other order (a head's pages side by side) was measured 3 % slower in the attention kernel
-    kv_q8_ = cfg_.kv_dtype == RETRO_ENGINE_KV_DTYPE_Q8_0 ? rk::KV_Q8 : cfg_.kv_dtype == RETRO_ENGINE_KV_DTYPE_Q4_0 ? rk::KV_Q4 : rk::KV_F16;
-    if (kv_q8_ != rk::KV_F16 && hp_.head_dim % 32 != 0) throw std::runtime_error("a Q8_0 or Q4_0 KV cache needs head_dim to be a multiple of 32");
-    kv_strides_ = rk::kv_strides(n_pages_, hp_.n_head_kv, hp_.head_dim, false, kv_q8_);
-    const int G = hp_.n_head / hp_.n_head_kv;
-    if (hp_.n_head % hp_.n_head_kv != 0 || G > 16) throw std::runtime_error("unsupported attention head grouping");
-    qt_ = rk::attention_tile_tokens(G);
+    if (stack_) {
+        build_stack();
+    } else {
+        // [page][kv head]: the other order (a head's pages side by side) was measured 3 % slower in the attention kernel
+        kv_q8_ = cfg_.kv_dtype == RETRO_ENGINE_KV_DTYPE_Q8_0 ? rk::KV_Q8 : cfg_.kv_dtype == RETRO_ENGINE_KV_DTYPE_Q4_0 ? rk::KV_Q4 : rk::KV_F16;
+        if (kv_q8_ != rk::KV_F16 && hp_.head_dim % 32 != 0) throw std::runtime_error("a Q8_0 or Q4_0 KV cache needs head_dim to be a multiple of 32");
+        kv_strides_ = rk::kv_strides(n_pages_, hp_.n_head_kv, hp_.head_dim, false, kv_q8_);
+        const int G = hp_.n_head / hp_.n_head_kv;
+        if (hp_.n_head % hp_.n_head_kv != 0 || G > 16) throw std::runtime_error("unsupported attention head grouping");
+        qt_ = rk::attention_tile_tokens(G);
 
-    const size_t pool_halves = (size_t)n_pages_ * hp_.n_head_kv * rk::kv_block_halves(hp_.head_dim, kv_q8_);
-    k_pool_.resize((size_t)hp_.n_layer);
-    v_pool_.resize((size_t)hp_.n_layer);
-    const size_t pool_bytes = (pool_halves * 2 + 255) / 256 * 256;
-    kv_slab_.alloc(pool_bytes * 2 * (size_t)hp_.n_layer);
-    // Pages must never hold non-finite bit patterns: a masked score times a
-    // NaN value would poison the output.
-    hip_check(hipMemsetAsync(kv_slab_.ptr, 0, kv_slab_.bytes, stream_), "hipMemsetAsync");
-    for (int l = 0; l < hp_.n_layer; ++l) {
-        k_pool_[(size_t)l] = PoolView{(uint8_t *)kv_slab_.ptr + pool_bytes * (2 * (size_t)l), pool_halves * 2};
-        v_pool_[(size_t)l] = PoolView{(uint8_t *)kv_slab_.ptr + pool_bytes * (2 * (size_t)l + 1), pool_halves * 2};
+        const size_t pool_halves = (size_t)n_pages_ * hp_.n_head_kv * rk::kv_block_halves(hp_.head_dim, kv_q8_);
+        k_pool_.resize((size_t)hp_.n_layer);
+        v_pool_.resize((size_t)hp_.n_layer);
+        const size_t pool_bytes = (pool_halves * 2 + 255) / 256 * 256;
+        kv_slab_.alloc(pool_bytes * 2 * (size_t)hp_.n_layer);
+        // Pages must never hold non-finite bit patterns: a masked score times a
+        // NaN value would poison the output.
+        hip_check(hipMemsetAsync(kv_slab_.ptr, 0, kv_slab_.bytes, stream_), "hipMemsetAsync");
+        for (int l = 0; l < hp_.n_layer; ++l) {
+            k_pool_[(size_t)l] = PoolView{(uint8_t *)kv_slab_.ptr + pool_bytes * (2 * (size_t)l), pool_halves * 2};
+            v_pool_[(size_t)l] = PoolView{(uint8_t *)kv_slab_.ptr + pool_bytes * (2 * (size_t)l + 1), pool_halves * 2};
+        }
+        for (int l = 0; l < hp_.n_layer; ++l)
+            for (int v = 0; v < 2; ++v)
+                cache_parts_.push_back({l, v != 0, rk::kv_row_halves(hp_.n_head_kv, hp_.head_dim, kv_q8_) * 2});
     }
+    for (const CachePart & p : cache_parts_) cache_row_bytes_ += p.row_bytes;
     table_.alloc((size_t)cfg_.n_seq_max * max_pages_ * sizeof(int32_t));
     hip_check(hipMemsetAsync(table_.ptr, 0xff, table_.bytes, stream_), "hipMemsetAsync");
     slots_.resize(cfg_.n_seq_max);
@@ -128,7 +137,7 @@ Engine::Engine(const std::string & path, const retro_engine_config & config) : c
     page_ref_.assign((size_t)n_pages_, 0);
     for (int p = 0; p < n_pages_; ++p) free_pages_.push(p);
 
-    build_buffers();
+    if (!stack_) build_buffers();
     hip_check(hipStreamSynchronize(stream_), "hipStreamSynchronize");
 }
 
@@ -246,13 +255,14 @@ bool Engine::upload_gate_up_interleaved(const TensorInfo & g, const TensorInfo &
 }
 
 void Engine::load_model(const std::string & path) {
+    if (cfg_.kv_dtype == RETRO_ENGINE_KV_DTYPE_F32) throw std::runtime_error("the f32 KV cache is not implemented for GGUF models (f16, q8_0 and q4_0 are)");
     GgufFile g(path);
     g.rewrite_as_q8_0();      // Q4_0, Q5_0, IQ4_NL and Q3_K tensors become the Q8_0 rows that hold the same values
     HParams & h = hp_;
     h.arch = g.get_string("general.architecture");
-    if (h.arch == "llama") h.rope_neox = false;
-    else if (h.arch == "qwen2" || h.arch == "qwen3" || h.arch == "qwen3moe") h.rope_neox = true;
-    else throw std::runtime_error("unsupported model architecture: " + h.arch);
+    const GgufArch * known = find_gguf_arch(h.arch);
+    if (!known) throw std::runtime_error("unsupported model architecture: " + h.arch);
+    h.rope_neox = known->rope_neox;
     const std::string a = h.arch + ".";
     h.n_layer = (int)g.need_int(a + "block_count");
     h.n_embd = (int)g.need_int(a + "embedding_length");
@@ -432,9 +442,9 @@ void Engine::load_model(const std::string & path) {
     fingerprint_ = hash;
 }
 
-void Engine::build_buffers() {
+// Arrays of the packed step, the same for every model.
+void Engine::build_pack_buffers() {
     const int B = (int)cfg_.n_batch;
-    const int E = hp_.n_embd, QD = hp_.n_head * hp_.head_dim, KD = hp_.n_head_kv * hp_.head_dim, F = hp_.n_ff;
     auto i32 = [&](size_t n) {
         pk_store_.emplace_back();
         pk_store_.back().alloc(n * 4);
@@ -452,7 +462,25 @@ void Engine::build_buffers() {
     pk_.tok_merge = (int4 *)i32((size_t)B * 4);
     pk_.rope_cos = (float *)i32((size_t)B * (hp_.rope_dim / 2));
     pk_.rope_sin = (float *)i32((size_t)B * (hp_.rope_dim / 2));
+}
 
+// Staging of the step's plan and of what sampling reads back, the same for every model.
+void Engine::build_step_buffers() {
+    const int B = (int)cfg_.n_batch;
+    sample_k_.alloc((size_t)B * 4);
+    sample_out_.alloc((size_t)B * sizeof(rk::SampleOut));
+    sample_scratch_.alloc(rk::sample_scratch_bytes(B));
+    const size_t stage = (size_t)B * (sizeof(rk::RowDesc) + 4) + 65536;
+    d_stage_.alloc(stage);
+    h_stage_.ensure(stage);
+    h_sample_.ensure((size_t)B * sizeof(rk::SampleOut));
+}
+
+void Engine::build_buffers() {
+    const int B = (int)cfg_.n_batch;
+    const int E = hp_.n_embd, QD = hp_.n_head * hp_.head_dim, KD = hp_.n_head_kv * hp_.head_dim, F = hp_.n_ff;
+    build_pack_buffers();
+    build_step_buffers();
     x_.alloc((size_t)B * E * 4);
     qkv_.alloc((size_t)B * (QD + 2 * KD) * 4);
     gu_.alloc((size_t)B * 2 * std::max(F, 1) * 4);
@@ -511,13 +539,6 @@ void Engine::build_buffers() {
     q_half_lo_.alloc((size_t)B * QD * 2);
     mm_ws_.alloc(rk::matmul_workspace_bytes());
     hip_check(hipMemsetAsync(mm_ws_.ptr, 0, mm_ws_.bytes, stream_), "hipMemsetAsync");
-    sample_k_.alloc((size_t)B * 4);
-    sample_out_.alloc((size_t)B * sizeof(rk::SampleOut));
-    sample_scratch_.alloc(rk::sample_scratch_bytes(B));
-    const size_t stage = (size_t)B * (sizeof(rk::RowDesc) + 4) + 65536;
-    d_stage_.alloc(stage);
-    h_stage_.ensure(stage);
-    h_sample_.ensure((size_t)B * sizeof(rk::SampleOut));
 }
 
 // ---- pages ---------------------------------------------------------------------------
@@ -535,7 +556,32 @@ void Engine::release_page(int32_t page) {
     if (--page_ref_[(size_t)page] == 0) free_pages_.push(page);
 }
 
+void Engine::cells_gather(const CachePart & part, const int32_t * cells, int n, void * out) {
+    const PoolView & pool = (part.v ? v_pool_ : k_pool_)[(size_t)part.layer];
+    if (stack_) {
+        const int elem = arith_;
+        rk::latent_cells(stream_, pool.ptr, (int)(part.row_bytes / (32 * (size_t)elem)), elem, cells, n, out, true);
+    } else {
+        rk::kv_gather(stream_, pool.as<__half>(), kv_strides_, hp_.n_head_kv, hp_.head_dim, part.v, cells, n, (__half *)out, kv_q8_);
+    }
+}
+
+void Engine::cells_scatter(const CachePart & part, const int32_t * cells, int n, const void * in) {
+    const PoolView & pool = (part.v ? v_pool_ : k_pool_)[(size_t)part.layer];
+    if (stack_) {
+        const int elem = arith_;
+        rk::latent_cells(stream_, pool.ptr, (int)(part.row_bytes / (32 * (size_t)elem)), elem, cells, n, const_cast<void *>(in), false);
+    } else {
+        rk::kv_scatter(stream_, pool.as<__half>(), kv_strides_, hp_.n_head_kv, hp_.head_dim, part.v, cells, n, (const __half *)in, kv_q8_);
+    }
+}
+
 void Engine::copy_page(int32_t src, int32_t dst) {
+    if (stack_) {
+        for (const CachePart & p : cache_parts_)
+            rk::latent_copy_page(stream_, k_pool_[(size_t)p.layer].ptr, p.row_bytes * rk::PAGE, src, dst);
+        return;
+    }
     for (int l = 0; l < hp_.n_layer; ++l) {
         rk::kv_copy_page(stream_, k_pool_[(size_t)l].as<__half>(), v_pool_[(size_t)l].as<__half>(), kv_strides_,
                          hp_.n_head_kv, hp_.head_dim, src, dst, kv_q8_);
@@ -569,6 +615,10 @@ bool Engine::seq_rm(int32_t slot, int32_t p0, int32_t p1) {
     if (p0 <= s.begin && p1 >= s.end) {
         clear_slot(s, slot);
         return true;
+    }
+    if (is_hybrid()) {                       // the recurrent state holds every resident token and cannot forget some of them
+        set_error("a recurrent model's memory cannot remove a partial range; remove the whole sequence instead");
+        return false;
     }
     if (p1 >= s.end) {                       // drop a suffix: keep [begin, p0)
         const int keep_last = (p0 - 1) / rk::PAGE;
@@ -606,6 +656,10 @@ bool Engine::seq_cp(int32_t src, int32_t dst, int32_t p0, int32_t p1) {
     if (p1 < 0) p1 = INT_MAX;
     const int lo = std::max(p0, a.begin), hi = std::min(p1, a.end);
     if (a.end <= a.begin || hi <= lo) return true;
+    if (is_hybrid() && (!(whole || (lo == a.begin && hi == a.end)) || b.end > b.begin)) {
+        set_error("a recurrent model only supports whole-sequence copies into an empty slot");
+        return false;
+    }
     if (!cfg_.kv_unified && !(whole || (lo == a.begin && hi == a.end))) {
         set_error("a partitioned KV pool only supports whole-sequence copies");
         return false;
@@ -648,25 +702,22 @@ bool Engine::seq_cp(int32_t src, int32_t dst, int32_t p0, int32_t p1) {
                 cells_src.push_back(sp * rk::PAGE + p % rk::PAGE);
                 cells_dst.push_back(target * rk::PAGE + p % rk::PAGE);
             }
-            const size_t kd = rk::kv_row_halves(hp_.n_head_kv, hp_.head_dim, kv_q8_);      // halves of a cell's row
             DevBuf cs, cd, tmp;
             cs.alloc(cells_src.size() * 4);
             cd.alloc(cells_dst.size() * 4);
-            tmp.alloc(cells_src.size() * kd * 2);
+            tmp.alloc(cells_src.size() * cache_row_bytes_);
             hip_check(hipMemcpyAsync(cs.ptr, cells_src.data(), cs.bytes, hipMemcpyHostToDevice, stream_), "hipMemcpyAsync");
             hip_check(hipMemcpyAsync(cd.ptr, cells_dst.data(), cd.bytes, hipMemcpyHostToDevice, stream_), "hipMemcpyAsync");
-            for (int l = 0; l < hp_.n_layer; ++l) {
-                for (int v = 0; v < 2; ++v) {
-                    __half * pool = v ? v_pool_[(size_t)l].as<__half>() : k_pool_[(size_t)l].as<__half>();
-                    rk::kv_gather(stream_, pool, kv_strides_, hp_.n_head_kv, hp_.head_dim, v != 0, cs.as<int32_t>(), (int)cells_src.size(), tmp.as<__half>(), kv_q8_);
-                    rk::kv_scatter(stream_, pool, kv_strides_, hp_.n_head_kv, hp_.head_dim, v != 0, cd.as<int32_t>(), (int)cells_dst.size(), tmp.as<__half>(), kv_q8_);
-                }
+            for (const CachePart & p : cache_parts_) {
+                cells_gather(p, cs.as<int32_t>(), (int)cells_src.size(), tmp.ptr);
+                cells_scatter(p, cd.as<int32_t>(), (int)cells_dst.size(), tmp.ptr);
             }
             hip_check(hipStreamSynchronize(stream_), "seq_cp merge");
         }
     }
     if (b.end <= b.begin) { b.begin = lo; b.end = hi; }
     else { b.begin = std::min(b.begin, lo); b.end = std::max(b.end, hi); }
+    if (is_hybrid()) state_copy(src, dst);
     return true;
 }
 
@@ -700,7 +751,7 @@ int Engine::memory(retro_engine_memory_info * out) {
     for (const auto & b : k_pool_) kv += b.bytes;
     for (const auto & b : v_pool_) kv += b.bytes;
     out->kv_bytes = kv;
-    out->recurrent_bytes = 0;
+    out->recurrent_bytes = recurrent_slab_.bytes;
     return 0;
 }
 
@@ -716,9 +767,14 @@ struct SnapHeader { uint32_t magic, flags; int32_t n_layer, kv_dim, begin, end; 
 constexpr uint32_t kSnapMagic = 0x31564b52u;
 constexpr uint32_t kSnapMagicQ8 = 0x38564b52u;
 constexpr uint32_t kSnapMagicQ4 = 0x34564b52u;        // "RKV4"
+constexpr uint32_t kSnapMagicLatent16 = 0x32434c52u;  // "RLC2", "RLC4": latent caches in f16 / f32, then the recurrent state
+constexpr uint32_t kSnapMagicLatent32 = 0x34434c52u;
 }
 
-uint32_t Engine::snap_magic() const { return kv_q8_ == rk::KV_Q8 ? kSnapMagicQ8 : kv_q8_ == rk::KV_Q4 ? kSnapMagicQ4 : kSnapMagic; }
+uint32_t Engine::snap_magic() const {
+    if (stack_) return arith_ == rk::ARITH_16 ? kSnapMagicLatent16 : kSnapMagicLatent32;
+    return kv_q8_ == rk::KV_Q8 ? kSnapMagicQ8 : kv_q8_ == rk::KV_Q4 ? kSnapMagicQ4 : kSnapMagic;
+}
 
 int Engine::seq_save(int32_t slot, uint32_t flags, uint8_t * buffer, size_t n_buffer, size_t * out_n_bytes) {
     if (!out_n_bytes) {
@@ -734,34 +790,36 @@ int Engine::seq_save(int32_t slot, uint32_t flags, uint8_t * buffer, size_t n_bu
         return -1;
     }
     const Slot & s = slots_[(size_t)slot];
-    const size_t kd = rk::kv_row_halves(hp_.n_head_kv, hp_.head_dim, kv_q8_);
+    const size_t kd = cache_row_bytes_ / std::max<size_t>(1, cache_parts_.size()) / 2;
     const bool partial_only = (flags & RETRO_STATE_SEQ_FLAGS_PARTIAL_ONLY) != 0;
-    const int n_pos = partial_only ? 0 : std::max(0, s.end - s.begin);   // no recurrent or SWA state exists
-    const size_t required = sizeof(SnapHeader) + (size_t)hp_.n_layer * 2 * (size_t)n_pos * kd * 2;
+    const int n_pos = partial_only ? 0 : std::max(0, s.end - s.begin);   // PARTIAL_ONLY: what is not addressed by position, the recurrent state
+    const size_t state_bytes = s.end > s.begin ? recurrent_floats() * 4 : 0;
+    const size_t required = sizeof(SnapHeader) + (size_t)n_pos * cache_row_bytes_ + state_bytes;
     *out_n_bytes = required;
     if (!buffer) return 0;
     if (n_buffer < required) {
         set_error("the save buffer is too small for this sequence's state");
         return -2;
     }
-    SnapHeader h{snap_magic(), flags, hp_.n_layer, (int32_t)kd, partial_only ? 0 : s.begin, partial_only ? 0 : s.begin + n_pos};
+    // a recurrent PARTIAL_ONLY snapshot still says which span its state stands for
+    const bool span = !partial_only || state_bytes > 0;
+    SnapHeader h{snap_magic(), flags, hp_.n_layer, (int32_t)kd, span ? s.begin : 0, span ? std::max(s.begin, s.end) : 0};
     std::memcpy(buffer, &h, sizeof(h));
+    if (state_bytes > 0) state_pack(slot, (float *)(buffer + required - state_bytes));
     if (n_pos > 0) {
         std::vector<int32_t> cells((size_t)n_pos);
         for (int p = s.begin; p < s.end; ++p) cells[(size_t)(p - s.begin)] = s.pages[(size_t)(p / rk::PAGE)] * rk::PAGE + p % rk::PAGE;
         DevBuf dc, tmp;
         dc.alloc(cells.size() * 4);
-        tmp.alloc((size_t)n_pos * kd * 2);
+        tmp.alloc((size_t)n_pos * cache_row_bytes_);
         hip_check(hipMemcpyAsync(dc.ptr, cells.data(), dc.bytes, hipMemcpyHostToDevice, stream_), "hipMemcpyAsync");
         uint8_t * at = buffer + sizeof(h);
-        for (int l = 0; l < hp_.n_layer; ++l) {
-            for (int v = 0; v < 2; ++v) {
-                const __half * pool = v ? v_pool_[(size_t)l].as<__half>() : k_pool_[(size_t)l].as<__half>();
-                rk::kv_gather(stream_, pool, kv_strides_, hp_.n_head_kv, hp_.head_dim, v != 0, dc.as<int32_t>(), n_pos, tmp.as<__half>(), kv_q8_);
-                hip_check(hipMemcpyAsync(at, tmp.ptr, tmp.bytes, hipMemcpyDeviceToHost, stream_), "hipMemcpyAsync");
-                hip_check(hipStreamSynchronize(stream_), "seq_save");
-                at += tmp.bytes;
-            }
+        for (const CachePart & p : cache_parts_) {
+            const size_t bytes = (size_t)n_pos * p.row_bytes;
+            cells_gather(p, dc.as<int32_t>(), n_pos, tmp.ptr);
+            hip_check(hipMemcpyAsync(at, tmp.ptr, bytes, hipMemcpyDeviceToHost, stream_), "hipMemcpyAsync");
+            hip_check(hipStreamSynchronize(stream_), "seq_save");
+            at += bytes;
         }
     }
     return 0;
@@ -788,16 +846,23 @@ int Engine::seq_load(int32_t slot, uint32_t flags, const uint8_t * buffer, size_
     SnapHeader h;
     if (n_bytes < sizeof(h)) { set_error(refused); return -1; }
     std::memcpy(&h, buffer, sizeof(h));
-    const size_t kd = rk::kv_row_halves(hp_.n_head_kv, hp_.head_dim, kv_q8_);
+    const size_t kd = cache_row_bytes_ / std::max<size_t>(1, cache_parts_.size()) / 2;
     if (h.magic != snap_magic() || h.flags != flags || h.n_layer != hp_.n_layer || h.kv_dim != (int32_t)kd
             || h.begin < 0 || h.end < h.begin || h.end > n_ctx_seq_) {
         set_error(refused);
         return -1;
     }
     const int n_pos = h.end - h.begin;
-    const size_t required = sizeof(h) + (size_t)hp_.n_layer * 2 * (size_t)n_pos * kd * 2;
+    const bool partial_only = (flags & RETRO_STATE_SEQ_FLAGS_PARTIAL_ONLY) != 0;
+    const size_t state_bytes = n_pos > 0 ? recurrent_floats() * 4 : 0;
+    const size_t required = sizeof(h) + (partial_only ? 0 : (size_t)n_pos * cache_row_bytes_) + state_bytes;
     if (n_bytes < required) { set_error(refused); return -1; }
-    if (flags & RETRO_STATE_SEQ_FLAGS_PARTIAL_ONLY) {
+    if (partial_only) {
+        if (state_bytes > 0) {
+            const Slot & have = slots_[(size_t)slot];
+            if (have.begin != h.begin || have.end != h.end) { set_error(refused); return -1; }     // the state of another span
+            state_unpack(slot, (const float *)(buffer + required - state_bytes));
+        }
         *out_n_read = required;
         return 0;
     }
@@ -816,18 +881,17 @@ int Engine::seq_load(int32_t slot, uint32_t flags, const uint8_t * buffer, size_
         for (int p = s.begin; p < s.end; ++p) cells[(size_t)(p - s.begin)] = s.pages[(size_t)(p / rk::PAGE)] * rk::PAGE + p % rk::PAGE;
         DevBuf dc, tmp;
         dc.alloc(cells.size() * 4);
-        tmp.alloc((size_t)n_pos * kd * 2);
+        tmp.alloc((size_t)n_pos * cache_row_bytes_);
         hip_check(hipMemcpyAsync(dc.ptr, cells.data(), dc.bytes, hipMemcpyHostToDevice, stream_), "hipMemcpyAsync");
         const uint8_t * at = buffer + sizeof(h);
-        for (int l = 0; l < hp_.n_layer; ++l) {
-            for (int v = 0; v < 2; ++v) {
-                __half * pool = v ? v_pool_[(size_t)l].as<__half>() : k_pool_[(size_t)l].as<__half>();
-                hip_check(hipMemcpyAsync(tmp.ptr, at, tmp.bytes, hipMemcpyHostToDevice, stream_), "hipMemcpyAsync");
-                rk::kv_scatter(stream_, pool, kv_strides_, hp_.n_head_kv, hp_.head_dim, v != 0, dc.as<int32_t>(), n_pos, tmp.as<__half>(), kv_q8_);
-                hip_check(hipStreamSynchronize(stream_), "seq_load");
-                at += tmp.bytes;
-            }
+        for (const CachePart & p : cache_parts_) {
+            const size_t bytes = (size_t)n_pos * p.row_bytes;
+            hip_check(hipMemcpyAsync(tmp.ptr, at, bytes, hipMemcpyHostToDevice, stream_), "hipMemcpyAsync");
+            cells_scatter(p, dc.as<int32_t>(), n_pos, tmp.ptr);
+            hip_check(hipStreamSynchronize(stream_), "seq_load");
+            at += bytes;
         }
+        if (state_bytes > 0) state_unpack(slot, (const float *)(buffer + required - state_bytes));
     }
     *out_n_read = required;
     return 0;
@@ -921,6 +985,34 @@ bool valid_sampling_v2(const retro_sampling_params_v2 & s, int32_t n_vocab) {
 int Engine::step(const retro_step_row_v2 * rows2, const retro_step_row * rows1, size_t n_rows,
                  retro_step_out_row_v2 * out2, retro_step_out_row * out1,
                  int32_t * out_top_ids, float * out_top_logprobs, size_t n_top_stride) {
+    return run_step(rows2, rows1, n_rows, out2, out1, out_top_ids, out_top_logprobs, n_top_stride, nullptr);
+}
+
+int Engine::step_logits(const retro_step_row_v2 * rows, size_t n_rows, const WantLogits & want) {
+    size_t total = 0;
+    for (size_t r = 0; r < n_rows; ++r) {
+        if (rows[r].sample) {
+            set_error("a step for logits samples nothing");
+            return -3;
+        }
+        total += rows[r].n;
+    }
+    if (want.n > total || (want.n > 0 && (!want.row || !want.index || !want.out))) {
+        set_error("more logits are wanted than the step has tokens, or their places or buffer are missing");
+        return -3;
+    }
+    for (size_t i = 0; i < want.n; ++i)
+        if (want.row[i] >= n_rows || want.index[i] >= rows[want.row[i]].n) {
+            set_error("logits are wanted outside the step's rows");
+            return -3;
+        }
+    std::vector<retro_step_out_row_v2> outs(n_rows);
+    return run_step(rows, nullptr, n_rows, outs.data(), nullptr, nullptr, nullptr, 0, &want);
+}
+
+int Engine::run_step(const retro_step_row_v2 * rows2, const retro_step_row * rows1, size_t n_rows,
+                     retro_step_out_row_v2 * out2, retro_step_out_row * out1,
+                     int32_t * out_top_ids, float * out_top_logprobs, size_t n_top_stride, const WantLogits * want) {
     const bool is_v2 = rows2 != nullptr;
     if ((!rows2 && !rows1) || n_rows == 0 || (!out2 && !out1)) {
         set_error("step rows and output rows are required");
@@ -1086,6 +1178,8 @@ int Engine::step(const retro_step_row_v2 * rows2, const retro_step_row * rows1, 
             return -1;
         }
     }
+    std::vector<std::pair<int, int>> before(stack_ ? slots_.size() : 0);      // the spans the step found
+    for (size_t i = 0; i < before.size(); ++i) before[i] = {slots_[i].begin, slots_[i].end};
     for (const RowView & row : rows) {
         Slot & s = slots_[(size_t)row.slot];
         if (s.end <= s.begin) { s.begin = row.pos0; s.end = row.pos0; }
@@ -1119,9 +1213,14 @@ int Engine::step(const retro_step_row_v2 * rows2, const retro_step_row * rows1, 
     const size_t n_upd = pending_updates_.size();
     const size_t off_tok = n_rows * sizeof(rk::RowDesc);
     const size_t off_upd = off_tok + (size_t)T * 4;
-    const size_t stage_bytes = off_upd + n_upd * sizeof(rk::TableUpdate);
+    const size_t off_want = off_upd + n_upd * sizeof(rk::TableUpdate);
+    const size_t n_want = want ? want->n : 0;
+    const size_t off_plan = (off_want + n_want * 4 + 15) / 16 * 16;
+    if (stack_) plan_stack(rows, before);
+    const size_t stage_bytes = off_plan + (stack_ ? stack_plan_bytes() : 0);
     h_stage_.ensure(stage_bytes);
     d_stage_.ensure(stage_bytes);
+    if (stack_) stage_stack_plan(h_stage_.as<uint8_t>() + off_plan, d_stage_.as<uint8_t>() + off_plan);
     rk::RowDesc * hd = h_stage_.as<rk::RowDesc>();
     int32_t * ht = (int32_t *)((uint8_t *)h_stage_.ptr + off_tok);
     int n_out = 0;
@@ -1157,8 +1256,13 @@ int Engine::step(const retro_step_row_v2 * rows2, const retro_step_row * rows1, 
         }
         pending_updates_.clear();
     }
+    if (want) {
+        int32_t * hw = (int32_t *)((uint8_t *)h_stage_.ptr + off_want);
+        for (size_t i = 0; i < n_want; ++i) hw[i] = hd[want->row[i]].tok_off + (int32_t)want->index[i];
+        n_out = (int)n_want;
+    }
     int n_tiles = 0, n_items = 0;
-    rk::count_attention_work(hd, (int)n_rows, qt_, hp_.n_head_kv, &n_tiles, &n_items, &pk_.split_pages);
+    if (!stack_) rk::count_attention_work(hd, (int)n_rows, qt_, hp_.n_head_kv, &n_tiles, &n_items, &pk_.split_pages);
 
     if ((size_t)n_items * 32 > item_meta_.bytes) item_meta_.ensure((size_t)n_items * 48);      // some room to grow into
     pk_.item_a = item_meta_.as<int4>();
@@ -1173,7 +1277,19 @@ int Engine::step(const retro_step_row_v2 * rows2, const retro_step_row * rows1, 
                       table_.as<int32_t>(), max_pages_, qt_, hp_.n_head_kv, inv_freq_.as<double>(),
                       hp_.rope_dim / 2, pk_);
         prof_end(PC_PACK, pt_pack);
-        forward(T, n_out, n_tiles, n_items, (size_t)T == n_rows, routed);
+        if (n_want > 0)
+            rk::copy_floats(stream_, (const float *)((const uint8_t *)d_stage_.ptr + off_want), (float *)pk_.out_tok, n_want);
+        if (stack_) forward_stack(T, n_out);
+        else forward(T, n_out, n_tiles, n_items, (size_t)T == n_rows, routed);
+        if (want) {
+            if (n_want > 0)
+                hip_check(hipMemcpyAsync(want->out, logits_.ptr, n_want * (size_t)n_vocab * 4, hipMemcpyDeviceToHost, stream_), "hipMemcpyAsync");
+            hip_check(hipStreamSynchronize(stream_), "step");
+            if (prof_level_) prof_resolve();
+            last_n_out_ = n_out;
+            ++steps_run_;
+            return 0;
+        }
 
         // ---- sampling: the device scans the vocabulary, the host draws.
         std::vector<int32_t> kreq((size_t)std::max(n_out, 1), 0);
@@ -1779,6 +1895,10 @@ void Engine::forget_generation_kv() {
 }
 
 int Engine::read_adapter(const std::string & path, float scale, RowAdapterData & data) {
+    if (stack_) {
+        set_error("adapters are not supported for layer-stack models");
+        return -1;
+    }
     std::unique_ptr<GgufFile> file;
     try {
         file.reset(new GgufFile(path));
@@ -1998,16 +2118,19 @@ int Engine::debug_read_kv(int layer, int32_t slot, int32_t pos, int want_v, uint
     }
     const int32_t cell = s.pages[(size_t)(pos / rk::PAGE)] * rk::PAGE + pos % rk::PAGE;
     // the row as kv_gather writes it: kv_dim f16 values, or (a Q8_0 cache) per kv head the code bytes and block scales
-    const size_t kd = rk::kv_row_halves(hp_.n_head_kv, hp_.head_dim, kv_q8_);
-    DevBuf dc, tmp;
-    dc.alloc(4);
-    tmp.alloc(kd * 2);
-    hip_check(hipMemcpy(dc.ptr, &cell, 4, hipMemcpyHostToDevice), "hipMemcpy");
-    const __half * pool = want_v ? v_pool_[(size_t)layer].as<__half>() : k_pool_[(size_t)layer].as<__half>();
-    rk::kv_gather(stream_, pool, kv_strides_, hp_.n_head_kv, hp_.head_dim, want_v != 0, dc.as<int32_t>(), 1, tmp.as<__half>(), kv_q8_);
-    hip_check(hipStreamSynchronize(stream_), "debug_read_kv");
-    hip_check(hipMemcpy(out, tmp.ptr, kd * 2, hipMemcpyDeviceToHost), "hipMemcpy");
-    return 0;
+    for (const CachePart & p : cache_parts_) {
+        if (p.layer != layer || p.v != (want_v != 0)) continue;
+        DevBuf dc, tmp;
+        dc.alloc(4);
+        tmp.alloc(p.row_bytes);
+        hip_check(hipMemcpy(dc.ptr, &cell, 4, hipMemcpyHostToDevice), "hipMemcpy");
+        cells_gather(p, dc.as<int32_t>(), 1, tmp.ptr);
+        hip_check(hipStreamSynchronize(stream_), "debug_read_kv");
+        hip_check(hipMemcpy(out, tmp.ptr, p.row_bytes, hipMemcpyDeviceToHost), "hipMemcpy");
+        return 0;
+    }
+    set_error("the layer caches no such rows");
+    return -1;
 }
 
 int Engine::debug_pack(int32_t * tok, int32_t * pos, int32_t * seq, int32_t * cell, int32_t * out_index,

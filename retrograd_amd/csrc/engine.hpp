@@ -8,6 +8,7 @@
 #include "../../include/retro_step.h"
 #include "gguf_file.hpp"
 #include "kernels.hpp"
+#include "model_registry.hpp"
 #include "tokenizer.hpp"
 #include "grammar.hpp"
 #include "sampler.hpp"
@@ -79,7 +80,26 @@ struct LayerWeights {
     DevWeight router, gate_exps, up_exps, down_exps;
 };
 
+// A layer of a layer-stack model on the device. Everything that reads the layer's norm is one matrix (w_in: the mixer's
+// input projections as f32 columns, then the feed-forward's up rows), everything that adds to the stream another (w_out:
+// the mixer's output projection and the feed-forward's down projection side by side along K).
+struct StackLayer {
+    struct Matrix { rk::DenseWeight w; DevBuf buf; };
+    LayerSpec spec;
+    DevBuf norm, scale_mix, scale_ff;
+    Matrix w_in, w_out;
+    int in_tiles = 0, in_rows = 0;          // row tiles and rows of w_in that belong to the mixer
+    int kv_col = 0, gate_col = 0;           // columns of the input product: the latent, the head gates
+    DevBuf q_norm, kv_norm;
+    Matrix uq, uk, uv;                      // queries from their latent; per head: absorption and value up-projection
+    DevBuf conv_w, conv_b, dt_bias, A_log, D, gate_norm;
+    int pool_layer = -1;                    // the layer whose latent pool is attended to
+    float * conv_state = nullptr, * state = nullptr;       // the layer's part of the recurrent state
+    size_t conv_slot = 0, state_slot = 0;   // floats per slot (a plane of the convolution inputs holds every slot)
+};
+
 struct Slot {
+    int plane = 0;                  // recurrent models: the plane that holds the slot's convolution inputs
     int begin = 0, end = 0;         // resident positions [begin, end)
     std::vector<int32_t> pages;     // page id per page index (position / PAGE), -1 = none
 };
@@ -152,6 +172,10 @@ public:
     int step(const retro_step_row_v2 * rows2, const retro_step_row * rows1, size_t n_rows,
              retro_step_out_row_v2 * out2, retro_step_out_row * out1,
              int32_t * out_top_ids, float * out_top_logprobs, size_t n_top_stride);
+    // The same step without sampling: rows as in step(), none of which samples, and the logits of chosen tokens
+    // (token index[i] of row row[i]) in that order.
+    struct WantLogits { const uint32_t * row; const uint32_t * index; size_t n; float * out; };
+    int step_logits(const retro_step_row_v2 * rows, size_t n_rows, const WantLogits & want);
 
     bool seq_rm(int32_t slot, int32_t p0, int32_t p1);
     bool seq_cp(int32_t src, int32_t dst, int32_t p0, int32_t p1);
@@ -182,6 +206,7 @@ public:
     int adapter_load(const std::string & path, float scale, int32_t * out_id);
     // Rows of token_embd.weight of a model file, read from its header alone.
     static uint64_t vocab_size_of(const std::string & path) {
+        if (StackConfig::is_folder(path)) return (uint64_t)StackConfig::read(path).vocab;
         GgufFile file(path);
         return (uint64_t)file.require("token_embd.weight").ne[1];
     }
@@ -208,6 +233,7 @@ public:
     uint64_t weights_version() const { return weights_version_; }
     uint64_t fingerprint() const { return fingerprint_; }
     uint64_t steps_run() const { return steps_run_; }
+    bool is_hybrid() const { return stack_ && stack_->recurrent(); }
 
     // Event timing of kernel categories: level 0 off, 1 attention only, 2 all.
     void profile_level(int level) { prof_level_ = level; }
@@ -224,6 +250,10 @@ public:
     int debug_pack(int32_t * tok, int32_t * pos, int32_t * seq, int32_t * cell, int32_t * out_index,
                    int32_t * last_index, size_t cap_tokens, size_t cap_rows, int32_t * counts);
     int debug_page_table(int32_t slot, int32_t * out, size_t cap, size_t * out_n);
+    // Layer-stack models: keeps the residual stream after every layer of each step while on; read returns the last
+    // step's, [layer][token][width].
+    int debug_keep_residual(bool on);
+    int debug_read_residual(float * out, size_t n_floats, size_t * out_tokens);
 
 private:
     struct RowView {      // the fields both row versions share
@@ -247,6 +277,16 @@ private:
     void upload_f32(const TensorInfo * t, DevBuf & out, size_t expect);
     void upload_experts(const TensorInfo & t, int64_t K, int64_t N, DevWeight & out);
     void build_buffers();
+    void build_pack_buffers();
+    void build_step_buffers();
+
+    // layer-stack models (engine_stack.cpp)
+    void load_stack(const std::string & path);
+    void build_stack();
+    void forward_stack(int T, int n_out);
+    void plan_stack(const std::vector<RowView> & rows, const std::vector<std::pair<int, int>> & before);
+    size_t stack_plan_bytes() const;
+    void stage_stack_plan(uint8_t * host, const uint8_t * device);
 
     int32_t alloc_page();
     void release_page(int32_t page);
@@ -254,6 +294,22 @@ private:
     void set_page(int32_t slot, int idx, int32_t page);
     void clear_slot(Slot & s, int32_t slot);
     void forward(int T, int n_out, int n_tiles, int n_items, bool one_token_rows, bool routed);
+    int run_step(const retro_step_row_v2 * rows2, const retro_step_row * rows1, size_t n_rows,
+                 retro_step_out_row_v2 * out2, retro_step_out_row * out1,
+                 int32_t * out_top_ids, float * out_top_logprobs, size_t n_top_stride, const WantLogits * want);
+
+    // What a cell of the cache consists of: one part per layer and kind, its values in natural order on the way in and
+    // out of snapshots and merges.
+    struct CachePart { int layer; bool v; size_t row_bytes; };
+    std::vector<CachePart> cache_parts_;
+    size_t cache_row_bytes_ = 0;            // of all parts
+    void cells_gather(const CachePart & part, const int32_t * cells, int n, void * out);
+    void cells_scatter(const CachePart & part, const int32_t * cells, int n, const void * in);
+    // Recurrent state of a slot beside the cache (zero floats for attention-only models).
+    size_t recurrent_floats() const { return recurrent_slot_floats_; }
+    void state_copy(int32_t src, int32_t dst);
+    void state_pack(int32_t slot, float * out);             // device -> host buffer of recurrent_floats()
+    void state_unpack(int32_t slot, const float * in);
 
     retro_engine_config cfg_ {};
     HParams hp_;
@@ -268,6 +324,28 @@ private:
     rk::KvStrides kv_strides_ {};   // layout of every KV pool
 
     hipStream_t stream_ = nullptr;
+
+    // layer-stack models: configuration, weights, state and the step's buffers
+    std::unique_ptr<StackConfig> stack_;
+    int arith_ = rk::ARITH_16;
+    std::vector<StackLayer> stack_layers_;
+    StackLayer::Matrix stack_head_;
+    DevBuf recurrent_slab_;
+    size_t recurrent_slot_floats_ = 0, conv_plane_floats_ = 0;
+    DevBuf st_h_, st_proj_, st_cq_, st_q_, st_qa_, st_ol_, st_mix_, st_ff_, st_out_, st_partial_, st_xbc_, st_y_, st_chunk_;
+    int st_proj_ld_ = 0;
+    struct BlockPlan { int heads; int cols; size_t first, n; };    // attention blocks of the step for one head count
+    std::vector<BlockPlan> block_plans_;
+    std::vector<rk::LatentBlock> plan_blocks_;
+    std::vector<rk::SeqRun> plan_runs_;
+    std::vector<int32_t> plan_run_tok_;
+    int plan_max_run_ = 0;
+    const rk::LatentBlock * d_blocks_ = nullptr;
+    const rk::SeqRun * d_runs_ = nullptr;
+    const int32_t * d_run_tok_ = nullptr;
+    bool keep_residual_ = false;
+    DevBuf kept_residual_;
+    int kept_tokens_ = 0;
 
     // weights
     DevWeight tok_embd_;      // raw rows, gathered per token

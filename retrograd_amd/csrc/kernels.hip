@@ -1354,18 +1354,29 @@ __global__ __launch_bounds__(1024) void k_pack(const RowDesc * __restrict__ rows
     __shared__ int carry[3];
     __shared__ int len_count[MAX_SPLIT_PAGES + 1], len_base[MAX_SPLIT_PAGES + 1];
     __shared__ int row_len[1024];
+    __shared__ int long_rows[1024], long_out[1024], n_long;      // rows whose tokens the whole workgroup writes
     for (int i = threadIdx.x; i < n_upd; i += 1024) table[(size_t)upd[i].slot * max_pages + upd[i].index] = upd[i].page;
     if (threadIdx.x == 0) { carry[0] = 0; carry[1] = 0; carry[2] = 0; }
     __syncthreads();
+    auto write_token = [&](const RowDesc & d, int r, int i, int out_at) {
+        const int t = d.tok_off + i, p = d.pos0 + i;
+        o.tok[t] = toks[t];
+        o.pos[t] = p;
+        o.seq[t] = d.slot;
+        o.row[t] = r;
+        o.cell[t] = table[(size_t)d.slot * max_pages + p / PAGE] * PAGE + p % PAGE;
+        o.out_index[t] = (d.sample && i + 1 == d.n) ? out_at : -1;
+    };
 
     // rows in chunks of 1024: per-row tile / item / output counts -> bases
     for (int base = 0; base < n_rows; base += 1024) {
         const int r = base + threadIdx.x;
         int tiles = 0, items = 0, outs = 0;
         RowDesc d;
+        if (threadIdx.x == 0) n_long = 0;
         if (r < n_rows) {
             d = rows[r];
-            tiles = (d.n + qt - 1) / qt;
+            tiles = qt > 0 ? (d.n + qt - 1) / qt : 0;
             for (int j = 0; j < tiles; ++j) {
                 const int hi = d.pos0 + min(d.n, (j + 1) * qt);
                 items += n_kv * tile_splits(d.kv_begin, hi, o.split_pages);
@@ -1400,18 +1411,19 @@ __global__ __launch_bounds__(1024) void k_pack(const RowDesc * __restrict__ rows
                 item_at += n_kv * ns;
                 ++tile_at;
             }
-            for (int i = 0; i < d.n; ++i) {
-                const int t = d.tok_off + i;
-                const int p = d.pos0 + i;
-                o.tok[t] = toks[t];
-                o.pos[t] = p;
-                o.seq[t] = d.slot;
-                o.row[t] = r;
-                o.cell[t] = table[(size_t)d.slot * max_pages + p / PAGE] * PAGE + p % PAGE;
-                o.out_index[t] = (d.sample && i + 1 == d.n) ? out_at : -1;
+            if (d.n > 8) {
+                const int at = atomicAdd(&n_long, 1);
+                long_rows[at] = r;
+                long_out[at] = out_at;
+            } else {
+                for (int i = 0; i < d.n; ++i) write_token(d, r, i, out_at);
             }
         }
         __syncthreads();
+        for (int k = 0; k < n_long; ++k) {
+            const RowDesc ld = rows[long_rows[k]];
+            for (int i = threadIdx.x; i < ld.n; i += 1024) write_token(ld, long_rows[k], i, long_out[k]);
+        }
         // rows past n_rows contribute zero, so the last thread's inclusive
         // sums are the chunk totals
         if (threadIdx.x == 1023) {

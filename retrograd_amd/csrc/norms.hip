@@ -1,0 +1,77 @@
+// Row norms of layer-stack models: the residual stream (completed with the K-slices the product before left) through an
+// RMS or layer norm into activations. Statistics in f32, two passes over the row held in LDS.
+#include "stack_dev.hpp"
+
+namespace rk {
+
+namespace {
+
+template <int ARITH, int KIND>
+__global__ __launch_bounds__(256) void k_norm_act(float * __restrict__ x, const float * __restrict__ w, int E, float eps,
+                                                  const int32_t * __restrict__ rows, void * __restrict__ act, int kf, Slices add) {
+    extern __shared__ float row[];
+    __shared__ float scratch[16];
+    const int t = rows ? rows[blockIdx.x] : (int)blockIdx.x;
+    float * xr = x + (size_t)t * E;
+    float sum = 0.0f;
+    for (int k = threadIdx.x; k < E; k += 256) {
+        float v = xr[k];
+        if (add.n > 0) {
+            float d = 0.0f;
+            for (int i = 0; i < add.n; ++i) d += add.data[(size_t)i * add.stride + (size_t)t * E + k];
+            v += d;
+            xr[k] = v;
+        }
+        row[k] = v;
+        sum += KIND == NORM_LAYER ? v : v * v;
+    }
+    sum = block_sum(sum, scratch);
+    float mean = 0.0f;
+    if constexpr (KIND == NORM_LAYER) {
+        mean = sum / (float)E;
+        float q = 0.0f;
+        for (int k = threadIdx.x; k < E; k += 256) { const float d = row[k] - mean; q += d * d; }
+        sum = block_sum(q, scratch);
+    }
+    const float inv = 1.0f / sqrtf(sum / (float)E + eps);
+    for (int k = 8 * threadIdx.x; k < E; k += 8 * 256) {
+        float v[8];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[i] = k + i < E ? (row[k + i] - mean) * inv * w[k + i] : 0.0f;
+        store_frag8<ARITH>(act, kf, blockIdx.x, k, v);
+    }
+}
+
+__global__ void k_add_slices(float * __restrict__ x, size_t n, Slices add) {
+    for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) {
+        float d = 0.0f;
+        for (int k = 0; k < add.n; ++k) d += add.data[(size_t)k * add.stride + i];
+        x[i] += d;
+    }
+}
+
+}  // namespace
+
+void norm_act(hipStream_t s, int arith, int kind, float * x, const float * w, int E, float eps, const int32_t * rows,
+              int n_rows, void * act, int act_kf, const Slices & add) {
+    if (n_rows <= 0) return;
+    const size_t lds = (size_t)E * 4;
+    const dim3 grid((unsigned)n_rows), block(256);
+    if (arith == ARITH_16) {
+        if (kind == NORM_LAYER) hipLaunchKernelGGL((k_norm_act<ARITH_16, NORM_LAYER>), grid, block, lds, s, x, w, E, eps, rows, act, act_kf, add);
+        else hipLaunchKernelGGL((k_norm_act<ARITH_16, NORM_RMS>), grid, block, lds, s, x, w, E, eps, rows, act, act_kf, add);
+    } else {
+        if (kind == NORM_LAYER) hipLaunchKernelGGL((k_norm_act<ARITH_32, NORM_LAYER>), grid, block, lds, s, x, w, E, eps, rows, act, act_kf, add);
+        else hipLaunchKernelGGL((k_norm_act<ARITH_32, NORM_RMS>), grid, block, lds, s, x, w, E, eps, rows, act, act_kf, add);
+    }
+    check_launch("norm_act");
+}
+
+void add_slices(hipStream_t s, float * x, int E, int T, const Slices & add) {
+    if (add.n <= 0 || T <= 0) return;
+    const size_t n = (size_t)T * E;
+    hipLaunchKernelGGL(k_add_slices, dim3((unsigned)std::min<size_t>((n + 255) / 256, 4096)), dim3(256), 0, s, x, n, add);
+    check_launch("add_slices");
+}
+
+}  // namespace rk

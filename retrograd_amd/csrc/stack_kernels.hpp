@@ -1,0 +1,158 @@
+// Launch interface of the kernels behind layer-stack models (safetensors checkpoints whose config lists every layer):
+// bf16-weight matrix products in two arithmetics, layer norm, latent attention, the state-space mixer.
+#pragma once
+
+#include "kernels.hpp"
+
+namespace rk {
+
+// The two arithmetics of a layer-stack model. ARITH_16: matrix products and the activations between kernels in
+// bfloat16 with f32 accumulation, the latent cache in f16. ARITH_32: everything in f32 (products on the f32 matrix
+// instruction; the stored bf16 weights widen exactly).
+enum : int { ARITH_16 = 2, ARITH_32 = 4 };       // the value is the bytes of an activation element
+
+// ---- dense matrices and activations in operand ("fragment") order -------------------------------
+// Rows (of a weight, or tokens of an activation buffer) in tiles of 16, columns in fragments of 32:
+//   [row / 16][k / 32][lane = 16 * ((k % 32) / 8) + row % 16][k % 8]
+// so that a wave's operand of a 16x16x32 product is one contiguous load. Padding rows and columns of weights are zero;
+// padding columns of activations only have to be finite. Activation buffers hold a multiple of FRAG_ROWS tokens.
+constexpr int FRAG_ROWS = 128;
+constexpr int frags_of(int k) { return (k + 31) / 32; }
+constexpr size_t frag_elems(int rows, int kf) { return (size_t)((rows + FRAG_ROWS - 1) / FRAG_ROWS) * FRAG_ROWS * (size_t)kf * 32; }
+constexpr size_t frag_weight_elems(int row_tiles, int kf) { return (size_t)row_tiles * (size_t)kf * 512; }
+
+// `batch` matrices of `tiles` row tiles (n true rows) and kf fragments, one behind the other, stored as bf16.
+struct DenseWeight {
+    const uint16_t * w = nullptr;
+    int n = 0, tiles = 0, kf = 0, batch = 1;
+    size_t bytes() const { return frag_weight_elems(tiles, kf) * 2 * (size_t)batch; }
+};
+// dst(row0 + r, k0 + k) = src[r * row_stride + k * k_stride] for r < rows, k < cols; dst has kf fragments per row tile.
+void dense_pack(hipStream_t s, const uint16_t * src, int rows, int cols, int64_t row_stride, int64_t k_stride,
+                uint16_t * dst, int kf, int row0, int k0);
+
+// Where a product's rows go. col0 + b * col_batch + n is the output column of row n of batch b.
+enum : int {
+    OUT_F32 = 0,        // f32 rows dst[t * ld + col] = scale * v
+    OUT_ACT,            // activations in fragment order, ld fragments per token tile: scale * v
+    OUT_ACT_RELU2,      // ... max(v, 0)^2
+    OUT_ACT_GATED,      // ... v * sigmoid(gate[t * ld_gate + b])
+    OUT_QUERY,          // rows [t][batch][ld] in the latent cache's element type (f16 or f32): scale * v
+    OUT_RESIDUAL,       // f32 rows dst[t * ld + col] += v
+};
+struct DenseOut {
+    int kind = OUT_F32;
+    void * dst = nullptr;
+    int ld = 0, col0 = 0, col_batch = 0;
+    float scale = 1.0f;
+    const float * gate = nullptr;
+    int ld_gate = 0;
+};
+struct DenseIn {
+    const void * x = nullptr;   // activations in fragment order
+    int kf = 0;                 // fragments per token tile of that buffer
+    int kf_batch = 0;           // batch b reads from fragment b * kf_batch on
+};
+// One product, or two with one weight buffer [first | second] along K whose results are scaled element by element and
+// added: v = scale1[n] * (W1 x1) + scale2[n] * (W2 x2) (kf1 fragments belong to the first; scale1 null: plain product).
+struct DenseJob {
+    DenseWeight w;
+    DenseIn x, x2;
+    int kf1 = 0;
+    const float * scale1 = nullptr, * scale2 = nullptr;
+    int split_tile = 0;         // row tiles below go to `a`, the others (their rows counted from there) to `b`
+    DenseOut a, b;
+    int n_a = 0;                // true rows of part a when there is a part b
+};
+// Runs the product over T tokens. Where `ws` (dense_workspace_floats() floats) is given and the output is OUT_RESIDUAL,
+// a decode-sized product may come back as K-slices for the next norm to add instead.
+size_t dense_workspace_floats();
+Slices dense(hipStream_t s, int arith, const DenseJob & job, int T, float * ws);
+
+// ---- norms ----------------------------------------------------------------------------------------
+enum : int { NORM_RMS = 0, NORM_LAYER = 1 };
+// act[i] = norm(x[rows[i]] (+ slices, written back)) * w; statistics and products in f32.
+void norm_act(hipStream_t s, int arith, int kind, float * x, const float * w, int E, float eps, const int32_t * rows,
+              int n_rows, void * act, int act_kf, const Slices & add);
+// x[t][:] += the slices, for a stream that is read elsewhere than in the next norm.
+void add_slices(hipStream_t s, float * x, int E, int T, const Slices & add);
+
+// ---- latent attention --------------------------------------------------------------------------------
+// A page of the latent cache: PAGE tokens x kf fragments of 32 columns, f16 or f32,
+//   [column / 32][token / 16][lane = 16 * ((column % 32) / 8) + token % 16][column % 8]
+constexpr size_t latent_page_elems(int kf) { return (size_t)kf * 32 * PAGE; }
+// Queries' latent: act_q = RMS norm of proj[t][0, q_rank) times q_w. With kv_w also the cached latent: RMS norm of
+// proj[t][kv_col, kv_col + kv_rank) times kv_w into cell[t] of the pool.
+struct LatentNorms {
+    const float * proj = nullptr;
+    int ld = 0, q_rank = 0, kv_col = 0, kv_rank = 0;
+    const float * q_w = nullptr, * kv_w = nullptr;
+    float eps = 0.0f;
+    void * act_q = nullptr;
+    int act_q_kf = 0;
+    void * pool = nullptr;
+    int pool_kf = 0;
+    const int32_t * cell = nullptr;
+};
+void latent_norms(hipStream_t s, int arith, const LatentNorms & a, int T);
+
+// Attention of absorbed queries over the cached latents. A block serves up to `block_cols` of the T x H query columns
+// (token-major) of one row of the step.
+struct LatentBlock { int32_t row, col0; };       // row of the step, first of its n * H columns
+struct LatentAttn {
+    const void * q = nullptr;      // [T][H][kf * 32], already scaled by scale * log2(e)
+    int H = 0, kf = 0, window = 0; // window 0: every earlier position
+    const RowDesc * rows = nullptr;
+    const LatentBlock * blocks = nullptr;
+    int n_blocks = 0, block_cols = 0, splits = 1;
+    const int32_t * table = nullptr;
+    int max_pages = 0;
+    const void * pool = nullptr;
+    float * partial = nullptr;     // [T * H][splits][kf * 32 + 2] when splits > 1
+    void * out = nullptr;          // activations: column h * kf * 32 + c
+    int out_kf = 0;
+};
+int latent_block_cols(int arith, int H, int n_tokens, int n_rows);
+// Workgroups that share a block's keys, given the longest resident span among the step's rows.
+int latent_splits(int arith, const LatentAttn & a, int max_resident);
+size_t latent_partial_floats(int T, int H, int kf, int splits);
+void latent_attention(hipStream_t s, int arith, const LatentAttn & a, int T);
+
+// Page copies and cell gathers of any pool of pages (elem bytes 2 or 4).
+void latent_copy_page(hipStream_t s, void * pool, size_t page_bytes, int src, int dst);
+void latent_cells(hipStream_t s, void * pool, int kf, int elem, const int32_t * cells, int n, void * rows, bool gather);
+
+// ---- state-space mixer (Mamba-2) ------------------------------------------------------------------------
+// The tokens of one sequence in a step, in order: seg_tok[start .. start + n) are flat token indices.
+struct SeqRun { int32_t slot, start, n, flags; };      // flags bit 0: the sequence starts here (state is zero), bit 1: the
+                                                       // plane of the slot's convolution inputs that holds the current ones
+struct MambaShape {
+    int heads = 0, vdim = 0, state = 0, groups = 0, taps = 0, norm_groups = 0;
+    constexpr int inner() const { return heads * vdim; }
+    constexpr int channels() const { return inner() + 2 * groups * state; }
+    constexpr int rows() const { return inner() + channels() + heads; }      // of the input projection
+};
+struct MambaJob {
+    MambaShape sh;
+    const float * proj = nullptr;  // [T][ld]: z | x | B | C | dt
+    int ld = 0;
+    const float * conv_w = nullptr, * conv_b = nullptr, * dt_bias = nullptr, * A_log = nullptr, * D = nullptr, * norm_w = nullptr;
+    float eps = 0.0f;
+    const SeqRun * runs = nullptr;
+    int n_runs = 0, max_run = 0;
+    const int32_t * run_tok = nullptr;
+    float * conv_state = nullptr;  // [2 planes][slots][taps - 1][channels]
+    size_t conv_plane = 0;         // floats of a plane
+    float * state = nullptr;       // [slots][heads][state][vdim]
+    float * xbc = nullptr;         // scratch [T][channels]
+    float * y = nullptr;           // scratch [T][inner]
+    float * chunk_ws = nullptr;    // scratch of long runs (mamba_chunk_floats)
+    void * out = nullptr;          // activations, inner wide
+    int out_kf = 0;
+};
+size_t mamba_chunk_floats(const MambaShape & sh, int T, int n_seq);
+void mamba_mix(hipStream_t s, int arith, const MambaJob & j, int T);
+// dst slot's state = src slot's (floats each), and zeroing.
+void copy_floats(hipStream_t s, const float * src, float * dst, size_t n);
+
+}  // namespace rk

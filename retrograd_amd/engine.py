@@ -165,6 +165,7 @@ KERNEL_SYMBOLS = [
     "retro_engine_debug_logits", "retro_engine_debug_kv", "retro_engine_debug_pack", "retro_engine_debug_pages",
     "retro_engine_debug_profile", "retro_engine_debug_profile_categories", "retro_engine_debug_profile_read",
     "retro_engine_debug_attention_timeline", "retro_engine_debug_attention_timeline_read", "retro_engine_debug_single_token_matvec",
+    "retro_engine_step_logits", "retro_engine_debug_keep_residual", "retro_engine_debug_read_residual",
 ]
 PROFILE_CATEGORIES = ["pack", "embed", "norm", "qkv", "rope", "attention", "combine", "o_proj", "gate_up", "swiglu",
                       "down", "head", "sample"]
@@ -193,6 +194,10 @@ def load_library() -> C.CDLL:
                                       _i32p, _f32p, C.c_size_t]
     lib.retro_engine_step_v2.argtypes = [C.c_void_p, C.POINTER(CStepRowV2), C.c_size_t, C.POINTER(CStepOutRowV2),
                                          _i32p, _f32p, C.c_size_t]
+    lib.retro_engine_step_logits.argtypes = [C.c_void_p, C.POINTER(CStepRowV2), C.c_size_t, C.POINTER(C.c_uint32),
+                                             C.POINTER(C.c_uint32), C.c_size_t, _f32p]
+    lib.retro_engine_debug_keep_residual.argtypes = [C.c_void_p, C.c_bool]
+    lib.retro_engine_debug_read_residual.argtypes = [C.c_void_p, _f32p, C.c_size_t, C.POINTER(C.c_size_t)]
     lib.retro_engine_generate_batch.argtypes = [C.c_void_p, _i32p, C.c_size_t, C.POINTER(CSamplingParams), C.c_size_t,
                                                 _i32p, _f32p, C.c_size_t, C.POINTER(C.c_size_t), _u8p]
     lib.retro_engine_generate_continuous_batch.argtypes = [C.c_void_p, C.POINTER(CGenerationSequence), C.c_size_t,
@@ -515,6 +520,42 @@ class Engine:
         if status != 0:
             _raise(status)
         out.n_rows = n
+
+    def step_logits(self, rows: Sequence[tuple], want: Sequence[tuple]) -> np.ndarray:
+        """A step that samples nothing: rows of (slot, tokens, pos0), and the logits [len(want), vocab] of the tokens
+        (row, index in the row) of `want`."""
+        n = len(rows)
+        ffi = (CStepRowV2 * max(n, 1))()
+        keep = []
+        for f, (slot, tokens, pos0) in zip(ffi, rows):
+            toks = np.ascontiguousarray(tokens, dtype=np.int32)
+            keep.append(toks)
+            f.struct_size = C.sizeof(CStepRowV2)
+            f.request, f.slot, f.tokens, f.n, f.pos0 = -1, slot, toks.ctypes.data_as(_i32p), toks.size, pos0
+            f.sample = False
+            f.sampling.struct_size = C.sizeof(CSamplingParamsV2)
+        places = np.ascontiguousarray(np.asarray(want, dtype=np.uint32).reshape(-1, 2).T)
+        out = np.empty((len(want), self.vocab_size()), np.float32)
+        u32p = C.POINTER(C.c_uint32)
+        status = self._lib.retro_engine_step_logits(self._h, ffi, n, places[0].ctypes.data_as(u32p),
+                                                    places[1].ctypes.data_as(u32p), len(want), out.ctypes.data_as(_f32p))
+        if status != 0:
+            _raise(status)
+        return out
+
+    def keep_residual(self, on: bool) -> None:
+        if self._lib.retro_engine_debug_keep_residual(self._h, on) != 0:
+            _raise(-1)
+
+    def residual(self, n_layer: int, width: int) -> np.ndarray:
+        """The residual stream after every layer of the last step: [n_layer, tokens, width]."""
+        n = C.c_size_t()
+        if self._lib.retro_engine_debug_read_residual(self._h, None, 0, C.byref(n)) != 0:
+            _raise(-1)
+        out = np.empty((n_layer, n.value, width), np.float32)
+        if self._lib.retro_engine_debug_read_residual(self._h, out.ctypes.data_as(_f32p), out.size, C.byref(n)) != 0:
+            _raise(-1)
+        return out
 
     @staticmethod
     def _check_rows(rows, lens, requests, pos0, sample, sp) -> None:
