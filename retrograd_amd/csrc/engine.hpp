@@ -160,7 +160,7 @@ struct Vocab {
 // Kernel categories of one step, for the optional event-based timing.
 enum ProfCat : int {
     PC_PACK = 0, PC_EMBED, PC_NORM, PC_QKV, PC_ROPE, PC_ATTN, PC_COMBINE, PC_OPROJ, PC_GATEUP, PC_SWIGLU,
-    PC_DOWN, PC_HEAD, PC_SAMPLE, PC_COUNT
+    PC_DOWN, PC_HEAD, PC_SAMPLE, PC_ABSORB, PC_SCAN, PC_COUNT
 };
 
 class Engine {
@@ -334,12 +334,12 @@ private:
     size_t recurrent_slot_floats_ = 0, conv_plane_floats_ = 0;
     DevBuf st_h_, st_proj_, st_cq_, st_q_, st_qa_, st_ol_, st_mix_, st_ff_, st_out_, st_partial_, st_xbc_, st_y_, st_chunk_;
     int st_proj_ld_ = 0;
-    struct BlockPlan { int heads; int cols; size_t first, n; };    // attention blocks of the step for one head count
+    struct BlockPlan { int heads, cols; size_t first, n; };    // attention blocks of the step for one head count and width
     std::vector<BlockPlan> block_plans_;
     std::vector<rk::LatentBlock> plan_blocks_;
     std::vector<rk::SeqRun> plan_runs_;
     std::vector<int32_t> plan_run_tok_;
-    int plan_max_run_ = 0;
+    int plan_max_run_ = 0, step_rows_ = 0;
     const rk::LatentBlock * d_blocks_ = nullptr;
     const rk::SeqRun * d_runs_ = nullptr;
     const int32_t * d_run_tok_ = nullptr;

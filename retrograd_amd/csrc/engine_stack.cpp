@@ -326,13 +326,14 @@ void Engine::plan_stack(const std::vector<RowView> & rows, const std::vector<std
     plan_runs_.clear();
     plan_run_tok_.clear();
     plan_max_run_ = 0;
+    step_rows_ = (int)rows.size();
     int total = 0;
     for (const RowView & r : rows) total += (int)r.n;
     for (const LayerSpec & sp : stack_->layers) {
         if (sp.mixer != Mixer::LATENT_ATTENTION) continue;
-        const int H = sp.latent.heads;
-        if (std::any_of(block_plans_.begin(), block_plans_.end(), [&](const BlockPlan & b) { return b.heads == H; })) continue;
-        BlockPlan plan{H, rk::latent_block_cols(arith_, H, total, (int)rows.size()), plan_blocks_.size(), 0};
+        const int H = sp.latent.heads, cols = rk::latent_block_cols(arith_, H, rk::frags_of(sp.latent.kv_rank), total, (int)rows.size());
+        if (std::any_of(block_plans_.begin(), block_plans_.end(), [&](const BlockPlan & b) { return b.heads == H && b.cols == cols; })) continue;
+        BlockPlan plan{H, cols, plan_blocks_.size(), 0};
         for (size_t r = 0; r < rows.size(); ++r)
             for (int64_t c = 0; c < (int64_t)rows[r].n * H; c += plan.cols) plan_blocks_.push_back({(int32_t)r, (int32_t)c});
         plan.n = plan_blocks_.size() - plan.first;
@@ -422,6 +423,8 @@ void Engine::forward_stack(int T, int n_out) {
             n.act_q = st_cq_.ptr; n.act_q_kf = rk::frags_of(a.q_rank);
             n.pool = k_pool_[(size_t)L.pool_layer].ptr; n.pool_kf = R; n.cell = pk_.cell;
             rk::latent_norms(stream_, arith_, n, T);
+            prof_end(PC_ROPE, pt);
+            pt = prof_begin(PC_ABSORB);
             rk::DenseJob uq;
             uq.w = L.uq.w;
             uq.x = {st_cq_.ptr, rk::frags_of(a.q_rank), 0};
@@ -433,10 +436,11 @@ void Engine::forward_stack(int T, int n_out) {
             uk.a.kind = rk::OUT_QUERY; uk.a.dst = st_qa_.ptr; uk.a.ld = R * 32; uk.a.col_batch = H;
             uk.a.scale = (float)((double)a.scale * 1.4426950408889634);      // the softmax runs on powers of two
             rk::dense(stream_, arith_, uk, T, ws);
-            prof_end(PC_ROPE, pt);
+            prof_end(PC_ABSORB, pt);
             pt = prof_begin(PC_ATTN);
             const BlockPlan * plan = nullptr;
-            for (const BlockPlan & b : block_plans_) if (b.heads == H) plan = &b;
+            const int cols = rk::latent_block_cols(arith_, H, R, T, step_rows_);
+            for (const BlockPlan & b : block_plans_) if (b.heads == H && b.cols == cols) plan = &b;
             rk::LatentAttn at;
             at.q = st_qa_.ptr; at.H = H; at.kf = R; at.window = a.window;
             at.rows = rows; at.blocks = d_blocks_ + plan->first; at.n_blocks = (int)plan->n; at.block_cols = plan->cols;
@@ -457,7 +461,7 @@ void Engine::forward_stack(int T, int n_out) {
             rk::dense(stream_, arith_, uv, T, ws);
             prof_end(PC_OPROJ, pt);
         } else {
-            pt = prof_begin(PC_ATTN);
+            pt = prof_begin(PC_SCAN);
             rk::MambaJob j;
             j.sh = sp.mamba;
             j.proj = proj; j.ld = ld;
@@ -469,7 +473,7 @@ void Engine::forward_stack(int T, int n_out) {
             j.xbc = st_xbc_.as<float>(); j.y = st_y_.as<float>(); j.chunk_ws = st_chunk_.as<float>();
             j.out = st_mix_.ptr; j.out_kf = KM;
             rk::mamba_mix(stream_, arith_, j, T);
-            prof_end(PC_ATTN, pt);
+            prof_end(PC_SCAN, pt);
         }
         pt = prof_begin(PC_DOWN);
         rk::DenseJob out;

@@ -116,6 +116,216 @@ __global__ __launch_bounds__(256) void k_latent_attention_any(LatentAttn a) {
     }
 }
 
+typedef __fp16 q4 __attribute__((ext_vector_type(4)));
+typedef __attribute__((address_space(3))) q4 lds_q4;
+
+// Matrix-core form over f16 latents of at most MAXKF fragments. A workgroup serves CT * WC * 16 query columns; WC waves
+// share a page (staged once into LDS, double buffered, by direct-to-LDS loads), WK such groups take pages in turn and
+// merge at the end. Scores S^T = C q'^T and outputs O^T = C^T P^T both read the page's one layout: the second product's
+// operand is its transpose, which the LDS transpose read delivers. With several splits (blockIdx.y) every one leaves an
+// unnormalised partial result.
+template <int MAXKF, int CT, int WC, int WK>
+__global__ __launch_bounds__(64 * WC * WK, 1) void k_latent_attention(LatentAttn a) {
+    extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
+    __shared__ float merge_ml[WC][CT][2][64];
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int wc = wave % WC, wk = wave / WC, g = lane >> 4;
+    const int kf = a.kf;
+    const int page_bytes = kf * 2048;
+    const LatentBlock blk = a.blocks[blockIdx.x];
+    const RowDesc row = a.rows[blk.row];
+    const int n_cols = row.n * a.H;
+    auto low_of = [&](int pos) { return a.window > 0 ? max(row.kv_begin, pos - a.window + 1) : row.kv_begin; };
+
+    // this lane's column of every column tile: its token and head, and the keys it sees
+    int col[CT], lo[CT], hi[CT], lo_max = 0, hi_min = 1 << 30;
+    h8 q[CT][MAXKF];
+#pragma unroll
+    for (int c = 0; c < CT; ++c) {
+        col[c] = blk.col0 + (wc * CT + c) * 16 + (lane & 15);
+        const int cc = min(col[c], n_cols - 1);
+        const int tok = cc / a.H, h = cc - tok * a.H;
+        hi[c] = row.pos0 + tok;
+        lo[c] = low_of(hi[c]);
+        lo_max = max(lo_max, lo[c]);
+        hi_min = min(hi_min, hi[c]);
+        const __half * qr = (const __half *)a.q + ((size_t)(row.tok_off + tok) * a.H + h) * (size_t)(kf * 32) + 8 * g;
+#pragma unroll
+        for (int j = 0; j < MAXKF; ++j) if (j < kf) q[c][j] = load_h8(qr + 32 * j);
+    }
+#pragma unroll
+    for (int o = 8; o > 0; o >>= 1) {
+        lo_max = max(lo_max, __shfl_xor(lo_max, o, 64));
+        hi_min = min(hi_min, __shfl_xor(hi_min, o, 64));
+    }
+    // the block's pages, dealt to the splits
+    const int last_tok = min(blk.col0 + a.block_cols, n_cols) - 1;
+    const int page_lo = low_of(row.pos0 + blk.col0 / a.H) / PAGE, page_hi = (row.pos0 + last_tok / a.H) / PAGE + 1;
+    const int n_all = page_hi - page_lo, sp = blockIdx.y;
+    const int first = page_lo + (int)((int64_t)n_all * sp / a.splits), end = page_lo + (int)((int64_t)n_all * (sp + 1) / a.splits);
+    const int n_iter = (end - first + WK - 1) / WK;
+    const int32_t * table = a.table + (size_t)row.slot * a.max_pages;
+    uint8_t * buf = lds + (size_t)wk * 2 * page_bytes;
+
+    auto stage = [&](int page, int b) {
+        if (page >= end) return;
+        const int id = __builtin_amdgcn_readfirstlane(table[page]);
+        const uint8_t * src = (const uint8_t *)a.pool + (size_t)id * page_bytes;
+        for (int ch = wc; ch < 2 * kf; ch += WC)
+            lds_dma16(src + ch * 1024, (uint32_t)lane * 16, lds_offset(buf + (size_t)b * page_bytes + ch * 1024));
+    };
+    f4 acc[CT][2 * MAXKF];
+    float m[CT], l[CT];
+#pragma unroll
+    for (int c = 0; c < CT; ++c) {
+        m[c] = -INFINITY;
+        l[c] = 0.0f;
+#pragma unroll
+        for (int d = 0; d < 2 * MAXKF; ++d) acc[c][d] = f4{0, 0, 0, 0};
+    }
+    stage(first + wk, 0);
+    const int idx = lane & 15;
+    const int tr_lane = ((((idx >> 1) & 1) * 16 + 4 * g + (idx >> 2)) * 8 + (idx & 1) * 4) * 2;       // bytes into a 1 KiB piece
+    for (int it = 0; it < n_iter; ++it) {
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads();
+        const int page = first + it * WK + wk;
+        stage(page + WK, (it + 1) & 1);
+        if (page >= end) continue;
+        const uint8_t * cur = buf + (size_t)(it & 1) * page_bytes;
+        f4 s[2][CT];
+#pragma unroll
+        for (int hf = 0; hf < 2; ++hf) {
+#pragma unroll
+            for (int c = 0; c < CT; ++c) s[hf][c] = f4{0, 0, 0, 0};
+#pragma unroll
+            for (int j = 0; j < MAXKF; ++j) {
+                if (j < kf) {
+                    const h8 k = *(const h8 *)(cur + (j * 2 + hf) * 1024 + lane * 16);
+#pragma unroll
+                    for (int c = 0; c < CT; ++c) s[hf][c] = __builtin_amdgcn_mfma_f32_16x16x32_f16(k, q[c][j], s[hf][c], 0, 0, 0);
+                }
+            }
+        }
+        const int key0 = page * PAGE;
+        const bool inside = key0 >= lo_max && key0 + PAGE - 1 <= hi_min;
+        h8 p[CT];
+#pragma unroll
+        for (int c = 0; c < CT; ++c) {
+            if (!inside) {
+#pragma unroll
+                for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) {
+                        const int key = key0 + hf * 16 + 4 * g + i;
+                        if (key < lo[c] || key > hi[c]) s[hf][c][i] = -INFINITY;
+                    }
+            }
+            float mx = fmaxf(fmaxf(fmaxf(s[0][c][0], s[0][c][1]), fmaxf(s[0][c][2], s[0][c][3])),
+                             fmaxf(fmaxf(s[1][c][0], s[1][c][1]), fmaxf(s[1][c][2], s[1][c][3])));
+            mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+            mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+            const float m2 = fmaxf(m[c], mx), base = m2 == -INFINITY ? 0.0f : m2;
+            if (__ballot(m2 > m[c])) {
+                const float f = exp2f(m[c] - base);
+                l[c] *= f;
+#pragma unroll
+                for (int d = 0; d < 2 * MAXKF; ++d) acc[c][d] *= f;
+                m[c] = m2;
+            }
+#pragma unroll
+            for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const float e = exp2f(s[hf][c][i] - base);
+                    l[c] += e;
+                    p[c][hf * 4 + i] = (_Float16)e;
+                }
+        }
+#pragma unroll
+        for (int d = 0; d < 2 * MAXKF; ++d) {
+            if ((d >> 1) < kf) {
+                const uint8_t * v0 = cur + (d >> 1) * 2048 + (d & 1) * 512 + tr_lane;
+                union { q4 half[2]; h8 all; } v;
+                v.half[0] = __builtin_amdgcn_ds_read_tr16_b64_v4f16((lds_q4 *)(v0));
+                v.half[1] = __builtin_amdgcn_ds_read_tr16_b64_v4f16((lds_q4 *)(v0 + 1024));
+#pragma unroll
+                for (int c = 0; c < CT; ++c) acc[c][d] = __builtin_amdgcn_mfma_f32_16x16x32_f16(v.all, p[c], acc[c][d], 0, 0, 0);
+            }
+        }
+    }
+#pragma unroll
+    for (int c = 0; c < CT; ++c) {
+        l[c] += __shfl_xor(l[c], 16, 64);
+        l[c] += __shfl_xor(l[c], 32, 64);
+    }
+    if constexpr (WK > 1) {       // the groups' results, one after the other, into the first group's
+        static_assert(WK == 2 && CT == 1);
+        __syncthreads();
+        f4 * park = (f4 *)lds + (size_t)wc * 2 * kf * 64;
+        if (wk == 1) {
+            merge_ml[wc][0][0][lane] = m[0];
+            merge_ml[wc][0][1][lane] = l[0];
+#pragma unroll
+            for (int d = 0; d < 2 * MAXKF; ++d) if ((d >> 1) < kf) park[d * 64 + lane] = acc[0][d];
+        }
+        __syncthreads();
+        if (wk == 1) return;
+        const float mo = merge_ml[wc][0][0][lane], lo2 = merge_ml[wc][0][1][lane];
+        const float m2 = fmaxf(m[0], mo), base = m2 == -INFINITY ? 0.0f : m2;
+        const float f0 = exp2f(m[0] - base), f1 = exp2f(mo - base);
+        l[0] = l[0] * f0 + lo2 * f1;
+        m[0] = m2;
+#pragma unroll
+        for (int d = 0; d < 2 * MAXKF; ++d) if ((d >> 1) < kf) acc[0][d] = acc[0][d] * f0 + park[d * 64 + lane] * f1;
+    }
+#pragma unroll
+    for (int c = 0; c < CT; ++c) {
+        if (col[c] >= min(blk.col0 + a.block_cols, n_cols)) continue;
+        const int tok = col[c] / a.H, h = col[c] - tok * a.H, t = row.tok_off + tok;
+        if (a.splits > 1) {
+            float * o = a.partial + (((size_t)t * a.H + h) * a.splits + sp) * (size_t)(kf * 32 + 4);
+            if (g == 0) { o[kf * 32] = m[c]; o[kf * 32 + 1] = l[c]; }
+#pragma unroll
+            for (int d = 0; d < 2 * MAXKF; ++d) if ((d >> 1) < kf) *(f4 *)(o + d * 16 + 4 * g) = acc[c][d];
+        } else {
+            const float inv = 1.0f / l[c];
+#pragma unroll
+            for (int d = 0; d < 2 * MAXKF; ++d) {
+                if ((d >> 1) < kf) {
+                    const f4 v = acc[c][d] * inv;
+                    uint2 u;
+                    u.x = (uint32_t)bf16_bits(v[0]) | ((uint32_t)bf16_bits(v[1]) << 16);
+                    u.y = (uint32_t)bf16_bits(v[2]) | ((uint32_t)bf16_bits(v[3]) << 16);
+                    *(uint2 *)((uint16_t *)a.out + frag_at(t, h * kf * 32 + d * 16 + 4 * g, a.out_kf)) = u;
+                }
+            }
+        }
+    }
+}
+
+// Merges the splits of one query column: a wave per column, eight latent columns per lane and pass.
+__global__ __launch_bounds__(64) void k_latent_combine(LatentAttn a) {
+    const int R = a.kf * 32, t = blockIdx.x / a.H, h = blockIdx.x - t * a.H;
+    const float * p = a.partial + (size_t)blockIdx.x * a.splits * (R + 4);
+    float m = -INFINITY;
+    for (int s = 0; s < a.splits; ++s) m = fmaxf(m, p[(size_t)s * (R + 4) + R]);
+    float l = 0.0f;
+    for (int s = 0; s < a.splits; ++s) l += p[(size_t)s * (R + 4) + R + 1] * exp2f(p[(size_t)s * (R + 4) + R] - m);
+    const float inv = 1.0f / l;
+    for (int k = 8 * (int)threadIdx.x; k < R; k += 512) {
+        f4 x = {0, 0, 0, 0}, y = {0, 0, 0, 0};
+        for (int s = 0; s < a.splits; ++s) {
+            const float * o = p + (size_t)s * (R + 4);
+            const float f = exp2f(o[R] - m) * inv;
+            x += *(const f4 *)(o + k) * f;
+            y += *(const f4 *)(o + k + 4) * f;
+        }
+        const float v[8] = {x[0], x[1], x[2], x[3], y[0], y[1], y[2], y[3]};
+        store_frag8<ARITH_16>(a.out, a.out_kf, t, h * R + k, v);
+    }
+}
+
 __global__ void k_copy16(const u4 * __restrict__ src, u4 * __restrict__ dst, size_t n) {
     for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) dst[i] = src[i];
 }
@@ -148,13 +358,60 @@ void latent_norms(hipStream_t s, int arith, const LatentNorms & a, int T) {
     check_launch("latent_norms");
 }
 
-int latent_block_cols(int arith, int H, int n_tokens, int n_rows) { return 1; }
-int latent_splits(int arith, const LatentAttn & a, int max_resident) { return 1; }
-size_t latent_partial_floats(int T, int H, int kf, int splits) { return splits > 1 ? (size_t)T * H * splits * (kf * 32 + 2) : 0; }
+namespace {
+constexpr int kMatrixKf = 16;       // widest latent (in fragments) of the matrix-core kernel
+bool on_matrix_cores(int arith, int kf) { return arith == ARITH_16 && kf <= kMatrixKf; }
+
+template <int MAXKF, int CT, int WC, int WK> void launch_attention(hipStream_t s, const LatentAttn & a) {
+    const size_t lds = (size_t)WK * 2 * a.kf * 2048;
+    auto kernel = k_latent_attention<MAXKF, CT, WC, WK>;
+    static const bool allowed = hipFuncSetAttribute((const void *)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, WK * 2 * MAXKF * 2048) == hipSuccess;
+    if (!allowed) throw std::runtime_error("latent attention: the page buffers do not fit the LDS");
+    hipLaunchKernelGGL(kernel, dim3((unsigned)a.n_blocks, (unsigned)a.splits), dim3(64 * WC * WK), lds, s, a);
+}
+template <int MAXKF> void launch_columns(hipStream_t s, const LatentAttn & a) {
+    switch (a.block_cols) {
+        case 16: launch_attention<MAXKF, 1, 1, 2>(s, a); break;
+        case 32: launch_attention<MAXKF, 1, 2, 2>(s, a); break;
+        case 64: launch_attention<MAXKF, 1, 4, 1>(s, a); break;
+        case 128:
+            if constexpr (MAXKF <= 8) { launch_attention<MAXKF, 2, 4, 1>(s, a); break; }      // wider: the registers do not suffice
+            [[fallthrough]];
+        default: throw std::runtime_error("latent attention: no kernel for this many columns per block");
+    }
+}
+}  // namespace
+
+int latent_block_cols(int arith, int H, int kf, int n_tokens, int n_rows) {
+    if (!on_matrix_cores(arith, kf)) return 1;
+    if (n_tokens == n_rows) return H <= 16 ? 16 : H <= 32 ? 32 : 64;      // one token per row
+    return kf <= 8 && (int64_t)n_tokens * H >= 256 * 128 ? 128 : 64;
+}
+
+int latent_splits(int arith, const LatentAttn & a, int max_resident) {
+    if (!on_matrix_cores(arith, a.kf)) return 1;
+    const int keys = a.window > 0 ? std::min(a.window, max_resident) : max_resident;
+    const int pages = (keys + PAGE - 1) / PAGE + 1, per = a.block_cols <= 32 ? 2 : 1;
+    return std::max(1, std::min({256 / std::max(a.n_blocks, 1), pages / per, 32}));
+}
+
+size_t latent_partial_floats(int T, int H, int kf, int splits) { return splits > 1 ? (size_t)T * H * splits * (kf * 32 + 4) : 0; }
 
 void latent_attention(hipStream_t s, int arith, const LatentAttn & a, int T) {
     if (a.n_blocks <= 0) return;
     if (a.kf * 32 > 1024) throw std::runtime_error("latent attention: latents of at most 1024 columns");
+    if (on_matrix_cores(arith, a.kf)) {
+        if (a.kf <= 2) launch_columns<2>(s, a);
+        else if (a.kf <= 4) launch_columns<4>(s, a);
+        else if (a.kf <= 8) launch_columns<8>(s, a);
+        else launch_columns<16>(s, a);
+        check_launch("latent_attention");
+        if (a.splits > 1) {
+            hipLaunchKernelGGL(k_latent_combine, dim3((unsigned)(T * a.H)), dim3(64), 0, s, a);
+            check_launch("latent_combine");
+        }
+        return;
+    }
     const size_t lds = ((size_t)a.kf * 32 + 256) * 4;
     const dim3 grid((unsigned)a.n_blocks);
     if (arith == ARITH_16) hipLaunchKernelGGL(k_latent_attention_any<ARITH_16>, grid, dim3(256), lds, s, a);

@@ -108,11 +108,11 @@ struct LatentAttn {
     const int32_t * table = nullptr;
     int max_pages = 0;
     const void * pool = nullptr;
-    float * partial = nullptr;     // [T * H][splits][kf * 32 + 2] when splits > 1
+    float * partial = nullptr;     // [T * H][splits][kf * 32 + 4]: values, maximum, sum; when splits > 1
     void * out = nullptr;          // activations: column h * kf * 32 + c
     int out_kf = 0;
 };
-int latent_block_cols(int arith, int H, int n_tokens, int n_rows);
+int latent_block_cols(int arith, int H, int kf, int n_tokens, int n_rows);
 // Workgroups that share a block's keys, given the longest resident span among the step's rows.
 int latent_splits(int arith, const LatentAttn & a, int max_resident);
 size_t latent_partial_floats(int T, int H, int kf, int splits);

@@ -1,0 +1,147 @@
+"""Random-weight checkpoint folders (config.json + model.safetensors) of layer-stack models, for benchmarks and tests:
+the tensors a configuration asks for, values that keep activations of order one, and the safetensors writer."""
+
+from __future__ import annotations
+
+import json
+import struct
+from pathlib import Path
+
+import numpy as np
+
+
+def latent_layer(heads, dim, vdim, q_rank, kv_rank, window, ff, scale=None, kv_from=None):
+    m = {"heads": heads, "dim": dim, "vdim": vdim, "q_rank": q_rank, "kv_rank": kv_rank,
+         "scale": dim ** -0.5 if scale is None else scale, "mask": {"size": window}}
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return {"type": "latent_attention", "mixer": m, "mlp": {"kind": "dense", "ff": ff} if ff else None}
+
+
+def mamba2_layer(heads, vdim, state, groups, conv, norm_groups, ff):
+    m = {"heads": heads, "vdim": vdim, "state": state, "groups": groups, "conv": conv, "norm_groups": norm_groups}
+    return {"type": "mamba2", "mixer": m, "mlp": {"kind": "dense", "ff": ff} if ff else None}
+
+
+def dibosun(width, vocab, layers, eps=1e-5):
+    return {"architecture": "Dibosun", "width": width, "vocab": vocab, "norm": {"eps": eps}, "layers": layers}
+
+
+def tensor_shapes(cfg) -> dict:
+    E = cfg["width"]
+    out = {"embed": (cfg["vocab"], E)}
+    for i, layer in enumerate(cfg["layers"]):
+        p, m = "l%d." % i, layer["mixer"]
+        out[p + "norm1"] = (E,)
+        if layer["type"] == "latent_attention":
+            H = m["heads"]
+            out[p + "mix.dq"] = (m["q_rank"], E)
+            out[p + "mix.dq.norm"] = (m["q_rank"],)
+            out[p + "mix.uq"] = (H * m["dim"], m["q_rank"])
+            if m.get("kv_from") is None:
+                out[p + "mix.dkv"] = (m["kv_rank"], E)
+                out[p + "mix.dkv.norm"] = (m["kv_rank"],)
+            out[p + "mix.uk"] = (H * m["dim"], m["kv_rank"])
+            out[p + "mix.uv"] = (H * m["vdim"], m["kv_rank"])
+            out[p + "mix.g"] = (H, E)
+            out[p + "mix.o"] = (E, H * m["vdim"])
+        else:
+            inner, bc = m["heads"] * m["vdim"], 2 * m["groups"] * m["state"]
+            out[p + "mix.in"] = (2 * inner + bc + m["heads"], E)
+            out[p + "mix.conv"] = (inner + bc, m["conv"])
+            out[p + "mix.conv.b"] = (inner + bc,)
+            for name in ("dt_bias", "A_log", "D"):
+                out[p + "mix." + name] = (m["heads"],)
+            out[p + "mix.norm"] = (inner,)
+            out[p + "mix.o"] = (E, inner)
+        out[p + "ls1"] = (E,)
+        if layer.get("mlp"):
+            out[p + "mlp.up"] = (layer["mlp"]["ff"], E)
+            out[p + "mlp.down"] = (E, layer["mlp"]["ff"])
+            out[p + "ls2"] = (E,)
+    out["final.norm"] = (E,)
+    return out
+
+
+def mean_and_std(name, shape):
+    """Of a tensor's normal distribution."""
+    leaf = name.rsplit(".", 1)[-1]
+    if leaf == "dt_bias":
+        return -2.0, 0.7
+    if leaf == "A_log":
+        return -0.5, 1.0
+    if leaf == "D" or leaf == "norm" or leaf.startswith("norm") or leaf.startswith("ls"):
+        return 0.9, 0.2
+    if leaf == "b":
+        return 0.0, 0.1
+    if leaf == "conv":
+        return 0.0, 0.5
+    if name == "embed":
+        return 0.0, 1.0
+    return 0.0, shape[-1] ** -0.5
+
+
+def _header(items):
+    head, at = {}, 0
+    for name, shape in items.items():
+        n = 2 * int(np.prod(shape))
+        head[name] = {"dtype": "BF16", "shape": list(shape), "data_offsets": [at, at + n]}
+        at += n
+    raw = json.dumps(head).encode()
+    raw += b" " * (-len(raw) % 8)
+    return struct.pack("<Q", len(raw)) + raw
+
+
+def to_bf16(x) -> np.ndarray:
+    """f32 -> bf16 bits, to nearest even."""
+    b = np.ascontiguousarray(x, np.float32).view(np.uint32).astype(np.uint64)
+    return ((b + 0x7FFF + ((b >> 16) & 1)) >> 16).astype(np.uint16)
+
+
+def from_bf16(b) -> np.ndarray:
+    return (np.asarray(b, np.uint32) << 16).view(np.float32)
+
+
+def random_tensors(cfg, seed) -> dict:
+    """name -> f32 array whose values are exact in bf16."""
+    rng = np.random.default_rng(seed)
+    out = {}
+    for name, shape in tensor_shapes(cfg).items():
+        mean, std = mean_and_std(name, shape)
+        out[name] = from_bf16(to_bf16(mean + std * rng.standard_normal(shape)))
+    return out
+
+
+def write_checkpoint(folder, cfg, tensors) -> Path:
+    """The folder with the given tensors (values exact in bf16)."""
+    folder = Path(folder)
+    folder.mkdir(parents=True, exist_ok=True)
+    (folder / "config.json").write_text(json.dumps(cfg))
+    with open(folder / "model.safetensors", "wb") as f:
+        f.write(_header({k: v.shape for k, v in tensors.items()}))
+        for v in tensors.values():
+            f.write(to_bf16(v).tobytes())
+    return folder
+
+
+def write_random_checkpoint(folder, cfg, seed, device="cuda") -> Path:
+    """A large random checkpoint, generated tensor by tensor with torch."""
+    import torch
+
+    folder = Path(folder)
+    folder.mkdir(parents=True, exist_ok=True)
+    (folder / "config.json").write_text(json.dumps(cfg))
+    gen = torch.Generator(device=device).manual_seed(seed)
+    shapes = tensor_shapes(cfg)
+    with open(folder / "model.safetensors", "wb") as f:
+        f.write(_header(shapes))
+        for name, shape in shapes.items():
+            mean, std = mean_and_std(name, shape)
+            t = torch.empty(shape, device=device, dtype=torch.float32).normal_(mean, std, generator=gen).to(torch.bfloat16)
+            f.write(t.view(torch.int16).cpu().numpy().tobytes())
+    return folder
+
+
+def matrix_bytes(cfg) -> int:
+    """Bytes of the matrices one step streams (the embedding counted once, as the output head)."""
+    return sum(2 * int(np.prod(s)) for n, s in tensor_shapes(cfg).items() if len(s) == 2 and not n.endswith(".conv"))
