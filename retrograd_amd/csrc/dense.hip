@@ -17,73 +17,67 @@ struct DenseArgs {
     size_t slice;
 };
 
-__device__ __forceinline__ void store_out(const DenseOut & o, int arith, int t, int b, int n, int n_end, f4 v) {
+// One compiled form per pair of output kinds (part a, part b): a kernel that chose among all of them at run time would
+// spend more on fetching its epilogue's instructions than on a product of a few hundred columns.
+template <int KIND, int ARITH>
+__device__ __forceinline__ void store_out(const DenseOut & o, int t, int b, int n, int n_end, f4 v) {
     // rows n .. n + 3 of token t (those below n_end are real)
-    const int col = o.col0 + b * o.col_batch + n;
-    const int cnt = n_end - n < 4 ? n_end - n : 4;
+    const int cnt = n_end - n;
     if (cnt <= 0) return;
-    switch (o.kind) {
-        case OUT_ACT_RELU2:
+    if constexpr (KIND == OUT_ACT_RELU2) {
 #pragma unroll
-            for (int i = 0; i < 4; ++i) { const float r = fmaxf(v[i], 0.0f); v[i] = r * r; }
-            break;
-        case OUT_ACT_GATED: {
-            const float g = o.gate[(size_t)t * o.ld_gate + b];
-            const float sg = 1.0f / (1.0f + expf(-g));
-#pragma unroll
-            for (int i = 0; i < 4; ++i) v[i] *= sg;
-            break;
-        }
-        default:
-#pragma unroll
-            for (int i = 0; i < 4; ++i) v[i] *= o.scale;
+        for (int i = 0; i < 4; ++i) { const float r = fmaxf(v[i], 0.0f); v[i] = r * r; }
+    } else if constexpr (KIND == OUT_ACT_GATED) {
+        v *= 1.0f / (1.0f + expf(-o.gate[(size_t)t * o.ld_gate + b]));
+    } else if constexpr (KIND != OUT_RESIDUAL) {
+        v *= o.scale;
     }
-    if (o.kind == OUT_F32 || o.kind == OUT_RESIDUAL) {
-        float * y = (float *)o.dst + (size_t)t * o.ld + col;
-        if (cnt == 4 && (((size_t)t * o.ld + col) & 3) == 0) {
-            if (o.kind == OUT_RESIDUAL) v += *(const f4 *)y;
+    const int col = o.col0 + (KIND == OUT_QUERY ? 0 : b * o.col_batch) + n;
+    if constexpr (KIND == OUT_F32 || KIND == OUT_RESIDUAL) {
+        const size_t at = (size_t)t * o.ld + col;
+        float * y = (float *)o.dst + at;
+        if (cnt >= 4 && (at & 3) == 0) {
+            if constexpr (KIND == OUT_RESIDUAL) v += *(const f4 *)y;
             *(f4 *)y = v;
         } else {
-            for (int i = 0; i < cnt; ++i) y[i] = o.kind == OUT_RESIDUAL ? y[i] + v[i] : v[i];
-        }
-        return;
-    }
-    if (o.kind == OUT_QUERY) {
-        const size_t at = ((size_t)t * o.col_batch + b) * o.ld + n;      // col_batch holds the number of batches here
-        if (arith == ARITH_16) {
-            __half * q = (__half *)o.dst + at;
-            if (cnt == 4) {
-                union { __half h[4]; uint2 u; } w;
 #pragma unroll
-                for (int i = 0; i < 4; ++i) w.h[i] = sat_half(v[i]);
-                *(uint2 *)q = w.u;
-            } else for (int i = 0; i < cnt; ++i) q[i] = sat_half(v[i]);
-        } else {
-            float * q = (float *)o.dst + at;
-            for (int i = 0; i < cnt; ++i) q[i] = v[i];
+            for (int i = 0; i < 4; ++i) if (i < cnt) y[i] = KIND == OUT_RESIDUAL ? y[i] + v[i] : v[i];
         }
-        return;
-    }
-    // activations: four consecutive columns share a group of eight when the first is a multiple of four
-    if (arith == ARITH_16) {
-        uint16_t * a = (uint16_t *)o.dst;
-        if (cnt == 4 && (col & 3) == 0) {
+    } else if constexpr (KIND == OUT_QUERY) {
+        const size_t at = ((size_t)t * o.col_batch + b) * o.ld + n;      // col_batch holds the number of batches here
+        if constexpr (ARITH == ARITH_16) {                               // whole fragments: n_end and ld are multiples of 32
+            union { __half h[4]; uint2 u; } w;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) w.h[i] = sat_half(v[i]);
+            *(uint2 *)((__half *)o.dst + at) = w.u;
+        } else {
+            *(f4 *)((float *)o.dst + at) = v;
+        }
+    } else if (cnt >= 4 && (col & 3) == 0) {       // activations: four columns from a multiple of four share a group of eight
+        if constexpr (ARITH == ARITH_16) {
             uint2 u;
             u.x = (uint32_t)bf16_bits(v[0]) | ((uint32_t)bf16_bits(v[1]) << 16);
             u.y = (uint32_t)bf16_bits(v[2]) | ((uint32_t)bf16_bits(v[3]) << 16);
-            *(uint2 *)(a + frag_at(t, col, o.ld)) = u;
-        } else for (int i = 0; i < cnt; ++i) a[frag_at(t, col + i, o.ld)] = bf16_bits(v[i]);
+            *(uint2 *)((uint16_t *)o.dst + frag_at(t, col, o.ld)) = u;
+        } else {
+            *(f4 *)((float *)o.dst + frag_at(t, col, o.ld)) = v;
+        }
     } else {
-        float * a = (float *)o.dst;
-        if (cnt == 4 && (col & 3) == 0) *(f4 *)(a + frag_at(t, col, o.ld)) = v;
-        else for (int i = 0; i < cnt; ++i) a[frag_at(t, col + i, o.ld)] = v[i];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            if (i >= cnt) break;
+            const size_t at = frag_at(t, col + i, o.ld);
+            if constexpr (ARITH == ARITH_16) ((uint16_t *)o.dst)[at] = bf16_bits(v[i]);
+            else ((float *)o.dst)[at] = v[i];
+        }
     }
 }
 
-// Rows tile * 16 + 4 g .. + 3 of token t to the part they belong to.
-__device__ __forceinline__ void store_rows(const DenseJob & j, int arith, int t, int b, int tile, int g, const f4 & v) {
-    if (tile < j.split_tile) store_out(j.a, arith, t, b, tile * 16 + 4 * g, j.n_a, v);
-    else store_out(j.b, arith, t, b, (tile - j.split_tile) * 16 + 4 * g, j.w.n - j.split_tile * 16, v);
+// Rows tile * 16 + 4 g .. + 3 of token t to the part they belong to (KB < 0: there is only part a).
+template <int KA, int KB, int ARITH>
+__device__ __forceinline__ void store_rows(const DenseJob & j, int t, int b, int tile, int g, const f4 & v) {
+    if (KB < 0 || tile < j.split_tile) store_out<KA, ARITH>(j.a, t, b, tile * 16 + 4 * g, j.n_a, v);
+    else if constexpr (KB >= 0) store_out<KB, ARITH>(j.b, t, b, (tile - j.split_tile) * 16 + 4 * g, j.w.n - j.split_tile * 16, v);
 }
 
 template <typename TA> struct Operand;      // one lane's eight activation values of a fragment
@@ -111,8 +105,9 @@ __device__ __forceinline__ void mac(f4 & acc, const b8 & w, const Operand<float>
 
 // Operands straight from memory to registers: a wave multiplies RT row tiles with CT token tiles; KW waves of the
 // workgroup share the rows and split K, RW sets of them split the rows.
-template <typename TA, int RT, int CT, int KW, int RW, bool DUAL>
+template <typename TA, int KA, int KB, int RT, int CT, int KW, int RW>
 __global__ __launch_bounds__(64 * KW * RW) void k_dense(DenseArgs A) {
+    constexpr bool DUAL = KA == OUT_RESIDUAL;
     constexpr int U = sizeof(TA) == 4 ? 2 : (RT * CT >= 8 ? 2 : 4);      // fragments in flight per operand
     const DenseJob & j = A.j;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -215,7 +210,7 @@ __global__ __launch_bounds__(64 * KW * RW) void k_dense(DenseArgs A) {
         }
         if (kw != 0) return;
     }
-    const int arith = (int)sizeof(TA);
+    constexpr int ARITH = (int)sizeof(TA);
 #pragma unroll
     for (int r = 0; r < RT; ++r) {
         const int tile = tile0 + r;
@@ -224,13 +219,13 @@ __global__ __launch_bounds__(64 * KW * RW) void k_dense(DenseArgs A) {
         for (int c = 0; c < CT; ++c) {
             const int t = (tok_tile0 + c) * 16 + (lane & 15);
             if (t >= A.T) continue;
-            if (A.ksplit > 1) {
+            if (DUAL && A.ksplit > 1) {
                 const int n = tile * 16 + 4 * (lane >> 4);
                 float * p = A.partial + (size_t)ks * A.slice + (size_t)t * j.w.n + n;
                 if (n + 4 <= j.w.n && (j.w.n & 3) == 0) *(f4 *)p = acc[r][c];
                 else for (int i = 0; i < 4 && n + i < j.w.n; ++i) p[i] = acc[r][c][i];
             } else {
-                store_rows(j, arith, t, b, tile, lane >> 4, acc[r][c]);
+                store_rows<KA, KB, ARITH>(j, t, b, tile, lane >> 4, acc[r][c]);
             }
         }
     }
@@ -245,18 +240,172 @@ __global__ void k_dense_pack(const uint16_t * __restrict__ src, int rows, int co
     }
 }
 
-template <typename TA, int RT, int CT, int KW, int RW>
-void launch(hipStream_t s, DenseArgs & A) {
+// Operands through LDS, for steps of many tokens in bf16: a workgroup of four waves owns 32 RT rows x 32 CT tokens, two
+// waves along each, a wave RT x CT tiles. Fragments of both operands go to LDS by direct loads in the order they are
+// stored in; three buffers, so that two fragments are on their way while one is multiplied. A two-part product adds its
+// first part to the residual, then its second.
+template <int KA, int KB, int RT, int CT>
+__global__ __launch_bounds__(256, 2) void k_dense_lds(DenseArgs A, int n_tok_blocks) {
+    constexpr bool DUAL = KA == OUT_RESIDUAL;
+    constexpr int PIECES = 2 * RT + 2 * CT;                   // KiB of a stage: its row tiles, then its token tiles
+    constexpr int PER_WAVE = (PIECES + 3) / 4;
+    static_assert(PIECES % 4 == 0);
+    __shared__ __attribute__((aligned(16))) uint8_t lds[3][PIECES * 1024];
+    const DenseJob & j = A.j;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), wn = wave & 1, wt = wave >> 1;
+    // workgroup b runs on XCD b % 8: an XCD takes every eighth row block, and walks eight token blocks per row block, so
+    // that its concurrent workgroups share both operands in its L2
+    const int n_groups = A.n_groups;
+    int gb, tb;
+    {
+        const int xcd = blockIdx.x & 7, i = blockIdx.x >> 3, per = (n_groups + 7) / 8, group = 8 * per;
+        const int band = i / group, r = i - band * group, tn = min(8, n_tok_blocks - band * 8);
+        gb = (r / tn) * 8 + xcd;
+        tb = band * 8 + r % tn;
+        if (gb >= n_groups || tb >= n_tok_blocks || r / tn >= per) return;
+    }
+    const int tile0 = gb * 2 * RT, tok_tile0 = tb * 2 * CT;
+    f4 acc[RT][CT];
+    auto clear = [&]() {
+#pragma unroll
+        for (int r = 0; r < RT; ++r)
+#pragma unroll
+            for (int c = 0; c < CT; ++c) acc[r][c] = f4{0, 0, 0, 0};
+    };
+    auto run = [&](const DenseIn & in, int lo, int hi, int base) {
+        const int n = hi - lo;
+        if (n <= 0) return;
+        const uint8_t * src[PER_WAVE];
+#pragma unroll
+        for (int i = 0; i < PER_WAVE; ++i) {
+            const int piece = wave + 4 * i;
+            if (piece < 2 * RT) src[i] = (const uint8_t *)(j.w.w + ((size_t)min(tile0 + piece, j.w.tiles - 1) * j.w.kf + lo) * 512);
+            else src[i] = (const uint8_t *)((const uint16_t *)in.x + ((size_t)(tok_tile0 + piece - 2 * RT) * in.kf + (lo - base)) * 512);
+        }
+        const uint32_t to = lds_offset(lds);
+        auto stage = [&](int k, int b) {
+            const int kk = min(k, n - 1);
+#pragma unroll
+            for (int i = 0; i < PER_WAVE; ++i)
+                lds_dma16(src[i] + (size_t)kk * 1024, (uint32_t)lane * 16, to + (uint32_t)(b * PIECES + wave + 4 * i) * 1024);
+        };
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");      // the part before has stored, and the counted waits start at none
+        __syncthreads();                                      // the buffers may still be read by the part before
+        stage(0, 0);
+        stage(1, 1);
+        int b = 0;
+        for (int k = 0; k < n; ++k) {
+            asm volatile("s_waitcnt vmcnt(%0)" :: "n"(PER_WAVE) : "memory");
+            __syncthreads();
+            stage(k + 2, b == 0 ? 2 : b - 1);
+            const uint8_t * cur = lds[b];
+            b8 w[RT], x[CT];
+#pragma unroll
+            for (int r = 0; r < RT; ++r) w[r] = *(const b8 *)(cur + (wn * RT + r) * 1024 + lane * 16);
+#pragma unroll
+            for (int c = 0; c < CT; ++c) x[c] = *(const b8 *)(cur + (2 * RT + wt * CT + c) * 1024 + lane * 16);
+#pragma unroll
+            for (int r = 0; r < RT; ++r)
+#pragma unroll
+                for (int c = 0; c < CT; ++c) acc[r][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[r], x[c], acc[r][c], 0, 0, 0);
+            b = b == 2 ? 0 : b + 1;
+        }
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");      // nothing may land in LDS that another workgroup owns by then
+    };
+    auto store = [&](const float * scale) {
+#pragma unroll
+        for (int r = 0; r < RT; ++r) {
+            const int tile = tile0 + wn * RT + r;
+            if (tile >= j.w.tiles) break;
+            f4 f = {1, 1, 1, 1};
+            if (scale) {
+                const int n = tile * 16 + 4 * (lane >> 4);
+#pragma unroll
+                for (int i = 0; i < 4; ++i) f[i] = n + i < j.w.n ? scale[n + i] : 0.0f;
+            }
+#pragma unroll
+            for (int c = 0; c < CT; ++c) {
+                const int t = (tok_tile0 + wt * CT + c) * 16 + (lane & 15);
+                if (t < A.T) store_rows<KA, KB, ARITH_16>(j, t, 0, tile, lane >> 4, acc[r][c] * f);
+            }
+        }
+    };
+    clear();
+    if constexpr (DUAL) {
+        run(j.x, 0, j.kf1, 0);
+        store(j.scale1);
+        if (j.x2.x) {
+            clear();
+            run(j.x2, j.kf1, j.w.kf, j.kf1);
+            store(j.scale2);
+        }
+    } else {
+        run(j.x, 0, j.w.kf, 0);
+        store(nullptr);
+    }
+}
+
+template <int KA, int KB, int RT, int CT> void launch_lds(hipStream_t s, DenseArgs & A) {
+    A.n_groups = (A.j.w.tiles + 2 * RT - 1) / (2 * RT);
+    const int tok_blocks = (A.T + 32 * CT - 1) / (32 * CT), bands = (tok_blocks + 7) / 8;
+    const dim3 grid((unsigned)(8 * bands * 8 * ((A.n_groups + 7) / 8)));
+    hipLaunchKernelGGL((k_dense_lds<KA, KB, RT, CT>), grid, dim3(256), 0, s, A, tok_blocks);
+}
+
+template <typename TA, int KA, int KB, int RT, int CT, int KW, int RW> void launch(hipStream_t s, DenseArgs & A) {
     const DenseJob & j = A.j;
     A.n_groups = (j.w.tiles + RT * RW - 1) / (RT * RW);
     const dim3 grid((unsigned)(A.n_groups * A.ksplit), (unsigned)((A.T + 16 * CT - 1) / (16 * CT)), (unsigned)j.w.batch);
-    if (j.kf1 > 0) hipLaunchKernelGGL((k_dense<TA, RT, CT, KW, RW, true>), grid, dim3(64 * KW * RW), 0, s, A);
-    else hipLaunchKernelGGL((k_dense<TA, RT, CT, KW, RW, false>), grid, dim3(64 * KW * RW), 0, s, A);
-    check_launch("dense");
+    hipLaunchKernelGGL((k_dense<TA, KA, KB, RT, CT, KW, RW>), grid, dim3(64 * KW * RW), 0, s, A);
 }
 
 constexpr int kMaxSlices = 8;
 constexpr size_t kSliceFloats = (size_t)64 * 32768;      // tokens x rows of one slice
+
+template <int KA, int KB> Slices run(hipStream_t s, int arith, DenseArgs & A, float * ws) {
+    Slices out;
+    const int T = A.T;
+    const DenseWeight & w = A.j.w;
+    if (arith == ARITH_32) {
+        if (T <= 16) launch<float, KA, KB, 1, 1, 4, 1>(s, A);
+        else launch<float, KA, KB, 2, 4, 1, 4>(s, A);
+        return out;
+    }
+    if constexpr (KA != OUT_QUERY && KA != OUT_ACT_GATED) {        // products of one matrix
+        if (w.batch == 1 && T > 128) {
+            // the largest tile that leaves every CU a workgroup
+            auto blocks = [&](int rt, int ct) { return (int64_t)((w.tiles + 2 * rt - 1) / (2 * rt)) * ((T + 32 * ct - 1) / (32 * ct)); };
+            if constexpr (KA != OUT_RESIDUAL) {
+                if (blocks(8, 4) >= 448) { launch_lds<KA, KB, 8, 4>(s, A); return out; }
+            }
+            if (blocks(4, 4) >= 256) launch_lds<KA, KB, 4, 4>(s, A);
+            else launch_lds<KA, KB, 4, 2>(s, A);
+            return out;
+        }
+    }
+    const bool deep = w.kf >= 16;
+    if (KA == OUT_RESIDUAL && deep && ws && (size_t)T * w.n <= kSliceFloats) {
+        // few rows: the workgroups that share a row group leave K-slices, added by the next norm
+        const int groups = T <= 16 ? w.tiles : (w.tiles + 1) / 2;
+        A.ksplit = std::max(1, std::min({kMaxSlices, 512 / std::max(groups, 1), w.kf / 64}));
+        if (A.ksplit > 1) {
+            A.partial = ws;
+            A.slice = (size_t)T * w.n;
+            out.data = ws;
+            out.n = A.ksplit;
+            out.stride = A.slice;
+            out.N = w.n;
+        }
+    }
+    if (!deep) {                        // one wave has too little of K to share it
+        if (T <= 16) launch<uint16_t, KA, KB, 1, 1, 1, 4>(s, A);
+        else if (T <= 32) launch<uint16_t, KA, KB, 1, 2, 1, 4>(s, A);
+        else launch<uint16_t, KA, KB, 1, 4, 1, 4>(s, A);
+    } else if (T <= 16) launch<uint16_t, KA, KB, 1, 1, 8, 1>(s, A);
+    else if (T <= 32) launch<uint16_t, KA, KB, 2, 2, 8, 1>(s, A);
+    else launch<uint16_t, KA, KB, 2, 4, 8, 1>(s, A);
+    return out;
+}
 
 }  // namespace
 
@@ -272,23 +421,30 @@ void dense_pack(hipStream_t s, const uint16_t * src, int rows, int cols, int64_t
 size_t dense_workspace_floats() { return kMaxSlices * kSliceFloats; }
 
 Slices dense(hipStream_t s, int arith, const DenseJob & job, int T, float * ws) {
-    Slices out;
-    if (T <= 0 || job.w.n <= 0) return out;
+    if (T <= 0 || job.w.n <= 0) return Slices();
     DenseArgs A;
     A.j = job;
     A.T = T;
     A.ksplit = 1;
     A.partial = nullptr;
     A.slice = 0;
-    if (A.j.split_tile == 0 && A.j.n_a == 0) { A.j.split_tile = A.j.w.tiles; A.j.n_a = A.j.w.n; }      // one part
-    if (arith == ARITH_32) {
-        if (T <= 16) launch<float, 1, 1, 4, 1>(s, A);
-        else launch<float, 2, 4, 1, 4>(s, A);
-        return out;
+    const bool two = A.j.n_a > 0 && A.j.split_tile < A.j.w.tiles;
+    if (!two) { A.j.split_tile = A.j.w.tiles; A.j.n_a = A.j.w.n; }
+    Slices out;
+    if (two) {
+        if (job.a.kind != OUT_F32 || job.b.kind != OUT_ACT_RELU2) throw std::runtime_error("dense: this pair of outputs is not compiled");
+        out = run<OUT_F32, OUT_ACT_RELU2>(s, arith, A, ws);
+    } else {
+        switch (job.a.kind) {
+            case OUT_F32: out = run<OUT_F32, -1>(s, arith, A, ws); break;
+            case OUT_ACT: out = run<OUT_ACT, -1>(s, arith, A, ws); break;
+            case OUT_ACT_GATED: out = run<OUT_ACT_GATED, -1>(s, arith, A, ws); break;
+            case OUT_QUERY: out = run<OUT_QUERY, -1>(s, arith, A, ws); break;
+            case OUT_RESIDUAL: out = run<OUT_RESIDUAL, -1>(s, arith, A, ws); break;
+            default: throw std::runtime_error("dense: this output is not compiled");
+        }
     }
-    if (T <= 16) launch<uint16_t, 1, 1, 8, 1>(s, A);
-    else if (T <= 32) launch<uint16_t, 2, 2, 4, 1>(s, A);
-    else launch<uint16_t, 4, 4, 1, 4>(s, A);
+    check_launch("dense");
     return out;
 }
 
