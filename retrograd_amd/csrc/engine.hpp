@@ -332,7 +332,7 @@ private:
     StackLayer::Matrix stack_head_;
     DevBuf recurrent_slab_;
     size_t recurrent_slot_floats_ = 0, conv_plane_floats_ = 0;
-    DevBuf st_h_, st_proj_, st_cq_, st_q_, st_qa_, st_ol_, st_mix_, st_ff_, st_out_, st_partial_, st_xbc_, st_y_, st_chunk_;
+    DevBuf st_h_, st_proj_, st_cq_, st_q_, st_qa_, st_ol_, st_mix_, st_ff_, st_out_, st_partial_, st_xbc_, st_y_;
     int st_proj_ld_ = 0;
     struct BlockPlan { int heads, cols; size_t first, n; };    // attention blocks of the step for one head count and width
     std::vector<BlockPlan> block_plans_;

@@ -143,7 +143,7 @@ void Engine::load_stack(const std::string & path) {
             }
             ld.matrix(m + "g", a.heads, E, L.w_in, L.gate_col);
             // queries head by head, every head padded to whole fragments
-            const int D = up32(a.dim), R = up32(a.kv_rank);
+            const int D = up32(a.dim), R = 32 * rk::latent_frags(a.kv_rank);
             ld.shape(L.uq, a.heads * D, rk::frags_of(a.q_rank));
             const uint16_t * uq = ld.raw(m + "uq", a.heads * a.dim, a.q_rank);
             for (int h = 0; h < a.heads; ++h)
@@ -197,7 +197,7 @@ void Engine::build_stack() {
     for (size_t l = 0; l < n_layer; ++l) {
         const LatentSpec & a = c.layers[l].latent;
         if (c.layers[l].mixer != Mixer::LATENT_ATTENTION || a.kv_from >= 0) continue;
-        const int kf = rk::frags_of(a.kv_rank);
+        const int kf = rk::latent_frags(a.kv_rank);
         bytes[l] = (size_t)n_pages_ * rk::latent_page_elems(kf) * elem;
         at[l] = total;
         total += (bytes[l] + 255) / 256 * 256;
@@ -238,7 +238,7 @@ void Engine::build_stack() {
     inv_freq_.alloc(sizeof(double));
     hip_check(hipMemcpy(inv_freq_.ptr, &magnitude, sizeof(double), hipMemcpyHostToDevice), "hipMemcpy");
 
-    size_t h = rk::frag_elems(B, rk::frags_of(E)), cq = 0, q = 0, qa = 0, ol = 0, mix = 0, ff = 0, xbc = 0, y = 0, chunk = 0;
+    size_t h = rk::frag_elems(B, rk::frags_of(E)), cq = 0, q = 0, qa = 0, ol = 0, mix = 0, ff = 0, xbc = 0, y = 0;
     for (const LayerSpec & sp : c.layers) {
         mix = std::max(mix, rk::frag_elems(B, rk::frags_of(sp.mix_width())));
         if (sp.ff > 0) ff = std::max(ff, rk::frag_elems(B, rk::frags_of(sp.ff)));
@@ -246,12 +246,11 @@ void Engine::build_stack() {
             const LatentSpec & a = sp.latent;
             cq = std::max(cq, rk::frag_elems(B, rk::frags_of(a.q_rank)));
             q = std::max(q, rk::frag_elems(B, a.heads * rk::frags_of(a.dim)));
-            qa = std::max(qa, (size_t)B * a.heads * up32(a.kv_rank));
-            ol = std::max(ol, rk::frag_elems(B, a.heads * rk::frags_of(a.kv_rank)));
+            qa = std::max(qa, (size_t)B * a.heads * 32 * rk::latent_frags(a.kv_rank));
+            ol = std::max(ol, rk::frag_elems(B, a.heads * rk::latent_frags(a.kv_rank)));
         } else {
             xbc = std::max(xbc, (size_t)B * sp.mamba.channels());
             y = std::max(y, (size_t)B * sp.mamba.inner());
-            chunk = std::max(chunk, rk::mamba_chunk_floats(sp.mamba, B, n_slots));
         }
     }
     for (const StackLayer & L : stack_layers_) st_proj_ld_ = std::max(st_proj_ld_, L.in_tiles * 16);
@@ -271,7 +270,6 @@ void Engine::build_stack() {
     zeroed(st_ff_, ff * elem);
     zeroed(st_xbc_, xbc * 4);
     zeroed(st_y_, y * 4);
-    zeroed(st_chunk_, chunk * 4);
     mm_ws_.alloc(rk::dense_workspace_floats() * 4);
 }
 
@@ -331,7 +329,7 @@ void Engine::plan_stack(const std::vector<RowView> & rows, const std::vector<std
     for (const RowView & r : rows) total += (int)r.n;
     for (const LayerSpec & sp : stack_->layers) {
         if (sp.mixer != Mixer::LATENT_ATTENTION) continue;
-        const int H = sp.latent.heads, cols = rk::latent_block_cols(arith_, H, rk::frags_of(sp.latent.kv_rank), total, (int)rows.size());
+        const int H = sp.latent.heads, cols = rk::latent_block_cols(arith_, H, rk::latent_frags(sp.latent.kv_rank), total, (int)rows.size());
         if (std::any_of(block_plans_.begin(), block_plans_.end(), [&](const BlockPlan & b) { return b.heads == H && b.cols == cols; })) continue;
         BlockPlan plan{H, cols, plan_blocks_.size(), 0};
         for (size_t r = 0; r < rows.size(); ++r)
@@ -415,7 +413,7 @@ void Engine::forward_stack(int T, int n_out) {
         const int KM = rk::frags_of(sp.mix_width());
         if (sp.mixer == Mixer::LATENT_ATTENTION) {
             const LatentSpec & a = sp.latent;
-            const int D = rk::frags_of(a.dim), R = rk::frags_of(a.kv_rank), H = a.heads;
+            const int D = rk::frags_of(a.dim), R = rk::latent_frags(a.kv_rank), H = a.heads;
             pt = prof_begin(PC_ROPE);
             rk::LatentNorms n;
             n.proj = proj; n.ld = ld; n.q_rank = a.q_rank; n.kv_col = L.kv_col; n.kv_rank = a.kv_rank;
@@ -470,7 +468,7 @@ void Engine::forward_stack(int T, int n_out) {
             j.eps = c.eps;
             j.runs = d_runs_; j.n_runs = (int)plan_runs_.size(); j.max_run = plan_max_run_; j.run_tok = d_run_tok_;
             j.conv_state = L.conv_state; j.conv_plane = conv_plane_floats_; j.state = L.state;
-            j.xbc = st_xbc_.as<float>(); j.y = st_y_.as<float>(); j.chunk_ws = st_chunk_.as<float>();
+            j.xbc = st_xbc_.as<float>(); j.y = st_y_.as<float>();
             j.out = st_mix_.ptr; j.out_kf = KM;
             rk::mamba_mix(stream_, arith_, j, T);
             prof_end(PC_SCAN, pt);

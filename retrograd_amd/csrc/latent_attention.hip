@@ -29,7 +29,7 @@ __global__ __launch_bounds__(64) void k_latent_norms(LatentNorms a) {
     const float inv = 1.0f / sqrtf(q / (float)n + a.eps);
     const int cell = kv ? a.cell[t] : 0;
     EL * page = kv ? (EL *)a.pool + (size_t)(cell / PAGE) * latent_page_elems(a.pool_kf) : nullptr;
-    const int padded = (n + 31) / 32 * 32;
+    const int padded = 32 * (kv ? a.pool_kf : a.act_q_kf);
     for (int k = 8 * lane; k < padded; k += 512) {
         float v[8];
 #pragma unroll
@@ -119,19 +119,20 @@ __global__ __launch_bounds__(256) void k_latent_attention_any(LatentAttn a) {
 typedef __fp16 q4 __attribute__((ext_vector_type(4)));
 typedef __attribute__((address_space(3))) q4 lds_q4;
 
-// Matrix-core form over f16 latents of at most MAXKF fragments. A workgroup serves CT * WC * 16 query columns; WC waves
+// Matrix-core form over f16 latents of KF fragments. A workgroup serves CT * WC * 16 query columns; WC waves
 // share a page (staged once into LDS, double buffered, by direct-to-LDS loads), WK such groups take pages in turn and
 // merge at the end. Scores S^T = C q'^T and outputs O^T = C^T P^T both read the page's one layout: the second product's
 // operand is its transpose, which the LDS transpose read delivers. With several splits (blockIdx.y) every one leaves an
 // unnormalised partial result.
-template <int MAXKF, int CT, int WC, int WK>
-__global__ __launch_bounds__(64 * WC * WK, 1) void k_latent_attention(LatentAttn a) {
+template <int KF, int CT, int WC, int WK>
+__global__ __launch_bounds__(64 * WC * WK) __attribute__((amdgpu_waves_per_eu(2, 2)))
+void k_latent_attention(LatentAttn a) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
     __shared__ float merge_ml[WC][CT][2][64];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int wc = wave % WC, wk = wave / WC, g = lane >> 4;
-    const int kf = a.kf;
-    const int page_bytes = kf * 2048;
+    constexpr int AHEAD = KF >= 4 ? 6 : 2 * KF;
+    constexpr int kf = KF, page_bytes = KF * 2048;
     const LatentBlock blk = a.blocks[blockIdx.x];
     const RowDesc row = a.rows[blk.row];
     const int n_cols = row.n * a.H;
@@ -139,7 +140,7 @@ __global__ __launch_bounds__(64 * WC * WK, 1) void k_latent_attention(LatentAttn
 
     // this lane's column of every column tile: its token and head, and the keys it sees
     int col[CT], lo[CT], hi[CT], lo_max = 0, hi_min = 1 << 30;
-    h8 q[CT][MAXKF];
+    h8 q[CT][KF];
 #pragma unroll
     for (int c = 0; c < CT; ++c) {
         col[c] = blk.col0 + (wc * CT + c) * 16 + (lane & 15);
@@ -151,7 +152,7 @@ __global__ __launch_bounds__(64 * WC * WK, 1) void k_latent_attention(LatentAttn
         hi_min = min(hi_min, hi[c]);
         const __half * qr = (const __half *)a.q + ((size_t)(row.tok_off + tok) * a.H + h) * (size_t)(kf * 32) + 8 * g;
 #pragma unroll
-        for (int j = 0; j < MAXKF; ++j) if (j < kf) q[c][j] = load_h8(qr + 32 * j);
+        for (int j = 0; j < KF; ++j) q[c][j] = load_h8(qr + 32 * j);
     }
 #pragma unroll
     for (int o = 8; o > 0; o >>= 1) {
@@ -174,14 +175,14 @@ __global__ __launch_bounds__(64 * WC * WK, 1) void k_latent_attention(LatentAttn
         for (int ch = wc; ch < 2 * kf; ch += WC)
             lds_dma16(src + ch * 1024, (uint32_t)lane * 16, lds_offset(buf + (size_t)b * page_bytes + ch * 1024));
     };
-    f4 acc[CT][2 * MAXKF];
+    f4 acc[CT][2 * KF];
     float m[CT], l[CT];
 #pragma unroll
     for (int c = 0; c < CT; ++c) {
         m[c] = -INFINITY;
         l[c] = 0.0f;
 #pragma unroll
-        for (int d = 0; d < 2 * MAXKF; ++d) acc[c][d] = f4{0, 0, 0, 0};
+        for (int d = 0; d < 2 * KF; ++d) acc[c][d] = f4{0, 0, 0, 0};
     }
     stage(first + wk, 0);
     const int idx = lane & 15;
@@ -199,14 +200,20 @@ __global__ __launch_bounds__(64 * WC * WK, 1) void k_latent_attention(LatentAttn
 #pragma unroll
             for (int c = 0; c < CT; ++c) s[hf][c] = f4{0, 0, 0, 0};
 #pragma unroll
-            for (int j = 0; j < MAXKF; ++j) {
-                if (j < kf) {
-                    const h8 k = *(const h8 *)(cur + (j * 2 + hf) * 1024 + lane * 16);
+            for (int j = 0; j < KF; ++j) {
+                const h8 k = *(const h8 *)(cur + (j * 2 + hf) * 1024 + lane * 16);
 #pragma unroll
-                    for (int c = 0; c < CT; ++c) s[hf][c] = __builtin_amdgcn_mfma_f32_16x16x32_f16(k, q[c][j], s[hf][c], 0, 0, 0);
-                }
+                for (int c = 0; c < CT; ++c) s[hf][c] = __builtin_amdgcn_mfma_f32_16x16x32_f16(k, q[c][j], s[hf][c], 0, 0, 0);
             }
         }
+        // eight reads ahead of the products: the scheduler would otherwise wait for every read it issues
+        __builtin_amdgcn_sched_group_barrier(0x100, AHEAD, 0);
+#pragma unroll
+        for (int i = 0; i < 2 * KF - AHEAD; ++i) {
+            __builtin_amdgcn_sched_group_barrier(0x008, CT, 0);
+            __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
+        }
+        __builtin_amdgcn_sched_group_barrier(0x008, AHEAD * CT, 0);
         const int key0 = page * PAGE;
         const bool inside = key0 >= lo_max && key0 + PAGE - 1 <= hi_min;
         h8 p[CT];
@@ -230,7 +237,7 @@ __global__ __launch_bounds__(64 * WC * WK, 1) void k_latent_attention(LatentAttn
                 const float f = exp2f(m[c] - base);
                 l[c] *= f;
 #pragma unroll
-                for (int d = 0; d < 2 * MAXKF; ++d) acc[c][d] *= f;
+                for (int d = 0; d < 2 * KF; ++d) acc[c][d] *= f;
                 m[c] = m2;
             }
 #pragma unroll
@@ -243,16 +250,21 @@ __global__ __launch_bounds__(64 * WC * WK, 1) void k_latent_attention(LatentAttn
                 }
         }
 #pragma unroll
-        for (int d = 0; d < 2 * MAXKF; ++d) {
-            if ((d >> 1) < kf) {
-                const uint8_t * v0 = cur + (d >> 1) * 2048 + (d & 1) * 512 + tr_lane;
-                union { q4 half[2]; h8 all; } v;
-                v.half[0] = __builtin_amdgcn_ds_read_tr16_b64_v4f16((lds_q4 *)(v0));
-                v.half[1] = __builtin_amdgcn_ds_read_tr16_b64_v4f16((lds_q4 *)(v0 + 1024));
+        for (int d = 0; d < 2 * KF; ++d) {
+            const uint8_t * v0 = cur + (d >> 1) * 2048 + (d & 1) * 512 + tr_lane;
+            union { q4 half[2]; h8 all; } v;
+            v.half[0] = __builtin_amdgcn_ds_read_tr16_b64_v4f16((lds_q4 *)(v0));
+            v.half[1] = __builtin_amdgcn_ds_read_tr16_b64_v4f16((lds_q4 *)(v0 + 1024));
 #pragma unroll
-                for (int c = 0; c < CT; ++c) acc[c][d] = __builtin_amdgcn_mfma_f32_16x16x32_f16(v.all, p[c], acc[c][d], 0, 0, 0);
-            }
+            for (int c = 0; c < CT; ++c) acc[c][d] = __builtin_amdgcn_mfma_f32_16x16x32_f16(v.all, p[c], acc[c][d], 0, 0, 0);
         }
+        __builtin_amdgcn_sched_group_barrier(0x100, 2 * AHEAD, 1);
+#pragma unroll
+        for (int i = 0; i < 2 * KF - AHEAD; ++i) {
+            __builtin_amdgcn_sched_group_barrier(0x008, CT, 1);
+            __builtin_amdgcn_sched_group_barrier(0x100, 2, 1);
+        }
+        __builtin_amdgcn_sched_group_barrier(0x008, AHEAD * CT, 1);
     }
 #pragma unroll
     for (int c = 0; c < CT; ++c) {
@@ -267,7 +279,7 @@ __global__ __launch_bounds__(64 * WC * WK, 1) void k_latent_attention(LatentAttn
             merge_ml[wc][0][0][lane] = m[0];
             merge_ml[wc][0][1][lane] = l[0];
 #pragma unroll
-            for (int d = 0; d < 2 * MAXKF; ++d) if ((d >> 1) < kf) park[d * 64 + lane] = acc[0][d];
+            for (int d = 0; d < 2 * KF; ++d) park[d * 64 + lane] = acc[0][d];
         }
         __syncthreads();
         if (wk == 1) return;
@@ -277,7 +289,7 @@ __global__ __launch_bounds__(64 * WC * WK, 1) void k_latent_attention(LatentAttn
         l[0] = l[0] * f0 + lo2 * f1;
         m[0] = m2;
 #pragma unroll
-        for (int d = 0; d < 2 * MAXKF; ++d) if ((d >> 1) < kf) acc[0][d] = acc[0][d] * f0 + park[d * 64 + lane] * f1;
+        for (int d = 0; d < 2 * KF; ++d) acc[0][d] = acc[0][d] * f0 + park[d * 64 + lane] * f1;
     }
 #pragma unroll
     for (int c = 0; c < CT; ++c) {
@@ -287,18 +299,16 @@ __global__ __launch_bounds__(64 * WC * WK, 1) void k_latent_attention(LatentAttn
             float * o = a.partial + (((size_t)t * a.H + h) * a.splits + sp) * (size_t)(kf * 32 + 4);
             if (g == 0) { o[kf * 32] = m[c]; o[kf * 32 + 1] = l[c]; }
 #pragma unroll
-            for (int d = 0; d < 2 * MAXKF; ++d) if ((d >> 1) < kf) *(f4 *)(o + d * 16 + 4 * g) = acc[c][d];
+            for (int d = 0; d < 2 * KF; ++d) *(f4 *)(o + d * 16 + 4 * g) = acc[c][d];
         } else {
             const float inv = 1.0f / l[c];
 #pragma unroll
-            for (int d = 0; d < 2 * MAXKF; ++d) {
-                if ((d >> 1) < kf) {
-                    const f4 v = acc[c][d] * inv;
-                    uint2 u;
-                    u.x = (uint32_t)bf16_bits(v[0]) | ((uint32_t)bf16_bits(v[1]) << 16);
-                    u.y = (uint32_t)bf16_bits(v[2]) | ((uint32_t)bf16_bits(v[3]) << 16);
-                    *(uint2 *)((uint16_t *)a.out + frag_at(t, h * kf * 32 + d * 16 + 4 * g, a.out_kf)) = u;
-                }
+            for (int d = 0; d < 2 * KF; ++d) {
+                const f4 v = acc[c][d] * inv;
+                uint2 u;
+                u.x = (uint32_t)bf16_bits(v[0]) | ((uint32_t)bf16_bits(v[1]) << 16);
+                u.y = (uint32_t)bf16_bits(v[2]) | ((uint32_t)bf16_bits(v[3]) << 16);
+                *(uint2 *)((uint16_t *)a.out + frag_at(t, h * kf * 32 + d * 16 + 4 * g, a.out_kf)) = u;
             }
         }
     }
@@ -362,25 +372,31 @@ namespace {
 constexpr int kMatrixKf = 16;       // widest latent (in fragments) of the matrix-core kernel
 bool on_matrix_cores(int arith, int kf) { return arith == ARITH_16 && kf <= kMatrixKf; }
 
-template <int MAXKF, int CT, int WC, int WK> void launch_attention(hipStream_t s, const LatentAttn & a) {
-    const size_t lds = (size_t)WK * 2 * a.kf * 2048;
-    auto kernel = k_latent_attention<MAXKF, CT, WC, WK>;
-    static const bool allowed = hipFuncSetAttribute((const void *)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, WK * 2 * MAXKF * 2048) == hipSuccess;
+template <int KF, int CT, int WC, int WK> void launch_attention(hipStream_t s, const LatentAttn & a) {
+    const size_t lds = (size_t)WK * 2 * KF * 2048;
+    auto kernel = k_latent_attention<KF, CT, WC, WK>;
+    static const bool allowed = hipFuncSetAttribute((const void *)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, WK * 2 * KF * 2048) == hipSuccess;
     if (!allowed) throw std::runtime_error("latent attention: the page buffers do not fit the LDS");
     hipLaunchKernelGGL(kernel, dim3((unsigned)a.n_blocks, (unsigned)a.splits), dim3(64 * WC * WK), lds, s, a);
 }
-template <int MAXKF> void launch_columns(hipStream_t s, const LatentAttn & a) {
+template <int KF> void launch_columns(hipStream_t s, const LatentAttn & a) {
     switch (a.block_cols) {
-        case 16: launch_attention<MAXKF, 1, 1, 2>(s, a); break;
-        case 32: launch_attention<MAXKF, 1, 2, 2>(s, a); break;
-        case 64: launch_attention<MAXKF, 1, 4, 1>(s, a); break;
+        case 16: launch_attention<KF, 1, 1, 2>(s, a); break;
+        case 32: launch_attention<KF, 1, 2, 2>(s, a); break;
+        case 64: launch_attention<KF, 1, 4, 1>(s, a); break;
         case 128:
-            if constexpr (MAXKF <= 8) { launch_attention<MAXKF, 2, 4, 1>(s, a); break; }      // wider: the registers do not suffice
+            if constexpr (KF <= 8) { launch_attention<KF, 2, 4, 1>(s, a); break; }      // wider: the registers do not suffice
             [[fallthrough]];
         default: throw std::runtime_error("latent attention: no kernel for this many columns per block");
     }
 }
 }  // namespace
+
+int latent_frags(int kv_rank) {
+    const int kf = frags_of(kv_rank);
+    for (int w : {1, 2, 3, 4, 6, 8, 12, 16}) if (kf <= w) return w;
+    return kf;
+}
 
 int latent_block_cols(int arith, int H, int kf, int n_tokens, int n_rows) {
     if (!on_matrix_cores(arith, kf)) return 1;
@@ -401,10 +417,17 @@ void latent_attention(hipStream_t s, int arith, const LatentAttn & a, int T) {
     if (a.n_blocks <= 0) return;
     if (a.kf * 32 > 1024) throw std::runtime_error("latent attention: latents of at most 1024 columns");
     if (on_matrix_cores(arith, a.kf)) {
-        if (a.kf <= 2) launch_columns<2>(s, a);
-        else if (a.kf <= 4) launch_columns<4>(s, a);
-        else if (a.kf <= 8) launch_columns<8>(s, a);
-        else launch_columns<16>(s, a);
+        switch (a.kf) {                   // the widths latent_frags() rounds to
+            case 1: launch_columns<1>(s, a); break;
+            case 2: launch_columns<2>(s, a); break;
+            case 3: launch_columns<3>(s, a); break;
+            case 4: launch_columns<4>(s, a); break;
+            case 6: launch_columns<6>(s, a); break;
+            case 8: launch_columns<8>(s, a); break;
+            case 12: launch_columns<12>(s, a); break;
+            case 16: launch_columns<16>(s, a); break;
+            default: throw std::runtime_error("latent attention: no kernel for this latent width");
+        }
         check_launch("latent_attention");
         if (a.splits > 1) {
             hipLaunchKernelGGL(k_latent_combine, dim3((unsigned)(T * a.H)), dim3(64), 0, s, a);

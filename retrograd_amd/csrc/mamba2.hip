@@ -14,9 +14,10 @@ constexpr int kConvTokens = 16;       // tokens of a run one workgroup convolves
 
 // xbc[t][c] = silu(bias + sum over the taps); inputs before the run come from the slot's current plane, and the run's
 // last taps - 1 inputs go to the other plane (the workgroups of a run read the one while the other is written).
+template <int TAPS>
 __global__ __launch_bounds__(256) void k_mamba_conv(MambaJob j) {
     const MambaShape sh = j.sh;
-    const int C = sh.channels(), c = blockIdx.y * 256 + threadIdx.x, K = sh.taps;
+    const int C = sh.channels(), c = blockIdx.y * 256 + threadIdx.x, K = TAPS > 0 ? TAPS : sh.taps;
     const SeqRun run = j.runs[blockIdx.z];
     const int first = blockIdx.x * kConvTokens;
     if (c >= C || first >= run.n) return;
@@ -30,11 +31,31 @@ __global__ __launch_bounds__(256) void k_mamba_conv(MambaJob j) {
         return fresh ? 0.0f : old_in[(size_t)(i + K - 1) * C + c];
     };
     const float * w = j.conv_w + (size_t)c * K;
+    const float bias = j.conv_b[c];
     const int last = min(first + kConvTokens, run.n);
-    for (int i = first; i < last; ++i) {
-        float s = 0.0f;
-        for (int k = 0; k < K; ++k) s += w[k] * input(i - (K - 1) + k);
-        j.xbc[(size_t)j.run_tok[run.start + i] * C + c] = silu_f(s + j.conv_b[c]);
+    if constexpr (TAPS > 0) {                   // the window and the taps in registers
+        float win[TAPS], tap[TAPS];
+#pragma unroll
+        for (int k = 0; k < TAPS; ++k) {
+            tap[k] = w[k];
+            win[k] = k > 0 ? input(first - TAPS + k) : 0.0f;
+        }
+        for (int i = first; i < last; ++i) {
+            const int t = j.run_tok[run.start + i];
+            float v = 0.0f;
+#pragma unroll
+            for (int k = 0; k + 1 < TAPS; ++k) win[k] = win[k + 1];
+            win[TAPS - 1] = j.proj[(size_t)t * j.ld + off];
+#pragma unroll
+            for (int k = 0; k < TAPS; ++k) v += tap[k] * win[k];
+            j.xbc[(size_t)t * C + c] = silu_f(v + bias);
+        }
+    } else {
+        for (int i = first; i < last; ++i) {
+            float v = 0.0f;
+            for (int k = 0; k < K; ++k) v += w[k] * input(i - (K - 1) + k);
+            j.xbc[(size_t)j.run_tok[run.start + i] * C + c] = silu_f(v + bias);
+        }
     }
     if (last == run.n)
         for (int k = 0; k < K - 1; ++k) new_in[(size_t)k * C + c] = input(run.n - (K - 1) + k);
@@ -109,6 +130,214 @@ __global__ __launch_bounds__(256) void k_mamba_scan(MambaJob j) {
     }
 }
 
+constexpr int kChunk = 64;            // tokens of a chunk
+constexpr int kChunkP = 32;           // state columns of a workgroup
+constexpr int kChunkN = 128;          // most state rows of the chunked kernel
+
+// The recurrence in chunks of 64 tokens on the f32 matrix instruction. With l_t the running sum of -exp(A_log) dt in a
+// chunk (kept in double: differences of it are what is exponentiated) and S the state before the chunk,
+//   y_t = exp(l_t) S^T C_t + sum over s <= t of exp(l_t - l_s) dt_s (C_t . B_s) x_s + D x_t,
+//   S  <- exp(l_last) S + sum over s of exp(l_last - l_s) dt_s B_s x_s^T.
+// One workgroup walks a run's chunks for 32 columns of one head; wave w owns the chunk's token tile w. Tokens past the
+// run's end count as dt = 0, which leaves everything unchanged. VEC: rows can be read four columns at a time, and the next
+// chunk's rows are on their way while a chunk is worked on.
+template <bool VEC>
+__global__ __launch_bounds__(256) void k_mamba_chunks(MambaJob j) {
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    const MambaShape sh = j.sh;
+    const int N = sh.state, Np = (N + 15) / 16 * 16, P = sh.vdim, C = sh.channels(), LB = Np + 4;
+    const int h = blockIdx.x, g = h / (sh.heads / sh.groups), p0 = blockIdx.y * kChunkP;
+    const SeqRun run = j.runs[blockIdx.z];
+    const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, r16 = lane & 15, kg = lane >> 4;
+    float * sB = sm, * sC = sB + kChunk * LB, * sX = sC + kChunk * LB, * sM = sX + kChunk * 36, * sS = sM + kChunk * 68;
+    __shared__ double s_l[kChunk];
+    __shared__ float s_dt[kChunk], s_w[kChunk];
+    __shared__ int s_tok[kChunk];
+    const float a = expf(j.A_log[h]), Dh = j.D[h], bias = j.dt_bias[h];
+    float * st = j.state + (((size_t)run.slot * sh.heads + h) * N) * P + p0;
+    const int n_tiles = Np / 16;
+    // the state in registers: wave w holds row tiles w, w + 4, both column tiles
+    f4 S[kChunkN / 64][2];
+#pragma unroll
+    for (int q = 0; q < kChunkN / 64; ++q)
+#pragma unroll
+        for (int c = 0; c < 2; ++c)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int n = (w + 4 * q) * 16 + 4 * kg + i, p = c * 16 + r16;
+                S[q][c][i] = (n < N && p0 + p < P && !(run.flags & 1)) ? st[(size_t)n * P + p] : 0.0f;
+            }
+    constexpr int RB = kChunk * kChunkN / 4 / 256, RX = kChunk * kChunkP / 4 / 256;
+    f4 nB[VEC ? RB : 1], nC[VEC ? RB : 1], nX[VEC ? RX : 1];
+    float n_dt = 0.0f;
+    int n_tok = 0;
+    auto token = [&](int base, int tk) { return j.run_tok[run.start + min(base + tk, run.n - 1)]; };
+    auto fetch = [&](int base) {                // of the chunk at base into registers; nothing past the run's end is used
+        if (w == 0) {
+            n_tok = token(base, lane);
+            n_dt = j.proj[(size_t)n_tok * j.ld + sh.inner() + C + h];
+        }
+        if constexpr (VEC) {
+            const int n = 4 * (threadIdx.x & 31);
+#pragma unroll
+            for (int i = 0; i < RB; ++i) {
+                const float * row = j.xbc + (size_t)token(base, (threadIdx.x >> 5) + 8 * i) * C + sh.inner() + g * N + min(n, N - 4);
+                nB[i] = *(const f4 *)row;
+                nC[i] = *(const f4 *)(row + (size_t)sh.groups * N);
+            }
+            const int p = 4 * (threadIdx.x & 7);
+#pragma unroll
+            for (int i = 0; i < RX; ++i)
+                nX[i] = *(const f4 *)(j.xbc + (size_t)token(base, (threadIdx.x >> 3) + 32 * i) * C + h * P + min(p0 + p, P - 4));
+        }
+    };
+    fetch(0);
+    for (int base = 0; base < run.n; base += kChunk) {
+        const int cnt = min(kChunk, run.n - base);
+        __syncthreads();
+        if (w == 0) {
+            s_tok[lane] = n_tok;
+            const float dt = lane < cnt ? softplus_f(n_dt + bias) : 0.0f;
+            double l = -(double)a * (double)dt;
+#pragma unroll
+            for (int o = 1; o < 64; o <<= 1) {
+                const double up = __shfl_up(l, o, 64);
+                if (lane >= o) l += up;
+            }
+            s_l[lane] = l;
+            s_dt[lane] = dt;
+            s_w[lane] = expf((float)(__shfl(l, 63, 64) - l)) * dt;
+        }
+#pragma unroll
+        for (int q = 0; q < kChunkN / 64; ++q)
+#pragma unroll
+            for (int c = 0; c < 2; ++c)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const int n = (w + 4 * q) * 16 + 4 * kg + i;
+                    if (n < Np) sS[n * 36 + c * 16 + r16] = S[q][c][i];
+                }
+        if constexpr (VEC) {
+            const f4 zero = {0, 0, 0, 0};
+            const int n = 4 * (threadIdx.x & 31), p = 4 * (threadIdx.x & 7);
+            if (n < Np) {
+#pragma unroll
+                for (int i = 0; i < RB; ++i) {
+                    const int tk = (threadIdx.x >> 5) + 8 * i;
+                    const bool in = n < N && tk < cnt;
+                    *(f4 *)(sB + tk * LB + n) = in ? nB[i] : zero;
+                    *(f4 *)(sC + tk * LB + n) = in ? nC[i] : zero;
+                }
+            }
+#pragma unroll
+            for (int i = 0; i < RX; ++i) {
+                const int tk = (threadIdx.x >> 3) + 32 * i;
+                *(f4 *)(sX + tk * 36 + p) = p0 + p < P && tk < cnt ? nX[i] : zero;
+            }
+        } else {
+            __syncthreads();
+            for (int i = threadIdx.x; i < kChunk * Np; i += 256) {
+                const int tk = i / Np, n = i - tk * Np;
+                const float * row = j.xbc + (size_t)s_tok[tk] * C + sh.inner() + g * N + n;
+                const bool in = n < N && tk < cnt;
+                sB[tk * LB + n] = in ? row[0] : 0.0f;
+                sC[tk * LB + n] = in ? row[(size_t)sh.groups * N] : 0.0f;
+            }
+            for (int i = threadIdx.x; i < kChunk * kChunkP; i += 256) {
+                const int tk = i / kChunkP, p = i - tk * kChunkP;
+                sX[tk * 36 + p] = (p0 + p < P && tk < cnt) ? j.xbc[(size_t)s_tok[tk] * C + h * P + p0 + p] : 0.0f;
+            }
+        }
+        __syncthreads();
+        if (base + kChunk < run.n) fetch(base + kChunk);
+        const int t0 = 16 * w;
+        double lt[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) lt[i] = s_l[t0 + 4 * kg + i];
+        // decayed C B^T of this wave's tokens with everything before them
+        for (int q = 0; q <= w; ++q) {
+            f4 d = {0, 0, 0, 0};
+            const float * ca = sC + (t0 + r16) * LB + 4 * kg, * cb = sB + (16 * q + r16) * LB + 4 * kg;
+            for (int k = 0; k < Np; k += 16) {
+                const f4 x = *(const f4 *)(ca + k), y = *(const f4 *)(cb + k);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) d = __builtin_amdgcn_mfma_f32_16x16x4f32(x[e], y[e], d, 0, 0, 0);
+            }
+            const int sk = 16 * q + r16;
+            const double ls = s_l[sk];
+            const float dt = s_dt[sk];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int t = t0 + 4 * kg + i;
+                sM[t * 68 + sk] = sk <= t ? d[i] * expf((float)(lt[i] - ls)) * dt : 0.0f;
+            }
+        }
+        // (a wave reads only the rows of sM that it wrote)
+        f4 y[2] = {{0, 0, 0, 0}, {0, 0, 0, 0}};
+        {
+            const float * ca = sC + (t0 + r16) * LB + 4 * kg;
+            for (int k = 0; k < Np; k += 16) {
+                const f4 x = *(const f4 *)(ca + k);
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+#pragma unroll
+                    for (int c = 0; c < 2; ++c)
+                        y[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(x[e], sS[(k + 4 * kg + e) * 36 + c * 16 + r16], y[c], 0, 0, 0);
+            }
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const float f = expf((float)lt[i]);
+                y[0][i] *= f;
+                y[1][i] *= f;
+            }
+            __builtin_amdgcn_wave_barrier();
+            const float * ma = sM + (t0 + r16) * 68 + 4 * kg;
+            for (int k = 0; k < t0 + 16; k += 16) {
+                const f4 x = *(const f4 *)(ma + k);
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+#pragma unroll
+                    for (int c = 0; c < 2; ++c)
+                        y[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(x[e], sX[(k + 4 * kg + e) * 36 + c * 16 + r16], y[c], 0, 0, 0);
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int tk = t0 + 4 * kg + i;
+            if (tk >= cnt) break;
+#pragma unroll
+            for (int c = 0; c < 2; ++c) {
+                const int p = c * 16 + r16;
+                if (p0 + p < P) j.y[(size_t)s_tok[tk] * sh.inner() + h * P + p0 + p] = y[c][i] + Dh * sX[tk * 36 + p];
+            }
+        }
+        const float decay = expf((float)s_l[kChunk - 1]);
+#pragma unroll
+        for (int q = 0; q < kChunkN / 64; ++q) {
+            if (w + 4 * q >= n_tiles) break;
+            f4 d[2] = {S[q][0] * decay, S[q][1] * decay};
+            const int n = (w + 4 * q) * 16 + r16;
+            for (int k = 0; k < cnt; k += 4) {
+                const int sk = k + kg;
+                const float bw = sB[sk * LB + n] * s_w[sk];
+#pragma unroll
+                for (int c = 0; c < 2; ++c) d[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(bw, sX[sk * 36 + c * 16 + r16], d[c], 0, 0, 0);
+            }
+            S[q][0] = d[0];
+            S[q][1] = d[1];
+        }
+    }
+#pragma unroll
+    for (int q = 0; q < kChunkN / 64; ++q)
+#pragma unroll
+        for (int c = 0; c < 2; ++c)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int n = (w + 4 * q) * 16 + 4 * kg + i, p = c * 16 + r16;
+                if (n < N && p0 + p < P) st[(size_t)n * P + p] = S[q][c][i];
+            }
+}
+
 // act[t] = norm over each of the equal parts of (y * silu(z)), times the weight: one workgroup per token and part.
 template <int ARITH>
 __global__ __launch_bounds__(256) void k_mamba_gate_norm(MambaJob j) {
@@ -144,24 +373,41 @@ __global__ __launch_bounds__(256) void k_mamba_gate_norm(MambaJob j) {
 
 }  // namespace
 
-size_t mamba_chunk_floats(const MambaShape & sh, int T, int n_seq) { return 0; }
-
 void mamba_mix(hipStream_t s, int arith, const MambaJob & j, int T) {
     if (j.n_runs <= 0 || T <= 0) return;
     const MambaShape & sh = j.sh;
     if (sh.state > 512) throw std::runtime_error("mamba2: at most 512 state rows per head");
-    hipLaunchKernelGGL(k_mamba_conv, dim3((unsigned)((j.max_run + kConvTokens - 1) / kConvTokens), (unsigned)((sh.channels() + 255) / 256), (unsigned)j.n_runs),
-                       dim3(256), 0, s, j);
+    const dim3 conv((unsigned)((j.max_run + kConvTokens - 1) / kConvTokens), (unsigned)((sh.channels() + 255) / 256), (unsigned)j.n_runs);
+    switch (sh.taps) {
+        case 2: hipLaunchKernelGGL(k_mamba_conv<2>, conv, dim3(256), 0, s, j); break;
+        case 3: hipLaunchKernelGGL(k_mamba_conv<3>, conv, dim3(256), 0, s, j); break;
+        case 4: hipLaunchKernelGGL(k_mamba_conv<4>, conv, dim3(256), 0, s, j); break;
+        default: hipLaunchKernelGGL(k_mamba_conv<0>, conv, dim3(256), 0, s, j);
+    }
     check_launch("mamba_conv");
-    const dim3 grid((unsigned)sh.heads, (unsigned)((sh.vdim + kScanP - 1) / kScanP), (unsigned)j.n_runs);
-    const size_t lds = (size_t)(2 * kScanTokens * sh.state + kScanTokens * 256) * 4;
-    const int npt = (sh.state + 3) / 4;
-    if (npt <= 8) hipLaunchKernelGGL(k_mamba_scan<8>, grid, dim3(256), lds, s, j);
-    else if (npt <= 16) hipLaunchKernelGGL(k_mamba_scan<16>, grid, dim3(256), lds, s, j);
-    else if (npt <= 32) hipLaunchKernelGGL(k_mamba_scan<32>, grid, dim3(256), lds, s, j);
-    else if (npt <= 64) hipLaunchKernelGGL(k_mamba_scan<64>, grid, dim3(256), lds, s, j);
-    else hipLaunchKernelGGL(k_mamba_scan<128>, grid, dim3(256), lds, s, j);
-    check_launch("mamba_scan");
+    if (j.max_run >= kChunk / 2 && sh.state <= kChunkN) {
+        const int Np = (sh.state + 15) / 16 * 16;
+        const size_t lds = ((size_t)2 * kChunk * (Np + 4) + kChunk * 36 + kChunk * 68 + (size_t)Np * 36) * 4;
+        constexpr int most = (2 * kChunk * (kChunkN + 4) + kChunk * 36 + kChunk * 68 + kChunkN * 36) * 4;
+        static const bool allowed = hipFuncSetAttribute((const void *)k_mamba_chunks<true>, hipFuncAttributeMaxDynamicSharedMemorySize, most) == hipSuccess
+                                 && hipFuncSetAttribute((const void *)k_mamba_chunks<false>, hipFuncAttributeMaxDynamicSharedMemorySize, most) == hipSuccess;
+        if (!allowed) throw std::runtime_error("mamba2: a chunk does not fit the LDS");
+        const dim3 grid((unsigned)sh.heads, (unsigned)((sh.vdim + kChunkP - 1) / kChunkP), (unsigned)j.n_runs);
+        // every row starts at a multiple of four floats
+        if (sh.vdim % 4 == 0 && sh.state % 4 == 0) hipLaunchKernelGGL(k_mamba_chunks<true>, grid, dim3(256), lds, s, j);
+        else hipLaunchKernelGGL(k_mamba_chunks<false>, grid, dim3(256), lds, s, j);
+        check_launch("mamba_chunks");
+    } else {
+        const dim3 grid((unsigned)sh.heads, (unsigned)((sh.vdim + kScanP - 1) / kScanP), (unsigned)j.n_runs);
+        const size_t lds = (size_t)(2 * kScanTokens * sh.state + kScanTokens * 256) * 4;
+        const int npt = (sh.state + 3) / 4;
+        if (npt <= 8) hipLaunchKernelGGL(k_mamba_scan<8>, grid, dim3(256), lds, s, j);
+        else if (npt <= 16) hipLaunchKernelGGL(k_mamba_scan<16>, grid, dim3(256), lds, s, j);
+        else if (npt <= 32) hipLaunchKernelGGL(k_mamba_scan<32>, grid, dim3(256), lds, s, j);
+        else if (npt <= 64) hipLaunchKernelGGL(k_mamba_scan<64>, grid, dim3(256), lds, s, j);
+        else hipLaunchKernelGGL(k_mamba_scan<128>, grid, dim3(256), lds, s, j);
+        check_launch("mamba_scan");
+    }
     const dim3 gn((unsigned)T, (unsigned)sh.norm_groups);
     const size_t nl = (size_t)(sh.inner() / sh.norm_groups) * 4;
     if (arith == ARITH_16) hipLaunchKernelGGL(k_mamba_gate_norm<ARITH_16>, gn, dim3(256), nl, s, j);

@@ -80,6 +80,8 @@ void add_slices(hipStream_t s, float * x, int E, int T, const Slices & add);
 // ---- latent attention --------------------------------------------------------------------------------
 // A page of the latent cache: PAGE tokens x kf fragments of 32 columns, f16 or f32,
 //   [column / 32][token / 16][lane = 16 * ((column % 32) / 8) + token % 16][column % 8]
+// Fragments a latent of kv_rank columns is stored in: the widths the attention kernel is compiled for, zero padded.
+int latent_frags(int kv_rank);
 constexpr size_t latent_page_elems(int kf) { return (size_t)kf * 32 * PAGE; }
 // Queries' latent: act_q = RMS norm of proj[t][0, q_rank) times q_w. With kv_w also the cached latent: RMS norm of
 // proj[t][kv_col, kv_col + kv_rank) times kv_w into cell[t] of the pool.
@@ -146,13 +148,10 @@ struct MambaJob {
     float * state = nullptr;       // [slots][heads][state][vdim]
     float * xbc = nullptr;         // scratch [T][channels]
     float * y = nullptr;           // scratch [T][inner]
-    float * chunk_ws = nullptr;    // scratch of long runs (mamba_chunk_floats)
     void * out = nullptr;          // activations, inner wide
     int out_kf = 0;
 };
-size_t mamba_chunk_floats(const MambaShape & sh, int T, int n_seq);
 void mamba_mix(hipStream_t s, int arith, const MambaJob & j, int T);
-// dst slot's state = src slot's (floats each), and zeroing.
 void copy_floats(hipStream_t s, const float * src, float * dst, size_t n);
 
 }  // namespace rk
