@@ -446,7 +446,8 @@ void Engine::forward_stack(int T, int n_out) {
             at.pool = k_pool_[(size_t)L.pool_layer].ptr;
             at.splits = rk::latent_splits(arith_, at, step_max_resident_);
             st_partial_.ensure(rk::latent_partial_floats(T, H, R, at.splits) * 4);
-            at.partial = st_partial_.as<float>();
+            at.partial_ml = st_partial_.as<float>();
+            at.partial = at.partial_ml + (size_t)T * H * at.splits * 2;
             at.out = st_ol_.ptr; at.out_kf = H * R;
             rk::latent_attention(stream_, arith_, at, T);
             prof_end(PC_ATTN, pt);

@@ -14,33 +14,64 @@ template <typename EL> __device__ __forceinline__ EL float_el(float v);
 template <> __device__ __forceinline__ __half float_el<__half>(float v) { return sat_half(v); }
 template <> __device__ __forceinline__ float float_el<float>(float v) { return v; }
 
-// One wave per token and norm: the queries' latent, and (blockIdx.y = 1) the latent that goes into the cache.
+// One workgroup per token and norm: the queries' latent, and (blockIdx.y = 1) the latent that goes into the cache. A
+// thread keeps its groups of eight columns in registers between the two passes.
 template <int ARITH>
-__global__ __launch_bounds__(64) void k_latent_norms(LatentNorms a) {
+__global__ __launch_bounds__(256) void k_latent_norms(LatentNorms a) {
     using EL = typename std::conditional<ARITH == ARITH_16, __half, float>::type;
-    const int t = blockIdx.x, lane = threadIdx.x;
+    __shared__ float scratch[16];
+    constexpr int KEEP = 2;                    // groups of eight per thread that stay in registers
+    const int t = blockIdx.x;
     const bool kv = blockIdx.y == 1;
     const int n = kv ? a.kv_rank : a.q_rank;
     const float * src = a.proj + (size_t)t * a.ld + (kv ? a.kv_col : 0);
     const float * w = kv ? a.kv_w : a.q_w;
-    float q = 0.0f;
-    for (int k = lane; k < n; k += 64) q += src[k] * src[k];
-    q = wave_sum(q);
+    float v[KEEP][8], q = 0.0f;
+    auto load = [&](int k, float (&o)[8]) {    // rows of the product start at multiples of four
+        if (k + 8 <= n) {
+            const f4 x = *(const f4 *)(src + k), y = *(const f4 *)(src + k + 4);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) { o[i] = x[i]; o[4 + i] = y[i]; }
+        } else {
+#pragma unroll
+            for (int i = 0; i < 8; ++i) o[i] = k + i < n ? src[k + i] : 0.0f;
+        }
+    };
+#pragma unroll
+    for (int g = 0; g < KEEP; ++g) {
+        load(8 * (int)(threadIdx.x + 256 * g), v[g]);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) q += v[g][i] * v[g][i];
+    }
+    for (int k = 8 * (int)(threadIdx.x + 256 * KEEP); k < n; k += 8 * 256) {
+        float o[8];
+        load(k, o);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) q += o[i] * o[i];
+    }
+    q = block_sum(q, scratch);
     const float inv = 1.0f / sqrtf(q / (float)n + a.eps);
     const int cell = kv ? a.cell[t] : 0;
     EL * page = kv ? (EL *)a.pool + (size_t)(cell / PAGE) * latent_page_elems(a.pool_kf) : nullptr;
     const int padded = 32 * (kv ? a.pool_kf : a.act_q_kf);
-    for (int k = 8 * lane; k < padded; k += 512) {
-        float v[8];
+    auto finish = [&](int k, float (&o)[8]) {
+        if (k >= padded) return;
 #pragma unroll
-        for (int i = 0; i < 8; ++i) v[i] = k + i < n ? src[k + i] * inv * w[k + i] : 0.0f;
+        for (int i = 0; i < 8; ++i) o[i] = k + i < n ? o[i] * inv * w[k + i] : 0.0f;
         if (kv) {
             EL * dst = page + latent_at(cell % PAGE, k);
 #pragma unroll
-            for (int i = 0; i < 8; ++i) dst[i] = float_el<EL>(v[i]);
+            for (int i = 0; i < 8; ++i) dst[i] = float_el<EL>(o[i]);
         } else {
-            store_frag8<ARITH>(a.act_q, a.act_q_kf, t, k, v);
+            store_frag8<ARITH>(a.act_q, a.act_q_kf, t, k, o);
         }
+    };
+#pragma unroll
+    for (int g = 0; g < KEEP; ++g) finish(8 * (int)(threadIdx.x + 256 * g), v[g]);
+    for (int k = 8 * (int)(threadIdx.x + 256 * KEEP); k < padded; k += 8 * 256) {
+        float o[8];
+        load(k, o);
+        finish(k, o);
     }
 }
 
@@ -138,6 +169,23 @@ void k_latent_attention(LatentAttn a) {
     const int n_cols = row.n * a.H;
     auto low_of = [&](int pos) { return a.window > 0 ? max(row.kv_begin, pos - a.window + 1) : row.kv_begin; };
 
+    // the block's pages, dealt to the splits
+    const int last_tok = min(blk.col0 + a.block_cols, n_cols) - 1;
+    const int page_lo = low_of(row.pos0 + blk.col0 / a.H) / PAGE, page_hi = (row.pos0 + last_tok / a.H) / PAGE + 1;
+    const int n_all = page_hi - page_lo, sp = blockIdx.y;
+    const int first = page_lo + (int)((int64_t)n_all * sp / a.splits), end = page_lo + (int)((int64_t)n_all * (sp + 1) / a.splits);
+    const int n_iter = (end - first + WK - 1) / WK;
+    const int32_t * table = a.table + (size_t)row.slot * a.max_pages;
+    uint8_t * buf = lds + (size_t)wk * 2 * page_bytes;
+
+    auto stage = [&](int page, int b) {
+        if (page >= end) return;
+        const int id = __builtin_amdgcn_readfirstlane(table[page]);
+        const uint8_t * src = (const uint8_t *)a.pool + (size_t)id * page_bytes;
+        for (int ch = wc; ch < 2 * kf; ch += WC)
+            lds_dma16(src + ch * 1024, (uint32_t)lane * 16, lds_offset(buf + (size_t)b * page_bytes + ch * 1024));
+    };
+    stage(first + wk, 0);
     // this lane's column of every column tile: its token and head, and the keys it sees
     int col[CT], lo[CT], hi[CT], lo_max = 0, hi_min = 1 << 30;
     h8 q[CT][KF];
@@ -159,22 +207,6 @@ void k_latent_attention(LatentAttn a) {
         lo_max = max(lo_max, __shfl_xor(lo_max, o, 64));
         hi_min = min(hi_min, __shfl_xor(hi_min, o, 64));
     }
-    // the block's pages, dealt to the splits
-    const int last_tok = min(blk.col0 + a.block_cols, n_cols) - 1;
-    const int page_lo = low_of(row.pos0 + blk.col0 / a.H) / PAGE, page_hi = (row.pos0 + last_tok / a.H) / PAGE + 1;
-    const int n_all = page_hi - page_lo, sp = blockIdx.y;
-    const int first = page_lo + (int)((int64_t)n_all * sp / a.splits), end = page_lo + (int)((int64_t)n_all * (sp + 1) / a.splits);
-    const int n_iter = (end - first + WK - 1) / WK;
-    const int32_t * table = a.table + (size_t)row.slot * a.max_pages;
-    uint8_t * buf = lds + (size_t)wk * 2 * page_bytes;
-
-    auto stage = [&](int page, int b) {
-        if (page >= end) return;
-        const int id = __builtin_amdgcn_readfirstlane(table[page]);
-        const uint8_t * src = (const uint8_t *)a.pool + (size_t)id * page_bytes;
-        for (int ch = wc; ch < 2 * kf; ch += WC)
-            lds_dma16(src + ch * 1024, (uint32_t)lane * 16, lds_offset(buf + (size_t)b * page_bytes + ch * 1024));
-    };
     f4 acc[CT][2 * KF];
     float m[CT], l[CT];
 #pragma unroll
@@ -184,7 +216,6 @@ void k_latent_attention(LatentAttn a) {
 #pragma unroll
         for (int d = 0; d < 2 * KF; ++d) acc[c][d] = f4{0, 0, 0, 0};
     }
-    stage(first + wk, 0);
     const int idx = lane & 15;
     const int tr_lane = ((((idx >> 1) & 1) * 16 + 4 * g + (idx >> 2)) * 8 + (idx & 1) * 4) * 2;       // bytes into a 1 KiB piece
     for (int it = 0; it < n_iter; ++it) {
@@ -296,10 +327,17 @@ void k_latent_attention(LatentAttn a) {
         if (col[c] >= min(blk.col0 + a.block_cols, n_cols)) continue;
         const int tok = col[c] / a.H, h = col[c] - tok * a.H, t = row.tok_off + tok;
         if (a.splits > 1) {
-            float * o = a.partial + (((size_t)t * a.H + h) * a.splits + sp) * (size_t)(kf * 32 + 4);
-            if (g == 0) { o[kf * 32] = m[c]; o[kf * 32 + 1] = l[c]; }
+            const size_t at = ((size_t)t * a.H + h) * a.splits + sp;
+            if (g == 0) *(float2 *)(a.partial_ml + 2 * at) = make_float2(m[c], l[c]);
+            __half * o = (__half *)a.partial + at * (size_t)(kf * 32);
+            const float inv = l[c] > 0.0f ? 1.0f / l[c] : 0.0f;      // a split may lie outside this column's window
 #pragma unroll
-            for (int d = 0; d < 2 * KF; ++d) *(f4 *)(o + d * 16 + 4 * g) = acc[c][d];
+            for (int d = 0; d < 2 * KF; ++d) {
+                union { __half h[4]; uint2 u; } w;
+#pragma unroll
+                for (int i = 0; i < 4; ++i) w.h[i] = __float2half_rn(acc[c][d][i] * inv);
+                *(uint2 *)(o + d * 16 + 4 * g) = w.u;
+            }
         } else {
             const float inv = 1.0f / l[c];
 #pragma unroll
@@ -314,25 +352,33 @@ void k_latent_attention(LatentAttn a) {
     }
 }
 
-// Merges the splits of one query column: a wave per column, eight latent columns per lane and pass.
+// Merges the splits of one query column (at most 32), each a mean in f16 with its maximum and sum: a wave per column,
+// lane i the weight of split i; eight latent columns per lane and pass, the splits' values requested four at a time.
 __global__ __launch_bounds__(64) void k_latent_combine(LatentAttn a) {
-    const int R = a.kf * 32, t = blockIdx.x / a.H, h = blockIdx.x - t * a.H;
-    const float * p = a.partial + (size_t)blockIdx.x * a.splits * (R + 4);
-    float m = -INFINITY;
-    for (int s = 0; s < a.splits; ++s) m = fmaxf(m, p[(size_t)s * (R + 4) + R]);
-    float l = 0.0f;
-    for (int s = 0; s < a.splits; ++s) l += p[(size_t)s * (R + 4) + R + 1] * exp2f(p[(size_t)s * (R + 4) + R] - m);
-    const float inv = 1.0f / l;
-    for (int k = 8 * (int)threadIdx.x; k < R; k += 512) {
-        f4 x = {0, 0, 0, 0}, y = {0, 0, 0, 0};
-        for (int s = 0; s < a.splits; ++s) {
-            const float * o = p + (size_t)s * (R + 4);
-            const float f = exp2f(o[R] - m) * inv;
-            x += *(const f4 *)(o + k) * f;
-            y += *(const f4 *)(o + k + 4) * f;
+    const int R = a.kf * 32, t = blockIdx.x / a.H, h = blockIdx.x - t * a.H, lane = threadIdx.x;
+    const __half * p = (const __half *)a.partial + (size_t)blockIdx.x * a.splits * R;
+    const float * ml = a.partial_ml + (size_t)blockIdx.x * a.splits * 2;
+    const float m = lane < a.splits ? ml[2 * lane] : -INFINITY, l = lane < a.splits ? ml[2 * lane + 1] : 0.0f;
+    float top = m;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) top = fmaxf(top, __shfl_xor(top, o, 64));
+    const float f = l * exp2f(m - top);
+    const float mine = f / wave_sum(f);
+    for (int k0 = 0; k0 < R; k0 += 512) {
+        const int k = k0 + 8 * lane, kc = min(k, R - 8);
+        float v[8] = {};
+        for (int s = 0; s < a.splits; s += 4) {
+            h8 u[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) u[i] = load_h8(p + (size_t)min(s + i, a.splits - 1) * R + kc);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const float c = s + i < a.splits ? __shfl(mine, s + i, 64) : 0.0f;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) v[e] += (float)u[i][e] * c;
+            }
         }
-        const float v[8] = {x[0], x[1], x[2], x[3], y[0], y[1], y[2], y[3]};
-        store_frag8<ARITH_16>(a.out, a.out_kf, t, h * R + k, v);
+        if (k < R) store_frag8<ARITH_16>(a.out, a.out_kf, t, h * R + k, v);
     }
 }
 
@@ -363,8 +409,8 @@ __global__ void k_latent_cells(EL * __restrict__ pool, int kf, const int32_t * _
 void latent_norms(hipStream_t s, int arith, const LatentNorms & a, int T) {
     if (T <= 0) return;
     const dim3 grid((unsigned)T, a.kv_w ? 2u : 1u);
-    if (arith == ARITH_16) hipLaunchKernelGGL(k_latent_norms<ARITH_16>, grid, dim3(64), 0, s, a);
-    else hipLaunchKernelGGL(k_latent_norms<ARITH_32>, grid, dim3(64), 0, s, a);
+    if (arith == ARITH_16) hipLaunchKernelGGL(k_latent_norms<ARITH_16>, grid, dim3(256), 0, s, a);
+    else hipLaunchKernelGGL(k_latent_norms<ARITH_32>, grid, dim3(256), 0, s, a);
     check_launch("latent_norms");
 }
 
@@ -411,7 +457,7 @@ int latent_splits(int arith, const LatentAttn & a, int max_resident) {
     return std::max(1, std::min({256 / std::max(a.n_blocks, 1), pages / per, 32}));
 }
 
-size_t latent_partial_floats(int T, int H, int kf, int splits) { return splits > 1 ? (size_t)T * H * splits * (kf * 32 + 4) : 0; }
+size_t latent_partial_floats(int T, int H, int kf, int splits) { return splits > 1 ? (size_t)T * H * splits * (kf * 16 + 2) : 0; }
 
 void latent_attention(hipStream_t s, int arith, const LatentAttn & a, int T) {
     if (a.n_blocks <= 0) return;

@@ -6,35 +6,55 @@ namespace rk {
 
 namespace {
 
-template <int ARITH, int KIND>
-__global__ __launch_bounds__(256) void k_norm_act(float * __restrict__ x, const float * __restrict__ w, int E, float eps,
-                                                  const int32_t * __restrict__ rows, void * __restrict__ act, int kf, Slices add) {
-    extern __shared__ float row[];
+// VEC: rows of whole groups of four, read and written as such; the slices of a group are all requested at once.
+template <int ARITH, int KIND, bool VEC>
+__global__ __launch_bounds__(1024) void k_norm_act(float * __restrict__ x, const float * __restrict__ w, int E, float eps,
+                                                   const int32_t * __restrict__ rows, void * __restrict__ act, int kf, Slices add) {
+    extern __shared__ __attribute__((aligned(16))) float row[];
     __shared__ float scratch[16];
-    const int t = rows ? rows[blockIdx.x] : (int)blockIdx.x;
+    const int t = rows ? rows[blockIdx.x] : (int)blockIdx.x, n_thr = blockDim.x;
     float * xr = x + (size_t)t * E;
     float sum = 0.0f;
-    for (int k = threadIdx.x; k < E; k += 256) {
-        float v = xr[k];
-        if (add.n > 0) {
-            float d = 0.0f;
-            for (int i = 0; i < add.n; ++i) d += add.data[(size_t)i * add.stride + (size_t)t * E + k];
-            v += d;
-            xr[k] = v;
+    if constexpr (VEC) {
+        for (int k = 4 * (int)threadIdx.x; k < E; k += 4 * n_thr) {
+            f4 v = *(const f4 *)(xr + k);
+            if (add.n > 0) {
+                const float * from = add.data + (size_t)t * E + k;
+                f4 d[8];
+#pragma unroll
+                for (int i = 0; i < 8; ++i) if (i < add.n) d[i] = *(const f4 *)(from + (size_t)i * add.stride);
+                f4 s = {0, 0, 0, 0};
+#pragma unroll
+                for (int i = 0; i < 8; ++i) if (i < add.n) s += d[i];
+                v += s;
+                *(f4 *)(xr + k) = v;
+            }
+            *(f4 *)(row + k) = v;
+            sum += KIND == NORM_LAYER ? v[0] + v[1] + v[2] + v[3] : v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
         }
-        row[k] = v;
-        sum += KIND == NORM_LAYER ? v : v * v;
+    } else {
+        for (int k = threadIdx.x; k < E; k += n_thr) {
+            float v = xr[k];
+            if (add.n > 0) {
+                float d = 0.0f;
+                for (int i = 0; i < add.n; ++i) d += add.data[(size_t)i * add.stride + (size_t)t * E + k];
+                v += d;
+                xr[k] = v;
+            }
+            row[k] = v;
+            sum += KIND == NORM_LAYER ? v : v * v;
+        }
     }
     sum = block_sum(sum, scratch);
     float mean = 0.0f;
     if constexpr (KIND == NORM_LAYER) {
         mean = sum / (float)E;
         float q = 0.0f;
-        for (int k = threadIdx.x; k < E; k += 256) { const float d = row[k] - mean; q += d * d; }
+        for (int k = threadIdx.x; k < E; k += n_thr) { const float d = row[k] - mean; q += d * d; }
         sum = block_sum(q, scratch);
     }
     const float inv = 1.0f / sqrtf(sum / (float)E + eps);
-    for (int k = 8 * threadIdx.x; k < E; k += 8 * 256) {
+    for (int k = 8 * (int)threadIdx.x; k < E; k += 8 * n_thr) {
         float v[8];
 #pragma unroll
         for (int i = 0; i < 8; ++i) v[i] = k + i < E ? (row[k + i] - mean) * inv * w[k + i] : 0.0f;
@@ -56,13 +76,15 @@ void norm_act(hipStream_t s, int arith, int kind, float * x, const float * w, in
               int n_rows, void * act, int act_kf, const Slices & add) {
     if (n_rows <= 0) return;
     const size_t lds = (size_t)E * 4;
-    const dim3 grid((unsigned)n_rows), block(256);
+    const bool vec = E % 4 == 0 && add.n <= 8;
+    const dim3 grid((unsigned)n_rows), block(n_rows <= 512 && E >= 2048 ? 1024 : 256);
+    auto go = [&](auto kernel) { hipLaunchKernelGGL(kernel, grid, block, lds, s, x, w, E, eps, rows, act, act_kf, add); };
     if (arith == ARITH_16) {
-        if (kind == NORM_LAYER) hipLaunchKernelGGL((k_norm_act<ARITH_16, NORM_LAYER>), grid, block, lds, s, x, w, E, eps, rows, act, act_kf, add);
-        else hipLaunchKernelGGL((k_norm_act<ARITH_16, NORM_RMS>), grid, block, lds, s, x, w, E, eps, rows, act, act_kf, add);
+        if (kind == NORM_LAYER) vec ? go(k_norm_act<ARITH_16, NORM_LAYER, true>) : go(k_norm_act<ARITH_16, NORM_LAYER, false>);
+        else vec ? go(k_norm_act<ARITH_16, NORM_RMS, true>) : go(k_norm_act<ARITH_16, NORM_RMS, false>);
     } else {
-        if (kind == NORM_LAYER) hipLaunchKernelGGL((k_norm_act<ARITH_32, NORM_LAYER>), grid, block, lds, s, x, w, E, eps, rows, act, act_kf, add);
-        else hipLaunchKernelGGL((k_norm_act<ARITH_32, NORM_RMS>), grid, block, lds, s, x, w, E, eps, rows, act, act_kf, add);
+        if (kind == NORM_LAYER) vec ? go(k_norm_act<ARITH_32, NORM_LAYER, true>) : go(k_norm_act<ARITH_32, NORM_LAYER, false>);
+        else vec ? go(k_norm_act<ARITH_32, NORM_RMS, true>) : go(k_norm_act<ARITH_32, NORM_RMS, false>);
     }
     check_launch("norm_act");
 }

@@ -110,7 +110,8 @@ struct LatentAttn {
     const int32_t * table = nullptr;
     int max_pages = 0;
     const void * pool = nullptr;
-    float * partial = nullptr;     // [T * H][splits][kf * 32 + 4]: values, maximum, sum; when splits > 1
+    void * partial = nullptr;      // several splits: [T * H][splits][kf * 32] means in f16 ...
+    float * partial_ml = nullptr;  // ... and [T * H][splits][2] maxima and sums (latent_partial_floats() for both)
     void * out = nullptr;          // activations: column h * kf * 32 + c
     int out_kf = 0;
 };
