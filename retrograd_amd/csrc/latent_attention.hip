@@ -177,15 +177,16 @@ void k_latent_attention(LatentAttn a) {
     const int n_iter = (end - first + WK - 1) / WK;
     const int32_t * table = a.table + (size_t)row.slot * a.max_pages;
     uint8_t * buf = lds + (size_t)wk * 2 * page_bytes;
+    const uint32_t to = lds_offset(lds) + (uint32_t)(wk * 2 * page_bytes);
 
     auto stage = [&](int page, int b) {
         if (page >= end) return;
-        const int id = __builtin_amdgcn_readfirstlane(table[page]);
+        // a scalar load, which no vector load is waited for with
+        const int id = __builtin_amdgcn_readfirstlane(((const __attribute__((address_space(4))) int32_t *)table)[__builtin_amdgcn_readfirstlane(page)]);
         const uint8_t * src = (const uint8_t *)a.pool + (size_t)id * page_bytes;
         for (int ch = wc; ch < 2 * kf; ch += WC)
-            lds_dma16(src + ch * 1024, (uint32_t)lane * 16, lds_offset(buf + (size_t)b * page_bytes + ch * 1024));
+            lds_dma16(src + ch * 1024, (uint32_t)lane * 16, __builtin_amdgcn_readfirstlane(to + (uint32_t)(b * page_bytes + ch * 1024)));
     };
-    stage(first + wk, 0);
     // this lane's column of every column tile: its token and head, and the keys it sees
     int col[CT], lo[CT], hi[CT], lo_max = 0, hi_min = 1 << 30;
     h8 q[CT][KF];
@@ -218,11 +219,22 @@ void k_latent_attention(LatentAttn a) {
     }
     const int idx = lane & 15;
     const int tr_lane = ((((idx >> 1) & 1) * 16 + 4 * g + (idx >> 2)) * 8 + (idx & 1) * 4) * 2;       // bytes into a 1 KiB piece
+    stage(first + wk, 0);
+    stage(first + wk + WK, 1);
+#pragma unroll
+    for (int c = 0; c < CT; ++c)
+#pragma unroll
+        for (int j = 0; j < KF; ++j) asm volatile("" :: "v"(q[c][j]));      // the queries are waited for here, not in the loop
     for (int it = 0; it < n_iter; ++it) {
-        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-        __syncthreads();
+        // a page's loads and the next one's are on their way: wait for the former
         const int page = first + it * WK + wk;
-        stage(page + WK, (it + 1) & 1);
+        if (it > 0) {
+            __syncthreads();
+            stage(page + WK, (it + 1) & 1);
+        }
+        if (page + WK < end) asm volatile("s_waitcnt vmcnt(%0)" :: "n"(2 * KF / WC) : "memory");
+        else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads();
         if (page >= end) continue;
         const uint8_t * cur = buf + (size_t)(it & 1) * page_bytes;
         f4 s[2][CT];
