@@ -15,6 +15,7 @@ struct DenseArgs {
     int ksplit;            // workgroups that share a row group along K
     float * partial;       // [ksplit][rows padded to 64][N]
     size_t slice;
+    int grid_k;            // workgroups of one K-slice (the LDS kernel)
 };
 
 // One compiled form per pair of output kinds (part a, part b): a kernel that chose among all of them at run time would
@@ -256,9 +257,11 @@ __global__ __launch_bounds__(256, 2) void k_dense_lds(DenseArgs A, int n_tok_blo
     // workgroup b runs on XCD b % 8: an XCD takes every eighth row block, and walks eight token blocks per row block, so
     // that its concurrent workgroups share both operands in its L2
     const int n_groups = A.n_groups;
-    int gb, tb;
+    int gb, tb, ks;
     {
-        const int xcd = blockIdx.x & 7, i = blockIdx.x >> 3, per = (n_groups + 7) / 8, group = 8 * per;
+        const int b = A.ksplit > 1 ? blockIdx.x % A.grid_k : blockIdx.x;
+        ks = A.ksplit > 1 ? blockIdx.x / A.grid_k : 0;
+        const int xcd = b & 7, i = b >> 3, per = (n_groups + 7) / 8, group = 8 * per;
         const int band = i / group, r = i - band * group, tn = min(8, n_tok_blocks - band * 8);
         gb = (r / tn) * 8 + xcd;
         tb = band * 8 + r % tn;
@@ -312,7 +315,7 @@ __global__ __launch_bounds__(256, 2) void k_dense_lds(DenseArgs A, int n_tok_blo
         }
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");      // nothing may land in LDS that another workgroup owns by then
     };
-    auto store = [&](const float * scale) {
+    auto store = [&](const float * scale, bool first) {
 #pragma unroll
         for (int r = 0; r < RT; ++r) {
             const int tile = tile0 + wn * RT + r;
@@ -326,30 +329,43 @@ __global__ __launch_bounds__(256, 2) void k_dense_lds(DenseArgs A, int n_tok_blo
 #pragma unroll
             for (int c = 0; c < CT; ++c) {
                 const int t = (tok_tile0 + wt * CT + c) * 16 + (lane & 15);
-                if (t < A.T) store_rows<KA, KB, ARITH_16>(j, t, 0, tile, lane >> 4, acc[r][c] * f);
+                if (t >= A.T) continue;
+                if (DUAL && A.ksplit > 1) {                   // whole groups of four rows (see run)
+                    const int n = tile * 16 + 4 * (lane >> 4);
+                    if (n >= j.w.n) continue;
+                    f4 * p = (f4 *)(A.partial + (size_t)ks * A.slice + (size_t)t * j.w.n + n);
+                    f4 v = acc[r][c] * f;
+                    if (!first) v += *p;
+                    *p = v;
+                } else {
+                    store_rows<KA, KB, ARITH_16>(j, t, 0, tile, lane >> 4, acc[r][c] * f);
+                }
             }
         }
     };
     clear();
     if constexpr (DUAL) {
-        run(j.x, 0, j.kf1, 0);
-        store(j.scale1);
-        if (j.x2.x) {
+        const int lo = (int)((int64_t)j.w.kf * ks / A.ksplit), hi = (int)((int64_t)j.w.kf * (ks + 1) / A.ksplit);
+        if (lo < j.kf1) {
+            run(j.x, lo, min(hi, j.kf1), 0);
+            store(j.scale1, true);
             clear();
-            run(j.x2, j.kf1, j.w.kf, j.kf1);
-            store(j.scale2);
+        }
+        if (hi > j.kf1) {
+            run(j.x2, max(lo, j.kf1), hi, j.kf1);
+            store(j.scale2, lo >= j.kf1);
         }
     } else {
         run(j.x, 0, j.w.kf, 0);
-        store(nullptr);
+        store(nullptr, true);
     }
 }
 
 template <int KA, int KB, int RT, int CT> void launch_lds(hipStream_t s, DenseArgs & A) {
     A.n_groups = (A.j.w.tiles + 2 * RT - 1) / (2 * RT);
     const int tok_blocks = (A.T + 32 * CT - 1) / (32 * CT), bands = (tok_blocks + 7) / 8;
-    const dim3 grid((unsigned)(8 * bands * 8 * ((A.n_groups + 7) / 8)));
-    hipLaunchKernelGGL((k_dense_lds<KA, KB, RT, CT>), grid, dim3(256), 0, s, A, tok_blocks);
+    A.grid_k = 8 * bands * 8 * ((A.n_groups + 7) / 8);
+    hipLaunchKernelGGL((k_dense_lds<KA, KB, RT, CT>), dim3((unsigned)(A.grid_k * A.ksplit)), dim3(256), 0, s, A, tok_blocks);
 }
 
 template <typename TA, int KA, int KB, int RT, int CT, int KW, int RW> void launch(hipStream_t s, DenseArgs & A) {
@@ -371,6 +387,18 @@ template <int KA, int KB> Slices run(hipStream_t s, int arith, DenseArgs & A, fl
         else launch<float, KA, KB, 2, 4, 1, 4>(s, A);
         return out;
     }
+    // K-slices: workgroups that share rows along K leave partial results, added by the next norm
+    auto slice_k = [&](int want) {
+        A.ksplit = std::max(1, std::min({kMaxSlices, want, w.kf / 64}));
+        if (A.ksplit == 1) return;
+        A.partial = ws;
+        A.slice = (size_t)T * w.n;
+        out.data = ws;
+        out.n = A.ksplit;
+        out.stride = A.slice;
+        out.N = w.n;
+    };
+    const bool sliceable = KA == OUT_RESIDUAL && ws && (size_t)T * w.n <= kSliceFloats;
     if constexpr (KA != OUT_QUERY && KA != OUT_ACT_GATED) {        // products of one matrix
         if (w.batch == 1 && T > 128) {
             // the largest tile that leaves every CU a workgroup
@@ -378,25 +406,16 @@ template <int KA, int KB> Slices run(hipStream_t s, int arith, DenseArgs & A, fl
             if constexpr (KA != OUT_RESIDUAL) {
                 if (blocks(8, 4) >= 448) { launch_lds<KA, KB, 8, 4>(s, A); return out; }
             }
-            if (blocks(4, 4) >= 256) launch_lds<KA, KB, 4, 4>(s, A);
+            if (sliceable && w.n % 4 == 0 && blocks(4, 4) < 256) {
+                slice_k((int)(512 / blocks(4, 4)));
+                launch_lds<KA, KB, 4, 4>(s, A);
+            } else if (blocks(4, 4) >= 256) launch_lds<KA, KB, 4, 4>(s, A);
             else launch_lds<KA, KB, 4, 2>(s, A);
             return out;
         }
     }
     const bool deep = w.kf >= 16;
-    if (KA == OUT_RESIDUAL && deep && ws && (size_t)T * w.n <= kSliceFloats) {
-        // few rows: the workgroups that share a row group leave K-slices, added by the next norm
-        const int groups = T <= 16 ? w.tiles : (w.tiles + 1) / 2;
-        A.ksplit = std::max(1, std::min({kMaxSlices, 512 / std::max(groups, 1), w.kf / 64}));
-        if (A.ksplit > 1) {
-            A.partial = ws;
-            A.slice = (size_t)T * w.n;
-            out.data = ws;
-            out.n = A.ksplit;
-            out.stride = A.slice;
-            out.N = w.n;
-        }
-    }
+    if (deep && sliceable) slice_k(512 / std::max(T <= 16 ? w.tiles : (w.tiles + 1) / 2, 1));
     if (!deep) {                        // one wave has too little of K to share it
         if (T <= 16) launch<uint16_t, KA, KB, 1, 1, 1, 4>(s, A);
         else if (T <= 32) launch<uint16_t, KA, KB, 1, 2, 1, 4>(s, A);

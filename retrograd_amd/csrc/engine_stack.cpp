@@ -449,8 +449,13 @@ void Engine::forward_stack(int T, int n_out) {
             at.partial_ml = st_partial_.as<float>();
             at.partial = at.partial_ml + (size_t)T * H * at.splits * 2;
             at.out = st_ol_.ptr; at.out_kf = H * R;
-            rk::latent_attention(stream_, arith_, at, T);
+            rk::latent_attention(stream_, arith_, at);
             prof_end(PC_ATTN, pt);
+            if (at.splits > 1) {
+                pt = prof_begin(PC_COMBINE);
+                rk::latent_combine(stream_, at, T);
+                prof_end(PC_COMBINE, pt);
+            }
             pt = prof_begin(PC_OPROJ);
             rk::DenseJob uv;
             uv.w = L.uv.w;

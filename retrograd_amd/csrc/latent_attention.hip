@@ -471,7 +471,7 @@ int latent_splits(int arith, const LatentAttn & a, int max_resident) {
 
 size_t latent_partial_floats(int T, int H, int kf, int splits) { return splits > 1 ? (size_t)T * H * splits * (kf * 16 + 2) : 0; }
 
-void latent_attention(hipStream_t s, int arith, const LatentAttn & a, int T) {
+void latent_attention(hipStream_t s, int arith, const LatentAttn & a) {
     if (a.n_blocks <= 0) return;
     if (a.kf * 32 > 1024) throw std::runtime_error("latent attention: latents of at most 1024 columns");
     if (on_matrix_cores(arith, a.kf)) {
@@ -487,10 +487,6 @@ void latent_attention(hipStream_t s, int arith, const LatentAttn & a, int T) {
             default: throw std::runtime_error("latent attention: no kernel for this latent width");
         }
         check_launch("latent_attention");
-        if (a.splits > 1) {
-            hipLaunchKernelGGL(k_latent_combine, dim3((unsigned)(T * a.H)), dim3(64), 0, s, a);
-            check_launch("latent_combine");
-        }
         return;
     }
     const size_t lds = ((size_t)a.kf * 32 + 256) * 4;
@@ -498,6 +494,12 @@ void latent_attention(hipStream_t s, int arith, const LatentAttn & a, int T) {
     if (arith == ARITH_16) hipLaunchKernelGGL(k_latent_attention_any<ARITH_16>, grid, dim3(256), lds, s, a);
     else hipLaunchKernelGGL(k_latent_attention_any<ARITH_32>, grid, dim3(256), lds, s, a);
     check_launch("latent_attention");
+}
+
+void latent_combine(hipStream_t s, const LatentAttn & a, int T) {
+    if (a.splits <= 1 || T <= 0) return;
+    hipLaunchKernelGGL(k_latent_combine, dim3((unsigned)(T * a.H)), dim3(64), 0, s, a);
+    check_launch("latent_combine");
 }
 
 void latent_copy_page(hipStream_t s, void * pool, size_t page_bytes, int src, int dst) {

@@ -119,7 +119,8 @@ int latent_block_cols(int arith, int H, int kf, int n_tokens, int n_rows);
 // Workgroups that share a block's keys, given the longest resident span among the step's rows.
 int latent_splits(int arith, const LatentAttn & a, int max_resident);
 size_t latent_partial_floats(int T, int H, int kf, int splits);
-void latent_attention(hipStream_t s, int arith, const LatentAttn & a, int T);
+void latent_attention(hipStream_t s, int arith, const LatentAttn & a);
+void latent_combine(hipStream_t s, const LatentAttn & a, int T);      // of several splits (nothing to do for one)
 
 // Page copies and cell gathers of any pool of pages (elem bytes 2 or 4).
 void latent_copy_page(hipStream_t s, void * pool, size_t page_bytes, int src, int dst);
