@@ -199,6 +199,72 @@ def test_many_decoding_sequences(models, name, kv):
                 close(got[i], m.plain(prompts[i])[len(prompts[i]) + k], kv, (count, i))
 
 
+@pytest.mark.parametrize("kv", KINDS)
+@pytest.mark.parametrize("kv_rank", [20, 56, 90, 100, 190, 250, 330, 500, 600])
+def test_latent_widths_and_head_counts(tmp_path, kv_rank, kv):
+    """Every latent width the attention kernels are compiled for (and one beyond), with few, some and many heads: whole
+    prompts, decoding one sequence (whose keys are shared out) and many."""
+    for heads in (5, 20, 40):
+        m = Model(tmp_path / ("r%dh%d" % (kv_rank, heads)), Y.dibosun(48, 60, [
+            Y.latent_layer(heads=heads, dim=16, vdim=12, q_rank=24, kv_rank=kv_rank, window=150, ff=0, scale=1.0)]))
+        toks = m.tokens(230, heads)
+        want = m.plain(toks)
+        with m.engine(kv, n_ctx=256 * 12, slots=12) as eng:
+            close(feed(eng, 0, toks, [227, 1]), want, kv, (heads, "one"))
+            for s in range(1, 12):
+                eng.step_logits([(s, toks[:20 * s], 0)], [])
+            got = eng.step_logits([(s, [toks[20 * s]], 20 * s) for s in range(1, 12)], [(s, 0) for s in range(11)])
+            close(got, want[[20 * s for s in range(1, 12)]], kv, (heads, "many"))
+
+
+@pytest.mark.parametrize("kv", KINDS)
+def test_long_portions_of_many_heads(tmp_path, kv):
+    m = Model(tmp_path / "heads", Y.dibosun(48, 60, [Y.latent_layer(heads=64, dim=16, vdim=12, q_rank=24, kv_rank=64, window=90, ff=0, scale=1.0)]))
+    toks = m.tokens(530, 1)
+    with m.engine(kv, n_ctx=1024, n_batch=1024) as eng:
+        close(feed(eng, 0, toks, [530]), m.plain(toks), kv)
+
+
+TILES = {
+    # more rows in the input product, in the residual, and columns in the residual's product than one workgroup's share
+    "rows": (Y.dibosun(64, 50, [Y.latent_layer(heads=2, dim=16, vdim=16, q_rank=16, kv_rank=16, window=40, ff=28684)]), (520, 300, 140)),
+    "stream": (Y.dibosun(8204, 50, [Y.latent_layer(heads=2, dim=16, vdim=16, q_rank=16, kv_rank=16, window=40, ff=52)]), (520, 140)),
+    "columns": (Y.dibosun(132, 50, [Y.latent_layer(heads=16, dim=16, vdim=130, q_rank=16, kv_rank=48, window=40, ff=4100),
+                                    Y.mamba2_layer(heads=8, vdim=40, state=20, groups=2, conv=4, norm_groups=2, ff=4200)]), (300, 140, 64, 30, 9)),
+    "columns-odd": (Y.dibosun(131, 50, [Y.latent_layer(heads=16, dim=16, vdim=130, q_rank=16, kv_rank=48, window=40, ff=4100)]), (300, 60, 9)),
+    "queries": (Y.dibosun(64, 50, [Y.latent_layer(heads=300, dim=96, vdim=8, q_rank=40, kv_rank=30, window=40, ff=0)]), (530, 200)),
+}
+
+
+@pytest.mark.parametrize("kv", KINDS)
+@pytest.mark.parametrize("name", sorted(TILES))
+def test_products_of_every_tile_shape(tmp_path, name, kv):
+    cfg, sizes = TILES[name]
+    m = Model(tmp_path / name, cfg)
+    with m.engine(kv, n_ctx=1024, n_batch=576) as eng:
+        for n in sizes:
+            toks = m.tokens(n + 3, n)
+            want = m.plain(toks)
+            got = eng.step_logits([(0, toks[:n], 0)], [(0, k) for k in range(n)])
+            close(got, want[:n], kv, n)
+            close(feed(eng, 0, toks, [1], n), want[n:], kv, n)
+            eng.seq_rm(0)
+
+
+@pytest.mark.parametrize("kv", KINDS)
+def test_recurrence_of_unusual_sizes(tmp_path, kv):
+    """States beyond the chunked form, taps without a compiled form, columns that are no multiple of four or of a tile."""
+    m = Model(tmp_path / "odd", Y.dibosun(72, 50, [
+        Y.mamba2_layer(heads=3, vdim=100, state=130, groups=1, conv=5, norm_groups=3, ff=0),
+        Y.mamba2_layer(heads=4, vdim=30, state=50, groups=4, conv=1, norm_groups=1, ff=20),
+        Y.mamba2_layer(heads=2, vdim=33, state=128, groups=1, conv=3, norm_groups=6, ff=0)]))
+    toks = m.tokens(200, 3)
+    want = m.plain(toks)
+    with m.engine(kv) as eng:
+        close(feed(eng, 0, toks, [200]), want, kv)
+        close(feed(eng, 1, toks, [70, 63, 1, 2, 40, 1]), want, kv)
+
+
 def sharpen(cfg, tensors):
     """Queries of every head point at the keys that token 7 leaves, far above all others."""
     m = cfg["layers"][0]["mixer"]
