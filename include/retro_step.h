@@ -36,7 +36,8 @@ typedef enum retro_device {
     RETRO_DEVICE_GPU  = 2,
 } retro_device;
 
-/* ref h:88-93. Only F16 is implemented; the others are refused at creation. */
+/* ref h:88-93. GGUF models take F16, Q8_0 and Q4_0. Layer-stack models (a checkpoint folder) take F16 - products in
+ * bfloat16 with 32-bit accumulation, the latent cache in f16 - or F32: everything in 32-bit. */
 typedef enum retro_engine_kv_dtype {
     RETRO_ENGINE_KV_DTYPE_F32  = 0,
     RETRO_ENGINE_KV_DTYPE_F16  = 1,

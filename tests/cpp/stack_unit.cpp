@@ -1,0 +1,35 @@
+// Reads a checkpoint folder's config.json and model.safetensors with the engine's readers and prints what they found, or
+// the refusal. Built and driven by tests/test_stack_files.py; CPU only.
+#include <cstdio>
+#include <exception>
+
+#include "../../retrograd_amd/csrc/model_registry.hpp"
+#include "../../retrograd_amd/csrc/safetensors_file.hpp"
+
+int main(int argc, char ** argv) {
+    if (argc != 3) return 2;
+    const std::string folder = argv[1], what = argv[2];
+    try {
+        if (what == "config") {
+            const retro::StackConfig c = retro::StackConfig::read(folder);
+            std::printf("%s width %d vocab %d eps %g\n", c.arch->name, c.width, c.vocab, (double)c.eps);
+            for (const retro::LayerSpec & l : c.layers) {
+                const retro::LatentSpec & a = l.latent;
+                const rk::MambaShape & s = l.mamba;
+                if (l.mixer == retro::Mixer::MAMBA2)
+                    std::printf("mamba2 heads %d vdim %d state %d groups %d taps %d norm_groups %d ff %d\n", s.heads, s.vdim, s.state, s.groups, s.taps, s.norm_groups, l.ff);
+                else
+                    std::printf("latent heads %d dim %d vdim %d q_rank %d kv_rank %d window %d from %d scale %g ff %d\n", a.heads, a.dim, a.vdim, a.q_rank, a.kv_rank,
+                                a.window, a.kv_from, (double)a.scale, l.ff);
+            }
+        } else {
+            retro::SafetensorsFile f(folder + "/model.safetensors");
+            const retro::StTensor * t = f.find(what);
+            std::printf("%llu bytes, %s %s\n", (unsigned long long)f.tensor_bytes(), what.c_str(), t ? t->dtype.c_str() : "missing");
+        }
+        return 0;
+    } catch (const std::exception & e) {
+        std::printf("refused: %s\n", e.what());
+        return 1;
+    }
+}
