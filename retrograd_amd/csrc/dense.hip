@@ -16,7 +16,73 @@ struct DenseArgs {
     float * partial;       // [ksplit][rows padded to 64][N]
     size_t slice;
     int grid_k;            // workgroups of one K-slice (the LDS kernel)
+    ExpertGroups groups;
 };
+
+// Slots of an expert product's tile (a plain product: its tokens), and whose row the lane reads of slot `slot`.
+struct Columns { int b, first, end; };
+template <bool GROUPED> __device__ __forceinline__ bool columns_of(const DenseArgs & A, int tile, Columns & c) {
+    if constexpr (GROUPED) {
+        if (tile >= *A.groups.n_tiles) return false;
+        const int4 e = ((const int4 *)A.groups.tiles)[tile];
+        c = {e.x, e.y, e.y + e.z};
+    }
+    return true;
+}
+template <bool GROUPED> __device__ __forceinline__ int row_of(const DenseArgs & A, const Columns & c, int slot) {
+    if constexpr (GROUPED) {
+        if (A.j.gather) return A.groups.slot_pair[min(slot, c.end - 1)] / A.groups.top;
+    }
+    return slot;
+}
+
+// Four columns n .. n + 3 of token t: two pairs of one head.
+template <int ARITH> __device__ __forceinline__ void store_rotary(const DenseOut & o, int t, int n, f4 v) {
+    using EL = typename std::conditional<ARITH == ARITH_16, __half, float>::type;
+    const RotaryOut & r = o.rot;
+    const int head = n / (r.kf * 32), c = n - head * r.kf * 32;
+    f4 y = v;
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+        const int pair = (c >> 1) + i;
+        if (pair < r.pairs) {
+            const float2 cs = *(const float2 *)(r.table + 2 * ((size_t)t * r.pairs + pair));
+            y[2 * i] = v[2 * i] * cs.x - v[2 * i + 1] * cs.y;
+            y[2 * i + 1] = v[2 * i + 1] * cs.x + v[2 * i] * cs.y;
+        }
+    }
+    auto put = [](EL * dst, const f4 & u) {
+        if constexpr (ARITH == ARITH_16) {
+            union { __half h[4]; uint2 w; } p;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) p.h[i] = sat_half(u[i]);
+            *(uint2 *)dst = p.w;
+        } else {
+            *(f4 *)dst = u;
+        }
+    };
+    if (head < r.H) {
+        put((EL *)o.dst + ((size_t)t * r.H + head) * (r.kf * 32) + c, y);
+    } else {
+        const int cell = r.cell[t];
+        const size_t at = (size_t)(cell / PAGE) * cache_page_elems(r.kf * r.G) + cache_at(cell % PAGE, (head - r.H) * r.kf * 32 + c);
+        put((EL *)r.k_pool + at, y);
+        put((EL *)r.v_pool + at, v);
+    }
+}
+
+// gate and up of the same four columns
+template <int KIND> __device__ __forceinline__ f4 glu(const f4 & gate, const f4 & up) {
+    f4 v;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const float z = gate[i];
+        // 0.5 (1 + tanh(u)) = sigmoid(2 u)
+        const float u = KIND == OUT_ACT_GEGLU ? 1.5957691216057308f * (z + 0.044715f * z * z * z) : z;
+        v[i] = z / (1.0f + expf(-u)) * up[i];
+    }
+    return v;
+}
 
 // One compiled form per pair of output kinds (part a, part b): a kernel that chose among all of them at run time would
 // spend more on fetching its epilogue's instructions than on a product of a few hundred columns.
@@ -25,12 +91,16 @@ __device__ __forceinline__ void store_out(const DenseOut & o, int t, int b, int 
     // rows n .. n + 3 of token t (those below n_end are real)
     const int cnt = n_end - n;
     if (cnt <= 0) return;
+    if constexpr (KIND == OUT_ROTARY) {
+        store_rotary<ARITH>(o, t, n, v);
+        return;
+    }
     if constexpr (KIND == OUT_ACT_RELU2) {
 #pragma unroll
         for (int i = 0; i < 4; ++i) { const float r = fmaxf(v[i], 0.0f); v[i] = r * r; }
     } else if constexpr (KIND == OUT_ACT_GATED) {
         v *= 1.0f / (1.0f + expf(-o.gate[(size_t)t * o.ld_gate + b]));
-    } else if constexpr (KIND != OUT_RESIDUAL) {
+    } else if constexpr (KIND != OUT_RESIDUAL && !out_is_glu(KIND) && KIND != OUT_EXPERT) {
         v *= o.scale;
     }
     const int col = o.col0 + (KIND == OUT_QUERY ? 0 : b * o.col_batch) + n;
@@ -75,10 +145,43 @@ __device__ __forceinline__ void store_out(const DenseOut & o, int t, int b, int 
 }
 
 // Rows tile * 16 + 4 g .. + 3 of token t to the part they belong to (KB < 0: there is only part a).
+// A gated part is stored at its gate tiles (the even ones of the part, which starts at an even tile): `next` holds the
+// rows of the tile behind, its up rows.
 template <int KA, int KB, int ARITH>
-__device__ __forceinline__ void store_rows(const DenseJob & j, int t, int b, int tile, int g, const f4 & v) {
-    if (KB < 0 || tile < j.split_tile) store_out<KA, ARITH>(j.a, t, b, tile * 16 + 4 * g, j.n_a, v);
-    else if constexpr (KB >= 0) store_out<KB, ARITH>(j.b, t, b, (tile - j.split_tile) * 16 + 4 * g, j.w.n - j.split_tile * 16, v);
+__device__ __forceinline__ void store_rows(const DenseJob & j, int t, int b, int tile, int g, const f4 & v, const f4 & next) {
+    if (KB < 0 || tile < j.split_tile) {
+        if constexpr (out_is_glu(KA)) {
+            if (tile & 1) return;
+            store_out<KA, ARITH>(j.a, t, b, tile * 8 + 4 * g, j.n_a / 2, glu<KA>(v, next));
+        } else {
+            store_out<KA, ARITH>(j.a, t, b, tile * 16 + 4 * g, j.n_a, v);
+        }
+    } else if constexpr (KB >= 0) {
+        const int rows = j.w.n - j.split_tile * 16, at = tile - j.split_tile;
+        if constexpr (out_is_glu(KB)) {
+            if (at & 1) return;
+            store_out<KB, ARITH>(j.b, t, b, at * 8 + 4 * g, rows / 2, glu<KB>(v, next));
+        } else {
+            store_out<KB, ARITH>(j.b, t, b, at * 16 + 4 * g, rows, v);
+        }
+    }
+}
+
+// An expert's rows of the pair in slot t.
+__device__ __forceinline__ void store_expert(const DenseArgs & A, int t, int n, f4 v) {
+    const DenseOut & o = A.j.a;
+    const int cnt = A.j.w.n - n;
+    if (cnt <= 0) return;
+    const int pair = A.groups.slot_pair[t], token = pair / A.groups.top, choice = pair - token * A.groups.top;
+    v *= A.groups.weight[pair];
+    float * y = (float *)o.dst + (size_t)choice * o.stride + (size_t)token * o.ld + n;
+    if (cnt >= 4 && (o.ld & 3) == 0) *(f4 *)y = v;
+    else
+        for (int i = 0; i < 4 && i < cnt; ++i) y[i] = v[i];
+}
+
+__device__ __forceinline__ float token_factor(const DenseJob & j, int t) {
+    return j.token_gate ? 1.0f / (1.0f + expf(-j.token_gate[(size_t)t * j.ld_token_gate])) : 1.0f;
 }
 
 template <typename TA> struct Operand;      // one lane's eight activation values of a fragment
@@ -106,16 +209,18 @@ __device__ __forceinline__ void mac(f4 & acc, const b8 & w, const Operand<float>
 
 // Operands straight from memory to registers: a wave multiplies RT row tiles with CT token tiles; KW waves of the
 // workgroup share the rows and split K, RW sets of them split the rows.
-template <typename TA, int KA, int KB, int RT, int CT, int KW, int RW>
+template <typename TA, int KA, int KB, int RT, int CT, int KW, int RW, bool GROUPED>
 __global__ __launch_bounds__(64 * KW * RW) void k_dense(DenseArgs A) {
     constexpr bool DUAL = KA == OUT_RESIDUAL;
+    static_assert(RT % 2 == 0 || !(out_is_glu(KA) || out_is_glu(KB)));
     constexpr int U = sizeof(TA) == 4 ? 2 : (RT * CT >= 8 ? 2 : 4);      // fragments in flight per operand
     const DenseJob & j = A.j;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int kw = wave % KW, rw = wave / KW;
     const int group = blockIdx.x % A.n_groups, ks = blockIdx.x / A.n_groups;
-    const int b = blockIdx.z;
-    const int tok_tile0 = blockIdx.y * CT;
+    Columns cols = {(int)blockIdx.z, (int)blockIdx.y * CT * 16, A.T};
+    if (!columns_of<GROUPED>(A, blockIdx.y, cols)) return;
+    const int b = cols.b;
     const int tile0 = (group * RW + rw) * RT;
     const uint16_t * wbase[RT];
 #pragma unroll
@@ -135,7 +240,10 @@ __global__ __launch_bounds__(64 * KW * RW) void k_dense(DenseArgs A) {
         const TA * xb[CT];
 #pragma unroll
         for (int c = 0; c < CT; ++c)
-            xb[c] = (const TA *)in.x + ((size_t)(tok_tile0 + c) * in.kf + (size_t)b * in.kf_batch) * 512 + lane * 8 - (ptrdiff_t)base * 512;
+        {
+            const int row = row_of<GROUPED>(A, cols, cols.first + c * 16 + (lane & 15));
+            xb[c] = (const TA *)in.x + ((size_t)(row >> 4) * in.kf + (GROUPED ? 0 : (size_t)b * in.kf_batch)) * 512 + ((lane & 48) | (row & 15)) * 8 - (ptrdiff_t)base * 512;
+        }
         int k = lo;
         for (; k + U <= hi; k += U) {
             b8 w[U][RT];
@@ -218,26 +326,29 @@ __global__ __launch_bounds__(64 * KW * RW) void k_dense(DenseArgs A) {
         if (tile >= j.w.tiles) break;
 #pragma unroll
         for (int c = 0; c < CT; ++c) {
-            const int t = (tok_tile0 + c) * 16 + (lane & 15);
-            if (t >= A.T) continue;
-            if (DUAL && A.ksplit > 1) {
+            const int t = cols.first + c * 16 + (lane & 15);
+            if (t >= cols.end) continue;
+            if constexpr (DUAL) acc[r][c] *= token_factor(j, t);
+            if constexpr (KA == OUT_EXPERT) {
+                store_expert(A, t, tile * 16 + 4 * (lane >> 4), acc[r][c]);
+            } else if (DUAL && A.ksplit > 1) {
                 const int n = tile * 16 + 4 * (lane >> 4);
                 float * p = A.partial + (size_t)ks * A.slice + (size_t)t * j.w.n + n;
                 if (n + 4 <= j.w.n && (j.w.n & 3) == 0) *(f4 *)p = acc[r][c];
                 else for (int i = 0; i < 4 && n + i < j.w.n; ++i) p[i] = acc[r][c][i];
             } else {
-                store_rows<KA, KB, ARITH>(j, t, b, tile, lane >> 4, acc[r][c]);
+                store_rows<KA, KB, ARITH>(j, t, GROUPED ? 0 : b, tile, lane >> 4, acc[r][c], acc[RT > 1 ? r ^ 1 : r][c]);
             }
         }
     }
 }
 
 __global__ void k_dense_pack(const uint16_t * __restrict__ src, int rows, int cols, int64_t rs, int64_t cs,
-                             uint16_t * __restrict__ dst, int kf, int row0, int k0) {
+                             uint16_t * __restrict__ dst, int kf, PackMap row, PackMap col) {
     const int64_t n = (int64_t)rows * cols;
     for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (int64_t)gridDim.x * blockDim.x) {
         const int r = (int)(i / cols), c = (int)(i % cols);
-        dst[frag_at(row0 + r, k0 + c, kf)] = src[r * rs + c * cs];
+        dst[frag_at(row.at + r / row.run * row.step + r % row.run, col.at + c / col.run * col.step + c % col.run, kf)] = src[r * rs + c * cs];
     }
 }
 
@@ -245,7 +356,7 @@ __global__ void k_dense_pack(const uint16_t * __restrict__ src, int rows, int co
 // waves along each, a wave RT x CT tiles. Fragments of both operands go to LDS by direct loads in the order they are
 // stored in; three buffers, so that two fragments are on their way while one is multiplied. A two-part product adds its
 // first part to the residual, then its second.
-template <int KA, int KB, int RT, int CT>
+template <int KA, int KB, int RT, int CT, bool GROUPED>
 __global__ __launch_bounds__(256, 2) void k_dense_lds(DenseArgs A, int n_tok_blocks) {
     constexpr bool DUAL = KA == OUT_RESIDUAL;
     constexpr int PIECES = 2 * RT + 2 * CT;                   // KiB of a stage: its row tiles, then its token tiles
@@ -258,7 +369,12 @@ __global__ __launch_bounds__(256, 2) void k_dense_lds(DenseArgs A, int n_tok_blo
     // that its concurrent workgroups share both operands in its L2
     const int n_groups = A.n_groups;
     int gb, tb, ks;
-    {
+    if constexpr (GROUPED) {           // the row blocks of a tile of slots on one XCD, which keeps the gathered rows in its L2
+        const int i = blockIdx.x >> 3;
+        gb = i % n_groups;
+        tb = (i / n_groups) * 8 + (blockIdx.x & 7);
+        ks = 0;
+    } else {
         const int b = A.ksplit > 1 ? blockIdx.x % A.grid_k : blockIdx.x;
         ks = A.ksplit > 1 ? blockIdx.x / A.grid_k : 0;
         const int xcd = b & 7, i = b >> 3, per = (n_groups + 7) / 8, group = 8 * per;
@@ -267,7 +383,10 @@ __global__ __launch_bounds__(256, 2) void k_dense_lds(DenseArgs A, int n_tok_blo
         tb = band * 8 + r % tn;
         if (gb >= n_groups || tb >= n_tok_blocks || r / tn >= per) return;
     }
-    const int tile0 = gb * 2 * RT, tok_tile0 = tb * 2 * CT;
+    Columns cols = {0, tb * 32 * CT, A.T};
+    if (!columns_of<GROUPED>(A, tb, cols)) return;
+    const int tile0 = gb * 2 * RT;
+    const uint16_t * weights = j.w.w + (size_t)cols.b * j.w.tiles * j.w.kf * 512;
     f4 acc[RT][CT];
     auto clear = [&]() {
 #pragma unroll
@@ -279,18 +398,24 @@ __global__ __launch_bounds__(256, 2) void k_dense_lds(DenseArgs A, int n_tok_blo
         const int n = hi - lo;
         if (n <= 0) return;
         const uint8_t * src[PER_WAVE];
+        uint32_t off[GROUPED ? PER_WAVE : 1];                 // the lane's place: a row of its own where rows are gathered
 #pragma unroll
         for (int i = 0; i < PER_WAVE; ++i) {
             const int piece = wave + 4 * i;
-            if (piece < 2 * RT) src[i] = (const uint8_t *)(j.w.w + ((size_t)min(tile0 + piece, j.w.tiles - 1) * j.w.kf + lo) * 512);
-            else src[i] = (const uint8_t *)((const uint16_t *)in.x + ((size_t)(tok_tile0 + piece - 2 * RT) * in.kf + (lo - base)) * 512);
+            if constexpr (GROUPED) off[i] = (uint32_t)lane * 16;
+            if (piece < 2 * RT) src[i] = (const uint8_t *)(weights + ((size_t)min(tile0 + piece, j.w.tiles - 1) * j.w.kf + lo) * 512);
+            else if constexpr (GROUPED) {
+                const int row = row_of<GROUPED>(A, cols, cols.first + (piece - 2 * RT) * 16 + (lane & 15));
+                src[i] = (const uint8_t *)((const uint16_t *)in.x + (size_t)(lo - base) * 512);
+                off[i] = (uint32_t)(row >> 4) * (uint32_t)in.kf * 1024 + (uint32_t)((lane & 48) | (row & 15)) * 16;
+            } else src[i] = (const uint8_t *)((const uint16_t *)in.x + ((size_t)((cols.first >> 4) + piece - 2 * RT) * in.kf + (lo - base)) * 512);
         }
         const uint32_t to = lds_offset(lds);
         auto stage = [&](int k, int b) {
             const int kk = min(k, n - 1);
 #pragma unroll
             for (int i = 0; i < PER_WAVE; ++i)
-                lds_dma16(src[i] + (size_t)kk * 1024, (uint32_t)lane * 16, to + (uint32_t)(b * PIECES + wave + 4 * i) * 1024);
+                lds_dma16(src[i] + (size_t)kk * 1024, GROUPED ? off[GROUPED ? i : 0] : (uint32_t)lane * 16, to + (uint32_t)(b * PIECES + wave + 4 * i) * 1024);
         };
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");      // the part before has stored, and the counted waits start at none
         __syncthreads();                                      // the buffers may still be read by the part before
@@ -328,17 +453,20 @@ __global__ __launch_bounds__(256, 2) void k_dense_lds(DenseArgs A, int n_tok_blo
             }
 #pragma unroll
             for (int c = 0; c < CT; ++c) {
-                const int t = (tok_tile0 + wt * CT + c) * 16 + (lane & 15);
-                if (t >= A.T) continue;
-                if (DUAL && A.ksplit > 1) {                   // whole groups of four rows (see run)
+                const int t = cols.first + (wt * CT + c) * 16 + (lane & 15);
+                if (t >= cols.end) continue;
+                f4 v = acc[r][c];
+                if constexpr (DUAL) v *= f * token_factor(j, t);
+                if constexpr (KA == OUT_EXPERT) {
+                    store_expert(A, t, tile * 16 + 4 * (lane >> 4), v);
+                } else if (DUAL && A.ksplit > 1) {            // whole groups of four rows (see run)
                     const int n = tile * 16 + 4 * (lane >> 4);
                     if (n >= j.w.n) continue;
                     f4 * p = (f4 *)(A.partial + (size_t)ks * A.slice + (size_t)t * j.w.n + n);
-                    f4 v = acc[r][c] * f;
                     if (!first) v += *p;
                     *p = v;
                 } else {
-                    store_rows<KA, KB, ARITH_16>(j, t, 0, tile, lane >> 4, acc[r][c] * f);
+                    store_rows<KA, KB, ARITH_16>(j, t, 0, tile, lane >> 4, v, acc[r ^ 1][c]);
                 }
             }
         }
@@ -361,18 +489,29 @@ __global__ __launch_bounds__(256, 2) void k_dense_lds(DenseArgs A, int n_tok_blo
     }
 }
 
+template <int KA, int RT, int CT> void launch_lds_groups(hipStream_t s, DenseArgs & A) {
+    A.n_groups = (A.j.w.tiles + 2 * RT - 1) / (2 * RT);
+    const int tiles = (A.groups.max_tiles + 7) / 8 * 8;
+    hipLaunchKernelGGL((k_dense_lds<KA, -1, RT, CT, true>), dim3((unsigned)(A.n_groups * tiles)), dim3(256), 0, s, A, tiles);
+}
+template <typename TA, int KA, int RT, int CT, int KW, int RW> void launch_groups(hipStream_t s, DenseArgs & A) {
+    A.n_groups = (A.j.w.tiles + RT * RW - 1) / (RT * RW);
+    const dim3 grid((unsigned)A.n_groups, (unsigned)A.groups.max_tiles);
+    hipLaunchKernelGGL((k_dense<TA, KA, -1, RT, CT, KW, RW, true>), grid, dim3(64 * KW * RW), 0, s, A);
+}
+
 template <int KA, int KB, int RT, int CT> void launch_lds(hipStream_t s, DenseArgs & A) {
     A.n_groups = (A.j.w.tiles + 2 * RT - 1) / (2 * RT);
     const int tok_blocks = (A.T + 32 * CT - 1) / (32 * CT), bands = (tok_blocks + 7) / 8;
     A.grid_k = 8 * bands * 8 * ((A.n_groups + 7) / 8);
-    hipLaunchKernelGGL((k_dense_lds<KA, KB, RT, CT>), dim3((unsigned)(A.grid_k * A.ksplit)), dim3(256), 0, s, A, tok_blocks);
+    hipLaunchKernelGGL((k_dense_lds<KA, KB, RT, CT, false>), dim3((unsigned)(A.grid_k * A.ksplit)), dim3(256), 0, s, A, tok_blocks);
 }
 
 template <typename TA, int KA, int KB, int RT, int CT, int KW, int RW> void launch(hipStream_t s, DenseArgs & A) {
     const DenseJob & j = A.j;
     A.n_groups = (j.w.tiles + RT * RW - 1) / (RT * RW);
     const dim3 grid((unsigned)(A.n_groups * A.ksplit), (unsigned)((A.T + 16 * CT - 1) / (16 * CT)), (unsigned)j.w.batch);
-    hipLaunchKernelGGL((k_dense<TA, KA, KB, RT, CT, KW, RW>), grid, dim3(64 * KW * RW), 0, s, A);
+    hipLaunchKernelGGL((k_dense<TA, KA, KB, RT, CT, KW, RW, false>), grid, dim3(64 * KW * RW), 0, s, A);
 }
 
 constexpr int kMaxSlices = 8;
@@ -382,8 +521,10 @@ template <int KA, int KB> Slices run(hipStream_t s, int arith, DenseArgs & A, fl
     Slices out;
     const int T = A.T;
     const DenseWeight & w = A.j.w;
+    constexpr bool PAIRS = out_is_glu(KA) || out_is_glu(KB);      // row tiles in pairs
+    constexpr int R1 = PAIRS ? 2 : 1;
     if (arith == ARITH_32) {
-        if (T <= 16) launch<float, KA, KB, 1, 1, 4, 1>(s, A);
+        if (T <= 16) launch<float, KA, KB, R1, 1, 4, 1>(s, A);
         else launch<float, KA, KB, 2, 4, 1, 4>(s, A);
         return out;
     }
@@ -417,23 +558,47 @@ template <int KA, int KB> Slices run(hipStream_t s, int arith, DenseArgs & A, fl
     const bool deep = w.kf >= 16;
     if (deep && sliceable) slice_k(512 / std::max(T <= 16 ? w.tiles : (w.tiles + 1) / 2, 1));
     if (!deep) {                        // one wave has too little of K to share it
-        if (T <= 16) launch<uint16_t, KA, KB, 1, 1, 1, 4>(s, A);
-        else if (T <= 32) launch<uint16_t, KA, KB, 1, 2, 1, 4>(s, A);
-        else launch<uint16_t, KA, KB, 1, 4, 1, 4>(s, A);
-    } else if (T <= 16) launch<uint16_t, KA, KB, 1, 1, 8, 1>(s, A);
+        if (T <= 16) launch<uint16_t, KA, KB, R1, 1, 1, 4>(s, A);
+        else if (T <= 32) launch<uint16_t, KA, KB, R1, 2, 1, 4>(s, A);
+        else launch<uint16_t, KA, KB, R1, 4, 1, 4>(s, A);
+    } else if (T <= 16) launch<uint16_t, KA, KB, R1, 1, 8, 1>(s, A);
     else if (T <= 32) launch<uint16_t, KA, KB, 2, 2, 8, 1>(s, A);
     else launch<uint16_t, KA, KB, 2, 4, 8, 1>(s, A);
     return out;
 }
 
+// Products of the pairs of every expert: short tiles straight to registers, longer ones through LDS.
+template <int KA> void run_groups(hipStream_t s, int arith, DenseArgs & A) {
+    constexpr int R1 = out_is_glu(KA) ? 2 : 1;
+    const int block = A.groups.block;
+    if (arith == ARITH_32) {
+        if (block == 16) launch_groups<float, KA, R1, 1, 4, 1>(s, A);
+        else launch_groups<float, KA, 2, 4, 1, 4>(s, A);
+        return;
+    }
+    const bool deep = A.j.w.kf >= 16;
+    switch (block) {
+        case 16: deep ? launch_groups<uint16_t, KA, R1, 1, 8, 1>(s, A) : launch_groups<uint16_t, KA, R1, 1, 1, 4>(s, A); break;
+        case 32: deep ? launch_groups<uint16_t, KA, 2, 2, 8, 1>(s, A) : launch_groups<uint16_t, KA, R1, 2, 1, 4>(s, A); break;
+        case 64: launch_lds_groups<KA, 4, 2>(s, A); break;
+        default: launch_lds_groups<KA, 4, 4>(s, A); break;
+    }
+}
+
 }  // namespace
 
+int expert_block(int arith, int T, int top, int experts) {
+    const int mean = (T * top + experts - 1) / experts;      // pairs of an expert
+    if (arith == ARITH_32) return mean <= 16 ? 16 : 64;
+    return mean <= 8 ? 16 : mean <= 24 ? 32 : mean <= 96 ? 64 : 128;
+}
+
 void dense_pack(hipStream_t s, const uint16_t * src, int rows, int cols, int64_t row_stride, int64_t k_stride,
-                uint16_t * dst, int kf, int row0, int k0) {
+                uint16_t * dst, int kf, PackMap row, PackMap column) {
     if (rows <= 0 || cols <= 0) return;
     const int64_t n = (int64_t)rows * cols;
     hipLaunchKernelGGL(k_dense_pack, dim3((unsigned)std::min<int64_t>((n + 255) / 256, 8192)), dim3(256), 0, s, src, rows, cols,
-                       row_stride, k_stride, dst, kf, row0, k0);
+                       row_stride, k_stride, dst, kf, row, column);
     check_launch("dense_pack");
 }
 
@@ -447,17 +612,35 @@ Slices dense(hipStream_t s, int arith, const DenseJob & job, int T, float * ws) 
     A.ksplit = 1;
     A.partial = nullptr;
     A.slice = 0;
+    if (job.groups) {
+        A.groups = *job.groups;
+        if (A.groups.max_tiles <= 0) return Slices();
+        A.j.split_tile = A.j.w.tiles;
+        A.j.n_a = A.j.w.n;
+        switch (job.a.kind) {
+            case OUT_ACT_SWIGLU: run_groups<OUT_ACT_SWIGLU>(s, arith, A); break;
+            case OUT_EXPERT: run_groups<OUT_EXPERT>(s, arith, A); break;
+            default: throw std::runtime_error("dense: this output of an expert product is not compiled");
+        }
+        check_launch("dense");
+        return Slices();
+    }
     const bool two = A.j.n_a > 0 && A.j.split_tile < A.j.w.tiles;
     if (!two) { A.j.split_tile = A.j.w.tiles; A.j.n_a = A.j.w.n; }
     Slices out;
     if (two) {
-        if (job.a.kind != OUT_F32 || job.b.kind != OUT_ACT_RELU2) throw std::runtime_error("dense: this pair of outputs is not compiled");
-        out = run<OUT_F32, OUT_ACT_RELU2>(s, arith, A, ws);
+        if (job.a.kind == OUT_F32 && job.b.kind == OUT_ACT_RELU2) out = run<OUT_F32, OUT_ACT_RELU2>(s, arith, A, ws);
+        else if (job.a.kind == OUT_F32 && job.b.kind == OUT_ACT_SWIGLU) out = run<OUT_F32, OUT_ACT_SWIGLU>(s, arith, A, ws);
+        else throw std::runtime_error("dense: this pair of outputs is not compiled");
     } else {
         switch (job.a.kind) {
             case OUT_F32: out = run<OUT_F32, -1>(s, arith, A, ws); break;
             case OUT_ACT: out = run<OUT_ACT, -1>(s, arith, A, ws); break;
             case OUT_ACT_GATED: out = run<OUT_ACT_GATED, -1>(s, arith, A, ws); break;
+            case OUT_ACT_GEGLU: out = run<OUT_ACT_GEGLU, -1>(s, arith, A, ws); break;
+            case OUT_ACT_SWIGLU: out = run<OUT_ACT_SWIGLU, -1>(s, arith, A, ws); break;
+            case OUT_ACT_RELU2: out = run<OUT_ACT_RELU2, -1>(s, arith, A, ws); break;
+            case OUT_ROTARY: out = run<OUT_ROTARY, -1>(s, arith, A, ws); break;
             case OUT_QUERY: out = run<OUT_QUERY, -1>(s, arith, A, ws); break;
             case OUT_RESIDUAL: out = run<OUT_RESIDUAL, -1>(s, arith, A, ws); break;
             default: throw std::runtime_error("dense: this output is not compiled");

@@ -560,7 +560,7 @@ void Engine::cells_gather(const CachePart & part, const int32_t * cells, int n, 
     const PoolView & pool = (part.v ? v_pool_ : k_pool_)[(size_t)part.layer];
     if (stack_) {
         const int elem = arith_;
-        rk::latent_cells(stream_, pool.ptr, (int)(part.row_bytes / (32 * (size_t)elem)), elem, cells, n, out, true);
+        rk::stack_cells(stream_, pool.ptr, (int)(part.row_bytes / (32 * (size_t)elem)), elem, cells, n, out, true);
     } else {
         rk::kv_gather(stream_, pool.as<__half>(), kv_strides_, hp_.n_head_kv, hp_.head_dim, part.v, cells, n, (__half *)out, kv_q8_);
     }
@@ -570,7 +570,7 @@ void Engine::cells_scatter(const CachePart & part, const int32_t * cells, int n,
     const PoolView & pool = (part.v ? v_pool_ : k_pool_)[(size_t)part.layer];
     if (stack_) {
         const int elem = arith_;
-        rk::latent_cells(stream_, pool.ptr, (int)(part.row_bytes / (32 * (size_t)elem)), elem, cells, n, const_cast<void *>(in), false);
+        rk::stack_cells(stream_, pool.ptr, (int)(part.row_bytes / (32 * (size_t)elem)), elem, cells, n, const_cast<void *>(in), false);
     } else {
         rk::kv_scatter(stream_, pool.as<__half>(), kv_strides_, hp_.n_head_kv, hp_.head_dim, part.v, cells, n, (const __half *)in, kv_q8_);
     }
@@ -579,7 +579,7 @@ void Engine::cells_scatter(const CachePart & part, const int32_t * cells, int n,
 void Engine::copy_page(int32_t src, int32_t dst) {
     if (stack_) {
         for (const CachePart & p : cache_parts_)
-            rk::latent_copy_page(stream_, k_pool_[(size_t)p.layer].ptr, p.row_bytes * rk::PAGE, src, dst);
+            rk::stack_copy_page(stream_, (p.v ? v_pool_ : k_pool_)[(size_t)p.layer].ptr, p.row_bytes * rk::PAGE, src, dst);
         return;
     }
     for (int l = 0; l < hp_.n_layer; ++l) {

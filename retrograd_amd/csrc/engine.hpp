@@ -81,20 +81,30 @@ struct LayerWeights {
 };
 
 // A layer of a layer-stack model on the device. Everything that reads the layer's norm is one matrix (w_in: the mixer's
-// input projections as f32 columns, then the feed-forward's up rows), everything that adds to the stream another (w_out:
-// the mixer's output projection and the feed-forward's down projection side by side along K).
+// input projections, of a parallel layer then the feed-forward's up rows), everything that adds to the stream another
+// (w_out: the mixer's output projection, of a parallel layer with the feed-forward's down projection beside it along K).
+// The feed-forward of a sequential layer: ff_in (gate and up rows in turn, tile by tile; with experts the router's
+// logits and the shared expert's gate before the shared expert's rows) and ff_out.
 struct StackLayer {
     struct Matrix { rk::DenseWeight w; DevBuf buf; };
     LayerSpec spec;
-    DevBuf norm, scale_mix, scale_ff;
-    Matrix w_in, w_out;
+    DevBuf norm, norm2, scale_mix, scale_ff;
+    Matrix w_in, w_out, ff_in, ff_out;
     int in_tiles = 0, in_rows = 0;          // row tiles and rows of w_in that belong to the mixer
+    int route_tiles = 0;                    // row tiles of ff_in that belong to the router
     int kv_col = 0, gate_col = 0;           // columns of the input product: the latent, the head gates
     DevBuf q_norm, kv_norm;
     Matrix uq, uk, uv;                      // queries from their latent; per head: absorption and value up-projection
     DevBuf conv_w, conv_b, dt_bias, A_log, D, gate_norm;
-    int pool_layer = -1;                    // the layer whose latent pool is attended to
-    float * conv_state = nullptr, * state = nullptr;       // the layer's part of the recurrent state
+    int rotary = -1;                        // index of the layer's rotary table
+    Matrix experts_in, experts_out;         // every expert's rows, gate and up in turn; down
+};
+
+// One pass through a layer: its cache and state.
+struct StackRun {
+    int layer = 0, pool = 0;                // the run whose pools are attended to
+    bool add_embedding = false;
+    float * conv_state = nullptr, * state = nullptr;       // the run's part of the recurrent state
     size_t conv_slot = 0, state_slot = 0;   // floats per slot (a plane of the convolution inputs holds every slot)
 };
 
@@ -160,7 +170,8 @@ struct Vocab {
 // Kernel categories of one step, for the optional event-based timing.
 enum ProfCat : int {
     PC_PACK = 0, PC_EMBED, PC_NORM, PC_QKV, PC_ROPE, PC_ATTN, PC_COMBINE, PC_OPROJ, PC_GATEUP, PC_SWIGLU,
-    PC_DOWN, PC_HEAD, PC_SAMPLE, PC_ABSORB, PC_SCAN, PC_COUNT
+    PC_DOWN, PC_HEAD, PC_SAMPLE, PC_ABSORB, PC_SCAN, PC_ROUTE, PC_EXPERTS_IN,
+    PC_EXPERTS_OUT, PC_COUNT
 };
 
 class Engine {
@@ -284,6 +295,12 @@ private:
     void load_stack(const std::string & path);
     void build_stack();
     void forward_stack(int T, int n_out);
+    void mix_latent(const StackLayer & L, const StackRun & run, int T);
+    void mix_mamba(const StackLayer & L, const StackRun & run, int T);
+    void mix_attention(const StackLayer & L, const StackRun & run, int T);
+    void attend(rk::StackAttn & at, int T);
+    rk::Slices stack_feed_forward(const StackLayer & L, int T);
+    rk::Slices stack_experts(const StackLayer & L, int T);
     void plan_stack(const std::vector<RowView> & rows, const std::vector<std::pair<int, int>> & before);
     size_t stack_plan_bytes() const;
     void stage_stack_plan(uint8_t * host, const uint8_t * device);
@@ -329,18 +346,24 @@ private:
     std::unique_ptr<StackConfig> stack_;
     int arith_ = rk::ARITH_16;
     std::vector<StackLayer> stack_layers_;
+    std::vector<StackRun> stack_runs_;
     StackLayer::Matrix stack_head_;
+    struct RotaryTable { RotarySpec spec; DevBuf freq, table; };      // of the layers that share it; filled once per step
+    std::vector<RotaryTable> rotary_;
+    bool looped_ = false;
+    size_t moe_ws_floats_ = 0;
     DevBuf recurrent_slab_;
     size_t recurrent_slot_floats_ = 0, conv_plane_floats_ = 0;
     DevBuf st_h_, st_proj_, st_cq_, st_q_, st_qa_, st_ol_, st_mix_, st_ff_, st_out_, st_partial_, st_xbc_, st_y_;
+    DevBuf st_embed_, st_route_, ex_sel_, ex_weight_, ex_slot_, ex_tiles_, ex_h_;
     int st_proj_ld_ = 0;
-    struct BlockPlan { int heads, cols; size_t first, n; };    // attention blocks of the step for one head count and width
+    struct BlockPlan { int heads, cols; size_t first, n; };    // attention blocks of the step for one number of query columns per token
     std::vector<BlockPlan> block_plans_;
-    std::vector<rk::LatentBlock> plan_blocks_;
+    std::vector<rk::AttnBlock> plan_blocks_;
     std::vector<rk::SeqRun> plan_runs_;
     std::vector<int32_t> plan_run_tok_;
     int plan_max_run_ = 0, step_rows_ = 0;
-    const rk::LatentBlock * d_blocks_ = nullptr;
+    const rk::AttnBlock * d_blocks_ = nullptr;
     const rk::SeqRun * d_runs_ = nullptr;
     const int32_t * d_run_tok_ = nullptr;
     bool keep_residual_ = false;

@@ -1,5 +1,5 @@
-// Layer-stack models in the engine: loading a checkpoint folder, the latent pools and recurrent state beside the paged
-// cache, the step's plan for them and the forward pass. Slots, pages, packing, sampling, sequence operations and the
+// Layer-stack models in the engine: loading a checkpoint folder, the cache pools and recurrent state of every pass
+// through a layer, the step's plan for them and the forward pass. Slots, pages, packing, sampling, sequence operations and the
 // generators are the engine's own (engine.cpp, generate.cpp).
 #include "engine.hpp"
 #include "safetensors_file.hpp"
@@ -24,7 +24,7 @@ class Loader {
 public:
     Loader(const SafetensorsFile & f, hipStream_t s) : file_(f), stream_(s) {}
 
-    void vector(const std::string & name, const std::vector<int64_t> & shape, DevBuf & out) {
+    void vector(const std::string & name, const std::vector<int64_t> & shape, DevBuf & out, float plus = 0.0f) {
         const StTensor & t = file_.require(name, shape);
         const size_t n = t.nbytes / (t.dtype == "F32" ? 4 : 2);
         std::vector<float> v(n);
@@ -40,6 +40,7 @@ public:
         } else {
             throw std::runtime_error("tensor " + name + " must be BF16 or F32");
         }
+        for (float & x : v) x += plus;
         out.alloc(n * 4);
         hip_check(hipMemcpy(out.ptr, v.data(), n * 4, hipMemcpyHostToDevice), "hipMemcpy");
     }
@@ -61,13 +62,42 @@ public:
         hip_check(hipMemcpyAsync(raw_.ptr, t.data, t.nbytes, hipMemcpyHostToDevice, stream_), "hipMemcpyAsync");
         return raw_.as<uint16_t>();
     }
-    // ... as rows row0 .. of m, its columns from k0 on.
-    void matrix(const std::string & name, int rows, int cols, StackLayer::Matrix & m, int row0 = 0, int k0 = 0) {
-        rk::dense_pack(stream_, raw(name, rows, cols), rows, cols, cols, 1, m.buf.as<uint16_t>(), m.w.kf, row0, k0);
+    // ... as rows of batch b of m.
+    void matrix(const std::string & name, int rows, int cols, StackLayer::Matrix & m, rk::PackMap row = 0, rk::PackMap col = 0, int b = 0) {
+        rk::dense_pack(stream_, raw(name, rows, cols), rows, cols, cols, 1, m.buf.as<uint16_t>() + b * rk::frag_weight_elems(m.w.tiles, m.w.kf), m.w.kf, row, col);
+    }
+    // A gate and an up matrix as row tiles in turn, from row tile tile0 on.
+    void gated(const std::string & p, int rows, int cols, StackLayer::Matrix & m, int tile0 = 0, int b = 0) {
+        matrix(p + "gate", rows, cols, m, {tile0 * 16, 16, 32}, 0, b);
+        matrix(p + "up", rows, cols, m, {tile0 * 16 + 16, 16, 32}, 0, b);
+    }
+    static int gated_rows(int ff) { return 2 * up16(ff); }
+    // The rows of `heads` heads, every head from a multiple of `padded` rows on, the columns of a rotated pair side by side.
+    void heads(const std::string & name, int heads, int dim, int padded, int rotated, int cols, StackLayer::Matrix & m, int head0) {
+        const uint16_t * src = raw(name, heads * dim, cols);
+        for (int h = 0; h < heads; ++h)
+            each_part(dim, rotated, [&](int from, int n, int to, int step) {
+                rk::dense_pack(stream_, src + ((size_t)h * dim + from) * cols, n, cols, cols, 1, m.buf.as<uint16_t>(), m.w.kf, {(head0 + h) * padded + to, 1, step}, 0);
+            });
+    }
+    // ... and the columns of a matrix that reads them.
+    void from_heads(const std::string & name, int rows, int heads, int dim, int padded, int rotated, StackLayer::Matrix & m) {
+        const uint16_t * src = raw(name, rows, heads * dim);
+        for (int h = 0; h < heads; ++h)
+            each_part(dim, rotated, [&](int from, int n, int to, int step) {
+                rk::dense_pack(stream_, src + h * dim + from, rows, n, heads * dim, 1, m.buf.as<uint16_t>(), m.w.kf, 0, {h * padded + to, 1, step});
+            });
     }
     void finish() { hip_check(hipStreamSynchronize(stream_), "hipStreamSynchronize"); }
 
 private:
+    template <typename F> static void each_part(int dim, int rotated, F f) {
+        if (rotated > 0) {
+            f(0, rotated / 2, 0, 2);
+            f(rotated / 2, rotated / 2, 1, 2);
+        }
+        if (dim > rotated) f(rotated, dim - rotated, rotated, 1);
+    }
     const SafetensorsFile & file_;
     hipStream_t stream_;
     DevBuf raw_;
@@ -85,7 +115,7 @@ void Engine::load_stack(const std::string & path) {
     SafetensorsFile file(path + "/model.safetensors");
     Loader ld(file, stream_);
     hp_.arch = c.arch->name;
-    hp_.n_layer = (int)c.layers.size();
+    hp_.n_layer = (int)c.runs.size();
     hp_.n_embd = c.width;
     hp_.n_vocab = c.vocab;
     hp_.eps = c.eps;
@@ -102,7 +132,8 @@ void Engine::load_stack(const std::string & path) {
     tok_embd_.w.raw = tok_embd_.buf.as<uint8_t>();
     ld.shape(stack_head_, c.vocab, KE);
     ld.matrix("embed", c.vocab, E, stack_head_);
-    ld.vector("final.norm", {E}, out_norm_);
+    const float norm_plus = c.arch->norm_around_one ? 1.0f : 0.0f;
+    ld.vector("final.norm", {E}, out_norm_, norm_plus);
 
     stack_layers_.resize(c.layers.size());
     for (size_t l = 0; l < c.layers.size(); ++l) {
@@ -110,29 +141,68 @@ void Engine::load_stack(const std::string & path) {
         L.spec = c.layers[l];
         const LayerSpec & sp = L.spec;
         const std::string p = "l" + std::to_string(l) + ".", m = p + "mix.";
-        ld.vector(p + "norm1", {E}, L.norm);
+        const bool parallel = c.arch->parallel;
+        if (parallel && sp.moe.experts > 0) throw std::runtime_error("experts in parallel layers are not supported");
+        ld.vector(p + "norm1", {E}, L.norm, norm_plus);
+        if (!parallel && sp.has_ff()) ld.vector(p + "norm2", {E}, L.norm2, norm_plus);
         if (c.arch->layer_scale) {
             ld.vector(p + "ls1", {E}, L.scale_mix);
             if (sp.ff > 0) ld.vector(p + "ls2", {E}, L.scale_ff);
         }
-        // input rows: the mixer's, in whole tiles, then the feed-forward's
+        // input rows: the mixer's, in whole tiles, then a parallel feed-forward's
         const LatentSpec & a = sp.latent;
+        const AttentionSpec & ga = sp.attention;
+        const int head_rows = 32 * rk::cache_frags(std::max(ga.dim, 1));
         if (sp.mixer == Mixer::LATENT_ATTENTION) {
             const bool own = a.kv_from < 0;
             L.kv_col = up16(a.q_rank);
             L.gate_col = L.kv_col + (own ? up16(a.kv_rank) : 0);
             L.in_rows = L.gate_col + a.heads;
-            L.pool_layer = own ? (int)l : a.kv_from;
+        } else if (sp.mixer == Mixer::ATTENTION) {
+            L.in_rows = (ga.heads + ga.kv_heads) * head_rows;
         } else {
             L.in_rows = sp.mamba.rows();
         }
         L.in_tiles = (L.in_rows + 15) / 16;
-        ld.shape(L.w_in, sp.ff > 0 ? L.in_tiles * 16 + sp.ff : L.in_rows, KE);
-        if (sp.ff > 0) ld.matrix(p + "mlp.up", sp.ff, E, L.w_in, L.in_tiles * 16);
+        const int beside = parallel ? sp.ff : 0;
+        ld.shape(L.w_in, beside > 0 ? L.in_tiles * 16 + beside : L.in_rows, KE);
+        if (beside > 0) ld.matrix(p + "mlp.up", beside, E, L.w_in, L.in_tiles * 16);
         const int mix = sp.mix_width(), KM = rk::frags_of(mix);
-        ld.shape(L.w_out, E, KM + (sp.ff > 0 ? rk::frags_of(sp.ff) : 0));
-        ld.matrix(m + "o", E, mix, L.w_out);
-        if (sp.ff > 0) ld.matrix(p + "mlp.down", E, sp.ff, L.w_out, 0, KM * 32);
+        ld.shape(L.w_out, E, KM + (beside > 0 ? rk::frags_of(beside) : 0));
+        if (sp.mixer == Mixer::ATTENTION) ld.from_heads(m + "o", E, ga.heads, ga.dim, head_rows, ga.rot.dims, L.w_out);
+        else ld.matrix(m + "o", E, mix, L.w_out);
+        if (beside > 0) ld.matrix(p + "mlp.down", E, beside, L.w_out, 0, KM * 32);
+        if (!parallel && sp.ff > 0) {
+            if (rk::out_is_glu(c.arch->ff_act)) {
+                ld.shape(L.ff_in, Loader::gated_rows(sp.ff), KE);
+                ld.gated(p + "mlp.", sp.ff, E, L.ff_in);
+            } else {
+                ld.shape(L.ff_in, sp.ff, KE);
+                ld.matrix(p + "mlp.up", sp.ff, E, L.ff_in);
+            }
+            ld.shape(L.ff_out, E, rk::frags_of(sp.ff));
+            ld.matrix(p + "mlp.down", E, sp.ff, L.ff_out);
+        } else if (sp.moe.experts > 0) {
+            const MoeSpec & e = sp.moe;
+            const std::string sh = p + "mlp.shared.";
+            const int route = e.experts + (e.shared_ff > 0 ? 1 : 0);
+            L.route_tiles = up32(route) / 16;
+            ld.shape(L.ff_in, e.shared_ff > 0 ? L.route_tiles * 16 + Loader::gated_rows(e.shared_ff) : route, KE);
+            ld.matrix(p + "mlp.router", e.experts, E, L.ff_in);
+            if (e.shared_ff > 0) {
+                ld.matrix(sh + "sg", 1, E, L.ff_in, e.experts);
+                ld.gated(sh, e.shared_ff, E, L.ff_in, L.route_tiles);
+                ld.shape(L.ff_out, E, rk::frags_of(e.shared_ff));
+                ld.matrix(sh + "down", E, e.shared_ff, L.ff_out);
+            }
+            ld.shape(L.experts_in, Loader::gated_rows(e.ff), KE, e.experts);
+            ld.shape(L.experts_out, E, rk::frags_of(e.ff), e.experts);
+            for (int x = 0; x < e.experts; ++x) {
+                const std::string ex = p + "mlp.e" + std::to_string(x) + ".";
+                ld.gated(ex, e.ff, E, L.experts_in, 0, x);
+                ld.matrix(ex + "down", E, e.ff, L.experts_out, 0, 0, x);
+            }
+        }
 
         if (sp.mixer == Mixer::LATENT_ATTENTION) {
             ld.matrix(m + "dq", a.q_rank, E, L.w_in);
@@ -143,7 +213,7 @@ void Engine::load_stack(const std::string & path) {
             }
             ld.matrix(m + "g", a.heads, E, L.w_in, L.gate_col);
             // queries head by head, every head padded to whole fragments
-            const int D = up32(a.dim), R = 32 * rk::latent_frags(a.kv_rank);
+            const int D = up32(a.dim), R = 32 * rk::cache_frags(a.kv_rank);
             ld.shape(L.uq, a.heads * D, rk::frags_of(a.q_rank));
             const uint16_t * uq = ld.raw(m + "uq", a.heads * a.dim, a.q_rank);
             for (int h = 0; h < a.heads; ++h)
@@ -159,6 +229,19 @@ void Engine::load_stack(const std::string & path) {
             const size_t uv_head = rk::frag_weight_elems(L.uv.w.tiles, L.uv.w.kf);
             for (int h = 0; h < a.heads; ++h)
                 rk::dense_pack(stream_, uv + (size_t)h * a.vdim * a.kv_rank, a.vdim, a.kv_rank, a.kv_rank, 1, L.uv.buf.as<uint16_t>() + h * uv_head, L.uv.w.kf, 0, 0);
+        } else if (sp.mixer == Mixer::ATTENTION) {
+            ld.heads(m + "q", ga.heads, ga.dim, head_rows, ga.rot.dims, E, L.w_in, 0);
+            ld.heads(m + "k", ga.kv_heads, ga.dim, head_rows, ga.rot.dims, E, L.w_in, ga.heads);
+            for (size_t r = 0; r < rotary_.size(); ++r) if (rotary_[r].spec == ga.rot) L.rotary = (int)r;
+            if (L.rotary < 0) {
+                L.rotary = (int)rotary_.size();
+                rotary_.emplace_back();
+                RotaryTable & t = rotary_.back();
+                t.spec = ga.rot;
+                const std::vector<double> f = ga.rot.frequencies();
+                t.freq.alloc(f.size() * sizeof(double));
+                if (!f.empty()) hip_check(hipMemcpy(t.freq.ptr, f.data(), t.freq.bytes, hipMemcpyHostToDevice), "hipMemcpy");
+            }
         } else {
             const rk::MambaShape & s = sp.mamba;
             ld.matrix(m + "in", s.rows(), E, L.w_in);
@@ -184,51 +267,68 @@ void Engine::load_stack(const std::string & path) {
     fingerprint_ = hash;
 }
 
-// Latent pools, recurrent state and the step's buffers.
+// Cache pools, recurrent state and the step's buffers.
 void Engine::build_stack() {
     const StackConfig & c = *stack_;
-    const size_t n_layer = c.layers.size(), elem = (size_t)arith_;
+    const size_t n_run = c.runs.size(), elem = (size_t)arith_;
     const int B = (int)cfg_.n_batch, E = c.width, n_slots = (int)cfg_.n_seq_max;
     qt_ = 0;                                  // attention plans its own blocks
-    k_pool_.resize(n_layer);
-    v_pool_.resize(n_layer);
+    stack_runs_.resize(n_run);
+    k_pool_.resize(n_run);
+    v_pool_.resize(n_run);
+    // per run: a pool of latents, or one of keys and one of values
+    struct Pool { size_t at = 0, bytes = 0; };
+    std::vector<Pool> pools(2 * n_run);
+    std::vector<int> last(c.layers.size(), 0);              // the latest run of a layer
     size_t total = 0;
-    std::vector<size_t> at(n_layer, 0), bytes(n_layer, 0);
-    for (size_t l = 0; l < n_layer; ++l) {
-        const LatentSpec & a = c.layers[l].latent;
-        if (c.layers[l].mixer != Mixer::LATENT_ATTENTION || a.kv_from >= 0) continue;
-        const int kf = rk::latent_frags(a.kv_rank);
-        bytes[l] = (size_t)n_pages_ * rk::latent_page_elems(kf) * elem;
-        at[l] = total;
-        total += (bytes[l] + 255) / 256 * 256;
-        cache_parts_.push_back({(int)l, false, (size_t)kf * 32 * elem});
+    auto pool = [&](size_t run, bool v, int kf) {
+        Pool & p = pools[2 * run + v];
+        p.bytes = (size_t)n_pages_ * rk::cache_page_elems(kf) * elem;
+        p.at = total;
+        total += (p.bytes + 255) / 256 * 256;
+        cache_parts_.push_back({(int)run, v, (size_t)kf * 32 * elem});
+    };
+    for (size_t r = 0; r < n_run; ++r) {
+        StackRun & R = stack_runs_[r];
+        R.layer = c.runs[r].layer;
+        R.add_embedding = c.runs[r].add_embedding;
+        looped_ |= R.add_embedding;
+        last[(size_t)R.layer] = (int)r;
+        R.pool = (int)r;
+        const LayerSpec & sp = c.layers[(size_t)R.layer];
+        if (sp.mixer == Mixer::LATENT_ATTENTION) {
+            if (sp.latent.kv_from >= 0) R.pool = last[(size_t)sp.latent.kv_from];
+            else pool(r, false, rk::cache_frags(sp.latent.kv_rank));
+        } else if (sp.mixer == Mixer::ATTENTION) {
+            for (int v = 0; v < 2; ++v) pool(r, v != 0, sp.attention.kv_heads * rk::cache_frags(sp.attention.dim));
+        }
     }
     kv_slab_.alloc(total);
     if (total) hip_check(hipMemsetAsync(kv_slab_.ptr, 0, total, stream_), "hipMemsetAsync");      // pages never hold non-finite values
-    for (size_t l = 0; l < n_layer; ++l)
-        if (bytes[l]) k_pool_[l] = PoolView{(uint8_t *)kv_slab_.ptr + at[l], bytes[l]};
+    for (size_t i = 0; i < pools.size(); ++i)
+        if (pools[i].bytes) (i & 1 ? v_pool_ : k_pool_)[i / 2] = PoolView{(uint8_t *)kv_slab_.ptr + pools[i].at, pools[i].bytes};
 
-    // recurrent state: [layer][slot] states, then two planes of [layer][slot] convolution inputs
+    // recurrent state: [run][slot] states, then two planes of [run][slot] convolution inputs
     size_t states = 0;
-    for (StackLayer & L : stack_layers_) {
-        if (L.spec.mixer != Mixer::MAMBA2) continue;
-        const rk::MambaShape & s = L.spec.mamba;
-        L.state_slot = (size_t)s.heads * s.state * s.vdim;
-        L.conv_slot = (size_t)(s.taps - 1) * s.channels();
-        states += L.state_slot * n_slots;
-        conv_plane_floats_ += L.conv_slot * n_slots;
-        recurrent_slot_floats_ += L.state_slot + L.conv_slot;
+    for (StackRun & R : stack_runs_) {
+        const LayerSpec & sp = c.layers[(size_t)R.layer];
+        if (sp.mixer != Mixer::MAMBA2) continue;
+        const rk::MambaShape & s = sp.mamba;
+        R.state_slot = (size_t)s.heads * s.state * s.vdim;
+        R.conv_slot = (size_t)(s.taps - 1) * s.channels();
+        states += R.state_slot * n_slots;
+        conv_plane_floats_ += R.conv_slot * n_slots;
+        recurrent_slot_floats_ += R.state_slot + R.conv_slot;
     }
     recurrent_slab_.alloc((states + 2 * conv_plane_floats_) * 4);
     if (recurrent_slab_.ptr) {
         hip_check(hipMemsetAsync(recurrent_slab_.ptr, 0, recurrent_slab_.bytes, stream_), "hipMemsetAsync");
         float * st = recurrent_slab_.as<float>(), * cv = st + states;
-        for (StackLayer & L : stack_layers_) {
-            if (L.spec.mixer != Mixer::MAMBA2) continue;
-            L.state = st;
-            L.conv_state = cv;
-            st += L.state_slot * n_slots;
-            cv += L.conv_slot * n_slots;
+        for (StackRun & R : stack_runs_) {
+            R.state = st;
+            R.conv_state = cv;
+            st += R.state_slot * n_slots;
+            cv += R.conv_slot * n_slots;
         }
     }
 
@@ -239,6 +339,7 @@ void Engine::build_stack() {
     hip_check(hipMemcpy(inv_freq_.ptr, &magnitude, sizeof(double), hipMemcpyHostToDevice), "hipMemcpy");
 
     size_t h = rk::frag_elems(B, rk::frags_of(E)), cq = 0, q = 0, qa = 0, ol = 0, mix = 0, ff = 0, xbc = 0, y = 0;
+    size_t route = 0, pairs = 0, slots = 0, tiles = 0, expert_h = 0;
     for (const LayerSpec & sp : c.layers) {
         mix = std::max(mix, rk::frag_elems(B, rk::frags_of(sp.mix_width())));
         if (sp.ff > 0) ff = std::max(ff, rk::frag_elems(B, rk::frags_of(sp.ff)));
@@ -246,14 +347,35 @@ void Engine::build_stack() {
             const LatentSpec & a = sp.latent;
             cq = std::max(cq, rk::frag_elems(B, rk::frags_of(a.q_rank)));
             q = std::max(q, rk::frag_elems(B, a.heads * rk::frags_of(a.dim)));
-            qa = std::max(qa, (size_t)B * a.heads * 32 * rk::latent_frags(a.kv_rank));
-            ol = std::max(ol, rk::frag_elems(B, a.heads * rk::latent_frags(a.kv_rank)));
+            qa = std::max(qa, (size_t)B * a.heads * 32 * rk::cache_frags(a.kv_rank));
+            ol = std::max(ol, rk::frag_elems(B, a.heads * rk::cache_frags(a.kv_rank)));
+        } else if (sp.mixer == Mixer::ATTENTION) {
+            qa = std::max(qa, (size_t)B * sp.mix_width());
         } else {
             xbc = std::max(xbc, (size_t)B * sp.mamba.channels());
             y = std::max(y, (size_t)B * sp.mamba.inner());
         }
+        if (sp.moe.experts > 0) {
+            const MoeSpec & e = sp.moe;
+            const size_t n = rk::expert_slots(B, e.top, e.experts);
+            if (e.shared_ff > 0) ff = std::max(ff, rk::frag_elems(B, rk::frags_of(e.shared_ff)));
+            route = std::max(route, (size_t)B * up32(e.experts + 1));
+            pairs = std::max(pairs, (size_t)B * e.top);
+            slots = std::max(slots, n);
+            tiles = std::max(tiles, (size_t)rk::expert_max_tiles(B, e.top, e.experts, 16));
+            expert_h = std::max(expert_h, rk::frag_elems((int)n, rk::frags_of(e.ff)));
+            moe_ws_floats_ = std::max(moe_ws_floats_, (size_t)B * E * e.top);
+        }
     }
-    for (const StackLayer & L : stack_layers_) st_proj_ld_ = std::max(st_proj_ld_, L.in_tiles * 16);
+    for (const StackLayer & L : stack_layers_)
+        if (L.spec.mixer != Mixer::ATTENTION) st_proj_ld_ = std::max(st_proj_ld_, L.in_tiles * 16);      // grouped attention's rows go to their places at once
+    for (RotaryTable & t : rotary_) t.table.alloc((size_t)B * t.spec.dims * 4);
+    if (looped_) st_embed_.alloc((size_t)B * E * 4);
+    st_route_.alloc(route * 4);
+    ex_sel_.alloc(pairs * 4);
+    ex_weight_.alloc(pairs * 4);
+    ex_slot_.alloc(slots * 4);
+    if (tiles) ex_tiles_.alloc((tiles + 1) * 16);           // the count behind the tiles
     auto zeroed = [&](DevBuf & b, size_t n) {       // padding that no producer writes has to be finite
         b.alloc(n);
         if (n) hip_check(hipMemsetAsync(b.ptr, 0, n, stream_), "hipMemsetAsync");
@@ -270,7 +392,8 @@ void Engine::build_stack() {
     zeroed(st_ff_, ff * elem);
     zeroed(st_xbc_, xbc * 4);
     zeroed(st_y_, y * 4);
-    mm_ws_.alloc(rk::dense_workspace_floats() * 4);
+    zeroed(ex_h_, expert_h * elem);
+    mm_ws_.alloc((rk::dense_workspace_floats() + moe_ws_floats_) * 4);
 }
 
 // ---- recurrent state of a slot --------------------------------------------------------------------
@@ -279,8 +402,8 @@ void Engine::state_copy(int32_t src, int32_t dst) {
     const Slot & a = slots_[(size_t)src];
     Slot & b = slots_[(size_t)dst];
     b.plane = 0;
-    for (const StackLayer & L : stack_layers_) {
-        if (L.spec.mixer != Mixer::MAMBA2) continue;
+    for (const StackRun & L : stack_runs_) {
+        if (L.state_slot == 0) continue;
         rk::copy_floats(stream_, L.state + src * L.state_slot, L.state + dst * L.state_slot, L.state_slot);
         rk::copy_floats(stream_, L.conv_state + a.plane * conv_plane_floats_ + src * L.conv_slot, L.conv_state + dst * L.conv_slot, L.conv_slot);
     }
@@ -292,8 +415,8 @@ void Engine::state_pack(int32_t slot, float * out) {
         if (n) hip_check(hipMemcpyAsync(out, src, n * 4, hipMemcpyDeviceToHost, stream_), "hipMemcpyAsync");
         out += n;
     };
-    for (const StackLayer & L : stack_layers_) {
-        if (L.spec.mixer != Mixer::MAMBA2) continue;
+    for (const StackRun & L : stack_runs_) {
+        if (L.state_slot == 0) continue;
         get(L.state + slot * L.state_slot, L.state_slot);
         get(L.conv_state + plane * conv_plane_floats_ + slot * L.conv_slot, L.conv_slot);
     }
@@ -306,8 +429,8 @@ void Engine::state_unpack(int32_t slot, const float * in) {
         if (n) hip_check(hipMemcpyAsync(dst, in, n * 4, hipMemcpyHostToDevice, stream_), "hipMemcpyAsync");
         in += n;
     };
-    for (const StackLayer & L : stack_layers_) {
-        if (L.spec.mixer != Mixer::MAMBA2) continue;
+    for (const StackRun & L : stack_runs_) {
+        if (L.state_slot == 0) continue;
         put(L.state + slot * L.state_slot, L.state_slot);
         put(L.conv_state + slot * L.conv_slot, L.conv_slot);
     }
@@ -315,7 +438,7 @@ void Engine::state_unpack(int32_t slot, const float * in) {
 }
 
 // ---- the step's plan ------------------------------------------------------------------------------
-// Blocks of query columns for every head count among the layers, and for recurrent models the tokens of every sequence
+// Blocks of query columns for every number of columns per token (heads of a key/value head) among the layers, and for recurrent models the tokens of every sequence
 // in order (a step may hold several rows of one slot).
 
 void Engine::plan_stack(const std::vector<RowView> & rows, const std::vector<std::pair<int, int>> & before) {
@@ -328,8 +451,10 @@ void Engine::plan_stack(const std::vector<RowView> & rows, const std::vector<std
     int total = 0;
     for (const RowView & r : rows) total += (int)r.n;
     for (const LayerSpec & sp : stack_->layers) {
-        if (sp.mixer != Mixer::LATENT_ATTENTION) continue;
-        const int H = sp.latent.heads, cols = rk::latent_block_cols(arith_, H, rk::latent_frags(sp.latent.kv_rank), total, (int)rows.size());
+        if (sp.mixer == Mixer::MAMBA2) continue;
+        const bool pair = sp.mixer == Mixer::ATTENTION;
+        const int H = pair ? sp.attention.heads / sp.attention.kv_heads : sp.latent.heads;
+        const int cols = rk::stack_block_cols(arith_, H, rk::cache_frags(pair ? sp.attention.dim : sp.latent.kv_rank), pair, total, (int)rows.size());
         if (std::any_of(block_plans_.begin(), block_plans_.end(), [&](const BlockPlan & b) { return b.heads == H && b.cols == cols; })) continue;
         BlockPlan plan{H, cols, plan_blocks_.size(), 0};
         for (size_t r = 0; r < rows.size(); ++r)
@@ -363,7 +488,7 @@ void Engine::plan_stack(const std::vector<RowView> & rows, const std::vector<std
 }
 
 size_t Engine::stack_plan_bytes() const {
-    return plan_runs_.size() * sizeof(rk::SeqRun) + plan_blocks_.size() * sizeof(rk::LatentBlock) + plan_run_tok_.size() * 4;
+    return plan_runs_.size() * sizeof(rk::SeqRun) + plan_blocks_.size() * sizeof(rk::AttnBlock) + plan_run_tok_.size() * 4;
 }
 
 void Engine::stage_stack_plan(uint8_t * host, const uint8_t * device) {
@@ -375,30 +500,219 @@ void Engine::stage_stack_plan(uint8_t * host, const uint8_t * device) {
         return d;
     };
     d_runs_ = (const rk::SeqRun *)put(plan_runs_.data(), plan_runs_.size() * sizeof(rk::SeqRun));
-    d_blocks_ = (const rk::LatentBlock *)put(plan_blocks_.data(), plan_blocks_.size() * sizeof(rk::LatentBlock));
+    d_blocks_ = (const rk::AttnBlock *)put(plan_blocks_.data(), plan_blocks_.size() * sizeof(rk::AttnBlock));
     d_run_tok_ = (const int32_t *)put(plan_run_tok_.data(), plan_run_tok_.size() * 4);
 }
 
 // ---- the forward pass -------------------------------------------------------------------------------
 
+// Attention over the caches of `at`, its blocks and splits filled in here.
+void Engine::attend(rk::StackAttn & at, int T) {
+    size_t pt = prof_begin(PC_ATTN);
+    const int per_token = at.H / at.G, cols = rk::stack_block_cols(arith_, per_token, at.kf, at.v_pool != nullptr, T, step_rows_);
+    const BlockPlan * plan = nullptr;
+    for (const BlockPlan & b : block_plans_) if (b.heads == per_token && b.cols == cols) plan = &b;
+    at.rows = d_stage_.as<rk::RowDesc>();
+    at.blocks = d_blocks_ + plan->first;
+    at.n_blocks = (int)plan->n;
+    at.block_cols = plan->cols;
+    at.table = table_.as<int32_t>();
+    at.max_pages = max_pages_;
+    at.splits = rk::stack_splits(arith_, at, step_max_resident_);
+    st_partial_.ensure(rk::stack_partial_floats(T, at.H, at.kf, at.splits) * 4);
+    at.partial_ml = st_partial_.as<float>();
+    at.partial = at.partial_ml + (size_t)T * at.H * at.splits * 2;
+    rk::stack_attention(stream_, arith_, at);
+    prof_end(PC_ATTN, pt);
+    if (at.splits > 1) {
+        pt = prof_begin(PC_COMBINE);
+        rk::stack_combine(stream_, at, T);
+        prof_end(PC_COMBINE, pt);
+    }
+}
+
+void Engine::mix_latent(const StackLayer & L, const StackRun & run, int T) {
+    const LatentSpec & a = L.spec.latent;
+    const int D = rk::frags_of(a.dim), R = rk::cache_frags(a.kv_rank), H = a.heads, ld = st_proj_ld_;
+    float * proj = st_proj_.as<float>(), * ws = mm_ws_.as<float>();
+    void * pool = k_pool_[(size_t)run.pool].ptr;
+    size_t pt = prof_begin(PC_ROPE);
+    rk::LatentNorms n;
+    n.proj = proj; n.ld = ld; n.q_rank = a.q_rank; n.kv_col = L.kv_col; n.kv_rank = a.kv_rank;
+    n.q_w = L.q_norm.as<float>(); n.kv_w = L.kv_norm.as<float>(); n.eps = stack_->eps;
+    n.act_q = st_cq_.ptr; n.act_q_kf = rk::frags_of(a.q_rank);
+    n.pool = pool; n.pool_kf = R; n.cell = pk_.cell;
+    rk::latent_norms(stream_, arith_, n, T);
+    prof_end(PC_ROPE, pt);
+    pt = prof_begin(PC_ABSORB);
+    rk::DenseJob uq;
+    uq.w = L.uq.w;
+    uq.x = {st_cq_.ptr, rk::frags_of(a.q_rank), 0};
+    uq.a.kind = rk::OUT_ACT; uq.a.dst = st_q_.ptr; uq.a.ld = H * D;
+    rk::dense(stream_, arith_, uq, T, ws);
+    rk::DenseJob uk;
+    uk.w = L.uk.w;
+    uk.x = {st_q_.ptr, H * D, D};
+    uk.a.kind = rk::OUT_QUERY; uk.a.dst = st_qa_.ptr; uk.a.ld = R * 32; uk.a.col_batch = H;
+    uk.a.scale = (float)((double)a.scale * 1.4426950408889634);      // the softmax runs on powers of two
+    rk::dense(stream_, arith_, uk, T, ws);
+    prof_end(PC_ABSORB, pt);
+    rk::StackAttn at;
+    at.q = st_qa_.ptr; at.H = H; at.kf = R; at.window = a.window;
+    at.pool = pool;
+    at.out = st_ol_.ptr; at.out_kf = H * R;
+    attend(at, T);
+    pt = prof_begin(PC_OPROJ);
+    rk::DenseJob uv;
+    uv.w = L.uv.w;
+    uv.x = {st_ol_.ptr, H * R, R};
+    uv.a.kind = rk::OUT_ACT_GATED; uv.a.dst = st_mix_.ptr; uv.a.ld = rk::frags_of(L.spec.mix_width()); uv.a.col_batch = a.vdim;
+    uv.a.gate = proj + L.gate_col; uv.a.ld_gate = ld;
+    rk::dense(stream_, arith_, uv, T, ws);
+    prof_end(PC_OPROJ, pt);
+}
+
+void Engine::mix_mamba(const StackLayer & L, const StackRun & run, int T) {
+    const size_t pt = prof_begin(PC_SCAN);
+    rk::MambaJob j;
+    j.sh = L.spec.mamba;
+    j.proj = st_proj_.as<float>(); j.ld = st_proj_ld_;
+    j.conv_w = L.conv_w.as<float>(); j.conv_b = L.conv_b.as<float>(); j.dt_bias = L.dt_bias.as<float>();
+    j.A_log = L.A_log.as<float>(); j.D = L.D.as<float>(); j.norm_w = L.gate_norm.as<float>();
+    j.eps = stack_->eps;
+    j.runs = d_runs_; j.n_runs = (int)plan_runs_.size(); j.max_run = plan_max_run_; j.run_tok = d_run_tok_;
+    j.conv_state = run.conv_state; j.conv_plane = conv_plane_floats_; j.state = run.state;
+    j.xbc = st_xbc_.as<float>(); j.y = st_y_.as<float>();
+    j.out = st_mix_.ptr; j.out_kf = rk::frags_of(L.spec.mix_width());
+    rk::mamba_mix(stream_, arith_, j, T);
+    prof_end(PC_SCAN, pt);
+}
+
+// Grouped attention: the input product has already left queries, keys and values in their places.
+void Engine::mix_attention(const StackLayer & L, const StackRun & run, int T) {
+    const AttentionSpec & a = L.spec.attention;
+    rk::StackAttn at;
+    at.q = st_qa_.ptr; at.H = a.heads; at.G = a.kv_heads; at.kf = rk::cache_frags(a.dim);
+    at.window = a.window; at.chunk = a.chunk;
+    at.scale = a.scale; at.softcap = a.softcap;
+    at.pool = k_pool_[(size_t)run.pool].ptr; at.v_pool = v_pool_[(size_t)run.pool].ptr;
+    at.out = st_mix_.ptr; at.out_kf = a.heads * at.kf;
+    attend(at, T);
+}
+
+// The feed-forward of a sequential layer over the normed rows in st_h_.
+rk::Slices Engine::stack_feed_forward(const StackLayer & L, int T) {
+    const StackConfig & c = *stack_;
+    const int E = c.width, KE = rk::frags_of(E), KF = rk::frags_of(L.spec.ff);
+    float * ws = mm_ws_.as<float>();
+    if (L.spec.moe.experts > 0) return stack_experts(L, T);
+    size_t pt = prof_begin(PC_GATEUP);
+    rk::DenseJob in;
+    in.w = L.ff_in.w;
+    in.x = {st_h_.ptr, KE, 0};
+    in.a.kind = c.arch->ff_act; in.a.dst = st_ff_.ptr; in.a.ld = KF;
+    rk::dense(stream_, arith_, in, T, ws);
+    prof_end(PC_GATEUP, pt);
+    pt = prof_begin(PC_DOWN);
+    rk::DenseJob out;
+    out.w = L.ff_out.w;
+    out.x = {st_ff_.ptr, KF, 0};
+    out.kf1 = KF;
+    out.a.kind = rk::OUT_RESIDUAL; out.a.dst = x_.ptr; out.a.ld = E;
+    const rk::Slices left = rk::dense(stream_, arith_, out, T, ws);
+    prof_end(PC_DOWN, pt);
+    return left;
+}
+
+// Router and shared expert in one product, the routing, the chosen experts; every choice leaves a slice of the residual.
+rk::Slices Engine::stack_experts(const StackLayer & L, int T) {
+    const StackConfig & c = *stack_;
+    const MoeSpec & e = L.spec.moe;
+    const int E = c.width, KE = rk::frags_of(E), KS = rk::frags_of(std::max(e.shared_ff, 1)), KX = rk::frags_of(e.ff);
+    float * ws = mm_ws_.as<float>(), * route = st_route_.as<float>();
+    const int ld = up32(e.experts + 1);
+    size_t pt = prof_begin(PC_GATEUP);
+    rk::DenseJob in;
+    in.w = L.ff_in.w;
+    in.x = {st_h_.ptr, KE, 0};
+    in.split_tile = L.route_tiles;
+    in.n_a = e.experts + (e.shared_ff > 0 ? 1 : 0);
+    in.a.kind = rk::OUT_F32; in.a.dst = route; in.a.ld = ld;
+    in.b.kind = c.arch->expert_act; in.b.dst = st_ff_.ptr; in.b.ld = KS;
+    rk::dense(stream_, arith_, in, T, ws);
+    prof_end(PC_GATEUP, pt);
+    pt = prof_begin(PC_ROUTE);
+    rk::ExpertRoute r;
+    r.logits = route; r.ld = ld; r.experts = e.experts; r.top = e.top;
+    r.block = rk::expert_block(arith_, T, e.top, e.experts);
+    r.sel = ex_sel_.as<int32_t>(); r.weight = ex_weight_.as<float>(); r.slot_pair = ex_slot_.as<int32_t>();
+    r.tiles = ex_tiles_.as<int32_t>();
+    r.n_tiles = r.tiles + (ex_tiles_.bytes / 16 - 1) * 4;
+    rk::expert_route(stream_, r, T);
+    prof_end(PC_ROUTE, pt);
+    rk::ExpertGroups g;
+    g.tiles = r.tiles; g.n_tiles = r.n_tiles; g.block = r.block; g.max_tiles = rk::expert_max_tiles(T, e.top, e.experts, r.block);
+    g.slot_pair = r.slot_pair; g.weight = r.weight; g.top = e.top; g.pairs = T * e.top;
+    pt = prof_begin(PC_EXPERTS_IN);
+    rk::DenseJob up;
+    up.w = L.experts_in.w;
+    up.x = in.x;
+    up.groups = &g;
+    up.gather = true;
+    up.a.kind = c.arch->expert_act; up.a.dst = ex_h_.ptr; up.a.ld = KX;
+    rk::dense(stream_, arith_, up, T, ws);
+    prof_end(PC_EXPERTS_IN, pt);
+    rk::Slices left;
+    if (e.shared_ff > 0) {
+        pt = prof_begin(PC_DOWN);
+        rk::DenseJob out;
+        out.w = L.ff_out.w;
+        out.x = {st_ff_.ptr, KS, 0};
+        out.kf1 = KS;
+        out.a.kind = rk::OUT_RESIDUAL; out.a.dst = x_.ptr; out.a.ld = E;
+        out.token_gate = route + e.experts; out.ld_token_gate = ld;
+        left = rk::dense(stream_, arith_, out, T, ws);
+        prof_end(PC_DOWN, pt);
+    }
+    pt = prof_begin(PC_EXPERTS_OUT);
+    const size_t slice = (size_t)T * E;
+    rk::DenseJob down;
+    down.w = L.experts_out.w;
+    down.x = {ex_h_.ptr, KX, 0};
+    down.groups = &g;
+    down.a.kind = rk::OUT_EXPERT; down.a.dst = ws + (size_t)left.n * slice; down.a.ld = E; down.a.stride = slice;
+    rk::dense(stream_, arith_, down, T, ws);
+    prof_end(PC_EXPERTS_OUT, pt);
+    left.data = ws;
+    left.n += e.top;
+    left.stride = slice;
+    left.N = E;
+    return left;
+}
+
 void Engine::forward_stack(int T, int n_out) {
     const StackConfig & c = *stack_;
-    const int E = c.width, KE = rk::frags_of(E), ld = st_proj_ld_;
-    float * x = x_.as<float>(), * proj = st_proj_.as<float>(), * ws = mm_ws_.as<float>();
-    const rk::RowDesc * rows = d_stage_.as<rk::RowDesc>();
+    const int E = c.width, KE = rk::frags_of(E);
+    float * x = x_.as<float>(), * ws = mm_ws_.as<float>();
     rk::Slices pending;
     size_t pt = prof_begin(PC_EMBED);
     rk::embed(stream_, tok_embd_.w, pk_.tok, T, x);
+    if (looped_) rk::copy_floats(stream_, x, st_embed_.as<float>(), (size_t)T * E);
+    for (RotaryTable & t : rotary_)
+        rk::rotary_table(stream_, t.freq.as<double>(), t.spec.dims / 2, t.spec.magnitude(), pk_.pos, T, t.table.as<float>());
     prof_end(PC_EMBED, pt);
     if (keep_residual_) {
-        kept_residual_.ensure(stack_layers_.size() * (size_t)cfg_.n_batch * E * 4);
+        kept_residual_.ensure(stack_runs_.size() * (size_t)cfg_.n_batch * E * 4);
         kept_tokens_ = T;
     }
-    for (size_t l = 0; l < stack_layers_.size(); ++l) {
-        const StackLayer & L = stack_layers_[l];
+    for (size_t r = 0; r < stack_runs_.size(); ++r) {
+        const StackRun & run = stack_runs_[r];
+        const StackLayer & L = stack_layers_[(size_t)run.layer];
         const LayerSpec & sp = L.spec;
+        const bool beside = c.arch->parallel && sp.ff > 0;
         pt = prof_begin(PC_NORM);
-        rk::norm_act(stream_, arith_, c.arch->norm, x, L.norm.as<float>(), E, c.eps, nullptr, T, st_h_.ptr, KE, pending);
+        rk::norm_act(stream_, arith_, c.arch->norm, x, L.norm.as<float>(), E, c.eps, nullptr, T, st_h_.ptr, KE, pending,
+                     run.add_embedding ? st_embed_.as<float>() : nullptr);
         prof_end(PC_NORM, pt);
         pt = prof_begin(PC_QKV);
         rk::DenseJob in;
@@ -406,94 +720,45 @@ void Engine::forward_stack(int T, int n_out) {
         in.x = {st_h_.ptr, KE, 0};
         in.split_tile = L.in_tiles;
         in.n_a = L.in_rows;
-        in.a.kind = rk::OUT_F32; in.a.dst = proj; in.a.ld = ld;
+        if (sp.mixer == Mixer::ATTENTION) {
+            const AttentionSpec & a = sp.attention;
+            const RotaryTable & t = rotary_[(size_t)L.rotary];
+            in.a.kind = rk::OUT_ROTARY; in.a.dst = st_qa_.ptr;
+            in.a.rot.H = a.heads; in.a.rot.G = a.kv_heads; in.a.rot.kf = rk::cache_frags(a.dim); in.a.rot.pairs = t.spec.dims / 2;
+            in.a.rot.table = t.table.as<float>();
+            in.a.rot.k_pool = k_pool_[(size_t)run.pool].ptr; in.a.rot.v_pool = v_pool_[(size_t)run.pool].ptr;
+            in.a.rot.cell = pk_.cell;
+        } else {
+            in.a.kind = rk::OUT_F32; in.a.dst = st_proj_.ptr; in.a.ld = st_proj_ld_;
+        }
         in.b.kind = c.arch->ff_act; in.b.dst = st_ff_.ptr; in.b.ld = rk::frags_of(std::max(sp.ff, 1));
         rk::dense(stream_, arith_, in, T, ws);
         prof_end(PC_QKV, pt);
-        const int KM = rk::frags_of(sp.mix_width());
-        if (sp.mixer == Mixer::LATENT_ATTENTION) {
-            const LatentSpec & a = sp.latent;
-            const int D = rk::frags_of(a.dim), R = rk::latent_frags(a.kv_rank), H = a.heads;
-            pt = prof_begin(PC_ROPE);
-            rk::LatentNorms n;
-            n.proj = proj; n.ld = ld; n.q_rank = a.q_rank; n.kv_col = L.kv_col; n.kv_rank = a.kv_rank;
-            n.q_w = L.q_norm.as<float>(); n.kv_w = L.kv_norm.as<float>(); n.eps = c.eps;
-            n.act_q = st_cq_.ptr; n.act_q_kf = rk::frags_of(a.q_rank);
-            n.pool = k_pool_[(size_t)L.pool_layer].ptr; n.pool_kf = R; n.cell = pk_.cell;
-            rk::latent_norms(stream_, arith_, n, T);
-            prof_end(PC_ROPE, pt);
-            pt = prof_begin(PC_ABSORB);
-            rk::DenseJob uq;
-            uq.w = L.uq.w;
-            uq.x = {st_cq_.ptr, rk::frags_of(a.q_rank), 0};
-            uq.a.kind = rk::OUT_ACT; uq.a.dst = st_q_.ptr; uq.a.ld = H * D;
-            rk::dense(stream_, arith_, uq, T, ws);
-            rk::DenseJob uk;
-            uk.w = L.uk.w;
-            uk.x = {st_q_.ptr, H * D, D};
-            uk.a.kind = rk::OUT_QUERY; uk.a.dst = st_qa_.ptr; uk.a.ld = R * 32; uk.a.col_batch = H;
-            uk.a.scale = (float)((double)a.scale * 1.4426950408889634);      // the softmax runs on powers of two
-            rk::dense(stream_, arith_, uk, T, ws);
-            prof_end(PC_ABSORB, pt);
-            pt = prof_begin(PC_ATTN);
-            const BlockPlan * plan = nullptr;
-            const int cols = rk::latent_block_cols(arith_, H, R, T, step_rows_);
-            for (const BlockPlan & b : block_plans_) if (b.heads == H && b.cols == cols) plan = &b;
-            rk::LatentAttn at;
-            at.q = st_qa_.ptr; at.H = H; at.kf = R; at.window = a.window;
-            at.rows = rows; at.blocks = d_blocks_ + plan->first; at.n_blocks = (int)plan->n; at.block_cols = plan->cols;
-            at.table = table_.as<int32_t>(); at.max_pages = max_pages_;
-            at.pool = k_pool_[(size_t)L.pool_layer].ptr;
-            at.splits = rk::latent_splits(arith_, at, step_max_resident_);
-            st_partial_.ensure(rk::latent_partial_floats(T, H, R, at.splits) * 4);
-            at.partial_ml = st_partial_.as<float>();
-            at.partial = at.partial_ml + (size_t)T * H * at.splits * 2;
-            at.out = st_ol_.ptr; at.out_kf = H * R;
-            rk::latent_attention(stream_, arith_, at);
-            prof_end(PC_ATTN, pt);
-            if (at.splits > 1) {
-                pt = prof_begin(PC_COMBINE);
-                rk::latent_combine(stream_, at, T);
-                prof_end(PC_COMBINE, pt);
-            }
-            pt = prof_begin(PC_OPROJ);
-            rk::DenseJob uv;
-            uv.w = L.uv.w;
-            uv.x = {st_ol_.ptr, H * R, R};
-            uv.a.kind = rk::OUT_ACT_GATED; uv.a.dst = st_mix_.ptr; uv.a.ld = KM; uv.a.col_batch = a.vdim;
-            uv.a.gate = proj + L.gate_col; uv.a.ld_gate = ld;
-            rk::dense(stream_, arith_, uv, T, ws);
-            prof_end(PC_OPROJ, pt);
-        } else {
-            pt = prof_begin(PC_SCAN);
-            rk::MambaJob j;
-            j.sh = sp.mamba;
-            j.proj = proj; j.ld = ld;
-            j.conv_w = L.conv_w.as<float>(); j.conv_b = L.conv_b.as<float>(); j.dt_bias = L.dt_bias.as<float>();
-            j.A_log = L.A_log.as<float>(); j.D = L.D.as<float>(); j.norm_w = L.gate_norm.as<float>();
-            j.eps = c.eps;
-            j.runs = d_runs_; j.n_runs = (int)plan_runs_.size(); j.max_run = plan_max_run_; j.run_tok = d_run_tok_;
-            j.conv_state = L.conv_state; j.conv_plane = conv_plane_floats_; j.state = L.state;
-            j.xbc = st_xbc_.as<float>(); j.y = st_y_.as<float>();
-            j.out = st_mix_.ptr; j.out_kf = KM;
-            rk::mamba_mix(stream_, arith_, j, T);
-            prof_end(PC_SCAN, pt);
-        }
-        pt = prof_begin(PC_DOWN);
+        if (sp.mixer == Mixer::LATENT_ATTENTION) mix_latent(L, run, T);
+        else if (sp.mixer == Mixer::ATTENTION) mix_attention(L, run, T);
+        else mix_mamba(L, run, T);
+        const int out_cat = c.arch->parallel ? PC_DOWN : PC_OPROJ, KM = rk::frags_of(sp.mix_width());
+        pt = prof_begin(out_cat);
         rk::DenseJob out;
         out.w = L.w_out.w;
         out.x = {st_mix_.ptr, KM, 0};
         out.kf1 = KM;
         out.scale1 = L.scale_mix.as<float>();
-        if (sp.ff > 0) {
+        if (beside) {
             out.x2 = {st_ff_.ptr, rk::frags_of(sp.ff), 0};
             out.scale2 = L.scale_ff.as<float>();
         }
         out.a.kind = rk::OUT_RESIDUAL; out.a.dst = x; out.a.ld = E;
         pending = rk::dense(stream_, arith_, out, T, ws);
-        prof_end(PC_DOWN, pt);
+        prof_end(out_cat, pt);
+        if (!c.arch->parallel && sp.has_ff()) {
+            pt = prof_begin(PC_NORM);
+            rk::norm_act(stream_, arith_, c.arch->norm, x, L.norm2.as<float>(), E, c.eps, nullptr, T, st_h_.ptr, KE, pending);
+            prof_end(PC_NORM, pt);
+            pending = stack_feed_forward(L, T);
+        }
         if (keep_residual_) {
-            float * kept = kept_residual_.as<float>() + l * (size_t)cfg_.n_batch * E;
+            float * kept = kept_residual_.as<float>() + r * (size_t)cfg_.n_batch * E;
             rk::copy_floats(stream_, x, kept, (size_t)T * E);
             rk::add_slices(stream_, kept, E, T, pending);
         }
@@ -528,12 +793,12 @@ int Engine::debug_read_residual(float * out, size_t n_floats, size_t * out_token
     if (out_tokens) *out_tokens = (size_t)kept_tokens_;
     if (!out) return 0;
     const size_t per = (size_t)kept_tokens_ * stack_->width;
-    if (n_floats < per * stack_layers_.size()) {
+    if (n_floats < per * stack_runs_.size()) {
         set_error("the residual buffer is too small");
         return -2;
     }
     hip_check(hipStreamSynchronize(stream_), "debug_read_residual");
-    for (size_t l = 0; l < stack_layers_.size(); ++l)
+    for (size_t l = 0; l < stack_runs_.size(); ++l)
         hip_check(hipMemcpy(out + l * per, kept_residual_.as<float>() + l * (size_t)cfg_.n_batch * stack_->width, per * 4, hipMemcpyDeviceToHost), "hipMemcpy");
     return 0;
 }

@@ -6,6 +6,8 @@
 #include "json_schema.hpp"
 #include "stack_kernels.hpp"
 
+#include <algorithm>
+#include <cmath>
 #include <fstream>
 #include <sstream>
 #include <stdexcept>
@@ -23,16 +25,22 @@ inline const GgufArch * find_gguf_arch(const std::string & name) {
     return nullptr;
 }
 
-// What an architecture fixes about its layers: x <- x + scale1 * mixer(norm(x)) + scale2 * ff(norm(x)), one norm for
-// both; the norm's kind, the feed-forward's activation (a DenseOut kind), element-wise layer scales or none.
-struct StackArch { const char * name; int norm; int ff_act; bool layer_scale; };
+// What an architecture fixes about its layers. Parallel layers: x <- x + scale1 * mixer(n(x)) + scale2 * ff(n(x)), one
+// norm for both; otherwise x <- x + mixer(n1(x)), then x <- x + ff(n2(x)). The norm's kind and whether its weights are
+// stored as differences from one; the activations (DenseOut kinds) of the feed-forward and of experts; element-wise
+// layer scales or none; what positions of grouped attention a mask of some size leaves.
+enum class Mask { WINDOW, CHUNK };
+struct StackArch { const char * name; int norm; bool norm_around_one; bool parallel; int ff_act, expert_act; bool layer_scale; Mask mask; };
 inline const StackArch * find_stack_arch(const std::string & name) {
-    static const StackArch known[] = {{"Dibosun", rk::NORM_LAYER, rk::OUT_ACT_RELU2, true}};
+    static const StackArch known[] = {
+        {"Dibosun", rk::NORM_LAYER, false, true, rk::OUT_ACT_RELU2, -1, true, Mask::WINDOW},
+        {"Pomisun", rk::NORM_RMS, true, false, rk::OUT_ACT_GEGLU, rk::OUT_ACT_SWIGLU, false, Mask::CHUNK},
+    };
     for (const StackArch & a : known) if (name == a.name) return &a;
     return nullptr;
 }
 
-enum class Mixer { LATENT_ATTENTION, MAMBA2 };
+enum class Mixer { LATENT_ATTENTION, MAMBA2, ATTENTION };
 
 struct LatentSpec {
     int heads = 0, dim = 0, vdim = 0, q_rank = 0, kv_rank = 0;
@@ -41,19 +49,66 @@ struct LatentSpec {
     float scale = 1.0f;
 };
 
+// Rotary positions on the first `dims` columns of a head, optionally stretched (YaRN): frequencies that turn fewer than
+// `slow` times within the original length are divided by the factor, those above `fast` kept, a ramp in between.
+struct RotarySpec {
+    int dims = 0;
+    double base = 10000.0, factor = 1.0, original = 0.0, fast = 0.0, slow = 0.0;      // original 0: not stretched
+    bool operator==(const RotarySpec & o) const {
+        return dims == o.dims && base == o.base && factor == o.factor && original == o.original && fast == o.fast && slow == o.slow;
+    }
+    // Radians per position of the dims / 2 pairs.
+    std::vector<double> frequencies() const {
+        std::vector<double> f((size_t)(dims / 2));
+        const double pi = 3.14159265358979323846;
+        auto pair_of = [&](double turns) { return dims * std::log(original / (2.0 * pi * turns)) / (2.0 * std::log(base)); };
+        const double lo = original > 0.0 ? std::max(std::floor(pair_of(fast)), 0.0) : 0.0;
+        const double hi = original > 0.0 ? std::min(std::ceil(pair_of(slow)), dims - 1.0) : 0.0;
+        for (size_t i = 0; i < f.size(); ++i) {
+            f[i] = std::pow(base, -2.0 * (double)i / dims);
+            if (original <= 0.0) continue;
+            const double ramp = std::min(std::max(((double)i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
+            f[i] = f[i] / factor * ramp + f[i] * (1.0 - ramp);
+        }
+        return f;
+    }
+    double magnitude() const { return original > 0.0 ? 0.1 * std::log(factor) + 1.0 : 1.0; }      // of cosines and sines
+};
+
+// Grouped attention whose values are its keys before rotation.
+struct AttentionSpec {
+    int heads = 0, kv_heads = 0, dim = 0;
+    int window = 0, chunk = 0;   // positions seen: the last `window`, or those of the same chunk (0: no bound)
+    float scale = 1.0f, softcap = 0.0f;
+    RotarySpec rot;
+};
+
+// Experts of a feed-forward: every token takes `top` of them, and the shared one (ff 0: none) behind a gate per token.
+struct MoeSpec { int experts = 0, top = 0, ff = 0, shared_ff = 0; };
+
 struct LayerSpec {
     Mixer mixer = Mixer::LATENT_ATTENTION;
     LatentSpec latent;
     rk::MambaShape mamba;
-    int ff = 0;                  // 0: no feed-forward
-    int mix_width() const { return mixer == Mixer::MAMBA2 ? mamba.inner() : latent.heads * latent.vdim; }
+    AttentionSpec attention;
+    int ff = 0;                  // of a dense feed-forward; 0 and no experts: no feed-forward
+    MoeSpec moe;
+    bool has_ff() const { return ff > 0 || moe.experts > 0; }
+    // Columns a mixer hands to its output projection (a head of grouped attention padded as its cache rows are).
+    int mix_width() const {
+        return mixer == Mixer::MAMBA2 ? mamba.inner() : mixer == Mixer::ATTENTION ? attention.heads * 32 * rk::cache_frags(attention.dim) : latent.heads * latent.vdim;
+    }
 };
+
+// One pass through a layer; a looped layer has several, each with its own cache or state.
+struct LayerRun { int layer; bool add_embedding; };      // the embedding output is added to the stream first
 
 struct StackConfig {
     const StackArch * arch = nullptr;
     int width = 0, vocab = 0;
     float eps = 0.0f;
     std::vector<LayerSpec> layers;
+    std::vector<LayerRun> runs;
     bool recurrent() const {
         for (const LayerSpec & l : layers) if (l.mixer == Mixer::MAMBA2) return true;
         return false;
@@ -78,8 +133,21 @@ struct StackConfig {
         c.width = size(v, "width");
         c.vocab = size(v, "vocab");
         c.eps = (float)number(need(v, "norm"), "eps");
-        for (const JsonValue & l : need(v, "layers").items) c.layers.push_back(layer(l, c.layers));
-        if (c.layers.empty() || c.layers.size() > 4096) throw std::runtime_error("config.json: 'layers' must list 1 to 4096 layers");
+        for (const JsonValue & l : need(v, "layers").items) c.layers.push_back(layer(*c.arch, l, c.layers));
+        const int n = (int)c.layers.size();
+        if (n < 1 || n > 4096) throw std::runtime_error("config.json: 'layers' must list 1 to 4096 layers");
+        int start = 0, stop = 0, times = 1;
+        if (present(v, "loop")) {
+            const JsonValue & l = need(v, "loop");
+            start = size(l, "start", 0);
+            stop = size(l, "stop", 0);
+            times = size(l, "times");
+            if (start > stop || stop > n || (int64_t)(stop - start) * times > 65536) throw std::runtime_error("config.json: 'loop' must name a range of layers");
+        }
+        for (int l = 0; l < start; ++l) c.runs.push_back({l, false});
+        for (int t = 0; t < times; ++t)
+            for (int l = start; l < stop; ++l) c.runs.push_back({l, t > 0 && l == start});
+        for (int l = stop; l < n; ++l) c.runs.push_back({l, false});
         return c;
     }
 
@@ -103,7 +171,25 @@ private:
         const JsonValue * m = v.get(key);
         return m && m->kind != JsonValue::NUL;
     }
-    static LayerSpec layer(const JsonValue & v, const std::vector<LayerSpec> & before) {
+    static bool positive(double v) { return v > 0.0 && std::isfinite(v); }
+    static RotarySpec rotary(const JsonValue & v, int dim) {
+        RotarySpec r;
+        r.dims = size(v, "dims", 0);
+        r.base = number(v, "base");
+        if (r.dims > dim || r.dims % 2 != 0) throw std::runtime_error("config.json: 'rot.dims' must be even and within a head");
+        if (!positive(r.base) || r.base == 1.0) throw std::runtime_error("config.json: 'rot.base' must be positive and not 1");
+        if (present(v, "scaling")) {
+            const JsonValue & s = need(v, "scaling");
+            r.factor = number(s, "factor");
+            r.original = number(s, "original");
+            r.fast = number(s, "fast");
+            r.slow = number(s, "slow");
+            if (!positive(r.factor) || !positive(r.original) || !positive(r.fast) || !positive(r.slow))
+                throw std::runtime_error("config.json: 'rot.scaling' must hold positive numbers");
+        }
+        return r;
+    }
+    static LayerSpec layer(const StackArch & arch, const JsonValue & v, const std::vector<LayerSpec> & before) {
         LayerSpec l;
         const std::string type = need(v, "type").text;
         const JsonValue & m = need(v, "mixer");
@@ -135,14 +221,39 @@ private:
             if (s.heads % s.groups != 0) throw std::runtime_error("mamba2: heads must be a multiple of groups");
             if (s.inner() % s.norm_groups != 0) throw std::runtime_error("mamba2: heads * vdim must be a multiple of norm_groups");
             if (s.state > 512) throw std::runtime_error("mamba2: a state above 512 rows is not supported");
+        } else if (type == "attention") {
+            l.mixer = Mixer::ATTENTION;
+            AttentionSpec & a = l.attention;
+            a.heads = size(m, "heads");
+            a.kv_heads = size(m, "kv_heads");
+            a.dim = size(m, "dim");
+            a.scale = (float)number(m, "scale");
+            if (present(m, "softcap")) a.softcap = (float)number(m, "softcap");
+            if (present(m, "mask") && present(need(m, "mask"), "size")) (arch.mask == Mask::CHUNK ? a.chunk : a.window) = size(need(m, "mask"), "size");
+            if (a.heads % a.kv_heads != 0) throw std::runtime_error("attention: heads must be a multiple of kv_heads");
+            if (size(m, "vdim") != a.dim) throw std::runtime_error("attention: the values are the keys, so vdim must be dim");
+            if (a.dim > 1024) throw std::runtime_error("attention: heads above 1024 columns are not supported");
+            if (!(a.softcap >= 0.0f)) throw std::runtime_error("attention: softcap must not be negative");
+            a.rot = rotary(need(m, "rot"), a.dim);
         } else {
             throw std::runtime_error("config.json: unknown layer type '" + type + "'");
         }
         if (present(v, "mlp")) {
             const JsonValue & f = need(v, "mlp");
             const std::string kind = need(f, "kind").text;
-            if (kind != "dense") throw std::runtime_error("config.json: unknown feed-forward kind '" + kind + "'");
-            l.ff = size(f, "ff");
+            if (kind == "dense") {
+                l.ff = size(f, "ff");
+            } else if (kind == "moe" && arch.expert_act >= 0) {
+                const JsonValue & r = need(f, "router");
+                l.moe.experts = size(r, "experts");
+                l.moe.top = size(r, "top");
+                l.moe.ff = size(need(f, "expert"), "ff");
+                if (present(f, "shared")) l.moe.shared_ff = size(need(f, "shared"), "ff");
+                if (l.moe.top > l.moe.experts) throw std::runtime_error("moe: 'top' exceeds 'experts'");
+                if (l.moe.experts > rk::MAX_EXPERTS || l.moe.top > rk::MAX_TOP) throw std::runtime_error("moe: more experts than are supported");
+            } else {
+                throw std::runtime_error("config.json: unknown feed-forward kind '" + kind + "'");
+            }
         }
         return l;
     }

@@ -1,4 +1,4 @@
-// Row norms of layer-stack models: the residual stream (completed with the K-slices the product before left) through an
+// Row norms of layer-stack models: the residual stream (completed with the slices the products before left) through an
 // RMS or layer norm into activations. Statistics in f32, two passes over the row held in LDS.
 #include "stack_dev.hpp"
 
@@ -9,7 +9,8 @@ namespace {
 // VEC: rows of whole groups of four, read and written as such; the slices of a group are all requested at once.
 template <int ARITH, int KIND, bool VEC>
 __global__ __launch_bounds__(1024) void k_norm_act(float * __restrict__ x, const float * __restrict__ w, int E, float eps,
-                                                   const int32_t * __restrict__ rows, void * __restrict__ act, int kf, Slices add) {
+                                                   const int32_t * __restrict__ rows, void * __restrict__ act, int kf, Slices add,
+                                                   const float * __restrict__ plus) {
     extern __shared__ __attribute__((aligned(16))) float row[];
     __shared__ float scratch[16];
     const int t = rows ? rows[blockIdx.x] : (int)blockIdx.x, n_thr = blockDim.x;
@@ -18,14 +19,18 @@ __global__ __launch_bounds__(1024) void k_norm_act(float * __restrict__ x, const
     if constexpr (VEC) {
         for (int k = 4 * (int)threadIdx.x; k < E; k += 4 * n_thr) {
             f4 v = *(const f4 *)(xr + k);
-            if (add.n > 0) {
-                const float * from = add.data + (size_t)t * E + k;
-                f4 d[8];
-#pragma unroll
-                for (int i = 0; i < 8; ++i) if (i < add.n) d[i] = *(const f4 *)(from + (size_t)i * add.stride);
+            if (add.n > 0 || plus) {
                 f4 s = {0, 0, 0, 0};
+                if (plus) s = *(const f4 *)(plus + (size_t)t * E + k);
+                for (int base = 0; base < add.n; base += 8) {
+                    const float * from = add.data + (size_t)base * add.stride + (size_t)t * E + k;
+                    const int n = add.n - base;
+                    f4 d[8];
 #pragma unroll
-                for (int i = 0; i < 8; ++i) if (i < add.n) s += d[i];
+                    for (int i = 0; i < 8; ++i) if (i < n) d[i] = *(const f4 *)(from + (size_t)i * add.stride);
+#pragma unroll
+                    for (int i = 0; i < 8; ++i) if (i < n) s += d[i];
+                }
                 v += s;
                 *(f4 *)(xr + k) = v;
             }
@@ -35,8 +40,8 @@ __global__ __launch_bounds__(1024) void k_norm_act(float * __restrict__ x, const
     } else {
         for (int k = threadIdx.x; k < E; k += n_thr) {
             float v = xr[k];
-            if (add.n > 0) {
-                float d = 0.0f;
+            if (add.n > 0 || plus) {
+                float d = plus ? plus[(size_t)t * E + k] : 0.0f;
                 for (int i = 0; i < add.n; ++i) d += add.data[(size_t)i * add.stride + (size_t)t * E + k];
                 v += d;
                 xr[k] = v;
@@ -73,12 +78,12 @@ __global__ void k_add_slices(float * __restrict__ x, size_t n, Slices add) {
 }  // namespace
 
 void norm_act(hipStream_t s, int arith, int kind, float * x, const float * w, int E, float eps, const int32_t * rows,
-              int n_rows, void * act, int act_kf, const Slices & add) {
+              int n_rows, void * act, int act_kf, const Slices & add, const float * plus) {
     if (n_rows <= 0) return;
     const size_t lds = (size_t)E * 4;
-    const bool vec = E % 4 == 0 && add.n <= 8;
+    const bool vec = E % 4 == 0;
     const dim3 grid((unsigned)n_rows), block(n_rows <= 512 && E >= 2048 ? 1024 : 256);
-    auto go = [&](auto kernel) { hipLaunchKernelGGL(kernel, grid, block, lds, s, x, w, E, eps, rows, act, act_kf, add); };
+    auto go = [&](auto kernel) { hipLaunchKernelGGL(kernel, grid, block, lds, s, x, w, E, eps, rows, act, act_kf, add, plus); };
     if (arith == ARITH_16) {
         if (kind == NORM_LAYER) vec ? go(k_norm_act<ARITH_16, NORM_LAYER, true>) : go(k_norm_act<ARITH_16, NORM_LAYER, false>);
         else vec ? go(k_norm_act<ARITH_16, NORM_RMS, true>) : go(k_norm_act<ARITH_16, NORM_RMS, false>);

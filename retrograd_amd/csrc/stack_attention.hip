@@ -1,6 +1,9 @@
-// Latent attention: keys and values of every head are up-projections of one cached latent per token, so a query is
-// absorbed into the latent space first (q' = W_uk^T q) and every head attends over the same cached rows, with a
-// sliding window. The attended latents leave as activations for the value up-projection.
+// Paged attention of layer-stack models, in two forms that share their kernels.
+// Latent: keys and values of every head are up-projections of one cached latent per token, so a query is absorbed into
+// the latent space first (q' = W_uk^T q) and every head attends over the same cached rows, which are keys and values at
+// once. The attended latents leave as activations for the value up-projection.
+// Grouped: a cache of keys and one of values, each with a part per key/value head, and optionally soft-capped scores.
+// Either sees all earlier positions, a sliding window of them, or those of the token's own chunk.
 #include "stack_dev.hpp"
 
 namespace rk {
@@ -52,14 +55,14 @@ __global__ __launch_bounds__(256) void k_latent_norms(LatentNorms a) {
     q = block_sum(q, scratch);
     const float inv = 1.0f / sqrtf(q / (float)n + a.eps);
     const int cell = kv ? a.cell[t] : 0;
-    EL * page = kv ? (EL *)a.pool + (size_t)(cell / PAGE) * latent_page_elems(a.pool_kf) : nullptr;
+    EL * page = kv ? (EL *)a.pool + (size_t)(cell / PAGE) * cache_page_elems(a.pool_kf) : nullptr;
     const int padded = 32 * (kv ? a.pool_kf : a.act_q_kf);
     auto finish = [&](int k, float (&o)[8]) {
         if (k >= padded) return;
 #pragma unroll
         for (int i = 0; i < 8; ++i) o[i] = k + i < n ? o[i] * inv * w[k + i] : 0.0f;
         if (kv) {
-            EL * dst = page + latent_at(cell % PAGE, k);
+            EL * dst = page + cache_at(cell % PAGE, k);
 #pragma unroll
             for (int i = 0; i < 8; ++i) dst[i] = float_el<EL>(o[i]);
         } else {
@@ -75,21 +78,28 @@ __global__ __launch_bounds__(256) void k_latent_norms(LatentNorms a) {
     }
 }
 
-// Any rank, either element type: one workgroup per query column, keys in batches of one per thread, f32 throughout.
+// First position a token at `pos` sees.
+__device__ __forceinline__ int low_key(const StackAttn & a, int kv_begin, int pos) {
+    return max(kv_begin, a.chunk > 0 ? pos - pos % a.chunk : a.window > 0 ? pos - a.window + 1 : 0);
+}
+
+// Any width, either element type: one workgroup per query column, keys in batches of one per thread, f32 throughout.
 template <int ARITH>
-__global__ __launch_bounds__(256) void k_latent_attention_any(LatentAttn a) {
+__global__ __launch_bounds__(256) void k_stack_attention_any(StackAttn a) {
     using EL = typename std::conditional<ARITH == ARITH_16, __half, float>::type;
     extern __shared__ float sm[];
-    const int R = a.kf * 32;
+    const int R = a.kf * 32, HG = a.H / a.G, kv_head = blockIdx.y;
     float * q = sm, * p = sm + R;             // [R], [256]
     __shared__ float scratch[16];
-    const LatentBlock blk = a.blocks[blockIdx.x];
+    const AttnBlock blk = a.blocks[blockIdx.x];
     const RowDesc row = a.rows[blk.row];
-    const int n_cols = row.n * a.H;
-    const size_t page_elems = latent_page_elems(a.kf);
+    const int n_cols = row.n * HG;
+    const size_t page_elems = cache_page_elems(a.kf * a.G), head_at = cache_page_elems(a.kf * kv_head);
+    const EL * keys = (const EL *)a.pool + head_at, * values = (const EL *)(a.v_pool ? a.v_pool : a.pool) + head_at;
+    constexpr float LOG2E = 1.4426950408889634f;
     for (int c = blk.col0; c < min(blk.col0 + a.block_cols, n_cols); ++c) {
-        const int tok = c / a.H, h = c % a.H, t = row.tok_off + tok, pos = row.pos0 + tok;
-        const int lo = a.window > 0 ? max(row.kv_begin, pos - a.window + 1) : row.kv_begin;
+        const int tok = c / HG, h = kv_head * HG + c % HG, t = row.tok_off + tok, pos = row.pos0 + tok;
+        const int lo = low_key(a, row.kv_begin, pos);
         const EL * qr = (const EL *)a.q + ((size_t)t * a.H + h) * R;
         __syncthreads();
         for (int k = threadIdx.x; k < R; k += 256) q[k] = el_float<EL>(qr[k]);
@@ -101,12 +111,17 @@ __global__ __launch_bounds__(256) void k_latent_attention_any(LatentAttn a) {
             float s = -INFINITY;
             if (key <= pos) {
                 const int pg = a.table[(size_t)row.slot * a.max_pages + key / PAGE];
-                const EL * page = (const EL *)a.pool + (size_t)pg * page_elems;
+                const EL * page = keys + (size_t)pg * page_elems;
                 s = 0.0f;
                 for (int k = 0; k < R; k += 8) {
-                    const EL * e = page + latent_at(key % PAGE, k);
+                    const EL * e = page + cache_at(key % PAGE, k);
 #pragma unroll
                     for (int i = 0; i < 8; ++i) s += q[k + i] * el_float<EL>(e[i]);
+                }
+                if (a.v_pool) {
+                    s *= a.scale;
+                    if (a.softcap > 0.0f) s = a.softcap * tanhf(s / a.softcap);
+                    s *= LOG2E;
                 }
             }
             float bm = s;
@@ -126,12 +141,12 @@ __global__ __launch_bounds__(256) void k_latent_attention_any(LatentAttn a) {
             for (int k = 0; k < n; ++k) {
                 const int kk = base + k;
                 const int pg = a.table[(size_t)row.slot * a.max_pages + kk / PAGE];
-                const EL * page = (const EL *)a.pool + (size_t)pg * page_elems;
+                const EL * page = values + (size_t)pg * page_elems;
                 const float pk = p[k];
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
                     const int col = threadIdx.x + 256 * i;
-                    if (col < R) acc[i] += pk * el_float<EL>(page[latent_at(kk % PAGE, col)]);
+                    if (col < R) acc[i] += pk * el_float<EL>(page[cache_at(kk % PAGE, col)]);
                 }
             }
         }
@@ -150,28 +165,31 @@ __global__ __launch_bounds__(256) void k_latent_attention_any(LatentAttn a) {
 typedef __fp16 q4 __attribute__((ext_vector_type(4)));
 typedef __attribute__((address_space(3))) q4 lds_q4;
 
-// Matrix-core form over f16 latents of KF fragments. A workgroup serves CT * WC * 16 query columns; WC waves
-// share a page (staged once into LDS, double buffered, by direct-to-LDS loads), WK such groups take pages in turn and
-// merge at the end. Scores S^T = C q'^T and outputs O^T = C^T P^T both read the page's one layout: the second product's
-// operand is its transpose, which the LDS transpose read delivers. With several splits (blockIdx.y) every one leaves an
-// unnormalised partial result.
-template <int KF, int CT, int WC, int WK>
+// Matrix-core form over f16 cache rows of KF fragments (per head). A workgroup serves CT * WC * 16 query columns of one
+// key/value head (blockIdx.z); WC waves share a page (staged once into LDS, double buffered, by direct-to-LDS loads), WK
+// such groups take pages in turn and merge at the end. Scores S^T = K q^T and outputs O^T = V^T P^T read pages of one
+// layout: the second product's operand is its transpose, which the LDS transpose read delivers, so rows that are keys
+// and values at once (KV false) are staged once; KV: a page of keys, then the page of values. With several splits
+// (blockIdx.y) every one leaves an unnormalised partial result.
+template <int KF, int CT, int WC, int WK, bool KV>
 __global__ __launch_bounds__(64 * WC * WK) __attribute__((amdgpu_waves_per_eu(2, 2)))
-void k_latent_attention(LatentAttn a) {
+void k_stack_attention(StackAttn a) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
     __shared__ float merge_ml[WC][CT][2][64];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int wc = wave % WC, wk = wave / WC, g = lane >> 4;
     constexpr int AHEAD = KF >= 4 ? 6 : 2 * KF;
-    constexpr int kf = KF, page_bytes = KF * 2048;
-    const LatentBlock blk = a.blocks[blockIdx.x];
+    constexpr int kf = KF, head_bytes = KF * 2048, page_bytes = (KV ? 2 : 1) * head_bytes;      // of a staged page
+    constexpr int PIECES = page_bytes / 1024;
+    const AttnBlock blk = a.blocks[blockIdx.x];
     const RowDesc row = a.rows[blk.row];
-    const int n_cols = row.n * a.H;
-    auto low_of = [&](int pos) { return a.window > 0 ? max(row.kv_begin, pos - a.window + 1) : row.kv_begin; };
+    const int HG = KV ? a.H / a.G : a.H, kv_head = KV ? blockIdx.z : 0;
+    const int n_cols = row.n * HG;
+    auto low_of = [&](int pos) { return low_key(a, row.kv_begin, pos); };
 
     // the block's pages, dealt to the splits
     const int last_tok = min(blk.col0 + a.block_cols, n_cols) - 1;
-    const int page_lo = low_of(row.pos0 + blk.col0 / a.H) / PAGE, page_hi = (row.pos0 + last_tok / a.H) / PAGE + 1;
+    const int page_lo = low_of(row.pos0 + blk.col0 / HG) / PAGE, page_hi = (row.pos0 + last_tok / HG) / PAGE + 1;
     const int n_all = page_hi - page_lo, sp = blockIdx.y;
     const int first = page_lo + (int)((int64_t)n_all * sp / a.splits), end = page_lo + (int)((int64_t)n_all * (sp + 1) / a.splits);
     const int n_iter = (end - first + WK - 1) / WK;
@@ -183,9 +201,11 @@ void k_latent_attention(LatentAttn a) {
         if (page >= end) return;
         // a scalar load, which no vector load is waited for with
         const int id = __builtin_amdgcn_readfirstlane(((const __attribute__((address_space(4))) int32_t *)table)[__builtin_amdgcn_readfirstlane(page)]);
-        const uint8_t * src = (const uint8_t *)a.pool + (size_t)id * page_bytes;
-        for (int ch = wc; ch < 2 * kf; ch += WC)
-            lds_dma16(src + ch * 1024, (uint32_t)lane * 16, __builtin_amdgcn_readfirstlane(to + (uint32_t)(b * page_bytes + ch * 1024)));
+        const size_t at = KV ? ((size_t)id * a.G + kv_head) * head_bytes : (size_t)id * head_bytes;
+        const uint8_t * src = (const uint8_t *)a.pool + at;
+        const uint8_t * src_v = KV ? (const uint8_t *)a.v_pool + at - head_bytes : src;
+        for (int ch = wc; ch < PIECES; ch += WC)
+            lds_dma16((ch < 2 * kf ? src : src_v) + ch * 1024, (uint32_t)lane * 16, __builtin_amdgcn_readfirstlane(to + (uint32_t)(b * page_bytes + ch * 1024)));
     };
     // this lane's column of every column tile: its token and head, and the keys it sees
     int col[CT], lo[CT], hi[CT], lo_max = 0, hi_min = 1 << 30;
@@ -194,7 +214,7 @@ void k_latent_attention(LatentAttn a) {
     for (int c = 0; c < CT; ++c) {
         col[c] = blk.col0 + (wc * CT + c) * 16 + (lane & 15);
         const int cc = min(col[c], n_cols - 1);
-        const int tok = cc / a.H, h = cc - tok * a.H;
+        const int tok = cc / HG, h = kv_head * HG + cc - tok * HG;
         hi[c] = row.pos0 + tok;
         lo[c] = low_of(hi[c]);
         lo_max = max(lo_max, lo[c]);
@@ -208,6 +228,9 @@ void k_latent_attention(LatentAttn a) {
         lo_max = max(lo_max, __shfl_xor(lo_max, o, 64));
         hi_min = min(hi_min, __shfl_xor(hi_min, o, 64));
     }
+    constexpr float LOG2E = 1.4426950408889634f;
+    const float cap_out = KV ? a.softcap * LOG2E : 0.0f;
+    const float score_in = KV ? (a.softcap > 0.0f ? 2.0f * LOG2E * a.scale / a.softcap : a.scale * LOG2E) : 1.0f;
     f4 acc[CT][2 * KF];
     float m[CT], l[CT];
 #pragma unroll
@@ -232,7 +255,7 @@ void k_latent_attention(LatentAttn a) {
             __syncthreads();
             stage(page + WK, (it + 1) & 1);
         }
-        if (page + WK < end) asm volatile("s_waitcnt vmcnt(%0)" :: "n"(2 * KF / WC) : "memory");
+        if (page + WK < end) asm volatile("s_waitcnt vmcnt(%0)" :: "n"(PIECES / WC) : "memory");
         else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         __syncthreads();
         if (page >= end) continue;
@@ -257,6 +280,24 @@ void k_latent_attention(LatentAttn a) {
             __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
         }
         __builtin_amdgcn_sched_group_barrier(0x008, AHEAD * CT, 0);
+        if constexpr (KV) {       // scores in powers of two; tanh(x) = 1 - 2 / (1 + e^2x)
+            if (cap_out > 0.0f) {
+#pragma unroll
+                for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+                    for (int c = 0; c < CT; ++c)
+#pragma unroll
+                        for (int i = 0; i < 4; ++i) {
+                            const float e = __builtin_amdgcn_exp2f(s[hf][c][i] * score_in);
+                            s[hf][c][i] = fmaf(-2.0f * cap_out, __builtin_amdgcn_rcpf(1.0f + e), cap_out);
+                        }
+            } else {
+#pragma unroll
+                for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+                    for (int c = 0; c < CT; ++c) s[hf][c] *= score_in;
+            }
+        }
         const int key0 = page * PAGE;
         const bool inside = key0 >= lo_max && key0 + PAGE - 1 <= hi_min;
         h8 p[CT];
@@ -294,7 +335,7 @@ void k_latent_attention(LatentAttn a) {
         }
 #pragma unroll
         for (int d = 0; d < 2 * KF; ++d) {
-            const uint8_t * v0 = cur + (d >> 1) * 2048 + (d & 1) * 512 + tr_lane;
+            const uint8_t * v0 = cur + (KV ? head_bytes : 0) + (d >> 1) * 2048 + (d & 1) * 512 + tr_lane;
             union { q4 half[2]; h8 all; } v;
             v.half[0] = __builtin_amdgcn_ds_read_tr16_b64_v4f16((lds_q4 *)(v0));
             v.half[1] = __builtin_amdgcn_ds_read_tr16_b64_v4f16((lds_q4 *)(v0 + 1024));
@@ -317,7 +358,7 @@ void k_latent_attention(LatentAttn a) {
     if constexpr (WK > 1) {       // the groups' results, one after the other, into the first group's
         static_assert(WK == 2 && CT == 1);
         __syncthreads();
-        f4 * park = (f4 *)lds + (size_t)wc * 2 * kf * 64;
+        f4 * park = (f4 *)lds + (size_t)wc * 2 * kf * 64;      // 2 KiB per fragment and wave: within the pages
         if (wk == 1) {
             merge_ml[wc][0][0][lane] = m[0];
             merge_ml[wc][0][1][lane] = l[0];
@@ -337,7 +378,7 @@ void k_latent_attention(LatentAttn a) {
 #pragma unroll
     for (int c = 0; c < CT; ++c) {
         if (col[c] >= min(blk.col0 + a.block_cols, n_cols)) continue;
-        const int tok = col[c] / a.H, h = col[c] - tok * a.H, t = row.tok_off + tok;
+        const int tok = col[c] / HG, h = kv_head * HG + col[c] - tok * HG, t = row.tok_off + tok;
         if (a.splits > 1) {
             const size_t at = ((size_t)t * a.H + h) * a.splits + sp;
             if (g == 0) *(float2 *)(a.partial_ml + 2 * at) = make_float2(m[c], l[c]);
@@ -366,7 +407,7 @@ void k_latent_attention(LatentAttn a) {
 
 // Merges the splits of one query column (at most 32), each a mean in f16 with its maximum and sum: a wave per column,
 // lane i the weight of split i; eight latent columns per lane and pass, the splits' values requested four at a time.
-__global__ __launch_bounds__(64) void k_latent_combine(LatentAttn a) {
+__global__ __launch_bounds__(64) void k_stack_combine(StackAttn a) {
     const int R = a.kf * 32, t = blockIdx.x / a.H, h = blockIdx.x - t * a.H, lane = threadIdx.x;
     const __half * p = (const __half *)a.partial + (size_t)blockIdx.x * a.splits * R;
     const float * ml = a.partial_ml + (size_t)blockIdx.x * a.splits * 2;
@@ -403,13 +444,13 @@ __global__ void k_copy4(const float * __restrict__ src, float * __restrict__ dst
 
 // rows[i][c] <-> column c of cell cells[i]; a column group of eight per thread.
 template <typename EL>
-__global__ void k_latent_cells(EL * __restrict__ pool, int kf, const int32_t * __restrict__ cells, int n, EL * __restrict__ rows, bool gather) {
+__global__ void k_stack_cells(EL * __restrict__ pool, int kf, const int32_t * __restrict__ cells, int n, EL * __restrict__ rows, bool gather) {
     const int groups = kf * 4;
     const int64_t total = (int64_t)n * groups;
     for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (int64_t)gridDim.x * blockDim.x) {
         const int r = (int)(i / groups), c = (int)(i % groups) * 8;
         const int cell = cells[r];
-        EL * p = pool + (size_t)(cell / PAGE) * latent_page_elems(kf) + latent_at(cell % PAGE, c);
+        EL * p = pool + (size_t)(cell / PAGE) * cache_page_elems(kf) + cache_at(cell % PAGE, c);
         EL * o = rows + (size_t)r * kf * 32 + c;
 #pragma unroll
         for (int k = 0; k < 8; ++k) { if (gather) o[k] = p[k]; else p[k] = o[k]; }
@@ -427,86 +468,92 @@ void latent_norms(hipStream_t s, int arith, const LatentNorms & a, int T) {
 }
 
 namespace {
-constexpr int kMatrixKf = 16;       // widest latent (in fragments) of the matrix-core kernel
-bool on_matrix_cores(int arith, int kf) { return arith == ARITH_16 && kf <= kMatrixKf; }
+// Widest cache rows (in fragments) of the matrix-core kernel: rows that are keys and values at once, and separate ones.
+constexpr int kMatrixKf = 16, kMatrixKfPair = 8;
+bool on_matrix_cores(int arith, int kf, bool pair) { return arith == ARITH_16 && kf <= (pair ? kMatrixKfPair : kMatrixKf); }
 
-template <int KF, int CT, int WC, int WK> void launch_attention(hipStream_t s, const LatentAttn & a) {
-    const size_t lds = (size_t)WK * 2 * KF * 2048;
-    auto kernel = k_latent_attention<KF, CT, WC, WK>;
-    static const bool allowed = hipFuncSetAttribute((const void *)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, WK * 2 * KF * 2048) == hipSuccess;
-    if (!allowed) throw std::runtime_error("latent attention: the page buffers do not fit the LDS");
-    hipLaunchKernelGGL(kernel, dim3((unsigned)a.n_blocks, (unsigned)a.splits), dim3(64 * WC * WK), lds, s, a);
+template <int KF, int CT, int WC, int WK, bool KV> void launch_attention(hipStream_t s, const StackAttn & a) {
+    constexpr int lds = WK * 2 * (KV ? 2 : 1) * KF * 2048;
+    auto kernel = k_stack_attention<KF, CT, WC, WK, KV>;
+    static const bool allowed = hipFuncSetAttribute((const void *)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, lds) == hipSuccess;
+    if (!allowed) throw std::runtime_error("attention: the page buffers do not fit the LDS");
+    hipLaunchKernelGGL(kernel, dim3((unsigned)a.n_blocks, (unsigned)a.splits, (unsigned)a.G), dim3(64 * WC * WK), lds, s, a);
 }
-template <int KF> void launch_columns(hipStream_t s, const LatentAttn & a) {
+template <int KF, bool KV> void launch_columns(hipStream_t s, const StackAttn & a) {
     switch (a.block_cols) {
-        case 16: launch_attention<KF, 1, 1, 2>(s, a); break;
-        case 32: launch_attention<KF, 1, 2, 2>(s, a); break;
-        case 64: launch_attention<KF, 1, 4, 1>(s, a); break;
+        case 16: launch_attention<KF, 1, 1, 2, KV>(s, a); break;
+        case 32: launch_attention<KF, 1, 2, 2, KV>(s, a); break;
+        case 64: launch_attention<KF, 1, 4, 1, KV>(s, a); break;
         case 128:
-            if constexpr (KF <= 8) { launch_attention<KF, 2, 4, 1>(s, a); break; }      // wider: the registers do not suffice
+            if constexpr (KF <= 8) { launch_attention<KF, 2, 4, 1, KV>(s, a); break; }      // wider: the registers do not suffice
             [[fallthrough]];
-        default: throw std::runtime_error("latent attention: no kernel for this many columns per block");
+        default: throw std::runtime_error("attention: no kernel for this many columns per block");
     }
+}
+template <bool KV> void launch_width(hipStream_t s, const StackAttn & a) {
+    switch (a.kf) {                   // the widths cache_frags() rounds to
+        case 1: return launch_columns<1, KV>(s, a);
+        case 2: return launch_columns<2, KV>(s, a);
+        case 3: return launch_columns<3, KV>(s, a);
+        case 4: return launch_columns<4, KV>(s, a);
+        case 6: return launch_columns<6, KV>(s, a);
+        case 8: return launch_columns<8, KV>(s, a);
+        case 12: if constexpr (!KV) return launch_columns<12, KV>(s, a); break;
+        case 16: if constexpr (!KV) return launch_columns<16, KV>(s, a); break;
+        default: break;
+    }
+    throw std::runtime_error("attention: no kernel for this cache width");
 }
 }  // namespace
 
-int latent_frags(int kv_rank) {
+int cache_frags(int kv_rank) {
     const int kf = frags_of(kv_rank);
     for (int w : {1, 2, 3, 4, 6, 8, 12, 16}) if (kf <= w) return w;
     return kf;
 }
 
-int latent_block_cols(int arith, int H, int kf, int n_tokens, int n_rows) {
-    if (!on_matrix_cores(arith, kf)) return 1;
-    if (n_tokens == n_rows) return H <= 16 ? 16 : H <= 32 ? 32 : 64;      // one token per row
-    return kf <= 8 && (int64_t)n_tokens * H >= 256 * 128 ? 128 : 64;
+int stack_block_cols(int arith, int cols_per_token, int kf, bool pair, int n_tokens, int n_rows) {
+    if (!on_matrix_cores(arith, kf, pair)) return 1;
+    if (n_tokens == n_rows) return cols_per_token <= 16 ? 16 : cols_per_token <= 32 ? 32 : 64;      // one token per row
+    return kf <= 8 && (int64_t)n_tokens * cols_per_token >= 256 * 128 ? 128 : 64;
 }
 
-int latent_splits(int arith, const LatentAttn & a, int max_resident) {
-    if (!on_matrix_cores(arith, a.kf)) return 1;
-    const int keys = a.window > 0 ? std::min(a.window, max_resident) : max_resident;
+int stack_splits(int arith, const StackAttn & a, int max_resident) {
+    if (!on_matrix_cores(arith, a.kf, a.v_pool)) return 1;
+    const int reach = a.chunk > 0 ? a.chunk : a.window, keys = reach > 0 ? std::min(reach, max_resident) : max_resident;
     const int pages = (keys + PAGE - 1) / PAGE + 1, per = a.block_cols <= 32 ? 2 : 1;
-    return std::max(1, std::min({256 / std::max(a.n_blocks, 1), pages / per, 32}));
+    return std::max(1, std::min({256 / std::max(a.n_blocks * a.G, 1), pages / per, 32}));
 }
 
-size_t latent_partial_floats(int T, int H, int kf, int splits) { return splits > 1 ? (size_t)T * H * splits * (kf * 16 + 2) : 0; }
+size_t stack_partial_floats(int T, int H, int kf, int splits) { return splits > 1 ? (size_t)T * H * splits * (kf * 16 + 2) : 0; }
 
-void latent_attention(hipStream_t s, int arith, const LatentAttn & a) {
+void stack_attention(hipStream_t s, int arith, const StackAttn & a) {
     if (a.n_blocks <= 0) return;
-    if (a.kf * 32 > 1024) throw std::runtime_error("latent attention: latents of at most 1024 columns");
-    if (on_matrix_cores(arith, a.kf)) {
-        switch (a.kf) {                   // the widths latent_frags() rounds to
-            case 1: launch_columns<1>(s, a); break;
-            case 2: launch_columns<2>(s, a); break;
-            case 3: launch_columns<3>(s, a); break;
-            case 4: launch_columns<4>(s, a); break;
-            case 6: launch_columns<6>(s, a); break;
-            case 8: launch_columns<8>(s, a); break;
-            case 12: launch_columns<12>(s, a); break;
-            case 16: launch_columns<16>(s, a); break;
-            default: throw std::runtime_error("latent attention: no kernel for this latent width");
-        }
-        check_launch("latent_attention");
+    if (a.kf * 32 > 1024) throw std::runtime_error("attention: cache rows of at most 1024 columns per head");
+    if (on_matrix_cores(arith, a.kf, a.v_pool)) {
+        if (a.v_pool) launch_width<true>(s, a);
+        else launch_width<false>(s, a);
+        check_launch("stack_attention");
         return;
     }
     const size_t lds = ((size_t)a.kf * 32 + 256) * 4;
-    const dim3 grid((unsigned)a.n_blocks);
-    if (arith == ARITH_16) hipLaunchKernelGGL(k_latent_attention_any<ARITH_16>, grid, dim3(256), lds, s, a);
-    else hipLaunchKernelGGL(k_latent_attention_any<ARITH_32>, grid, dim3(256), lds, s, a);
-    check_launch("latent_attention");
+    const dim3 grid((unsigned)a.n_blocks, (unsigned)a.G);
+    if (arith == ARITH_16) hipLaunchKernelGGL(k_stack_attention_any<ARITH_16>, grid, dim3(256), lds, s, a);
+    else hipLaunchKernelGGL(k_stack_attention_any<ARITH_32>, grid, dim3(256), lds, s, a);
+    check_launch("stack_attention");
 }
 
-void latent_combine(hipStream_t s, const LatentAttn & a, int T) {
+void stack_combine(hipStream_t s, const StackAttn & a, int T) {
     if (a.splits <= 1 || T <= 0) return;
-    hipLaunchKernelGGL(k_latent_combine, dim3((unsigned)(T * a.H)), dim3(64), 0, s, a);
-    check_launch("latent_combine");
+    hipLaunchKernelGGL(k_stack_combine, dim3((unsigned)(T * a.H)), dim3(64), 0, s, a);
+    check_launch("stack_combine");
 }
 
-void latent_copy_page(hipStream_t s, void * pool, size_t page_bytes, int src, int dst) {
+void stack_copy_page(hipStream_t s, void * pool, size_t page_bytes, int src, int dst) {
     const size_t n = page_bytes / 16;
     hipLaunchKernelGGL(k_copy16, dim3((unsigned)std::min<size_t>((n + 255) / 256, 256)), dim3(256), 0, s,
                        (const u4 *)((const uint8_t *)pool + (size_t)src * page_bytes), (u4 *)((uint8_t *)pool + (size_t)dst * page_bytes), n);
-    check_launch("latent_copy_page");
+    check_launch("stack_copy_page");
 }
 
 void copy_floats(hipStream_t s, const float * src, float * dst, size_t n) {
@@ -515,13 +562,13 @@ void copy_floats(hipStream_t s, const float * src, float * dst, size_t n) {
     check_launch("copy_floats");
 }
 
-void latent_cells(hipStream_t s, void * pool, int kf, int elem, const int32_t * cells, int n, void * rows, bool gather) {
+void stack_cells(hipStream_t s, void * pool, int kf, int elem, const int32_t * cells, int n, void * rows, bool gather) {
     if (n <= 0) return;
     const int64_t total = (int64_t)n * kf * 4;
     const dim3 grid((unsigned)std::min<int64_t>((total + 255) / 256, 4096));
-    if (elem == 2) hipLaunchKernelGGL(k_latent_cells<uint16_t>, grid, dim3(256), 0, s, (uint16_t *)pool, kf, cells, n, (uint16_t *)rows, gather);
-    else hipLaunchKernelGGL(k_latent_cells<uint32_t>, grid, dim3(256), 0, s, (uint32_t *)pool, kf, cells, n, (uint32_t *)rows, gather);
-    check_launch("latent_cells");
+    if (elem == 2) hipLaunchKernelGGL(k_stack_cells<uint16_t>, grid, dim3(256), 0, s, (uint16_t *)pool, kf, cells, n, (uint16_t *)rows, gather);
+    else hipLaunchKernelGGL(k_stack_cells<uint32_t>, grid, dim3(256), 0, s, (uint32_t *)pool, kf, cells, n, (uint32_t *)rows, gather);
+    check_launch("stack_cells");
 }
 
 }  // namespace rk

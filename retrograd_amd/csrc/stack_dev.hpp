@@ -34,7 +34,7 @@ template <int ARITH> __device__ __forceinline__ void store_frag8(void * act, int
 }
 
 // Element offset inside a latent page of column c of token t (both within the page).
-__device__ __forceinline__ size_t latent_at(int t, int c) {
+__device__ __forceinline__ size_t cache_at(int t, int c) {
     return ((size_t)(c >> 5) * 2 + (t >> 4)) * 512 + ((((c >> 3) & 3) * 16 + (t & 15)) * 8) + (c & 7);
 }
 

@@ -1,5 +1,6 @@
 // Launch interface of the kernels behind layer-stack models (safetensors checkpoints whose config lists every layer):
-// bf16-weight matrix products in two arithmetics, layer norm, latent attention, the state-space mixer.
+// bf16-weight matrix products in two arithmetics (also over the tokens of every expert), norms, rotary positions, paged
+// attention, expert routing, the state-space mixer.
 #pragma once
 
 #include "kernels.hpp"
@@ -27,9 +28,14 @@ struct DenseWeight {
     int n = 0, tiles = 0, kf = 0, batch = 1;
     size_t bytes() const { return frag_weight_elems(tiles, kf) * 2 * (size_t)batch; }
 };
-// dst(row0 + r, k0 + k) = src[r * row_stride + k * k_stride] for r < rows, k < cols; dst has kf fragments per row tile.
+// Places of consecutive rows or columns: `run` of them side by side, runs `step` apart.
+struct PackMap {
+    int at, run, step;
+    PackMap(int at, int run = 1 << 30, int step = 1 << 30) : at(at), run(run), step(step) {}
+};
+// dst(row(r), column(k)) = src[r * row_stride + k * k_stride] for r < rows, k < cols; dst has kf fragments per row tile.
 void dense_pack(hipStream_t s, const uint16_t * src, int rows, int cols, int64_t row_stride, int64_t k_stride,
-                uint16_t * dst, int kf, int row0, int k0);
+                uint16_t * dst, int kf, PackMap row, PackMap column);
 
 // Where a product's rows go. col0 + b * col_batch + n is the output column of row n of batch b.
 enum : int {
@@ -37,8 +43,23 @@ enum : int {
     OUT_ACT,            // activations in fragment order, ld fragments per token tile: scale * v
     OUT_ACT_RELU2,      // ... max(v, 0)^2
     OUT_ACT_GATED,      // ... v * sigmoid(gate[t * ld_gate + b])
-    OUT_QUERY,          // rows [t][batch][ld] in the latent cache's element type (f16 or f32): scale * v
+    OUT_QUERY,          // rows [t][batch][ld] in the cache's element type (f16 or f32): scale * v
     OUT_RESIDUAL,       // f32 rows dst[t * ld + col] += v
+    OUT_ACT_GEGLU,      // activations from pairs of row tiles (gate, then up): gelu(gate) * up, gelu in its tanh form
+    OUT_ACT_SWIGLU,     // ... silu(gate) * up
+    OUT_ROTARY,         // queries, keys and values of grouped attention (RotaryOut)
+    OUT_EXPERT,         // f32 rows dst[choice * stride + token * ld + col] = weight * v of an expert product's pairs
+};
+constexpr bool out_is_glu(int kind) { return kind == OUT_ACT_GEGLU || kind == OUT_ACT_SWIGLU; }
+
+// Rows of a product that are heads of kf * 32 columns, H of queries, then G of keys: rotated, the queries to rows
+// [t][H][kf * 32], the keys to their cells; the keys as projected are the values. The columns of a rotated pair are
+// neighbours (2 i, 2 i + 1).
+struct RotaryOut {
+    int H = 0, G = 0, kf = 0, pairs = 0;       // rotated pairs of a head
+    const float * table = nullptr;             // [T][pairs][2]: cosine and sine
+    void * k_pool = nullptr, * v_pool = nullptr;
+    const int32_t * cell = nullptr;
 };
 struct DenseOut {
     int kind = OUT_F32;
@@ -47,6 +68,8 @@ struct DenseOut {
     float scale = 1.0f;
     const float * gate = nullptr;
     int ld_gate = 0;
+    size_t stride = 0;
+    RotaryOut rot;
 };
 struct DenseIn {
     const void * x = nullptr;   // activations in fragment order
@@ -55,6 +78,17 @@ struct DenseIn {
 };
 // One product, or two with one weight buffer [first | second] along K whose results are scaled element by element and
 // added: v = scale1[n] * (W1 x1) + scale2[n] * (W2 x2) (kf1 fragments belong to the first; scale1 null: plain product).
+// With token_gate, v is multiplied by sigmoid(token_gate[t * ld_token_gate]) (OUT_RESIDUAL).
+// With groups, batch b of the weight multiplies the pairs (token, choice) that chose expert b: their slots are the
+// product's columns, read as tokens (gather) or as rows of a buffer in slot order.
+struct ExpertGroups {
+    const int32_t * tiles = nullptr;           // [max_tiles][4]: expert, first slot (a multiple of 16), slots
+    const int32_t * n_tiles = nullptr;
+    int max_tiles = 0, block = 0;              // most slots of a tile: expert_block()
+    const int32_t * slot_pair = nullptr;       // the pair of a slot
+    const float * weight = nullptr;            // of a pair
+    int top = 0, pairs = 0;
+};
 struct DenseJob {
     DenseWeight w;
     DenseIn x, x2;
@@ -63,6 +97,10 @@ struct DenseJob {
     int split_tile = 0;         // row tiles below go to `a`, the others (their rows counted from there) to `b`
     DenseOut a, b;
     int n_a = 0;                // true rows of part a when there is a part b
+    const float * token_gate = nullptr;
+    int ld_token_gate = 0;
+    const ExpertGroups * groups = nullptr;
+    bool gather = false;
 };
 // Runs the product over T tokens. Where `ws` (dense_workspace_floats() floats) is given and the output is OUT_RESIDUAL,
 // a decode-sized product may come back as K-slices for the next norm to add instead.
@@ -71,18 +109,19 @@ Slices dense(hipStream_t s, int arith, const DenseJob & job, int T, float * ws);
 
 // ---- norms ----------------------------------------------------------------------------------------
 enum : int { NORM_RMS = 0, NORM_LAYER = 1 };
-// act[i] = norm(x[rows[i]] (+ slices, written back)) * w; statistics and products in f32.
+// act[i] = norm(x[rows[i]] (+ slices + the row of `plus`, written back)) * w; statistics and products in f32.
 void norm_act(hipStream_t s, int arith, int kind, float * x, const float * w, int E, float eps, const int32_t * rows,
-              int n_rows, void * act, int act_kf, const Slices & add);
+              int n_rows, void * act, int act_kf, const Slices & add, const float * plus = nullptr);
 // x[t][:] += the slices, for a stream that is read elsewhere than in the next norm.
 void add_slices(hipStream_t s, float * x, int E, int T, const Slices & add);
 
-// ---- latent attention --------------------------------------------------------------------------------
-// A page of the latent cache: PAGE tokens x kf fragments of 32 columns, f16 or f32,
+// ---- attention ---------------------------------------------------------------------------------------
+// A page of a cache: PAGE tokens x kf fragments of 32 columns, f16 or f32,
 //   [column / 32][token / 16][lane = 16 * ((column % 32) / 8) + token % 16][column % 8]
-// Fragments a latent of kv_rank columns is stored in: the widths the attention kernel is compiled for, zero padded.
-int latent_frags(int kv_rank);
-constexpr size_t latent_page_elems(int kf) { return (size_t)kf * 32 * PAGE; }
+// (several key/value heads: one head's fragments behind the other's). Fragments a head's row of `columns` columns is
+// stored in: the widths the attention kernel is compiled for, zero padded.
+int cache_frags(int columns);
+constexpr size_t cache_page_elems(int kf) { return (size_t)kf * 32 * PAGE; }
 // Queries' latent: act_q = RMS norm of proj[t][0, q_rank) times q_w. With kv_w also the cached latent: RMS norm of
 // proj[t][kv_col, kv_col + kv_rank) times kv_w into cell[t] of the pool.
 struct LatentNorms {
@@ -98,33 +137,57 @@ struct LatentNorms {
 };
 void latent_norms(hipStream_t s, int arith, const LatentNorms & a, int T);
 
-// Attention of absorbed queries over the cached latents. A block serves up to `block_cols` of the T x H query columns
-// (token-major) of one row of the step.
-struct LatentBlock { int32_t row, col0; };       // row of the step, first of its n * H columns
-struct LatentAttn {
-    const void * q = nullptr;      // [T][H][kf * 32], already scaled by scale * log2(e)
-    int H = 0, kf = 0, window = 0; // window 0: every earlier position
+// Attention over paged caches: absorbed queries over latents (v_pool null, one head's worth of rows that are keys and
+// values at once), or grouped attention over keys and values of G heads. A block serves up to `block_cols` of the
+// T x (H / G) query columns (token-major) of one row of the step, for every key/value head.
+struct AttnBlock { int32_t row, col0; };         // row of the step, first of its n * (H / G) columns
+struct StackAttn {
+    const void * q = nullptr;      // [T][H][kf * 32]; latents: already scaled by scale * log2(e)
+    int H = 0, G = 1, kf = 0;
+    int window = 0, chunk = 0;     // positions seen: the last `window`, or those of the same chunk of positions (0: no bound)
+    float scale = 1.0f, softcap = 0.0f;          // with v_pool: score = scale * q.k, then softcap * tanh(score / softcap)
     const RowDesc * rows = nullptr;
-    const LatentBlock * blocks = nullptr;
+    const AttnBlock * blocks = nullptr;
     int n_blocks = 0, block_cols = 0, splits = 1;
     const int32_t * table = nullptr;
     int max_pages = 0;
-    const void * pool = nullptr;
+    const void * pool = nullptr, * v_pool = nullptr;
     void * partial = nullptr;      // several splits: [T * H][splits][kf * 32] means in f16 ...
-    float * partial_ml = nullptr;  // ... and [T * H][splits][2] maxima and sums (latent_partial_floats() for both)
+    float * partial_ml = nullptr;  // ... and [T * H][splits][2] maxima and sums (stack_partial_floats() for both)
     void * out = nullptr;          // activations: column h * kf * 32 + c
     int out_kf = 0;
 };
-int latent_block_cols(int arith, int H, int kf, int n_tokens, int n_rows);
+int stack_block_cols(int arith, int cols_per_token, int kf, bool pair, int n_tokens, int n_rows);
 // Workgroups that share a block's keys, given the longest resident span among the step's rows.
-int latent_splits(int arith, const LatentAttn & a, int max_resident);
-size_t latent_partial_floats(int T, int H, int kf, int splits);
-void latent_attention(hipStream_t s, int arith, const LatentAttn & a);
-void latent_combine(hipStream_t s, const LatentAttn & a, int T);      // of several splits (nothing to do for one)
+int stack_splits(int arith, const StackAttn & a, int max_resident);
+size_t stack_partial_floats(int T, int H, int kf, int splits);
+void stack_attention(hipStream_t s, int arith, const StackAttn & a);
+void stack_combine(hipStream_t s, const StackAttn & a, int T);      // of several splits (nothing to do for one)
+
+// ---- rotary positions ----------------------------------------------------------------------------------
+// table[t][i] = magnitude * (cos, sin)(pos[t] * freq[i]) for i < pairs; angles in double.
+void rotary_table(hipStream_t s, const double * freq, int pairs, double magnitude, const int32_t * pos, int T, float * table);
+
+// ---- expert routing --------------------------------------------------------------------------------------
+// Per token the `top` experts of largest logit (ties to the lower index) and the softmax over the chosen logits; then
+// the pairs sorted by expert into slots, every expert from a multiple of 16 on, cut into tiles of `block` slots.
+constexpr int MAX_EXPERTS = 1024, MAX_TOP = 64;
+struct ExpertRoute {
+    const float * logits = nullptr;            // [T][ld]
+    int ld = 0, experts = 0, top = 0, block = 0;
+    int32_t * sel = nullptr;                   // [T * top]
+    float * weight = nullptr;                  // [T * top]
+    int32_t * slot_pair = nullptr;             // [expert_slots()]
+    int32_t * tiles = nullptr, * n_tiles = nullptr;
+};
+int expert_block(int arith, int T, int top, int experts);
+size_t expert_slots(int T, int top, int experts);            // with room for a whole last tile
+int expert_max_tiles(int T, int top, int experts, int block);
+void expert_route(hipStream_t s, const ExpertRoute & r, int T);
 
 // Page copies and cell gathers of any pool of pages (elem bytes 2 or 4).
-void latent_copy_page(hipStream_t s, void * pool, size_t page_bytes, int src, int dst);
-void latent_cells(hipStream_t s, void * pool, int kf, int elem, const int32_t * cells, int n, void * rows, bool gather);
+void stack_copy_page(hipStream_t s, void * pool, size_t page_bytes, int src, int dst);
+void stack_cells(hipStream_t s, void * pool, int kf, int elem, const int32_t * cells, int n, void * rows, bool gather);
 
 // ---- state-space mixer (Mamba-2) ------------------------------------------------------------------------
 // The tokens of one sequence in a step, in order: seg_tok[start .. start + n) are flat token indices.

@@ -168,7 +168,8 @@ KERNEL_SYMBOLS = [
     "retro_engine_step_logits", "retro_engine_debug_keep_residual", "retro_engine_debug_read_residual",
 ]
 PROFILE_CATEGORIES = ["pack", "embed", "norm", "qkv", "rope", "attention", "combine", "o_proj", "gate_up", "swiglu",
-                      "down", "head", "sample", "absorb", "scan"]
+                      "down", "head", "sample", "absorb", "scan", "route", "experts_in",
+                      "experts_out"]
 
 _lib = None
 _i32p, _f32p, _u8p = C.POINTER(C.c_int32), C.POINTER(C.c_float), C.POINTER(C.c_uint8)

@@ -27,9 +27,68 @@ def dibosun(width, vocab, layers, eps=1e-5):
     return {"architecture": "Dibosun", "width": width, "vocab": vocab, "norm": {"eps": eps}, "layers": layers}
 
 
+def rotary(dims, base=10000.0, factor=None, original=64, fast=32.0, slow=1.0):
+    r = {"dims": dims, "base": base}
+    if factor is not None:
+        r["scaling"] = {"factor": factor, "original": original, "fast": fast, "slow": slow}
+    return r
+
+
+def dense_mlp(ff):
+    return {"kind": "dense", "ff": ff}
+
+
+def moe_mlp(experts, top, ff, shared_ff=None):
+    out = {"kind": "moe", "router": {"experts": experts, "top": top}, "expert": {"ff": ff}}
+    if shared_ff is not None:
+        out["shared"] = {"ff": shared_ff}
+    return out
+
+
+def attention_layer(heads, kv_heads, dim, mask, rot, mlp, scale=None, softcap=None):
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "mask": {"size": mask}, "rot": rot,
+         "scale": dim ** -0.5 if scale is None else scale}
+    if softcap is not None:
+        m["softcap"] = softcap
+    return {"type": "attention", "mixer": m, "mlp": mlp}
+
+
+def pomisun(width, vocab, layers, eps=1e-5, loop=None):
+    """loop: (start, stop, times) of the layers that run several times, or none."""
+    out = {"architecture": "Pomisun", "width": width, "vocab": vocab, "norm": {"eps": eps}, "layers": layers}
+    if loop:
+        out["loop"] = dict(zip(("start", "stop", "times"), loop))
+    return out
+
+
+def _gated_shapes(p, ff, E):
+    return {p + "gate": (ff, E), p + "up": (ff, E), p + "down": (E, ff)}
+
+
 def tensor_shapes(cfg) -> dict:
     E = cfg["width"]
     out = {"embed": (cfg["vocab"], E)}
+    if cfg["architecture"] == "Pomisun":
+        for i, layer in enumerate(cfg["layers"]):
+            p, m, mlp = "l%d." % i, layer["mixer"], layer.get("mlp")
+            out[p + "norm1"] = (E,)
+            out[p + "mix.q"] = (m["heads"] * m["dim"], E)
+            out[p + "mix.k"] = (m["kv_heads"] * m["dim"], E)
+            out[p + "mix.o"] = (E, m["heads"] * m["dim"])
+            if not mlp:
+                continue
+            out[p + "norm2"] = (E,)
+            if mlp["kind"] == "dense":
+                out.update(_gated_shapes(p + "mlp.", mlp["ff"], E))
+                continue
+            out[p + "mlp.router"] = (mlp["router"]["experts"], E)
+            for e in range(mlp["router"]["experts"]):
+                out.update(_gated_shapes(p + "mlp.e%d." % e, mlp["expert"]["ff"], E))
+            if mlp.get("shared"):
+                out.update(_gated_shapes(p + "mlp.shared.", mlp["shared"]["ff"], E))
+                out[p + "mlp.shared.sg"] = (1, E)
+        out["final.norm"] = (E,)
+        return out
     for i, layer in enumerate(cfg["layers"]):
         p, m = "l%d." % i, layer["mixer"]
         out[p + "norm1"] = (E,)
@@ -63,9 +122,13 @@ def tensor_shapes(cfg) -> dict:
     return out
 
 
-def mean_and_std(name, shape):
+def mean_and_std(name, shape, architecture="Dibosun"):
     """Of a tensor's normal distribution."""
     leaf = name.rsplit(".", 1)[-1]
+    if architecture == "Pomisun" and leaf.startswith("norm"):
+        return -0.1, 0.2                     # stored as the difference from one
+    if leaf == "router":
+        return 0.0, 2.0 * shape[-1] ** -0.5
     if leaf == "dt_bias":
         return -2.0, 0.7
     if leaf == "A_log":
@@ -107,7 +170,7 @@ def random_tensors(cfg, seed) -> dict:
     rng = np.random.default_rng(seed)
     out = {}
     for name, shape in tensor_shapes(cfg).items():
-        mean, std = mean_and_std(name, shape)
+        mean, std = mean_and_std(name, shape, cfg["architecture"])
         out[name] = from_bf16(to_bf16(mean + std * rng.standard_normal(shape)))
     return out
 
@@ -136,7 +199,7 @@ def write_random_checkpoint(folder, cfg, seed, device="cuda") -> Path:
     with open(folder / "model.safetensors", "wb") as f:
         f.write(_header(shapes))
         for name, shape in shapes.items():
-            mean, std = mean_and_std(name, shape)
+            mean, std = mean_and_std(name, shape, cfg["architecture"])
             t = torch.empty(shape, device=device, dtype=torch.float32).normal_(mean, std, generator=gen).to(torch.bfloat16)
             f.write(t.view(torch.int16).cpu().numpy().tobytes())
     return folder

@@ -13,7 +13,21 @@ int main(int argc, char ** argv) {
         if (what == "config") {
             const retro::StackConfig c = retro::StackConfig::read(folder);
             std::printf("%s width %d vocab %d eps %g\n", c.arch->name, c.width, c.vocab, (double)c.eps);
+            if (c.runs.size() != c.layers.size()) {
+                std::printf("runs");
+                for (const retro::LayerRun & r : c.runs) std::printf(" %s%d", r.add_embedding ? "+" : "", r.layer);
+                std::printf("\n");
+            }
             for (const retro::LayerSpec & l : c.layers) {
+                if (l.mixer == retro::Mixer::ATTENTION) {
+                    const retro::AttentionSpec & g = l.attention;
+                    std::printf("attention heads %d kv_heads %d dim %d window %d chunk %d scale %g softcap %g ff %d experts %d top %d of %d shared %d\n", g.heads, g.kv_heads,
+                                g.dim, g.window, g.chunk, (double)g.scale, (double)g.softcap, l.ff, l.moe.experts, l.moe.top, l.moe.ff, l.moe.shared_ff);
+                    std::printf("rotary %d magnitude %.17g", g.rot.dims, g.rot.magnitude());
+                    for (double f : g.rot.frequencies()) std::printf(" %.17g", f);
+                    std::printf("\n");
+                    continue;
+                }
                 const retro::LatentSpec & a = l.latent;
                 const rk::MambaShape & s = l.mamba;
                 if (l.mixer == retro::Mixer::MAMBA2)

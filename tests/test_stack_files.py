@@ -42,12 +42,106 @@ def test_every_field_of_a_configuration(reader, tmp_path):
     assert reader(tmp_path, "l2.mix.dkv").endswith("l2.mix.dkv missing\n")
 
 
+POMISUN = Y.pomisun(36, 30, [
+    Y.attention_layer(heads=6, kv_heads=2, dim=10, mask=9, rot=Y.rotary(6, 1000.0, factor=8.0, original=40, fast=4.0, slow=0.5), mlp=Y.moe_mlp(5, 2, 7, 11), softcap=3.5),
+    Y.attention_layer(heads=3, kv_heads=3, dim=8, mask=4, rot=Y.rotary(8, 50.0), mlp=None, scale=0.25),
+    Y.attention_layer(heads=1, kv_heads=1, dim=2, mask=1, rot=Y.rotary(2, 7.0, factor=2.0, original=9), mlp=Y.moe_mlp(3, 3, 2), scale=1),
+    Y.attention_layer(heads=2, kv_heads=1, dim=40, mask=4, rot=Y.rotary(40, 10000.0, factor=4.0, original=4096), mlp=Y.dense_mlp(13))], loop=(1, 3, 3))
+
+
+def test_every_field_of_a_pomisun_configuration(reader, tmp_path):
+    import plain_pomisun as PP
+
+    Y.write_checkpoint(tmp_path, POMISUN, Y.random_tensors(POMISUN, 1))
+    lines = reader(tmp_path, "config").splitlines()
+    assert lines[:2] == ["Pomisun width 36 vocab 30 eps 1e-05", "runs 0 1 2 +1 2 +1 2 3"]
+    assert lines[2::2] == [
+        "attention heads 6 kv_heads 2 dim 10 window 0 chunk 9 scale 0.316228 softcap 3.5 ff 0 experts 5 top 2 of 7 shared 11",
+        "attention heads 3 kv_heads 3 dim 8 window 0 chunk 4 scale 0.25 softcap 0 ff 0 experts 0 top 0 of 0 shared 0",
+        "attention heads 1 kv_heads 1 dim 2 window 0 chunk 1 scale 1 softcap 0 ff 0 experts 3 top 3 of 2 shared 0",
+        "attention heads 2 kv_heads 1 dim 40 window 0 chunk 4 scale 0.158114 softcap 0 ff 13 experts 0 top 0 of 0 shared 0"]
+    for line, layer in zip(lines[3::2], POMISUN["layers"]):
+        words = line.split()
+        freq, magnitude = PP.yarn_frequencies(layer["mixer"]["rot"])
+        assert int(words[1]) == layer["mixer"]["rot"]["dims"]
+        assert np.allclose([float(w) for w in words[3:]], [magnitude, *freq], rtol=1e-13)
+    assert reader(tmp_path, "l0.mlp.e4.down").endswith("l0.mlp.e4.down BF16\n")
+    assert [run for run, _ in PP.layer_order(POMISUN)] == [0, 1, 2, 1, 2, 1, 2, 3]
+
+
+@pytest.mark.parametrize("rot", [Y.rotary(64, 10000.0, factor=16.0, original=4096), Y.rotary(10, 3.0, factor=0.5, original=7, fast=2.0, slow=2.0),
+                                 Y.rotary(16, 1e6, factor=40.0, original=100000, fast=1.0, slow=32.0), Y.rotary(2, 10.0, factor=1.0, original=1e9)])
+def test_stretched_frequencies(reader, tmp_path, rot):
+    """Ramps inside the pairs, of no width, upside down, and outside the pairs."""
+    import plain_pomisun as PP
+
+    cfg = Y.pomisun(8, 8, [Y.attention_layer(1, 1, 64, 5, rot, None)])
+    (tmp_path / "config.json").write_text(json.dumps(cfg))
+    words = reader(tmp_path, "config").splitlines()[2].split()
+    freq, magnitude = PP.yarn_frequencies(rot)
+    assert np.allclose([float(w) for w in words[3:]], [magnitude, *freq], rtol=1e-13)
+
+
+@pytest.mark.parametrize("edit, message", [
+    (lambda c: c["layers"][0]["mixer"].update(kv_heads=4), "multiple of kv_heads"),
+    (lambda c: c["layers"][0]["mixer"].update(vdim=9), "vdim must be dim"),
+    (lambda c: c["layers"][0]["mixer"].pop("rot"), "lacks 'rot'"),
+    (lambda c: c["layers"][0]["mixer"]["rot"].update(dims=12), "within a head"),
+    (lambda c: c["layers"][0]["mixer"]["rot"].update(dims=5), "even"),
+    (lambda c: c["layers"][0]["mixer"]["rot"].update(base=0), "'rot.base'"),
+    (lambda c: c["layers"][0]["mixer"]["rot"]["scaling"].update(factor=0), "positive numbers"),
+    (lambda c: c["layers"][0]["mixer"]["rot"]["scaling"].pop("slow"), "lacks 'slow'"),
+    (lambda c: c["layers"][0]["mixer"].update(softcap=-1), "softcap"),
+    (lambda c: c["layers"][0]["mlp"]["router"].update(top=6), "exceeds 'experts'"),
+    (lambda c: c["layers"][0]["mlp"]["router"].update(experts=5000), "more experts"),
+    (lambda c: c["layers"][0]["mlp"].update(kind="sparse"), "unknown feed-forward kind 'sparse'"),
+    (lambda c: c["loop"].update(stop=5), "range of layers"),
+    (lambda c: c["loop"].update(start=4), "range of layers"),
+    (lambda c: c["loop"].update(times=0), "'times' is no size"),
+])
+def test_refused_pomisun_configurations(reader, tmp_path, edit, message):
+    cfg = copy.deepcopy(POMISUN)
+    edit(cfg)
+    (tmp_path / "config.json").write_text(json.dumps(cfg))
+    out = reader(tmp_path, "config")
+    assert out.startswith("refused: ") and message in out
+
+
+def test_the_plain_pomisun_statements_against_closed_forms():
+    import plain_pomisun as PP
+
+    rng = np.random.default_rng(0)
+    assert PP.chunk_mask(5, 2).sum(1).tolist() == [1, 2, 1, 2, 1] and PP.chunk_mask(4, 0).sum() == 10
+    assert np.allclose(PP.gelu_tanh(np.array([0.0, 20.0, -20.0, 1.0])), [0, 20, 0, 0.8411919906082768])
+    # a rotation keeps lengths (times its magnitude), and a score depends on the distance alone
+    rot = Y.rotary(8, 100.0, factor=4.0, original=16, fast=2.0, slow=0.25)
+    q, k = rng.standard_normal((1, 1, 10)), rng.standard_normal((1, 1, 10))
+    at = lambda x, p: PP.rotate_half(x, [p], rot)[0, 0]
+    m = PP.yarn_frequencies(rot)[1]
+    assert np.allclose(np.linalg.norm(at(q, 5)[:8]), m * np.linalg.norm(q[0, 0, :8])) and np.allclose(at(q, 5)[8:], q[0, 0, 8:])
+    assert np.allclose(at(q, 9) @ at(k, 4), at(q, 105) @ at(k, 100))
+    # one pair by hand: column 1 and column 1 + dims / 2
+    f = PP.yarn_frequencies(Y.rotary(4, 100.0))[0]
+    x = np.zeros((1, 1, 4))
+    x[..., 1] = 1
+    assert np.allclose(f, [1.0, 0.1]) and np.allclose(PP.rotate_half(x, [3], Y.rotary(4, 100.0))[0, 0], [0, np.cos(0.3), 0, np.sin(0.3)])
+    # far below the original length nothing is stretched, far above everything by the factor
+    assert np.allclose(PP.yarn_frequencies(Y.rotary(8, 2.0, factor=4.0, original=1e6))[0], PP.yarn_frequencies(Y.rotary(8, 2.0))[0])
+    assert np.allclose(PP.yarn_frequencies(Y.rotary(8, 2.0, factor=4.0, original=0.1))[0][1:], PP.yarn_frequencies(Y.rotary(8, 2.0))[0][1:] / 4)
+    assert np.allclose(PP.soft_capped(np.array([1e-3, 1e3]), 5.0), [1e-3, 5.0])
+    sel, w = PP.choose_experts(np.array([[0.0, 2.0, 1.0, 2.0]]), 3)
+    assert sel.tolist() == [[1, 3, 2]] and np.allclose(w, np.exp([[2, 2, 1]]) / np.exp([2, 2, 1]).sum())
+    assert PP.layer_order({"layers": [0] * 4}) == [(i, False) for i in range(4)]
+    assert PP.layer_order({"layers": [0] * 3, "loop": {"start": 0, "stop": 2, "times": 2}}) == [(0, False), (1, False), (0, True), (1, False), (2, False)]
+    assert np.allclose(PP.rms_norm_around_one(np.array([[3.0, 4.0]]), np.array([0.0, 1.0]), 0.0), [[3 / 12.5 ** 0.5, 8 / 12.5 ** 0.5]])
+
+
 @pytest.mark.parametrize("edit, message", [
     (lambda c: c.update(architecture="Other"), "unsupported model architecture: Other"),
     (lambda c: c.pop("width"), "lacks 'width'"),
     (lambda c: c.update(vocab=3.5), "'vocab' is no size"),
     (lambda c: c.update(layers=[]), "1 to 4096 layers"),
-    (lambda c: c["layers"][0].update(type="attention"), "unknown layer type 'attention'"),
+    (lambda c: c["layers"][0].update(type="rotary"), "unknown layer type 'rotary'"),
     (lambda c: c["layers"][0]["mlp"].update(kind="experts"), "unknown feed-forward kind 'experts'"),
     (lambda c: c["layers"][0]["mixer"].update(groups=4), "multiple of groups"),
     (lambda c: c["layers"][0]["mixer"].update(norm_groups=4), "multiple of norm_groups"),
