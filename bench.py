@@ -75,11 +75,11 @@ def parse_args():
     ap.add_argument("--single-token-matvec", action="store_true",
                     help="with --one-sequence in the exact arithmetic: the matrix-vector kernel with f32 rows instead of the tile kernels "
                          "(what RETRO_GEMV_EXACT=1 selects)")
-    ap.add_argument("--model", default="llama", choices=["llama", "dibosun"],
-                    help="dibosun: prefill and decode of the layer-stack design at a few sizes, beside the closest GGUF model "
+    ap.add_argument("--model", default="llama", choices=["llama", "dibosun", "pomisun"],
+                    help="dibosun, pomisun: prefill and decode of that layer-stack design at a few sizes, beside the closest GGUF models "
                          "(another workload than the headline, with its own JSON line)")
-    ap.add_argument("--stack-sizes", default="w2048,w4096", help="with --model dibosun: which sizes")
-    ap.add_argument("--no-closest-model", action="store_true", help="with --model dibosun: only that design")
+    ap.add_argument("--stack-sizes", default="w2048,w4096", help="with --model dibosun or pomisun: which sizes")
+    ap.add_argument("--no-closest-model", action="store_true", help="with --model dibosun or pomisun: only that design")
     return ap.parse_args()
 
 
@@ -364,7 +364,7 @@ def main() -> int:
     if args.gpus != 1:
         print("bench.py measures one GPU: the decode step has no multi-GPU path in this build (--gpus must be 1)", file=sys.stderr)
         return 2
-    if args.model == "dibosun":
+    if args.model != "llama":
         from retrograd_amd import bench_stack
         return bench_stack.main(args)
 

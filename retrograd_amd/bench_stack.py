@@ -1,5 +1,5 @@
-"""Prefill and decode of layer-stack models (Dibosun) at sizes that resemble a real model's layers, beside the closest
-GGUF model of the same width, feed-forward width and depth: what `bench.py --model dibosun` runs. Weights are random
+"""Prefill and decode of layer-stack models at sizes that resemble a real model's layers, beside the closest GGUF models
+of the same width, feed-forward width and depth: what `bench.py --model dibosun` and `--model pomisun` run. Weights are random
 (seeded), prompts random token ids. Every kernel category is also priced against its roofline, the larger of its
 algorithmic bytes over 8 TB/s and its products' flops over 2.5 PFLOP/s (a product counted once, however a model's
 arithmetic splits its operands; the scan's flops over the 157 TFLOP/s of f32)."""
@@ -19,7 +19,9 @@ N_SEQ_MAX, CONTEXT = 64, 1024
 
 # width, feed-forward, heads, dim, q_rank, kv_rank, mamba heads (of 64 x 128 state), groups
 SIZES = {"w2048": (2048, 8192, 16, 128, 768, 512, 64, 8), "w4096": (4096, 14336, 32, 128, 1536, 512, 128, 8)}
-VOCAB, WINDOW = 32000, 1024
+VOCAB, WINDOW, CHUNK = 32000, 1024, 2048
+# experts, experts per token, their width, the shared expert's
+EXPERTS = {"w2048": (64, 8, 768, 1536), "w4096": (32, 4, 1536, 3072)}
 
 
 def dibosun_config(size):
@@ -28,6 +30,22 @@ def dibosun_config(size):
     lat = lambda kv_from=None: Y.latent_layer(H, D, D, QR, R, WINDOW, F, kv_from=kv_from)
     mam = lambda: Y.mamba2_layer(MH, 64, 128, G, 4, G, F)
     return Y.dibosun(E, VOCAB, [lat(), mam(), lat(0), mam(), lat(), mam(), lat(4), mam()])
+
+
+def pomisun_config(size):
+    from . import synth_stack as Y
+    E, F, H, D = SIZES[size][:4]
+    layer = lambda mlp: Y.attention_layer(H, max(H // 4, 1), D, CHUNK, Y.rotary(D, 500000.0, factor=4.0, original=4096), mlp, softcap=50.0)
+    return Y.pomisun(E, VOCAB, [layer(Y.dense_mlp(F)), layer(Y.moe_mlp(*EXPERTS[size]))] * 4)
+
+
+def qwen3moe_shape(size):
+    from . import gguf_writer as gw
+    from . import synth
+    E, F, H, D = SIZES[size][:4]
+    n, top, fe, _ = EXPERTS[size]
+    return synth.ModelShape("qwen3moe", 8, E, H, max(H // 4, 1), D, F, VOCAB, 500000.0, gw.GGML_Q4_K, n_expert=n, n_expert_used=top, n_ff_exp=fe,
+                            name="qwen3moe-%s-mxfp4-8layers" % size)
 
 
 def llama_shape(size):
@@ -73,6 +91,53 @@ def dibosun_work(cfg, rows, ctx, n_out):
     return w
 
 
+def chosen_experts(n, top, rows):
+    """Expected number of experts that some token of a step chooses (uniformly)."""
+    return n * (1.0 - (1.0 - top / n) ** rows)
+
+
+def pomisun_work(cfg, rows, ctx, n_out):
+    E, T = cfg["width"], rows
+    w = {}
+
+    def add(k, by, fl=0.0):
+        a = w.setdefault(k, [0.0, 0.0, 0.0])
+        a[0] += by
+        a[1] += fl
+    for layer in cfg["layers"]:
+        m, mlp = layer["mixer"], layer["mlp"]
+        H, G, D = m["heads"], m["kv_heads"], m["dim"]
+        add("norm", 2 * T * E * (4 + 4 + 2))
+        add("qkv", 2 * (H + G) * D * E + T * (2 * E + 2 * H * D + 4 * G * D), 2 * T * E * (H + G) * D)
+        add("attention", ctx[1] * 4 * G * D + T * H * D * 4, 4 * T * H * ctx[0] * D)
+        add("o_proj", 2 * E * H * D + T * (2 * H * D + 8 * E), 2 * T * E * H * D)
+        if mlp["kind"] == "dense":
+            F = mlp["ff"]
+            add("gate_up", 4 * F * E + T * (2 * E + 2 * F), 4 * T * E * F)
+            add("down", 2 * E * F + T * (2 * F + 8 * E), 2 * T * E * F)
+            continue
+        n, top, F, S = mlp["router"]["experts"], mlp["router"]["top"], mlp["expert"]["ff"], mlp["shared"]["ff"]
+        used = chosen_experts(n, top, T)
+        add("shared", 2 * (n + 1 + 3 * S) * E + T * (2 * E + 4 * (n + 1) + 4 * S + 8 * E), 2 * T * E * (n + 1 + 3 * S))
+        add("route", T * (4 * n + 8 * top))
+        add("experts_in", 4 * used * F * E + T * 2 * E + T * top * 2 * F, 4 * T * top * E * F)
+        add("experts_out", 2 * used * F * E + T * top * (2 * F + 4 * E), 2 * T * top * E * F)
+    add("head", 2 * cfg["vocab"] * E + n_out * (2 * E + 4 * cfg["vocab"]), 2 * n_out * E * cfg["vocab"])
+    return w
+
+
+def qwen3moe_work(s, rows, ctx, n_out):
+    from . import gguf_writer as gw
+    w = llama_work(s, rows, ctx, n_out)
+    el, by = gw.BLOCK_GEOMETRY[s.expert_type]
+    E, F, top = s.n_embd, s.n_ff_exp, s.n_expert_used
+    used = chosen_experts(s.n_expert, top, rows)
+    # one category: router, routing, gate/up and down of the experts
+    w["gate_up"] = (s.n_layer * (4 * s.n_expert * E + 3 * used * E * F * by / el + rows * (4 * E + top * (4 * F + 4 * E))),
+                    s.n_layer * 2 * rows * E * (s.n_expert + 3 * top * F), 0.0)
+    return w
+
+
 def llama_work(s, rows, ctx, n_out):
     from . import gguf_writer as gw
     el, by = gw.BLOCK_GEOMETRY[s.matrix_type]
@@ -88,8 +153,15 @@ def roofline(work):
     return max(work[0] / HBM, work[1] / BF16, work[2] / F32)
 
 
+MOE = ("shared", "route", "experts_in", "experts_out")       # what a mixture of experts consists of, also reported as one
+
+
 def categories(prof, n_steps, work):
     out = {}
+    if prof.get("route", (0, 0))[1]:
+        parts = [k for k in MOE if k in prof]
+        prof = dict(prof, moe=(sum(prof[k][0] for k in parts), sum(prof[k][1] for k in parts)))
+        work = dict(work, moe=[sum(work[k][i] for k in parts) for i in range(3)])
     for k, (ms, n) in sorted(prof.items(), key=lambda kv: -kv[1][0]):
         if n:
             out[k] = {"us": round(ms / n_steps * 1e3, 1), "launches": n // n_steps}
@@ -98,7 +170,8 @@ def categories(prof, n_steps, work):
     return out
 
 
-def measure(path, E, vocab, work_of, window, n_batch, prefill_sizes, steps):
+def measure(path, E, vocab, work_of, keys_of, n_batch, prefill_sizes, steps):
+    """keys_of: positions -> the number of keys a token there attends."""
     import torch
 
     n_ctx = N_SEQ_MAX * (CONTEXT + 128) + 8192
@@ -130,7 +203,7 @@ def measure(path, E, vocab, work_of, window, n_batch, prefill_sizes, steps):
     for n in prefill_sizes:
         toks = draw(n)
         sec, prof = timed(lambda i: [E.StepRow(0, 0, toks, 0, sample=True, sampling=greedy)], 8, lambda i: (eng.seq_rm(0), eng.request_free(0)))
-        keys = float(np.mean(np.minimum(np.arange(n) + 1, window)))
+        keys = float(np.mean(keys_of(np.arange(n))))
         out["prefill"][n] = {"ms": round(sec * 1e3, 3), "tok_s": round(n / sec, 1),
                              "kernels": categories(prof, 2, work_of(n, (keys, n, 1), 1))}
         print("[bench] prefill", n, json.dumps(out["prefill"][n]), file=sys.stderr, flush=True)
@@ -145,7 +218,7 @@ def measure(path, E, vocab, work_of, window, n_batch, prefill_sizes, steps):
                 pos[s] += 1
         at = pos[0]
         sec, prof = timed(lambda i: [E.StepRow.decode(s, s, int(7 * s + i) % vocab, pos[s], greedy) for s in range(n)], steps, advance)
-        keys = float(min(at + steps / 2, window))
+        keys = float(np.mean(keys_of(at + np.arange(steps))))
         out["decode"][n] = {"ms": round(sec * 1e3, 3), "tok_s": round(n / sec, 1),
                             "kernels": categories(prof, 2, work_of(n, (keys, keys * n, n), n))}
         print("[bench] decode", n, json.dumps(out["decode"][n]), file=sys.stderr, flush=True)
@@ -163,26 +236,31 @@ def main(args) -> int:
     if not torch.cuda.is_available():
         print("this benchmark needs an MI355X: no HIP device is visible", file=sys.stderr)
         return 2
-    sizes = args.stack_sizes.split(",")
+    causal = lambda p: p + 1
+    design, closest = {
+        "dibosun": ((dibosun_config, dibosun_work, lambda p: np.minimum(p + 1, WINDOW)), [("llama", llama_shape, llama_work)]),
+        "pomisun": ((pomisun_config, pomisun_work, lambda p: p % CHUNK + 1),
+                    [("llama", llama_shape, llama_work), ("qwen3moe", qwen3moe_shape, qwen3moe_work)]),
+    }[args.model]
     steps = min(args.steps, 16)
-    result = {"metric": "prefill and decode throughput, Dibosun beside Llama (Q4_K) of equal width, feed-forward and depth",
-              "data": "synthetic", "context": CONTEXT, "window": WINDOW, "vocab": VOCAB, "layers": 8, "sizes": {}}
-    for size in sizes:
-        cfg = dibosun_config(size)
-        folder = Path(args.model_dir) / ("retro-bench-dibosun-%s" % size)
+    result = {"metric": "prefill and decode throughput, %s beside GGUF models (Q4_K, MXFP4 experts) of equal width, feed-forward and depth" % args.model.capitalize(),
+              "data": "synthetic", "context": CONTEXT, "vocab": VOCAB, "layers": 8, "sizes": {}}
+    for size in args.stack_sizes.split(","):
+        cfg = design[0](size)
+        folder = Path(args.model_dir) / ("retro-bench-%s-%s" % (args.model, size))
         if not (folder / "done").exists():
             Y.write_random_checkpoint(folder, cfg, args.seed)
             (folder / "done").write_text("")
-        print("[bench] dibosun", size, file=sys.stderr, flush=True)
-        entry = {"dibosun": measure(folder, E, VOCAB, lambda *a: dibosun_work(cfg, *a), WINDOW, 4096, (512, 4096), steps)}
-        if not args.no_closest_model:
-            shape = llama_shape(size)
+        print("[bench]", args.model, size, file=sys.stderr, flush=True)
+        entry = {args.model: measure(folder, E, VOCAB, lambda *a: design[1](cfg, *a), design[2], 4096, (512, 4096), steps)}
+        for name, shape_of, work in [] if args.no_closest_model else closest:
+            shape = shape_of(size)
             path = Path(args.model_dir) / ("retro-bench-%s.gguf" % shape.name)
             if not path.exists():
                 synth.write_model(path.with_suffix(".tmp"), shape, seed=args.seed, device="cuda")
                 os.replace(path.with_suffix(".tmp"), path)
-            print("[bench] llama", size, file=sys.stderr, flush=True)
-            entry["llama"] = measure(path, E, VOCAB, lambda *a: llama_work(shape, *a), 1 << 30, 4096, (512, 4096), steps)
+            print("[bench]", name, size, file=sys.stderr, flush=True)
+            entry[name] = measure(path, E, VOCAB, lambda *a: work(shape, *a), causal, 4096, (512, 4096), steps)
         result["sizes"][size] = entry
     print(json.dumps(result), flush=True)
     return 0

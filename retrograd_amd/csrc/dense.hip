@@ -242,8 +242,10 @@ __global__ __launch_bounds__(64 * KW * RW) void k_dense(DenseArgs A) {
         for (int c = 0; c < CT; ++c)
         {
             const int row = row_of<GROUPED>(A, cols, cols.first + c * 16 + (lane & 15));
-            xb[c] = (const TA *)in.x + ((size_t)(row >> 4) * in.kf + (GROUPED ? 0 : (size_t)b * in.kf_batch)) * 512 + ((lane & 48) | (row & 15)) * 8 - (ptrdiff_t)base * 512;
+            if (GROUPED && j.gather) xb[c] = (const TA *)in.x + (size_t)row * in.kf * 32 + (lane >> 4) * 8;
+            else xb[c] = (const TA *)in.x + ((size_t)(row >> 4) * in.kf + (GROUPED ? 0 : (size_t)b * in.kf_batch)) * 512 + ((lane & 48) | (row & 15)) * 8 - (ptrdiff_t)base * 512;
         }
+        const size_t step = GROUPED && j.gather ? 32 : 512;       // elements from one fragment of a row to the next
         int k = lo;
         for (; k + U <= hi; k += U) {
             b8 w[U][RT];
@@ -253,7 +255,7 @@ __global__ __launch_bounds__(64 * KW * RW) void k_dense(DenseArgs A) {
 #pragma unroll
                 for (int r = 0; r < RT; ++r) w[u][r] = *(const b8 *)(wbase[r] + (size_t)(k + u) * 512);
 #pragma unroll
-                for (int c = 0; c < CT; ++c) x[u][c].load(xb[c] + (size_t)(k + u) * 512);
+                for (int c = 0; c < CT; ++c) x[u][c].load(xb[c] + (size_t)(k + u) * step);
             }
 #pragma unroll
             for (int u = 0; u < U; ++u)
@@ -265,7 +267,7 @@ __global__ __launch_bounds__(64 * KW * RW) void k_dense(DenseArgs A) {
         for (; k < hi; ++k) {
             Operand<TA> x[CT];
 #pragma unroll
-            for (int c = 0; c < CT; ++c) x[c].load(xb[c] + (size_t)k * 512);
+            for (int c = 0; c < CT; ++c) x[c].load(xb[c] + (size_t)k * step);
 #pragma unroll
             for (int r = 0; r < RT; ++r) {
                 const b8 w = *(const b8 *)(wbase[r] + (size_t)k * 512);
@@ -405,9 +407,11 @@ __global__ __launch_bounds__(256, 2) void k_dense_lds(DenseArgs A, int n_tok_blo
             if constexpr (GROUPED) off[i] = (uint32_t)lane * 16;
             if (piece < 2 * RT) src[i] = (const uint8_t *)(weights + ((size_t)min(tile0 + piece, j.w.tiles - 1) * j.w.kf + lo) * 512);
             else if constexpr (GROUPED) {
-                const int row = row_of<GROUPED>(A, cols, cols.first + (piece - 2 * RT) * 16 + (lane & 15));
-                src[i] = (const uint8_t *)((const uint16_t *)in.x + (size_t)(lo - base) * 512);
-                off[i] = (uint32_t)(row >> 4) * (uint32_t)in.kf * 1024 + (uint32_t)((lane & 48) | (row & 15)) * 16;
+                // plain rows: four lanes take a row's 64 bytes, dealt so that the reads below meet no bank twice
+                src[i] = (const uint8_t *)((const uint16_t *)in.x + (size_t)(lo - base) * (j.gather ? 32 : 512));
+                const int row = row_of<GROUPED>(A, cols, cols.first + (piece - 2 * RT) * 16 + (j.gather ? lane >> 2 : lane & 15));
+                if (j.gather) off[i] = (uint32_t)row * (uint32_t)in.kf * 64 + (uint32_t)((lane & 3) ^ ((lane >> 4) & 3)) * 16;
+                else off[i] = (uint32_t)(row >> 4) * (uint32_t)in.kf * 1024 + (uint32_t)lane * 16;
             } else src[i] = (const uint8_t *)((const uint16_t *)in.x + ((size_t)((cols.first >> 4) + piece - 2 * RT) * in.kf + (lo - base)) * 512);
         }
         const uint32_t to = lds_offset(lds);
@@ -415,8 +419,9 @@ __global__ __launch_bounds__(256, 2) void k_dense_lds(DenseArgs A, int n_tok_blo
             const int kk = min(k, n - 1);
 #pragma unroll
             for (int i = 0; i < PER_WAVE; ++i)
-                lds_dma16(src[i] + (size_t)kk * 1024, GROUPED ? off[GROUPED ? i : 0] : (uint32_t)lane * 16, to + (uint32_t)(b * PIECES + wave + 4 * i) * 1024);
+                lds_dma16(src[i] + (size_t)kk * (GROUPED && wave + 4 * i >= 2 * RT && j.gather ? 64 : 1024), GROUPED ? off[GROUPED ? i : 0] : (uint32_t)lane * 16, to + (uint32_t)(b * PIECES + wave + 4 * i) * 1024);
         };
+        const int x_lane = GROUPED && j.gather ? ((lane & 15) * 4 + ((lane >> 4) ^ ((lane >> 2) & 3))) * 16 : lane * 16;
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");      // the part before has stored, and the counted waits start at none
         __syncthreads();                                      // the buffers may still be read by the part before
         stage(0, 0);
@@ -431,7 +436,7 @@ __global__ __launch_bounds__(256, 2) void k_dense_lds(DenseArgs A, int n_tok_blo
 #pragma unroll
             for (int r = 0; r < RT; ++r) w[r] = *(const b8 *)(cur + (wn * RT + r) * 1024 + lane * 16);
 #pragma unroll
-            for (int c = 0; c < CT; ++c) x[c] = *(const b8 *)(cur + (2 * RT + wt * CT + c) * 1024 + lane * 16);
+            for (int c = 0; c < CT; ++c) x[c] = *(const b8 *)(cur + (2 * RT + wt * CT + c) * 1024 + x_lane);
 #pragma unroll
             for (int r = 0; r < RT; ++r)
 #pragma unroll
@@ -529,8 +534,8 @@ template <int KA, int KB> Slices run(hipStream_t s, int arith, DenseArgs & A, fl
         return out;
     }
     // K-slices: workgroups that share rows along K leave partial results, added by the next norm
-    auto slice_k = [&](int want) {
-        A.ksplit = std::max(1, std::min({kMaxSlices, want, w.kf / 64}));
+    auto slice_k = [&](int want, int least) {            // least: fragments of a slice
+        A.ksplit = std::max(1, std::min({kMaxSlices, want, w.kf / least}));
         if (A.ksplit == 1) return;
         A.partial = ws;
         A.slice = (size_t)T * w.n;
@@ -541,14 +546,14 @@ template <int KA, int KB> Slices run(hipStream_t s, int arith, DenseArgs & A, fl
     };
     const bool sliceable = KA == OUT_RESIDUAL && ws && (size_t)T * w.n <= kSliceFloats;
     if constexpr (KA != OUT_QUERY && KA != OUT_ACT_GATED) {        // products of one matrix
+        auto blocks = [&](int rt, int ct) { return (int64_t)((w.tiles + 2 * rt - 1) / (2 * rt)) * ((T + 32 * ct - 1) / (32 * ct)); };
         if (w.batch == 1 && T > 128) {
             // the largest tile that leaves every CU a workgroup
-            auto blocks = [&](int rt, int ct) { return (int64_t)((w.tiles + 2 * rt - 1) / (2 * rt)) * ((T + 32 * ct - 1) / (32 * ct)); };
             if constexpr (KA != OUT_RESIDUAL) {
                 if (blocks(8, 4) >= 448) { launch_lds<KA, KB, 8, 4>(s, A); return out; }
             }
             if (sliceable && w.n % 4 == 0 && blocks(4, 4) < 256) {
-                slice_k((int)(512 / blocks(4, 4)));
+                slice_k((int)(512 / blocks(4, 4)), 16);
                 launch_lds<KA, KB, 4, 4>(s, A);
             } else if (blocks(4, 4) >= 256) launch_lds<KA, KB, 4, 4>(s, A);
             else launch_lds<KA, KB, 4, 2>(s, A);
@@ -556,13 +561,14 @@ template <int KA, int KB> Slices run(hipStream_t s, int arith, DenseArgs & A, fl
         }
     }
     const bool deep = w.kf >= 16;
-    if (deep && sliceable) slice_k(512 / std::max(T <= 16 ? w.tiles : (w.tiles + 1) / 2, 1));
+    if (deep && sliceable) slice_k(512 / std::max(T <= 16 ? w.tiles : (w.tiles + 1) / 2, 1), 64);
     if (!deep) {                        // one wave has too little of K to share it
         if (T <= 16) launch<uint16_t, KA, KB, R1, 1, 1, 4>(s, A);
         else if (T <= 32) launch<uint16_t, KA, KB, R1, 2, 1, 4>(s, A);
         else launch<uint16_t, KA, KB, R1, 4, 1, 4>(s, A);
     } else if (T <= 16) launch<uint16_t, KA, KB, R1, 1, 8, 1>(s, A);
     else if (T <= 32) launch<uint16_t, KA, KB, 2, 2, 8, 1>(s, A);
+    else if (!PAIRS && (int64_t)w.tiles * A.ksplit * w.batch <= 256) launch<uint16_t, KA, KB, R1, 4, 8, 1>(s, A);      // a workgroup for every row tile
     else launch<uint16_t, KA, KB, 2, 4, 8, 1>(s, A);
     return out;
 }
@@ -581,7 +587,10 @@ template <int KA> void run_groups(hipStream_t s, int arith, DenseArgs & A) {
         case 16: deep ? launch_groups<uint16_t, KA, R1, 1, 8, 1>(s, A) : launch_groups<uint16_t, KA, R1, 1, 1, 4>(s, A); break;
         case 32: deep ? launch_groups<uint16_t, KA, 2, 2, 8, 1>(s, A) : launch_groups<uint16_t, KA, R1, 2, 1, 4>(s, A); break;
         case 64: launch_lds_groups<KA, 4, 2>(s, A); break;
-        default: launch_lds_groups<KA, 4, 4>(s, A); break;
+        default:
+            if (out_is_glu(KA) && (int64_t)A.groups.max_tiles * ((A.j.w.tiles + 15) / 16) >= 448) launch_lds_groups<KA, 8, 4>(s, A);
+            else launch_lds_groups<KA, 4, 4>(s, A);
+            break;
     }
 }
 

@@ -171,7 +171,7 @@ struct Vocab {
 enum ProfCat : int {
     PC_PACK = 0, PC_EMBED, PC_NORM, PC_QKV, PC_ROPE, PC_ATTN, PC_COMBINE, PC_OPROJ, PC_GATEUP, PC_SWIGLU,
     PC_DOWN, PC_HEAD, PC_SAMPLE, PC_ABSORB, PC_SCAN, PC_ROUTE, PC_EXPERTS_IN,
-    PC_EXPERTS_OUT, PC_COUNT
+    PC_EXPERTS_OUT, PC_SHARED, PC_COUNT
 };
 
 class Engine {
@@ -355,7 +355,7 @@ private:
     DevBuf recurrent_slab_;
     size_t recurrent_slot_floats_ = 0, conv_plane_floats_ = 0;
     DevBuf st_h_, st_proj_, st_cq_, st_q_, st_qa_, st_ol_, st_mix_, st_ff_, st_out_, st_partial_, st_xbc_, st_y_;
-    DevBuf st_embed_, st_route_, ex_sel_, ex_weight_, ex_slot_, ex_tiles_, ex_h_;
+    DevBuf st_embed_, st_rows_, st_route_, ex_sel_, ex_weight_, ex_slot_, ex_tiles_, ex_h_;
     int st_proj_ld_ = 0;
     struct BlockPlan { int heads, cols; size_t first, n; };    // attention blocks of the step for one number of query columns per token
     std::vector<BlockPlan> block_plans_;

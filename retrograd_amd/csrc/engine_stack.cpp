@@ -339,6 +339,10 @@ void Engine::build_stack() {
     hip_check(hipMemcpy(inv_freq_.ptr, &magnitude, sizeof(double), hipMemcpyHostToDevice), "hipMemcpy");
 
     size_t h = rk::frag_elems(B, rk::frags_of(E)), cq = 0, q = 0, qa = 0, ol = 0, mix = 0, ff = 0, xbc = 0, y = 0;
+    auto zeroed = [&](DevBuf & b, size_t n) {       // padding that no producer writes has to be finite
+        b.alloc(n);
+        if (n) hip_check(hipMemsetAsync(b.ptr, 0, n, stream_), "hipMemsetAsync");
+    };
     size_t route = 0, pairs = 0, slots = 0, tiles = 0, expert_h = 0;
     for (const LayerSpec & sp : c.layers) {
         mix = std::max(mix, rk::frag_elems(B, rk::frags_of(sp.mix_width())));
@@ -371,15 +375,12 @@ void Engine::build_stack() {
         if (L.spec.mixer != Mixer::ATTENTION) st_proj_ld_ = std::max(st_proj_ld_, L.in_tiles * 16);      // grouped attention's rows go to their places at once
     for (RotaryTable & t : rotary_) t.table.alloc((size_t)B * t.spec.dims * 4);
     if (looped_) st_embed_.alloc((size_t)B * E * 4);
+    if (route) zeroed(st_rows_, (size_t)B * rk::frags_of(E) * 32 * elem);
     st_route_.alloc(route * 4);
     ex_sel_.alloc(pairs * 4);
     ex_weight_.alloc(pairs * 4);
     ex_slot_.alloc(slots * 4);
     if (tiles) ex_tiles_.alloc((tiles + 1) * 16);           // the count behind the tiles
-    auto zeroed = [&](DevBuf & b, size_t n) {       // padding that no producer writes has to be finite
-        b.alloc(n);
-        if (n) hip_check(hipMemsetAsync(b.ptr, 0, n, stream_), "hipMemsetAsync");
-    };
     x_.alloc((size_t)B * E * 4);
     zeroed(st_h_, h * elem);
     zeroed(st_out_, h * elem);
@@ -631,7 +632,7 @@ rk::Slices Engine::stack_experts(const StackLayer & L, int T) {
     const int E = c.width, KE = rk::frags_of(E), KS = rk::frags_of(std::max(e.shared_ff, 1)), KX = rk::frags_of(e.ff);
     float * ws = mm_ws_.as<float>(), * route = st_route_.as<float>();
     const int ld = up32(e.experts + 1);
-    size_t pt = prof_begin(PC_GATEUP);
+    size_t pt = prof_begin(PC_SHARED);
     rk::DenseJob in;
     in.w = L.ff_in.w;
     in.x = {st_h_.ptr, KE, 0};
@@ -640,7 +641,7 @@ rk::Slices Engine::stack_experts(const StackLayer & L, int T) {
     in.a.kind = rk::OUT_F32; in.a.dst = route; in.a.ld = ld;
     in.b.kind = c.arch->expert_act; in.b.dst = st_ff_.ptr; in.b.ld = KS;
     rk::dense(stream_, arith_, in, T, ws);
-    prof_end(PC_GATEUP, pt);
+    prof_end(PC_SHARED, pt);
     pt = prof_begin(PC_ROUTE);
     rk::ExpertRoute r;
     r.logits = route; r.ld = ld; r.experts = e.experts; r.top = e.top;
@@ -656,7 +657,7 @@ rk::Slices Engine::stack_experts(const StackLayer & L, int T) {
     pt = prof_begin(PC_EXPERTS_IN);
     rk::DenseJob up;
     up.w = L.experts_in.w;
-    up.x = in.x;
+    up.x = {st_rows_.ptr, KE, 0};
     up.groups = &g;
     up.gather = true;
     up.a.kind = c.arch->expert_act; up.a.dst = ex_h_.ptr; up.a.ld = KX;
@@ -664,7 +665,7 @@ rk::Slices Engine::stack_experts(const StackLayer & L, int T) {
     prof_end(PC_EXPERTS_IN, pt);
     rk::Slices left;
     if (e.shared_ff > 0) {
-        pt = prof_begin(PC_DOWN);
+        pt = prof_begin(PC_SHARED);
         rk::DenseJob out;
         out.w = L.ff_out.w;
         out.x = {st_ff_.ptr, KS, 0};
@@ -672,7 +673,7 @@ rk::Slices Engine::stack_experts(const StackLayer & L, int T) {
         out.a.kind = rk::OUT_RESIDUAL; out.a.dst = x_.ptr; out.a.ld = E;
         out.token_gate = route + e.experts; out.ld_token_gate = ld;
         left = rk::dense(stream_, arith_, out, T, ws);
-        prof_end(PC_DOWN, pt);
+        prof_end(PC_SHARED, pt);
     }
     pt = prof_begin(PC_EXPERTS_OUT);
     const size_t slice = (size_t)T * E;
@@ -753,7 +754,8 @@ void Engine::forward_stack(int T, int n_out) {
         prof_end(out_cat, pt);
         if (!c.arch->parallel && sp.has_ff()) {
             pt = prof_begin(PC_NORM);
-            rk::norm_act(stream_, arith_, c.arch->norm, x, L.norm2.as<float>(), E, c.eps, nullptr, T, st_h_.ptr, KE, pending);
+            rk::norm_act(stream_, arith_, c.arch->norm, x, L.norm2.as<float>(), E, c.eps, nullptr, T, st_h_.ptr, KE, pending, nullptr,
+                         sp.moe.experts > 0 ? st_rows_.ptr : nullptr);
             prof_end(PC_NORM, pt);
             pending = stack_feed_forward(L, T);
         }

@@ -7,52 +7,59 @@ namespace rk {
 
 namespace {
 
-constexpr int PER_LANE = MAX_EXPERTS / 64;
-
-// One wave: the experts of token t.
-__device__ __forceinline__ void choose(const ExpertRoute & r, int t, int lane) {
+// One wave: the experts of token t, lane l holding the logits of experts l + 64 i. Every expert's rank is the number of
+// logits before its own; rank j < top is choice j.
+template <int N> __device__ __forceinline__ void choose(const ExpertRoute & r, int t, int lane, int32_t * sel) {
     const float * z = r.logits + (size_t)t * r.ld;
-    float v[PER_LANE];
-    bool open[PER_LANE];
+    float v[N], largest = -INFINITY;
+    int rank[N];
 #pragma unroll
-    for (int i = 0; i < PER_LANE; ++i) {
+    for (int i = 0; i < N; ++i) {
         const int e = lane + 64 * i;
-        open[i] = e < r.experts;
-        v[i] = open[i] ? z[e] : 0.0f;
+        v[i] = e < r.experts ? fmaxf(z[e], -3.4e38f) : -INFINITY;      // any order is a total one: no NaN, and open places come last
+        rank[i] = 0;
+        largest = fmaxf(largest, v[i]);
     }
-    const int n = (r.experts + 63) / 64;
-    float mine = -INFINITY;                     // lane j: the j-th largest logit
-    float largest = 0.0f;
-    for (int j = 0; j < r.top; ++j) {
-        float best = 0.0f;
-        int at = -1;
+#pragma unroll 8
+    for (int o = 0; o < 64; ++o) {
 #pragma unroll
-        for (int i = 0; i < PER_LANE; ++i)
-            if (i < n && open[i] && (at < 0 || v[i] > best)) { best = v[i]; at = lane + 64 * i; }
+        for (int j = 0; j < N; ++j) {
+            const float other = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v[j]), o));
 #pragma unroll
-        for (int o = 32; o > 0; o >>= 1) {
-            const float b = __shfl_xor(best, o, 64);
-            const int a = __shfl_xor(at, o, 64);
-            if (a >= 0 && (at < 0 || b > best || (b == best && a < at))) { best = b; at = a; }
+            for (int i = 0; i < N; ++i) rank[i] += other > v[i] || (other == v[i] && (j < i || (j == i && o < lane))) ? 1 : 0;
         }
-#pragma unroll
-        for (int i = 0; i < PER_LANE; ++i) if (at == lane + 64 * i) open[i] = false;
-        if (j == 0) largest = best;
-        if (lane == j) { mine = best; r.sel[(size_t)t * r.top + j] = at; }
     }
-    const float p = lane < r.top ? expf(mine - largest) : 0.0f;
-    const float sum = wave_sum(p);
-    if (lane < r.top) r.weight[(size_t)t * r.top + lane] = p / sum;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) largest = fmaxf(largest, __shfl_xor(largest, o, 64));
+    float p[N], sum = 0.0f;
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+        p[i] = rank[i] < r.top ? expf(v[i] - largest) : 0.0f;
+        sum += p[i];
+    }
+    sum = wave_sum(sum);
+#pragma unroll
+    for (int i = 0; i < N; ++i)
+        if (rank[i] < r.top) {
+            sel[rank[i]] = lane + 64 * i;
+            r.weight[(size_t)t * r.top + rank[i]] = p[i] / sum;
+        }
+}
+__device__ __forceinline__ void choose_any(const ExpertRoute & r, int t, int lane, int32_t * sel) {
+    if (r.experts <= 64) choose<1>(r, t, lane, sel);
+    else if (r.experts <= 128) choose<2>(r, t, lane, sel);
+    else if (r.experts <= 256) choose<4>(r, t, lane, sel);
+    else choose<MAX_EXPERTS / 64>(r, t, lane, sel);
 }
 
 // One workgroup of 1024 threads: the pairs' slots and the tiles. The order of an expert's pairs is whatever the atomics
 // give; it changes no result, since a pair's column is computed alone.
-__device__ void group(const ExpertRoute & r, int n_pairs) {
+__device__ __forceinline__ void group(const ExpertRoute & r, const int32_t * sel, int n_pairs) {
     __shared__ int count[MAX_EXPERTS], base[MAX_EXPERTS], part[2][16];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     count[tid] = 0;
     __syncthreads();
-    for (int p = tid; p < n_pairs; p += 1024) atomicAdd(&count[r.sel[p]], 1);
+    for (int p = tid; p < n_pairs; p += 1024) atomicAdd(&count[sel[p]], 1);
     __syncthreads();
     const int n = count[tid], padded = (n + 15) / 16 * 16, tiles = (n + r.block - 1) / r.block;
     int a = padded, b = tiles;                  // inclusive sums over the wave, then over the waves
@@ -69,20 +76,22 @@ __device__ void group(const ExpertRoute & r, int n_pairs) {
     for (int i = 0; i < tiles; ++i)
         ((int4 *)r.tiles)[b - tiles + i] = make_int4(tid, a - padded + i * r.block, min(r.block, n - i * r.block), 0);
     __syncthreads();
-    for (int p = tid; p < n_pairs; p += 1024) r.slot_pair[atomicAdd(&base[r.sel[p]], 1)] = p;
+    for (int p = tid; p < n_pairs; p += 1024) r.slot_pair[atomicAdd(&base[sel[p]], 1)] = p;
 }
 
 __global__ __launch_bounds__(256) void k_expert_choose(ExpertRoute r, int T) {
     const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (t < T) choose(r, t, threadIdx.x & 63);
+    if (t < T) choose_any(r, t, threadIdx.x & 63, r.sel + (size_t)t * r.top);
 }
-__global__ __launch_bounds__(1024) void k_expert_group(ExpertRoute r, int n_pairs) { group(r, n_pairs); }
-// Short steps: both in one launch.
+__global__ __launch_bounds__(1024) void k_expert_group(ExpertRoute r, int n_pairs) { group(r, r.sel, n_pairs); }
+// Short steps: both in one launch, the choices in LDS.
+constexpr int ONE_LAUNCH_TOKENS = 16;
 __global__ __launch_bounds__(1024) void k_expert_route(ExpertRoute r, int T) {
-    for (int t = threadIdx.x >> 6; t < T; t += 16) choose(r, t, threadIdx.x & 63);
-    __threadfence_block();
+    __shared__ int32_t sel[ONE_LAUNCH_TOKENS * MAX_TOP];
+    const int t = threadIdx.x >> 6;               // a wave per token
+    if (t < T) choose_any(r, t, threadIdx.x & 63, sel + t * r.top);
     __syncthreads();
-    group(r, T * r.top);
+    group(r, sel, T * r.top);
 }
 
 }  // namespace
@@ -100,7 +109,7 @@ int expert_max_tiles(int T, int top, int experts, int block) {
 void expert_route(hipStream_t s, const ExpertRoute & r, int T) {
     if (T <= 0) return;
     if (r.experts > MAX_EXPERTS || r.top > MAX_TOP || r.top > r.experts) throw std::runtime_error("expert routing: too many experts");
-    if (T <= 64) {
+    if (T <= ONE_LAUNCH_TOKENS) {
         hipLaunchKernelGGL(k_expert_route, dim3(1), dim3(1024), 0, s, r, T);
     } else {
         hipLaunchKernelGGL(k_expert_choose, dim3((unsigned)((T + 3) / 4)), dim3(256), 0, s, r, T);

@@ -10,7 +10,7 @@ namespace {
 template <int ARITH, int KIND, bool VEC>
 __global__ __launch_bounds__(1024) void k_norm_act(float * __restrict__ x, const float * __restrict__ w, int E, float eps,
                                                    const int32_t * __restrict__ rows, void * __restrict__ act, int kf, Slices add,
-                                                   const float * __restrict__ plus) {
+                                                   const float * __restrict__ plus, void * __restrict__ act_rows) {
     extern __shared__ __attribute__((aligned(16))) float row[];
     __shared__ float scratch[16];
     const int t = rows ? rows[blockIdx.x] : (int)blockIdx.x, n_thr = blockDim.x;
@@ -64,6 +64,7 @@ __global__ __launch_bounds__(1024) void k_norm_act(float * __restrict__ x, const
 #pragma unroll
         for (int i = 0; i < 8; ++i) v[i] = k + i < E ? (row[k + i] - mean) * inv * w[k + i] : 0.0f;
         store_frag8<ARITH>(act, kf, blockIdx.x, k, v);
+        if (act_rows) store_act8_at<ARITH>(act_rows, (size_t)blockIdx.x * kf * 32 + k, v);
     }
 }
 
@@ -78,12 +79,12 @@ __global__ void k_add_slices(float * __restrict__ x, size_t n, Slices add) {
 }  // namespace
 
 void norm_act(hipStream_t s, int arith, int kind, float * x, const float * w, int E, float eps, const int32_t * rows,
-              int n_rows, void * act, int act_kf, const Slices & add, const float * plus) {
+              int n_rows, void * act, int act_kf, const Slices & add, const float * plus, void * act_rows) {
     if (n_rows <= 0) return;
     const size_t lds = (size_t)E * 4;
     const bool vec = E % 4 == 0;
     const dim3 grid((unsigned)n_rows), block(n_rows <= 512 && E >= 2048 ? 1024 : 256);
-    auto go = [&](auto kernel) { hipLaunchKernelGGL(kernel, grid, block, lds, s, x, w, E, eps, rows, act, act_kf, add, plus); };
+    auto go = [&](auto kernel) { hipLaunchKernelGGL(kernel, grid, block, lds, s, x, w, E, eps, rows, act, act_kf, add, plus, act_rows); };
     if (arith == ARITH_16) {
         if (kind == NORM_LAYER) vec ? go(k_norm_act<ARITH_16, NORM_LAYER, true>) : go(k_norm_act<ARITH_16, NORM_LAYER, false>);
         else vec ? go(k_norm_act<ARITH_16, NORM_RMS, true>) : go(k_norm_act<ARITH_16, NORM_RMS, false>);

@@ -19,21 +19,25 @@ __device__ __forceinline__ size_t frag_at(int row, int k, int kf) {
     return ((size_t)(row >> 4) * kf + (k >> 5)) * 512 + ((((k >> 3) & 3) * 16 + (row & 15)) * 8) + (k & 7);
 }
 
-// Eight consecutive values of a row (k a multiple of 8) as activations of either arithmetic.
-template <int ARITH> __device__ __forceinline__ void store_frag8(void * act, int kf, int row, int k, const float (&v)[8]) {
+// Eight consecutive values of a row (k a multiple of 8) as activations of either arithmetic, from element `at` of act on.
+template <int ARITH> __device__ __forceinline__ void store_act8_at(void * act, size_t at, const float (&v)[8]) {
     if constexpr (ARITH == ARITH_16) {
         u4 u;
 #pragma unroll
         for (int i = 0; i < 4; ++i) u[i] = (uint32_t)bf16_bits(v[2 * i]) | ((uint32_t)bf16_bits(v[2 * i + 1]) << 16);
-        *(u4 *)((uint16_t *)act + frag_at(row, k, kf)) = u;
+        *(u4 *)((uint16_t *)act + at) = u;
     } else {
-        float * p = (float *)act + frag_at(row, k, kf);
+        float * p = (float *)act + at;
         *(f4 *)p = f4{v[0], v[1], v[2], v[3]};
         *(f4 *)(p + 4) = f4{v[4], v[5], v[6], v[7]};
     }
 }
 
-// Element offset inside a latent page of column c of token t (both within the page).
+template <int ARITH> __device__ __forceinline__ void store_frag8(void * act, int kf, int row, int k, const float (&v)[8]) {
+    store_act8_at<ARITH>(act, frag_at(row, k, kf), v);
+}
+
+// Element offset inside a cache page of column c of token t (both within the page).
 __device__ __forceinline__ size_t cache_at(int t, int c) {
     return ((size_t)(c >> 5) * 2 + (t >> 4)) * 512 + ((((c >> 3) & 3) * 16 + (t & 15)) * 8) + (c & 7);
 }

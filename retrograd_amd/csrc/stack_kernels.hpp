@@ -80,7 +80,8 @@ struct DenseIn {
 // added: v = scale1[n] * (W1 x1) + scale2[n] * (W2 x2) (kf1 fragments belong to the first; scale1 null: plain product).
 // With token_gate, v is multiplied by sigmoid(token_gate[t * ld_token_gate]) (OUT_RESIDUAL).
 // With groups, batch b of the weight multiplies the pairs (token, choice) that chose expert b: their slots are the
-// product's columns, read as tokens (gather) or as rows of a buffer in slot order.
+// product's columns, read as tokens (gather; x then holds plain rows of kf * 32 columns, so that a gathered row's pieces
+// lie together) or as rows of a buffer in slot order.
 struct ExpertGroups {
     const int32_t * tiles = nullptr;           // [max_tiles][4]: expert, first slot (a multiple of 16), slots
     const int32_t * n_tiles = nullptr;
@@ -109,9 +110,10 @@ Slices dense(hipStream_t s, int arith, const DenseJob & job, int T, float * ws);
 
 // ---- norms ----------------------------------------------------------------------------------------
 enum : int { NORM_RMS = 0, NORM_LAYER = 1 };
-// act[i] = norm(x[rows[i]] (+ slices + the row of `plus`, written back)) * w; statistics and products in f32.
+// act[i] = norm(x[rows[i]] (+ slices + the row of `plus`, written back)) * w; statistics and products in f32. With
+// act_rows the same activations also as plain rows of act_kf * 32.
 void norm_act(hipStream_t s, int arith, int kind, float * x, const float * w, int E, float eps, const int32_t * rows,
-              int n_rows, void * act, int act_kf, const Slices & add, const float * plus = nullptr);
+              int n_rows, void * act, int act_kf, const Slices & add, const float * plus = nullptr, void * act_rows = nullptr);
 // x[t][:] += the slices, for a stream that is read elsewhere than in the next norm.
 void add_slices(hipStream_t s, float * x, int E, int T, const Slices & add);
 

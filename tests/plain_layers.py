@@ -96,14 +96,28 @@ def mamba2(h, w, m, eps):
     return y @ w["o"].T
 
 
+def layer_order(cfg):
+    """(layer, whether the embedding output is added before it) of every layer run."""
+    n, loop = len(cfg["layers"]), cfg.get("loop")
+    if not loop:
+        return [(i, False) for i in range(n)]
+    lo, hi = loop["start"], loop["stop"]
+    order = [(i, False) for i in range(lo)]
+    for turn in range(loop["times"]):
+        order += [(i, turn > 0 and i == lo) for i in range(lo, hi)]
+    return order + [(i, False) for i in range(hi, n)]
+
+
 def run_stack(cfg, tensors, tokens, dtype=np.float64, keep=None):
-    """Logits [T, vocab] of one sequence; keep: a list that receives the residual stream after every layer."""
+    """Logits [T, vocab] of one sequence; keep: a list that receives the residual stream after every layer run."""
     W = {k: np.asarray(v, dtype) for k, v in tensors.items()}
     eps = dtype(cfg["norm"]["eps"])
-    x = W["embed"][np.asarray(tokens)]
-    latents = {}
-    for i, layer in enumerate(cfg["layers"]):
-        p = "l%d." % i
+    first = x = W["embed"][np.asarray(tokens)]
+    latents = {}                                 # of a layer's latest pass
+    for i, add_first in layer_order(cfg):
+        p, layer = "l%d." % i, cfg["layers"][i]
+        if add_first:
+            x = x + first
         w = {k[len(p) + 4:]: v for k, v in W.items() if k.startswith(p + "mix.")}
         h = layer_norm(x, W[p + "norm1"], eps)
         m = layer["mixer"]

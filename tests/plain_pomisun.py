@@ -7,7 +7,7 @@ import math
 
 import numpy as np
 
-from plain_layers import silu, softmax_rows, sigmoid
+from plain_layers import layer_order, sigmoid, silu, softmax_rows
 
 
 def gelu_tanh(z):
@@ -99,18 +99,6 @@ def expert_ff(h, w, mlp):
         s = gated_ff(h, w["shared.gate"], w["shared.up"], w["shared.down"], silu)
         out = out + s * sigmoid(h @ w["shared.sg"].T)
     return out
-
-
-def layer_order(cfg):
-    """(layer, whether the embedding output is added before it) of every layer run."""
-    n, loop = len(cfg["layers"]), cfg.get("loop")
-    if not loop:
-        return [(i, False) for i in range(n)]
-    lo, hi = loop["start"], loop["stop"]
-    order = [(i, False) for i in range(lo)]
-    for turn in range(loop["times"]):
-        order += [(i, turn > 0 and i == lo) for i in range(lo, hi)]
-    return order + [(i, False) for i in range(hi, n)]
 
 
 def routing_lead(z, top):

@@ -233,6 +233,8 @@ TILES = {
     "stream": (Y.pomisun(8204, 50, [attention(mlp=Y.moe_mlp(3, 2, 30, 52))]), (300, 140, 20)),
     "columns": (Y.pomisun(132, 50, [attention(heads=16, kv_heads=4, dim=130, mlp=Y.dense_mlp(4100)), attention(mlp=Y.moe_mlp(3, 2, 4100, 4132))]), (300, 140, 64, 30, 9)),
     "columns-odd": (Y.pomisun(131, 50, [attention(heads=16, kv_heads=4, dim=130, mlp=Y.dense_mlp(4100)), attention(mlp=Y.moe_mlp(3, 2, 650, 670))]), (300, 60, 9)),
+    "shared": (Y.pomisun(64, 30, [attention(mlp=Y.moe_mlp(3, 2, 30, 14340))]), (520,)),
+    "experts": (Y.pomisun(64, 30, [attention(heads=2, mlp=Y.moe_mlp(8, 4, 1540))]), (1000,)),
     "queries": (Y.pomisun(64, 40, [attention(heads=300, kv_heads=60, dim=96)]), (530, 200)),
 }
 
@@ -242,7 +244,7 @@ TILES = {
 def test_products_of_every_tile_shape(tmp_path, name, kv):
     cfg, sizes = TILES[name]
     m = Pomisun(tmp_path / name, cfg, decide_routing)
-    with m.engine(kv, n_ctx=1024, n_batch=576) as eng:
+    with m.engine(kv, n_ctx=1152, n_batch=1024) as eng:
         for n in sizes:
             toks = m.tokens(n + 3, n)
             want = m.plain(toks)

@@ -29,6 +29,9 @@ CONFIGS = {
     "mamba": Y.dibosun(64, 50, [Y.mamba2_layer(**MAMBA, ff=0)]),
     "mamba-ff": Y.dibosun(56, 50, [Y.mamba2_layer(**MAMBA, ff=33)]),
     "shared": Y.dibosun(64, 50, [Y.latent_layer(**LATENT, ff=0), Y.latent_layer(**{**LATENT, "window": 90}, ff=0, kv_from=0)]),
+    # layers that run several times, every pass with its own latents and states
+    "loop": {**Y.dibosun(64, 50, [Y.mamba2_layer(**MAMBA, ff=0), Y.latent_layer(**LATENT, ff=40), Y.latent_layer(**{**LATENT, "window": 90}, ff=0, kv_from=1),
+                                  Y.mamba2_layer(**MAMBA, ff=33)]), "loop": {"start": 1, "stop": 4, "times": 3}},
     # sizes of one
     "ones": Y.dibosun(33, 40, [
         Y.latent_layer(heads=1, dim=1, vdim=1, q_rank=1, kv_rank=1, window=1, ff=1, scale=1.5),
@@ -73,7 +76,7 @@ def test_whole_prompts_and_every_layer(models, name, kv):
 
 
 @pytest.mark.parametrize("kv", KINDS)
-@pytest.mark.parametrize("name", ["all", "ones", "wide"])
+@pytest.mark.parametrize("name", ["all", "loop", "ones", "wide"])
 def test_token_by_token_is_the_prompt(models, name, kv):
     m = models(name)
     toks = m.tokens(130 if name != "wide" else 120)
@@ -84,7 +87,7 @@ def test_token_by_token_is_the_prompt(models, name, kv):
 
 
 @pytest.mark.parametrize("kv", KINDS)
-@pytest.mark.parametrize("name", ["all", "ones", "wide"])
+@pytest.mark.parametrize("name", ["all", "loop", "ones", "wide"])
 def test_portions_of_any_size(models, name, kv):
     m = models(name)
     toks = m.tokens(150)
