@@ -35,7 +35,7 @@ def dibosun_config(size):
 def pomisun_config(size):
     from . import synth_stack as Y
     E, F, H, D = SIZES[size][:4]
-    layer = lambda mlp: Y.attention_layer(H, max(H // 4, 1), D, CHUNK, Y.rotary(D, 500000.0, factor=4.0, original=4096), mlp, softcap=50.0)
+    layer = lambda mlp: Y.attention_layer(H, max(H // 4, 1), D, CHUNK, Y.rotary(D, 1e6, factor=8.0, original=8192), mlp, softcap=30.0)
     return Y.pomisun(E, VOCAB, [layer(Y.dense_mlp(F)), layer(Y.moe_mlp(*EXPERTS[size]))] * 4)
 
 

@@ -289,7 +289,7 @@ def test_chunk_edges(tmp_path, chunk, kv):
     """One key's score stands far out: it decides the output until its chunk ends and not a token longer, in prompts,
     portions and decoding; chunks are one page, one key to either side of one, and several pages. The plain statement
     with a chunk one key shorter or longer is far outside the limit at the edge."""
-    cfg = lambda size: Y.pomisun(96, 60, [attention(heads=4, kv_heads=2, dim=32, mask=size, rot=Y.rotary(8), scale=0.6, softcap=50.0)])
+    cfg = lambda size: Y.pomisun(96, 60, [attention(heads=4, kv_heads=2, dim=32, mask=size, rot=Y.rotary(8), scale=0.6, softcap=45.0)])
     m = Pomisun(tmp_path / ("edge%d" % chunk), cfg(chunk), sharpen)
     for place in (0, 5, chunk - 2, chunk - 1, chunk, chunk + 3, 2 * chunk - 1):
         last = (place // chunk + 1) * chunk - 1
@@ -310,7 +310,7 @@ def test_chunk_edges(tmp_path, chunk, kv):
 @pytest.mark.parametrize("kv", KINDS)
 def test_far_keys(tmp_path, kv):
     """A key hundreds of tokens back decides, at page borders and inside pages; without it the output is another."""
-    m = Pomisun(tmp_path / "far", Y.pomisun(96, 60, [attention(heads=4, kv_heads=2, dim=32, mask=700, rot=Y.rotary(8), scale=0.6, softcap=50.0)]), sharpen)
+    m = Pomisun(tmp_path / "far", Y.pomisun(96, 60, [attention(heads=4, kv_heads=2, dim=32, mask=700, rot=Y.rotary(8), scale=0.6, softcap=45.0)]), sharpen)
     for place in (0, 31, 32, 100):
         toks = m.tokens(620, place)
         toks[toks == 7] = 8
