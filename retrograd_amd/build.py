@@ -16,7 +16,8 @@ CSRC = PKG / "csrc"
 LIB_DIR = PKG / "lib"
 LIB_PATH = LIB_DIR / "libretro_hip.so"
 SOURCES = ["kernels.hip", "mm_lds.hip", "gemv.hip", "moe.hip", "mxfp4_scaled.hip", "dense.hip", "norms.hip",
-           "stack_attention.hip", "experts.hip", "rotary.hip", "mamba2.hip", "engine.cpp", "engine_stack.cpp", "generate.cpp", "capi.cpp", "capi_trainer.cpp", "capi_test.cpp"]
+           "stack_attention.hip", "experts.hip", "rotary.hip", "short_conv.hip",
+           "mamba2.hip", "delta.hip", "engine.cpp", "engine_stack.cpp", "generate.cpp", "capi.cpp", "capi_trainer.cpp", "capi_test.cpp"]
 # host-only sources (the step scheduler): plain C++, no device pass
 HOST_SOURCES = ["sched/prefix_tree.cpp", "sched/scheduler.cpp", "sched/fake_backend.cpp", "sched/engine_backend.cpp",
                 "sched/capi_sched.cpp"]

@@ -13,7 +13,7 @@ struct DenseArgs {
     int T;
     int n_groups;          // row groups of one batch
     int ksplit;            // workgroups that share a row group along K
-    float * partial;       // [ksplit][rows padded to 64][N]
+    float * partial;       // [ksplit][T][N]: the product leaves its K-slices here (null: it goes to its outputs)
     size_t slice;
     int grid_k;            // workgroups of one K-slice (the LDS kernel)
     ExpertGroups groups;
@@ -72,8 +72,16 @@ template <int ARITH> __device__ __forceinline__ void store_rotary(const DenseOut
 }
 
 // gate and up of the same four columns
-template <int KIND> __device__ __forceinline__ f4 glu(const f4 & gate, const f4 & up) {
+template <int KIND> __device__ __forceinline__ f4 glu(const DenseOut & o, const f4 & gate, const f4 & up) {
     f4 v;
+    if constexpr (KIND == OUT_ACT_CLAMPED) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const float g = fminf(gate[i], o.limit), u = fminf(fmaxf(up[i], -o.limit), o.limit);
+            v[i] = g / (1.0f + expf(-o.slope * g)) * (u + 1.0f);
+        }
+        return v;
+    }
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
         const float z = gate[i];
@@ -100,11 +108,14 @@ __device__ __forceinline__ void store_out(const DenseOut & o, int t, int b, int 
         for (int i = 0; i < 4; ++i) { const float r = fmaxf(v[i], 0.0f); v[i] = r * r; }
     } else if constexpr (KIND == OUT_ACT_GATED) {
         v *= 1.0f / (1.0f + expf(-o.gate[(size_t)t * o.ld_gate + b]));
+    } else if constexpr (KIND == OUT_F32_CAPPED) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = o.limit * tanhf(v[i] / o.limit);
     } else if constexpr (KIND != OUT_RESIDUAL && !out_is_glu(KIND) && KIND != OUT_EXPERT) {
         v *= o.scale;
     }
     const int col = o.col0 + (KIND == OUT_QUERY ? 0 : b * o.col_batch) + n;
-    if constexpr (KIND == OUT_F32 || KIND == OUT_RESIDUAL) {
+    if constexpr (KIND == OUT_F32 || KIND == OUT_F32_CAPPED || KIND == OUT_RESIDUAL) {
         const size_t at = (size_t)t * o.ld + col;
         float * y = (float *)o.dst + at;
         if (cnt >= 4 && (at & 3) == 0) {
@@ -152,7 +163,7 @@ __device__ __forceinline__ void store_rows(const DenseJob & j, int t, int b, int
     if (KB < 0 || tile < j.split_tile) {
         if constexpr (out_is_glu(KA)) {
             if (tile & 1) return;
-            store_out<KA, ARITH>(j.a, t, b, tile * 8 + 4 * g, j.n_a / 2, glu<KA>(v, next));
+            store_out<KA, ARITH>(j.a, t, b, tile * 8 + 4 * g, j.n_a / 2, glu<KA>(j.a, v, next));
         } else {
             store_out<KA, ARITH>(j.a, t, b, tile * 16 + 4 * g, j.n_a, v);
         }
@@ -160,7 +171,7 @@ __device__ __forceinline__ void store_rows(const DenseJob & j, int t, int b, int
         const int rows = j.w.n - j.split_tile * 16, at = tile - j.split_tile;
         if constexpr (out_is_glu(KB)) {
             if (at & 1) return;
-            store_out<KB, ARITH>(j.b, t, b, at * 8 + 4 * g, rows / 2, glu<KB>(v, next));
+            store_out<KB, ARITH>(j.b, t, b, at * 8 + 4 * g, rows / 2, glu<KB>(j.b, v, next));
         } else {
             store_out<KB, ARITH>(j.b, t, b, at * 16 + 4 * g, rows, v);
         }
@@ -178,6 +189,24 @@ __device__ __forceinline__ void store_expert(const DenseArgs & A, int t, int n, 
     if (cnt >= 4 && (o.ld & 3) == 0) *(f4 *)y = v;
     else
         for (int i = 0; i < 4 && i < cnt; ++i) y[i] = v[i];
+}
+
+// K-slice `ks` of rows n .. n + 3 of token t; `add`: to what is there.
+__device__ __forceinline__ void store_slice(const DenseArgs & A, int ks, int t, int n, f4 v, bool add) {
+    const int cnt = A.j.w.n - n;
+    if (cnt <= 0) return;
+    float * p = A.partial + (size_t)ks * A.slice + (size_t)t * A.j.w.n + n;
+    if (cnt >= 4 && (A.j.w.n & 3) == 0) {
+        if (add) v += *(const f4 *)p;
+        *(f4 *)p = v;
+    } else {
+        for (int i = 0; i < 4 && i < cnt; ++i) p[i] = add ? p[i] + v[i] : v[i];
+    }
+}
+
+// Biases of rows 4 g .. 4 g + 3 of a tile.
+__device__ __forceinline__ f4 bias_of(const DenseJob & j, int b, int tile, int g) {
+    return *(const f4 *)(j.bias + ((size_t)b * j.w.tiles + tile) * 16 + 4 * g);
 }
 
 __device__ __forceinline__ float token_factor(const DenseJob & j, int t) {
@@ -322,6 +351,22 @@ __global__ __launch_bounds__(64 * KW * RW) void k_dense(DenseArgs A) {
         if (kw != 0) return;
     }
     constexpr int ARITH = (int)sizeof(TA);
+    if constexpr (DUAL) {
+#pragma unroll
+        for (int c = 0; c < CT; ++c) {
+            const float f = token_factor(j, min(cols.first + c * 16 + (lane & 15), cols.end - 1));
+#pragma unroll
+            for (int r = 0; r < RT; ++r) acc[r][c] *= f;
+        }
+    }
+    if (j.bias && ks == 0) {
+#pragma unroll
+        for (int r = 0; r < RT; ++r) {
+            const f4 f = bias_of(j, b, min(tile0 + r, j.w.tiles - 1), lane >> 4);
+#pragma unroll
+            for (int c = 0; c < CT; ++c) acc[r][c] += f;
+        }
+    }
 #pragma unroll
     for (int r = 0; r < RT; ++r) {
         const int tile = tile0 + r;
@@ -330,14 +375,10 @@ __global__ __launch_bounds__(64 * KW * RW) void k_dense(DenseArgs A) {
         for (int c = 0; c < CT; ++c) {
             const int t = cols.first + c * 16 + (lane & 15);
             if (t >= cols.end) continue;
-            if constexpr (DUAL) acc[r][c] *= token_factor(j, t);
             if constexpr (KA == OUT_EXPERT) {
                 store_expert(A, t, tile * 16 + 4 * (lane >> 4), acc[r][c]);
-            } else if (DUAL && A.ksplit > 1) {
-                const int n = tile * 16 + 4 * (lane >> 4);
-                float * p = A.partial + (size_t)ks * A.slice + (size_t)t * j.w.n + n;
-                if (n + 4 <= j.w.n && (j.w.n & 3) == 0) *(f4 *)p = acc[r][c];
-                else for (int i = 0; i < 4 && n + i < j.w.n; ++i) p[i] = acc[r][c][i];
+            } else if (DUAL && A.partial) {
+                store_slice(A, ks, t, tile * 16 + 4 * (lane >> 4), acc[r][c], false);
             } else {
                 store_rows<KA, KB, ARITH>(j, t, GROUPED ? 0 : b, tile, lane >> 4, acc[r][c], acc[RT > 1 ? r ^ 1 : r][c]);
             }
@@ -446,6 +487,15 @@ __global__ __launch_bounds__(256, 2) void k_dense_lds(DenseArgs A, int n_tok_blo
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");      // nothing may land in LDS that another workgroup owns by then
     };
     auto store = [&](const float * scale, bool first) {
+        const bool biased = j.bias && ks == 0 && first;
+        if (!DUAL && biased) {
+#pragma unroll
+            for (int r = 0; r < RT; ++r) {
+                const f4 f = bias_of(j, cols.b, min(tile0 + wn * RT + r, j.w.tiles - 1), lane >> 4);
+#pragma unroll
+                for (int c = 0; c < CT; ++c) acc[r][c] += f;
+            }
+        }
 #pragma unroll
         for (int r = 0; r < RT; ++r) {
             const int tile = tile0 + wn * RT + r;
@@ -461,15 +511,14 @@ __global__ __launch_bounds__(256, 2) void k_dense_lds(DenseArgs A, int n_tok_blo
                 const int t = cols.first + (wt * CT + c) * 16 + (lane & 15);
                 if (t >= cols.end) continue;
                 f4 v = acc[r][c];
-                if constexpr (DUAL) v *= f * token_factor(j, t);
+                if constexpr (DUAL) {
+                    v *= f * token_factor(j, t);
+                    if (biased) v += bias_of(j, 0, tile, lane >> 4);
+                }
                 if constexpr (KA == OUT_EXPERT) {
                     store_expert(A, t, tile * 16 + 4 * (lane >> 4), v);
-                } else if (DUAL && A.ksplit > 1) {            // whole groups of four rows (see run)
-                    const int n = tile * 16 + 4 * (lane >> 4);
-                    if (n >= j.w.n) continue;
-                    f4 * p = (f4 *)(A.partial + (size_t)ks * A.slice + (size_t)t * j.w.n + n);
-                    if (!first) v += *p;
-                    *p = v;
+                } else if (DUAL && A.partial) {
+                    store_slice(A, ks, t, tile * 16 + 4 * (lane >> 4), v, !first);
                 } else {
                     store_rows<KA, KB, ARITH_16>(j, t, 0, tile, lane >> 4, v, acc[r ^ 1][c]);
                 }
@@ -528,6 +577,16 @@ template <int KA, int KB> Slices run(hipStream_t s, int arith, DenseArgs & A, fl
     const DenseWeight & w = A.j.w;
     constexpr bool PAIRS = out_is_glu(KA) || out_is_glu(KB);      // row tiles in pairs
     constexpr int R1 = PAIRS ? 2 : 1;
+    auto slices = [&](int n) {
+        A.ksplit = n;
+        A.partial = ws;
+        A.slice = (size_t)T * w.n;
+        out.data = ws;
+        out.n = n;
+        out.stride = A.slice;
+        out.N = w.n;
+    };
+    if (KA == OUT_RESIDUAL && !A.j.a.dst) slices(1);
     if (arith == ARITH_32) {
         if (T <= 16) launch<float, KA, KB, R1, 1, 4, 1>(s, A);
         else launch<float, KA, KB, 2, 4, 1, 4>(s, A);
@@ -535,14 +594,8 @@ template <int KA, int KB> Slices run(hipStream_t s, int arith, DenseArgs & A, fl
     }
     // K-slices: workgroups that share rows along K leave partial results, added by the next norm
     auto slice_k = [&](int want, int least) {            // least: fragments of a slice
-        A.ksplit = std::max(1, std::min({kMaxSlices, want, w.kf / least}));
-        if (A.ksplit == 1) return;
-        A.partial = ws;
-        A.slice = (size_t)T * w.n;
-        out.data = ws;
-        out.n = A.ksplit;
-        out.stride = A.slice;
-        out.N = w.n;
+        const int n = std::min({kMaxSlices, want, w.kf / least});
+        if (n > 1) slices(n);
     };
     const bool sliceable = KA == OUT_RESIDUAL && ws && (size_t)T * w.n <= kSliceFloats;
     if constexpr (KA != OUT_QUERY && KA != OUT_ACT_GATED) {        // products of one matrix
@@ -628,6 +681,7 @@ Slices dense(hipStream_t s, int arith, const DenseJob & job, int T, float * ws) 
         A.j.n_a = A.j.w.n;
         switch (job.a.kind) {
             case OUT_ACT_SWIGLU: run_groups<OUT_ACT_SWIGLU>(s, arith, A); break;
+            case OUT_ACT_CLAMPED: run_groups<OUT_ACT_CLAMPED>(s, arith, A); break;
             case OUT_EXPERT: run_groups<OUT_EXPERT>(s, arith, A); break;
             default: throw std::runtime_error("dense: this output of an expert product is not compiled");
         }
@@ -640,6 +694,8 @@ Slices dense(hipStream_t s, int arith, const DenseJob & job, int T, float * ws) 
     if (two) {
         if (job.a.kind == OUT_F32 && job.b.kind == OUT_ACT_RELU2) out = run<OUT_F32, OUT_ACT_RELU2>(s, arith, A, ws);
         else if (job.a.kind == OUT_F32 && job.b.kind == OUT_ACT_SWIGLU) out = run<OUT_F32, OUT_ACT_SWIGLU>(s, arith, A, ws);
+        else if (job.a.kind == OUT_F32 && job.b.kind == OUT_ACT_CLAMPED) out = run<OUT_F32, OUT_ACT_CLAMPED>(s, arith, A, ws);
+        else if (job.a.kind == OUT_F32 && job.b.kind == OUT_ACT) out = run<OUT_F32, OUT_ACT>(s, arith, A, ws);
         else throw std::runtime_error("dense: this pair of outputs is not compiled");
     } else {
         switch (job.a.kind) {
@@ -648,6 +704,8 @@ Slices dense(hipStream_t s, int arith, const DenseJob & job, int T, float * ws) 
             case OUT_ACT_GATED: out = run<OUT_ACT_GATED, -1>(s, arith, A, ws); break;
             case OUT_ACT_GEGLU: out = run<OUT_ACT_GEGLU, -1>(s, arith, A, ws); break;
             case OUT_ACT_SWIGLU: out = run<OUT_ACT_SWIGLU, -1>(s, arith, A, ws); break;
+            case OUT_ACT_CLAMPED: out = run<OUT_ACT_CLAMPED, -1>(s, arith, A, ws); break;
+            case OUT_F32_CAPPED: out = run<OUT_F32_CAPPED, -1>(s, arith, A, ws); break;
             case OUT_ACT_RELU2: out = run<OUT_ACT_RELU2, -1>(s, arith, A, ws); break;
             case OUT_ROTARY: out = run<OUT_ROTARY, -1>(s, arith, A, ws); break;
             case OUT_QUERY: out = run<OUT_QUERY, -1>(s, arith, A, ws); break;

@@ -84,18 +84,23 @@ struct LayerWeights {
 // input projections, of a parallel layer then the feed-forward's up rows), everything that adds to the stream another
 // (w_out: the mixer's output projection, of a parallel layer with the feed-forward's down projection beside it along K).
 // The feed-forward of a sequential layer: ff_in (gate and up rows in turn, tile by tile; with experts the router's
-// logits and the shared expert's gate before the shared expert's rows) and ff_out.
+// logits and the shared expert's gate before the shared expert's rows) and ff_out. Biases lie in their matrix's row order.
 struct StackLayer {
     struct Matrix { rk::DenseWeight w; DevBuf buf; };
     LayerSpec spec;
     DevBuf norm, norm2, scale_mix, scale_ff;
+    DevBuf hyper[2];                        // of the mixer and the feed-forward: what they read of the residual streams and write to them
     Matrix w_in, w_out, ff_in, ff_out;
+    DevBuf in_bias, ff_in_bias, ff_out_bias;
     int in_tiles = 0, in_rows = 0;          // row tiles and rows of w_in that belong to the mixer
     int route_tiles = 0;                    // row tiles of ff_in that belong to the router
     int kv_col = 0, gate_col = 0;           // columns of the input product: the latent, the head gates
-    DevBuf q_norm, kv_norm;
+    int k_col = 0, v_col = 0;               // ... of grouped attention's own keys and values
+    DevBuf q_norm, kv_norm, v_share;
     Matrix uq, uk, uv;                      // queries from their latent; per head: absorption and value up-projection
     DevBuf conv_w, conv_b, dt_bias, A_log, D, gate_norm;
+    Matrix low;                             // the delta rule's decays and gates from their inner widths (low_frags fragments each)
+    int low_frags = 0;
     int rotary = -1;                        // index of the layer's rotary table
     Matrix experts_in, experts_out;         // every expert's rows, gate and up in turn; down
 };
@@ -171,7 +176,7 @@ struct Vocab {
 enum ProfCat : int {
     PC_PACK = 0, PC_EMBED, PC_NORM, PC_QKV, PC_ROPE, PC_ATTN, PC_COMBINE, PC_OPROJ, PC_GATEUP, PC_SWIGLU,
     PC_DOWN, PC_HEAD, PC_SAMPLE, PC_ABSORB, PC_SCAN, PC_ROUTE, PC_EXPERTS_IN,
-    PC_EXPERTS_OUT, PC_SHARED, PC_COUNT
+    PC_EXPERTS_OUT, PC_SHARED, PC_LOW_RANK, PC_COUNT
 };
 
 class Engine {
@@ -298,6 +303,8 @@ private:
     void mix_latent(const StackLayer & L, const StackRun & run, int T);
     void mix_mamba(const StackLayer & L, const StackRun & run, int T);
     void mix_attention(const StackLayer & L, const StackRun & run, int T);
+    void mix_delta(const StackLayer & L, const StackRun & run, int T);
+    rk::SeqRuns step_runs() const;
     void attend(rk::StackAttn & at, int T);
     rk::Slices stack_feed_forward(const StackLayer & L, int T);
     rk::Slices stack_experts(const StackLayer & L, int T);
@@ -355,6 +362,7 @@ private:
     DevBuf recurrent_slab_;
     size_t recurrent_slot_floats_ = 0, conv_plane_floats_ = 0;
     DevBuf st_h_, st_proj_, st_cq_, st_q_, st_qa_, st_ol_, st_mix_, st_ff_, st_out_, st_partial_, st_xbc_, st_y_;
+    DevBuf st_first_, st_low_, st_decay_, st_chunks_;      // values of the first layer that mixes them; the delta rule's
     DevBuf st_embed_, st_rows_, st_route_, ex_sel_, ex_weight_, ex_slot_, ex_tiles_, ex_h_;
     int st_proj_ld_ = 0;
     struct BlockPlan { int heads, cols; size_t first, n; };    // attention blocks of the step for one number of query columns per token
@@ -362,7 +370,7 @@ private:
     std::vector<rk::AttnBlock> plan_blocks_;
     std::vector<rk::SeqRun> plan_runs_;
     std::vector<int32_t> plan_run_tok_;
-    int plan_max_run_ = 0, step_rows_ = 0;
+    int plan_max_run_ = 0, plan_min_run_ = 0, step_rows_ = 0;
     const rk::AttnBlock * d_blocks_ = nullptr;
     const rk::SeqRun * d_runs_ = nullptr;
     const int32_t * d_run_tok_ = nullptr;

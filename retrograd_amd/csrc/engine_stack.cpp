@@ -7,6 +7,7 @@
 #include <algorithm>
 #include <cmath>
 #include <cstring>
+#include <tuple>
 
 namespace retro {
 
@@ -16,6 +17,9 @@ void hip_check(hipError_t err, const char * what) {
     if (err != hipSuccess) throw std::runtime_error(std::string("HIP error in ") + what + ": " + hipGetErrorString(err));
 }
 
+constexpr float kGateSlope = 1.702f;           // of the clamped gated pair's sigmoid
+constexpr float kUnitEps = 1e-6f;              // under the root of the delta rule's unit vectors
+
 int up16(int n) { return (n + 15) / 16 * 16; }
 int up32(int n) { return (n + 31) / 32 * 32; }
 
@@ -24,7 +28,7 @@ class Loader {
 public:
     Loader(const SafetensorsFile & f, hipStream_t s) : file_(f), stream_(s) {}
 
-    void vector(const std::string & name, const std::vector<int64_t> & shape, DevBuf & out, float plus = 0.0f) {
+    std::vector<float> floats(const std::string & name, const std::vector<int64_t> & shape) {
         const StTensor & t = file_.require(name, shape);
         const size_t n = t.nbytes / (t.dtype == "F32" ? 4 : 2);
         std::vector<float> v(n);
@@ -40,9 +44,42 @@ public:
         } else {
             throw std::runtime_error("tensor " + name + " must be BF16 or F32");
         }
+        return v;
+    }
+    static void upload(const std::vector<float> & v, DevBuf & out) {
+        out.alloc(v.size() * 4);
+        if (!v.empty()) hip_check(hipMemcpy(out.ptr, v.data(), v.size() * 4, hipMemcpyHostToDevice), "hipMemcpy");
+    }
+    void vector(const std::string & name, const std::vector<int64_t> & shape, DevBuf & out, float plus = 0.0f) {
+        std::vector<float> v = floats(name, shape);
         for (float & x : v) x += plus;
-        out.alloc(n * 4);
-        hip_check(hipMemcpy(out.ptr, v.data(), n * 4, hipMemcpyHostToDevice), "hipMemcpy");
+        upload(v, out);
+    }
+    // Several tensors one behind the other.
+    void vectors(const std::vector<std::pair<std::string, std::vector<int64_t>>> & parts, DevBuf & out) {
+        std::vector<float> all;
+        for (const auto & p : parts) {
+            const std::vector<float> v = floats(p.first, p.second);
+            all.insert(all.end(), v.begin(), v.end());
+        }
+        upload(all, out);
+    }
+    // Biases of a matrix's rows, each tensor at its rows' places.
+    void biases(const StackLayer::Matrix & m, const std::vector<std::tuple<std::string, int, rk::PackMap>> & parts, DevBuf & out) {
+        std::vector<float> all((size_t)m.w.batch * m.w.tiles * 16, 0.0f);
+        for (const auto & p : parts) {
+            const rk::PackMap & at = std::get<2>(p);
+            const std::vector<float> v = floats(std::get<0>(p), {std::get<1>(p)});
+            for (int r = 0; r < (int)v.size(); ++r) all[(size_t)(at.at + r / at.run * at.step + r % at.run)] = v[(size_t)r];
+        }
+        upload(all, out);
+    }
+    // Rows of a matrix of `cols` columns.
+    int rows_of(const std::string & name, int cols) {
+        const StTensor * t = file_.find(name);
+        if (!t) throw std::runtime_error("model is missing tensor " + name);
+        if (t->shape.size() != 2 || t->shape[0] < 1 || t->shape[0] > (1 << 24) || t->shape[1] != cols) throw std::runtime_error("tensor " + name + " has an unexpected shape");
+        return (int)t->shape[0];
     }
     void shape(StackLayer::Matrix & m, int n, int kf, int batch = 1) {
         m.w.n = n;
@@ -68,11 +105,13 @@ public:
     }
     // A gate and an up matrix as row tiles in turn, from row tile tile0 on.
     void gated(const std::string & p, int rows, int cols, StackLayer::Matrix & m, int tile0 = 0, int b = 0) {
-        matrix(p + "gate", rows, cols, m, {tile0 * 16, 16, 32}, 0, b);
-        matrix(p + "up", rows, cols, m, {tile0 * 16 + 16, 16, 32}, 0, b);
+        matrix(p + "gate", rows, cols, m, gate_row(tile0), 0, b);
+        matrix(p + "up", rows, cols, m, up_row(tile0), 0, b);
     }
+    static rk::PackMap gate_row(int tile0 = 0) { return {tile0 * 16, 16, 32}; }
+    static rk::PackMap up_row(int tile0 = 0) { return {tile0 * 16 + 16, 16, 32}; }
     static int gated_rows(int ff) { return 2 * up16(ff); }
-    // The rows of `heads` heads, every head from a multiple of `padded` rows on, the columns of a rotated pair side by side.
+    // The rows of `heads` heads, every head from a multiple of `padded` rows on, the columns of a rotated pair (i and i + rotated / 2) side by side.
     void heads(const std::string & name, int heads, int dim, int padded, int rotated, int cols, StackLayer::Matrix & m, int head0) {
         const uint16_t * src = raw(name, heads * dim, cols);
         for (int h = 0; h < heads; ++h)
@@ -131,7 +170,7 @@ void Engine::load_stack(const std::string & path) {
     hip_check(hipMemcpy(tok_embd_.buf.ptr, emb.data, emb.nbytes, hipMemcpyHostToDevice), "hipMemcpy");
     tok_embd_.w.raw = tok_embd_.buf.as<uint8_t>();
     ld.shape(stack_head_, c.vocab, KE);
-    ld.matrix("embed", c.vocab, E, stack_head_);
+    ld.matrix(c.arch->own_head ? "head" : "embed", c.vocab, E, stack_head_);
     const float norm_plus = c.arch->norm_around_one ? 1.0f : 0.0f;
     ld.vector("final.norm", {E}, out_norm_, norm_plus);
 
@@ -143,6 +182,11 @@ void Engine::load_stack(const std::string & path) {
         const std::string p = "l" + std::to_string(l) + ".", m = p + "mix.";
         const bool parallel = c.arch->parallel;
         if (parallel && sp.moe.experts > 0) throw std::runtime_error("experts in parallel layers are not supported");
+        if (parallel && sp.mixer == Mixer::CHANNEL_DELTA) throw std::runtime_error("channel_delta in parallel layers is not supported");
+        for (int q = 0; q < (sp.has_ff() ? 2 : 1) && c.streams > 0; ++q) {
+            const std::string hc = p + (q == 0 ? "hc1." : "hc2.");
+            ld.vectors({{hc + "in", {c.streams}}, {hc + "out", {c.streams}}, {hc + "mix", {c.streams, c.streams}}}, L.hyper[q]);
+        }
         ld.vector(p + "norm1", {E}, L.norm, norm_plus);
         if (!parallel && sp.has_ff()) ld.vector(p + "norm2", {E}, L.norm2, norm_plus);
         if (c.arch->layer_scale) {
@@ -152,26 +196,38 @@ void Engine::load_stack(const std::string & path) {
         // input rows: the mixer's, in whole tiles, then a parallel feed-forward's
         const LatentSpec & a = sp.latent;
         const AttentionSpec & ga = sp.attention;
-        const int head_rows = 32 * rk::cache_frags(std::max(ga.dim, 1));
+        const rk::PairFrags head = ga.frags();
+        rk::DeltaShape & ds = L.spec.delta;
+        const bool own_values = sp.mixer == Mixer::ATTENTION && !c.arch->keys_are_values;
+        int beside = parallel ? sp.ff : 0;              // rows behind the mixer's that go elsewhere
         if (sp.mixer == Mixer::LATENT_ATTENTION) {
             const bool own = a.kv_from < 0;
             L.kv_col = up16(a.q_rank);
             L.gate_col = L.kv_col + (own ? up16(a.kv_rank) : 0);
             L.in_rows = L.gate_col + a.heads;
+        } else if (own_values) {
+            L.k_col = up16(ga.heads * ga.dim);
+            L.v_col = L.k_col + up16(ga.kv_heads * ga.dim);
+            L.in_rows = L.v_col + ga.kv_heads * ga.vdim;
         } else if (sp.mixer == Mixer::ATTENTION) {
-            L.in_rows = (ga.heads + ga.kv_heads) * head_rows;
+            L.in_rows = (ga.heads + ga.kv_heads) * head.k * 32;
+        } else if (sp.mixer == Mixer::CHANNEL_DELTA) {
+            ds.decay_rank = ld.rows_of(m + "a1", E);
+            ds.gate_rank = ld.rows_of(m + "g1", E);
+            L.low_frags = std::max(rk::frags_of(ds.decay_rank), rk::frags_of(ds.gate_rank));
+            L.in_rows = ds.channels() + ds.heads;
+            beside = L.low_frags * 32 + ds.gate_rank;
         } else {
             L.in_rows = sp.mamba.rows();
         }
         L.in_tiles = (L.in_rows + 15) / 16;
-        const int beside = parallel ? sp.ff : 0;
         ld.shape(L.w_in, beside > 0 ? L.in_tiles * 16 + beside : L.in_rows, KE);
-        if (beside > 0) ld.matrix(p + "mlp.up", beside, E, L.w_in, L.in_tiles * 16);
+        if (parallel && beside > 0) ld.matrix(p + "mlp.up", beside, E, L.w_in, L.in_tiles * 16);
         const int mix = sp.mix_width(), KM = rk::frags_of(mix);
-        ld.shape(L.w_out, E, KM + (beside > 0 ? rk::frags_of(beside) : 0));
-        if (sp.mixer == Mixer::ATTENTION) ld.from_heads(m + "o", E, ga.heads, ga.dim, head_rows, ga.rot.dims, L.w_out);
+        ld.shape(L.w_out, E, KM + (parallel && beside > 0 ? rk::frags_of(beside) : 0));
+        if (sp.mixer == Mixer::ATTENTION) ld.from_heads(m + "o", E, ga.heads, ga.vdim, head.v * 32, own_values ? 0 : ga.rot.dims, L.w_out);
         else ld.matrix(m + "o", E, mix, L.w_out);
-        if (beside > 0) ld.matrix(p + "mlp.down", E, beside, L.w_out, 0, KM * 32);
+        if (parallel && beside > 0) ld.matrix(p + "mlp.down", E, beside, L.w_out, 0, KM * 32);
         if (!parallel && sp.ff > 0) {
             if (rk::out_is_glu(c.arch->ff_act)) {
                 ld.shape(L.ff_in, Loader::gated_rows(sp.ff), KE);
@@ -182,15 +238,20 @@ void Engine::load_stack(const std::string & path) {
             }
             ld.shape(L.ff_out, E, rk::frags_of(sp.ff));
             ld.matrix(p + "mlp.down", E, sp.ff, L.ff_out);
+            if (c.arch->ff_bias) {
+                if (rk::out_is_glu(c.arch->ff_act)) ld.biases(L.ff_in, {{p + "mlp.gate.b", sp.ff, Loader::gate_row()}, {p + "mlp.up.b", sp.ff, Loader::up_row()}}, L.ff_in_bias);
+                else ld.biases(L.ff_in, {{p + "mlp.up.b", sp.ff, 0}}, L.ff_in_bias);
+                ld.biases(L.ff_out, {{p + "mlp.down.b", E, 0}}, L.ff_out_bias);
+            }
         } else if (sp.moe.experts > 0) {
             const MoeSpec & e = sp.moe;
             const std::string sh = p + "mlp.shared.";
-            const int route = e.experts + (e.shared_ff > 0 ? 1 : 0);
+            const int route = e.experts + (e.shared_ff > 0 && c.arch->shared_gate ? 1 : 0);
             L.route_tiles = up32(route) / 16;
             ld.shape(L.ff_in, e.shared_ff > 0 ? L.route_tiles * 16 + Loader::gated_rows(e.shared_ff) : route, KE);
             ld.matrix(p + "mlp.router", e.experts, E, L.ff_in);
             if (e.shared_ff > 0) {
-                ld.matrix(sh + "sg", 1, E, L.ff_in, e.experts);
+                if (c.arch->shared_gate) ld.matrix(sh + "sg", 1, E, L.ff_in, e.experts);
                 ld.gated(sh, e.shared_ff, E, L.ff_in, L.route_tiles);
                 ld.shape(L.ff_out, E, rk::frags_of(e.shared_ff));
                 ld.matrix(sh + "down", E, e.shared_ff, L.ff_out);
@@ -230,8 +291,19 @@ void Engine::load_stack(const std::string & path) {
             for (int h = 0; h < a.heads; ++h)
                 rk::dense_pack(stream_, uv + (size_t)h * a.vdim * a.kv_rank, a.vdim, a.kv_rank, a.kv_rank, 1, L.uv.buf.as<uint16_t>() + h * uv_head, L.uv.w.kf, 0, 0);
         } else if (sp.mixer == Mixer::ATTENTION) {
-            ld.heads(m + "q", ga.heads, ga.dim, head_rows, ga.rot.dims, E, L.w_in, 0);
-            ld.heads(m + "k", ga.kv_heads, ga.dim, head_rows, ga.rot.dims, E, L.w_in, ga.heads);
+            if (own_values) {
+                const int nq = ga.heads * ga.dim, nk = ga.kv_heads * ga.dim, nv = ga.kv_heads * ga.vdim;
+                ld.matrix(m + "q", nq, E, L.w_in);
+                ld.matrix(m + "k", nk, E, L.w_in, L.k_col);
+                ld.matrix(m + "v", nv, E, L.w_in, L.v_col);
+                ld.biases(L.w_in, {{m + "q.b", nq, 0}, {m + "k.b", nk, L.k_col}, {m + "v.b", nv, L.v_col}}, L.in_bias);
+                ld.vector(m + "q.norm", {nq}, L.q_norm);
+                ld.vector(m + "k.norm", {nk}, L.kv_norm);
+                if (ga.v_mix && !ga.v_first) ld.vector(m + "vmix", {}, L.v_share);
+            } else {
+                ld.heads(m + "q", ga.heads, ga.dim, head.k * 32, ga.rot.dims, E, L.w_in, 0);
+                ld.heads(m + "k", ga.kv_heads, ga.dim, head.k * 32, ga.rot.dims, E, L.w_in, ga.heads);
+            }
             for (size_t r = 0; r < rotary_.size(); ++r) if (rotary_[r].spec == ga.rot) L.rotary = (int)r;
             if (L.rotary < 0) {
                 L.rotary = (int)rotary_.size();
@@ -242,6 +314,21 @@ void Engine::load_stack(const std::string & path) {
                 t.freq.alloc(f.size() * sizeof(double));
                 if (!f.empty()) hip_check(hipMemcpy(t.freq.ptr, f.data(), t.freq.bytes, hipMemcpyHostToDevice), "hipMemcpy");
             }
+        } else if (sp.mixer == Mixer::CHANNEL_DELTA) {
+            const int at_a = L.in_tiles * 16, decays = ds.heads * ds.dim, gates = ds.inner();
+            ld.matrix(m + "q", ds.keys(), E, L.w_in);
+            ld.matrix(m + "k", ds.keys(), E, L.w_in, ds.keys());
+            ld.matrix(m + "v", ds.inner(), E, L.w_in, 2 * ds.keys());
+            ld.matrix(m + "b", ds.heads, E, L.w_in, ds.channels());
+            ld.matrix(m + "a1", ds.decay_rank, E, L.w_in, at_a);
+            ld.matrix(m + "g1", ds.gate_rank, E, L.w_in, at_a + L.low_frags * 32);
+            ld.shape(L.low, std::max(decays, gates), L.low_frags, 2);
+            ld.matrix(m + "a2", decays, ds.decay_rank, L.low, 0, 0, 0);
+            ld.matrix(m + "g2", gates, ds.gate_rank, L.low, 0, 0, 1);
+            ld.vectors({{m + "q.conv", {ds.keys(), ds.taps}}, {m + "k.conv", {ds.keys(), ds.taps}}, {m + "v.conv", {ds.inner(), ds.taps}}}, L.conv_w);
+            ld.vector(m + "dt_bias", {decays}, L.dt_bias);
+            ld.vector(m + "A_log", {ds.heads}, L.A_log);
+            ld.vector(m + "norm", {ds.vdim}, L.gate_norm);
         } else {
             const rk::MambaShape & s = sp.mamba;
             ld.matrix(m + "in", s.rows(), E, L.w_in);
@@ -300,7 +387,8 @@ void Engine::build_stack() {
             if (sp.latent.kv_from >= 0) R.pool = last[(size_t)sp.latent.kv_from];
             else pool(r, false, rk::cache_frags(sp.latent.kv_rank));
         } else if (sp.mixer == Mixer::ATTENTION) {
-            for (int v = 0; v < 2; ++v) pool(r, v != 0, sp.attention.kv_heads * rk::cache_frags(sp.attention.dim));
+            const rk::PairFrags f = sp.attention.frags();
+            for (int v = 0; v < 2; ++v) pool(r, v != 0, sp.attention.kv_heads * (v ? f.v : f.k));
         }
     }
     kv_slab_.alloc(total);
@@ -312,10 +400,12 @@ void Engine::build_stack() {
     size_t states = 0;
     for (StackRun & R : stack_runs_) {
         const LayerSpec & sp = c.layers[(size_t)R.layer];
-        if (sp.mixer != Mixer::MAMBA2) continue;
+        if (!sp.recurrent()) continue;
         const rk::MambaShape & s = sp.mamba;
-        R.state_slot = (size_t)s.heads * s.state * s.vdim;
-        R.conv_slot = (size_t)(s.taps - 1) * s.channels();
+        const rk::DeltaShape & d = sp.delta;
+        const bool delta = sp.mixer == Mixer::CHANNEL_DELTA;
+        R.state_slot = delta ? d.state_floats() : (size_t)s.heads * s.state * s.vdim;
+        R.conv_slot = delta ? (size_t)(d.taps - 1) * d.channels() : (size_t)(s.taps - 1) * s.channels();
         states += R.state_slot * n_slots;
         conv_plane_floats_ += R.conv_slot * n_slots;
         recurrent_slot_floats_ += R.state_slot + R.conv_slot;
@@ -343,8 +433,9 @@ void Engine::build_stack() {
         b.alloc(n);
         if (n) hip_check(hipMemsetAsync(b.ptr, 0, n, stream_), "hipMemsetAsync");
     };
-    size_t route = 0, pairs = 0, slots = 0, tiles = 0, expert_h = 0;
-    for (const LayerSpec & sp : c.layers) {
+    size_t route = 0, pairs = 0, slots = 0, tiles = 0, expert_h = 0, first = 0, low = 0, decay = 0, chunks = 0;
+    for (const StackLayer & L : stack_layers_) {
+        const LayerSpec & sp = L.spec;
         mix = std::max(mix, rk::frag_elems(B, rk::frags_of(sp.mix_width())));
         if (sp.ff > 0) ff = std::max(ff, rk::frag_elems(B, rk::frags_of(sp.ff)));
         if (sp.mixer == Mixer::LATENT_ATTENTION) {
@@ -354,7 +445,16 @@ void Engine::build_stack() {
             qa = std::max(qa, (size_t)B * a.heads * 32 * rk::cache_frags(a.kv_rank));
             ol = std::max(ol, rk::frag_elems(B, a.heads * rk::cache_frags(a.kv_rank)));
         } else if (sp.mixer == Mixer::ATTENTION) {
-            qa = std::max(qa, (size_t)B * sp.mix_width());
+            const AttentionSpec & a = sp.attention;
+            qa = std::max(qa, (size_t)B * a.heads * 32 * a.frags().k);
+            if (a.v_mix) first = std::max(first, (size_t)B * a.kv_heads * a.vdim);
+        } else if (sp.mixer == Mixer::CHANNEL_DELTA) {
+            const rk::DeltaShape & d = sp.delta;
+            xbc = std::max(xbc, (size_t)B * d.channels());
+            y = std::max(y, (size_t)B * d.inner());
+            low = std::max(low, rk::frag_elems(B, 2 * L.low_frags));
+            decay = std::max(decay, (size_t)B * 2 * up16(L.low.w.n));
+            chunks = std::max(chunks, rk::delta_chunk_floats(d, B, n_slots));
         } else {
             xbc = std::max(xbc, (size_t)B * sp.mamba.channels());
             y = std::max(y, (size_t)B * sp.mamba.inner());
@@ -372,7 +472,7 @@ void Engine::build_stack() {
         }
     }
     for (const StackLayer & L : stack_layers_)
-        if (L.spec.mixer != Mixer::ATTENTION) st_proj_ld_ = std::max(st_proj_ld_, L.in_tiles * 16);      // grouped attention's rows go to their places at once
+        if (L.spec.mixer != Mixer::ATTENTION || !c.arch->keys_are_values) st_proj_ld_ = std::max(st_proj_ld_, L.in_tiles * 16);      // grouped attention's rows go to their places at once
     for (RotaryTable & t : rotary_) t.table.alloc((size_t)B * t.spec.dims * 4);
     if (looped_) st_embed_.alloc((size_t)B * E * 4);
     if (route) zeroed(st_rows_, (size_t)B * rk::frags_of(E) * 32 * elem);
@@ -381,7 +481,11 @@ void Engine::build_stack() {
     ex_weight_.alloc(pairs * 4);
     ex_slot_.alloc(slots * 4);
     if (tiles) ex_tiles_.alloc((tiles + 1) * 16);           // the count behind the tiles
-    x_.alloc((size_t)B * E * 4);
+    x_.alloc((size_t)B * E * 4 * std::max(c.streams, 1));
+    st_first_.alloc(first * 4);
+    zeroed(st_low_, low * elem);
+    zeroed(st_decay_, decay * 4);
+    st_chunks_.alloc(chunks * 4);
     zeroed(st_h_, h * elem);
     zeroed(st_out_, h * elem);
     zeroed(st_proj_, (size_t)B * st_proj_ld_ * 4);
@@ -394,7 +498,7 @@ void Engine::build_stack() {
     zeroed(st_xbc_, xbc * 4);
     zeroed(st_y_, y * 4);
     zeroed(ex_h_, expert_h * elem);
-    mm_ws_.alloc((rk::dense_workspace_floats() + moe_ws_floats_) * 4);
+    mm_ws_.alloc((std::max(rk::dense_workspace_floats(), c.streams > 0 ? (size_t)B * E : 0) + moe_ws_floats_) * 4);
 }
 
 // ---- recurrent state of a slot --------------------------------------------------------------------
@@ -447,15 +551,16 @@ void Engine::plan_stack(const std::vector<RowView> & rows, const std::vector<std
     plan_blocks_.clear();
     plan_runs_.clear();
     plan_run_tok_.clear();
-    plan_max_run_ = 0;
+    plan_max_run_ = plan_min_run_ = 0;
     step_rows_ = (int)rows.size();
     int total = 0;
     for (const RowView & r : rows) total += (int)r.n;
     for (const LayerSpec & sp : stack_->layers) {
-        if (sp.mixer == Mixer::MAMBA2) continue;
+        if (sp.recurrent()) continue;
         const bool pair = sp.mixer == Mixer::ATTENTION;
-        const int H = pair ? sp.attention.heads / sp.attention.kv_heads : sp.latent.heads;
-        const int cols = rk::stack_block_cols(arith_, H, rk::cache_frags(pair ? sp.attention.dim : sp.latent.kv_rank), pair, total, (int)rows.size());
+        const int H = pair ? sp.attention.heads / sp.attention.kv_heads : sp.latent.heads, R = rk::cache_frags(std::max(sp.latent.kv_rank, 1));
+        const rk::PairFrags f = pair ? sp.attention.frags() : rk::PairFrags{R, R};
+        const int cols = rk::stack_block_cols(arith_, H, f.k, f.v, pair, total, (int)rows.size());
         if (std::any_of(block_plans_.begin(), block_plans_.end(), [&](const BlockPlan & b) { return b.heads == H && b.cols == cols; })) continue;
         BlockPlan plan{H, cols, plan_blocks_.size(), 0};
         for (size_t r = 0; r < rows.size(); ++r)
@@ -484,6 +589,7 @@ void Engine::plan_stack(const std::vector<RowView> & rows, const std::vector<std
         plan_runs_[k].start = (int32_t)plan_run_tok_.size();
         plan_runs_[k].n = (int32_t)toks[k].size();
         plan_max_run_ = std::max(plan_max_run_, plan_runs_[k].n);
+        plan_min_run_ = k == 0 ? plan_runs_[k].n : std::min(plan_min_run_, plan_runs_[k].n);
         plan_run_tok_.insert(plan_run_tok_.end(), toks[k].begin(), toks[k].end());
     }
 }
@@ -510,7 +616,7 @@ void Engine::stage_stack_plan(uint8_t * host, const uint8_t * device) {
 // Attention over the caches of `at`, its blocks and splits filled in here.
 void Engine::attend(rk::StackAttn & at, int T) {
     size_t pt = prof_begin(PC_ATTN);
-    const int per_token = at.H / at.G, cols = rk::stack_block_cols(arith_, per_token, at.kf, at.v_pool != nullptr, T, step_rows_);
+    const int per_token = at.H / at.G, cols = rk::stack_block_cols(arith_, per_token, at.kf, at.vf, at.v_pool != nullptr, T, step_rows_);
     const BlockPlan * plan = nullptr;
     for (const BlockPlan & b : block_plans_) if (b.heads == per_token && b.cols == cols) plan = &b;
     at.rows = d_stage_.as<rk::RowDesc>();
@@ -520,7 +626,7 @@ void Engine::attend(rk::StackAttn & at, int T) {
     at.table = table_.as<int32_t>();
     at.max_pages = max_pages_;
     at.splits = rk::stack_splits(arith_, at, step_max_resident_);
-    st_partial_.ensure(rk::stack_partial_floats(T, at.H, at.kf, at.splits) * 4);
+    st_partial_.ensure(rk::stack_partial_floats(T, at.H, at.vf, at.splits) * 4);
     at.partial_ml = st_partial_.as<float>();
     at.partial = at.partial_ml + (size_t)T * at.H * at.splits * 2;
     rk::stack_attention(stream_, arith_, at);
@@ -559,7 +665,7 @@ void Engine::mix_latent(const StackLayer & L, const StackRun & run, int T) {
     rk::dense(stream_, arith_, uk, T, ws);
     prof_end(PC_ABSORB, pt);
     rk::StackAttn at;
-    at.q = st_qa_.ptr; at.H = H; at.kf = R; at.window = a.window;
+    at.q = st_qa_.ptr; at.H = H; at.kf = at.vf = R; at.window = a.window;
     at.pool = pool;
     at.out = st_ol_.ptr; at.out_kf = H * R;
     attend(at, T);
@@ -581,7 +687,7 @@ void Engine::mix_mamba(const StackLayer & L, const StackRun & run, int T) {
     j.conv_w = L.conv_w.as<float>(); j.conv_b = L.conv_b.as<float>(); j.dt_bias = L.dt_bias.as<float>();
     j.A_log = L.A_log.as<float>(); j.D = L.D.as<float>(); j.norm_w = L.gate_norm.as<float>();
     j.eps = stack_->eps;
-    j.runs = d_runs_; j.n_runs = (int)plan_runs_.size(); j.max_run = plan_max_run_; j.run_tok = d_run_tok_;
+    j.runs = step_runs();
     j.conv_state = run.conv_state; j.conv_plane = conv_plane_floats_; j.state = run.state;
     j.xbc = st_xbc_.as<float>(); j.y = st_y_.as<float>();
     j.out = st_mix_.ptr; j.out_kf = rk::frags_of(L.spec.mix_width());
@@ -589,15 +695,66 @@ void Engine::mix_mamba(const StackLayer & L, const StackRun & run, int T) {
     prof_end(PC_SCAN, pt);
 }
 
-// Grouped attention: the input product has already left queries, keys and values in their places.
+rk::SeqRuns Engine::step_runs() const {
+    rk::SeqRuns r;
+    r.runs = d_runs_; r.n = (int)plan_runs_.size(); r.longest = plan_max_run_; r.shortest = plan_min_run_; r.tok = d_run_tok_;
+    return r;
+}
+
+// The input product has left queries, keys, values and write strengths as f32 rows, the inner columns of decays and gates as
+// activations.
+void Engine::mix_delta(const StackLayer & L, const StackRun & run, int T) {
+    const rk::DeltaShape & sh = L.spec.delta;
+    const int half = up16(L.low.w.n);
+    size_t pt = prof_begin(PC_LOW_RANK);
+    rk::DenseJob low;
+    low.w = L.low.w;
+    low.x = {st_low_.ptr, 2 * L.low_frags, L.low_frags};
+    low.a.kind = rk::OUT_F32; low.a.dst = st_decay_.ptr; low.a.ld = 2 * half; low.a.col_batch = half;
+    rk::dense(stream_, arith_, low, T, nullptr);
+    prof_end(PC_LOW_RANK, pt);
+    pt = prof_begin(PC_SCAN);
+    rk::DeltaJob j;
+    j.sh = sh;
+    j.proj = st_proj_.as<float>(); j.ld = st_proj_ld_;
+    j.decay = st_decay_.as<float>(); j.gate = j.decay + half; j.ld_low = 2 * half;
+    j.conv_w = L.conv_w.as<float>(); j.A_log = L.A_log.as<float>(); j.dt_bias = L.dt_bias.as<float>(); j.norm_w = L.gate_norm.as<float>();
+    j.eps = stack_->eps; j.unit_eps = kUnitEps;
+    j.runs = step_runs();
+    j.conv_state = run.conv_state; j.conv_plane = conv_plane_floats_; j.state = run.state;
+    j.qkv = st_xbc_.as<float>(); j.y = st_y_.as<float>(); j.chunks = st_chunks_.as<float>();
+    j.out = st_mix_.ptr; j.out_kf = rk::frags_of(L.spec.mix_width());
+    rk::delta_mix(stream_, arith_, j, T);
+    prof_end(PC_SCAN, pt);
+}
+
+// Grouped attention. Where the values are the keys the input product has already left queries, keys and values in their
+// places; own values come as f32 rows with queries and keys that are still to be normed.
 void Engine::mix_attention(const StackLayer & L, const StackRun & run, int T) {
     const AttentionSpec & a = L.spec.attention;
+    const rk::PairFrags f = a.frags();
+    void * keys = k_pool_[(size_t)run.pool].ptr, * values = v_pool_[(size_t)run.pool].ptr;
+    if (!stack_->arch->keys_are_values) {
+        const size_t pt = prof_begin(PC_ROPE);
+        const RotaryTable & t = rotary_[(size_t)L.rotary];
+        rk::HeadRows r;
+        r.proj = st_proj_.as<float>(); r.ld = st_proj_ld_;
+        r.H = a.heads; r.G = a.kv_heads; r.dim = a.dim; r.vdim = a.vdim; r.k_col = L.k_col; r.v_col = L.v_col;
+        r.q_w = L.q_norm.as<float>(); r.k_w = L.kv_norm.as<float>(); r.eps = stack_->eps;
+        r.pairs = t.spec.dims / 2; r.table = t.table.as<float>();
+        if (a.v_mix) r.first = st_first_.as<float>();
+        if (a.v_mix && !a.v_first) r.share = L.v_share.as<float>();
+        r.q = st_qa_.ptr; r.k_pool = keys; r.v_pool = values;
+        r.kf = f.k; r.vf = f.v; r.cell = pk_.cell;
+        rk::head_rows(stream_, arith_, r, T);
+        prof_end(PC_ROPE, pt);
+    }
     rk::StackAttn at;
-    at.q = st_qa_.ptr; at.H = a.heads; at.G = a.kv_heads; at.kf = rk::cache_frags(a.dim);
+    at.q = st_qa_.ptr; at.H = a.heads; at.G = a.kv_heads; at.kf = f.k; at.vf = f.v;
     at.window = a.window; at.chunk = a.chunk;
     at.scale = a.scale; at.softcap = a.softcap;
-    at.pool = k_pool_[(size_t)run.pool].ptr; at.v_pool = v_pool_[(size_t)run.pool].ptr;
-    at.out = st_mix_.ptr; at.out_kf = a.heads * at.kf;
+    at.pool = keys; at.v_pool = values;
+    at.out = st_mix_.ptr; at.out_kf = a.heads * f.v;
     attend(at, T);
 }
 
@@ -612,6 +769,8 @@ rk::Slices Engine::stack_feed_forward(const StackLayer & L, int T) {
     in.w = L.ff_in.w;
     in.x = {st_h_.ptr, KE, 0};
     in.a.kind = c.arch->ff_act; in.a.dst = st_ff_.ptr; in.a.ld = KF;
+    in.a.limit = L.spec.ff_limit; in.a.slope = kGateSlope;
+    in.bias = L.ff_in_bias.as<float>();
     rk::dense(stream_, arith_, in, T, ws);
     prof_end(PC_GATEUP, pt);
     pt = prof_begin(PC_DOWN);
@@ -619,7 +778,8 @@ rk::Slices Engine::stack_feed_forward(const StackLayer & L, int T) {
     out.w = L.ff_out.w;
     out.x = {st_ff_.ptr, KF, 0};
     out.kf1 = KF;
-    out.a.kind = rk::OUT_RESIDUAL; out.a.dst = x_.ptr; out.a.ld = E;
+    out.a.kind = rk::OUT_RESIDUAL; out.a.dst = c.streams > 0 ? nullptr : x_.ptr; out.a.ld = E;
+    out.bias = L.ff_out_bias.as<float>();
     const rk::Slices left = rk::dense(stream_, arith_, out, T, ws);
     prof_end(PC_DOWN, pt);
     return left;
@@ -637,15 +797,17 @@ rk::Slices Engine::stack_experts(const StackLayer & L, int T) {
     in.w = L.ff_in.w;
     in.x = {st_h_.ptr, KE, 0};
     in.split_tile = L.route_tiles;
-    in.n_a = e.experts + (e.shared_ff > 0 ? 1 : 0);
+    in.n_a = e.experts + (e.shared_ff > 0 && c.arch->shared_gate ? 1 : 0);
     in.a.kind = rk::OUT_F32; in.a.dst = route; in.a.ld = ld;
     in.b.kind = c.arch->expert_act; in.b.dst = st_ff_.ptr; in.b.ld = KS;
+    in.b.limit = e.shared_limit; in.b.slope = kGateSlope;
     rk::dense(stream_, arith_, in, T, ws);
     prof_end(PC_SHARED, pt);
     pt = prof_begin(PC_ROUTE);
     rk::ExpertRoute r;
     r.logits = route; r.ld = ld; r.experts = e.experts; r.top = e.top;
     r.block = rk::expert_block(arith_, T, e.top, e.experts);
+    r.groups = e.groups; r.keep = e.keep; r.over_all = c.arch->route_over_all; r.scale = e.scale;
     r.sel = ex_sel_.as<int32_t>(); r.weight = ex_weight_.as<float>(); r.slot_pair = ex_slot_.as<int32_t>();
     r.tiles = ex_tiles_.as<int32_t>();
     r.n_tiles = r.tiles + (ex_tiles_.bytes / 16 - 1) * 4;
@@ -661,6 +823,7 @@ rk::Slices Engine::stack_experts(const StackLayer & L, int T) {
     up.groups = &g;
     up.gather = true;
     up.a.kind = c.arch->expert_act; up.a.dst = ex_h_.ptr; up.a.ld = KX;
+    up.a.limit = e.limit; up.a.slope = kGateSlope;
     rk::dense(stream_, arith_, up, T, ws);
     prof_end(PC_EXPERTS_IN, pt);
     rk::Slices left;
@@ -670,8 +833,8 @@ rk::Slices Engine::stack_experts(const StackLayer & L, int T) {
         out.w = L.ff_out.w;
         out.x = {st_ff_.ptr, KS, 0};
         out.kf1 = KS;
-        out.a.kind = rk::OUT_RESIDUAL; out.a.dst = x_.ptr; out.a.ld = E;
-        out.token_gate = route + e.experts; out.ld_token_gate = ld;
+        out.a.kind = rk::OUT_RESIDUAL; out.a.dst = c.streams > 0 ? nullptr : x_.ptr; out.a.ld = E;
+        if (c.arch->shared_gate) { out.token_gate = route + e.experts; out.ld_token_gate = ld; }
         left = rk::dense(stream_, arith_, out, T, ws);
         prof_end(PC_SHARED, pt);
     }
@@ -695,9 +858,21 @@ void Engine::forward_stack(int T, int n_out) {
     const StackConfig & c = *stack_;
     const int E = c.width, KE = rk::frags_of(E);
     float * x = x_.as<float>(), * ws = mm_ws_.as<float>();
-    rk::Slices pending;
+    rk::Slices pending;                         // what the stream, or the streams by the weights `due`, have yet to take in
+    const float * due = nullptr;
+    rk::Streams streams;
+    streams.x = x; streams.n = c.streams; streams.stride = (size_t)cfg_.n_batch * E;
+    // the norm before a sublayer, which reads the streams by its weights `hyper`
+    auto norm = [&](const DevBuf & w, const DevBuf * hyper, const int32_t * rows, int n, void * act, const float * plus, void * act_rows) {
+        const size_t pt = prof_begin(rows ? PC_HEAD : PC_NORM);
+        if (c.streams > 0)
+            rk::streams_norm_act(stream_, arith_, streams, due, pending, hyper ? hyper->as<float>() : nullptr, w.as<float>(), E, c.eps, rows, n, act, KE, act_rows);
+        else
+            rk::norm_act(stream_, arith_, c.arch->norm, x, w.as<float>(), E, c.eps, rows, n, act, KE, pending, plus, act_rows);
+        prof_end(rows ? PC_HEAD : PC_NORM, pt);
+    };
     size_t pt = prof_begin(PC_EMBED);
-    rk::embed(stream_, tok_embd_.w, pk_.tok, T, x);
+    rk::embed_rows(stream_, (const uint16_t *)tok_embd_.w.raw, pk_.tok, E, c.embedding_scale, T, x, std::max(c.streams, 1), streams.stride);
     if (looped_) rk::copy_floats(stream_, x, st_embed_.as<float>(), (size_t)T * E);
     for (RotaryTable & t : rotary_)
         rk::rotary_table(stream_, t.freq.as<double>(), t.spec.dims / 2, t.spec.magnitude(), pk_.pos, T, t.table.as<float>());
@@ -711,32 +886,35 @@ void Engine::forward_stack(int T, int n_out) {
         const StackLayer & L = stack_layers_[(size_t)run.layer];
         const LayerSpec & sp = L.spec;
         const bool beside = c.arch->parallel && sp.ff > 0;
-        pt = prof_begin(PC_NORM);
-        rk::norm_act(stream_, arith_, c.arch->norm, x, L.norm.as<float>(), E, c.eps, nullptr, T, st_h_.ptr, KE, pending,
-                     run.add_embedding ? st_embed_.as<float>() : nullptr);
-        prof_end(PC_NORM, pt);
+        norm(L.norm, &L.hyper[0], nullptr, T, st_h_.ptr, run.add_embedding ? st_embed_.as<float>() : nullptr, nullptr);
         pt = prof_begin(PC_QKV);
         rk::DenseJob in;
         in.w = L.w_in.w;
         in.x = {st_h_.ptr, KE, 0};
         in.split_tile = L.in_tiles;
         in.n_a = L.in_rows;
-        if (sp.mixer == Mixer::ATTENTION) {
+        in.bias = L.in_bias.as<float>();
+        if (sp.mixer == Mixer::ATTENTION && c.arch->keys_are_values) {
             const AttentionSpec & a = sp.attention;
             const RotaryTable & t = rotary_[(size_t)L.rotary];
             in.a.kind = rk::OUT_ROTARY; in.a.dst = st_qa_.ptr;
-            in.a.rot.H = a.heads; in.a.rot.G = a.kv_heads; in.a.rot.kf = rk::cache_frags(a.dim); in.a.rot.pairs = t.spec.dims / 2;
+            in.a.rot.H = a.heads; in.a.rot.G = a.kv_heads; in.a.rot.kf = a.frags().k; in.a.rot.pairs = t.spec.dims / 2;
             in.a.rot.table = t.table.as<float>();
             in.a.rot.k_pool = k_pool_[(size_t)run.pool].ptr; in.a.rot.v_pool = v_pool_[(size_t)run.pool].ptr;
             in.a.rot.cell = pk_.cell;
         } else {
             in.a.kind = rk::OUT_F32; in.a.dst = st_proj_.ptr; in.a.ld = st_proj_ld_;
         }
-        in.b.kind = c.arch->ff_act; in.b.dst = st_ff_.ptr; in.b.ld = rk::frags_of(std::max(sp.ff, 1));
+        if (sp.mixer == Mixer::CHANNEL_DELTA) {
+            in.b.kind = rk::OUT_ACT; in.b.dst = st_low_.ptr; in.b.ld = 2 * L.low_frags;
+        } else {
+            in.b.kind = c.arch->ff_act; in.b.dst = st_ff_.ptr; in.b.ld = rk::frags_of(std::max(sp.ff, 1));
+        }
         rk::dense(stream_, arith_, in, T, ws);
         prof_end(PC_QKV, pt);
         if (sp.mixer == Mixer::LATENT_ATTENTION) mix_latent(L, run, T);
         else if (sp.mixer == Mixer::ATTENTION) mix_attention(L, run, T);
+        else if (sp.mixer == Mixer::CHANNEL_DELTA) mix_delta(L, run, T);
         else mix_mamba(L, run, T);
         const int out_cat = c.arch->parallel ? PC_DOWN : PC_OPROJ, KM = rk::frags_of(sp.mix_width());
         pt = prof_begin(out_cat);
@@ -749,30 +927,34 @@ void Engine::forward_stack(int T, int n_out) {
             out.x2 = {st_ff_.ptr, rk::frags_of(sp.ff), 0};
             out.scale2 = L.scale_ff.as<float>();
         }
-        out.a.kind = rk::OUT_RESIDUAL; out.a.dst = x; out.a.ld = E;
+        out.a.kind = rk::OUT_RESIDUAL; out.a.dst = c.streams > 0 ? nullptr : x; out.a.ld = E;
         pending = rk::dense(stream_, arith_, out, T, ws);
+        due = L.hyper[0].as<float>();
         prof_end(out_cat, pt);
         if (!c.arch->parallel && sp.has_ff()) {
-            pt = prof_begin(PC_NORM);
-            rk::norm_act(stream_, arith_, c.arch->norm, x, L.norm2.as<float>(), E, c.eps, nullptr, T, st_h_.ptr, KE, pending, nullptr,
-                         sp.moe.experts > 0 ? st_rows_.ptr : nullptr);
-            prof_end(PC_NORM, pt);
+            norm(L.norm2, &L.hyper[1], nullptr, T, st_h_.ptr, nullptr, sp.moe.experts > 0 ? st_rows_.ptr : nullptr);
             pending = stack_feed_forward(L, T);
+            due = L.hyper[1].as<float>();
         }
         if (keep_residual_) {
             float * kept = kept_residual_.as<float>() + r * (size_t)cfg_.n_batch * E;
-            rk::copy_floats(stream_, x, kept, (size_t)T * E);
-            rk::add_slices(stream_, kept, E, T, pending);
+            if (c.streams > 0) {
+                rk::streams_sum(stream_, streams, due, pending, E, T, kept);
+            } else {
+                rk::copy_floats(stream_, x, kept, (size_t)T * E);
+                rk::add_slices(stream_, kept, E, T, pending);
+            }
         }
     }
     if (n_out > 0) {
         logits_.ensure((size_t)n_out * c.vocab * 4);
+        norm(out_norm_, nullptr, pk_.out_tok, n_out, st_out_.ptr, nullptr, nullptr);
         pt = prof_begin(PC_HEAD);
-        rk::norm_act(stream_, arith_, c.arch->norm, x, out_norm_.as<float>(), E, c.eps, pk_.out_tok, n_out, st_out_.ptr, KE, pending);
         rk::DenseJob head;
         head.w = stack_head_.w;
         head.x = {st_out_.ptr, KE, 0};
-        head.a.kind = rk::OUT_F32; head.a.dst = logits_.ptr; head.a.ld = c.vocab;
+        head.a.kind = c.logit_softcap > 0.0f ? rk::OUT_F32_CAPPED : rk::OUT_F32; head.a.dst = logits_.ptr; head.a.ld = c.vocab;
+        head.a.limit = c.logit_softcap;
         rk::dense(stream_, arith_, head, n_out, ws);
         prof_end(PC_HEAD, pt);
     }

@@ -1,11 +1,47 @@
 // Routing of mixture-of-experts feed-forwards of layer-stack models: the choice of experts per token and the order in
 // which the expert products (dense.hip) take the chosen pairs. Logits arrive in f32; the weights of a token are the
-// softmax over its chosen logits.
+// softmax over its chosen logits, or over all its logits.
 #include "stack_dev.hpp"
 
 namespace rk {
 
 namespace {
+
+// Logits of experts outside the kept groups become -infinity: a group's rank is the number of groups whose largest logit
+// comes before its own (ties to the lower group).
+template <int N> __device__ __forceinline__ void keep_groups(const ExpertRoute & r, int lane, float (&v)[N]) {
+    const int size = r.experts / r.groups;
+    float best[N];                              // of the lane's experts' groups
+    int own[N], rank[N];
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+        own[i] = (lane + 64 * i) / size;
+        best[i] = -INFINITY;
+        rank[i] = 0;
+    }
+    auto best_of = [&](int g) {
+        float m = -INFINITY;
+#pragma unroll
+        for (int i = 0; i < N; ++i) m = own[i] == g ? fmaxf(m, v[i]) : m;
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) m = fmaxf(m, __shfl_xor(m, o, 64));
+        return m;
+    };
+#pragma unroll 1
+    for (int g = 0; g < r.groups; ++g) {
+        const float m = best_of(g);
+#pragma unroll
+        for (int i = 0; i < N; ++i) best[i] = own[i] == g ? m : best[i];
+    }
+#pragma unroll 1
+    for (int g = 0; g < r.groups; ++g) {
+        const float m = best_of(g);
+#pragma unroll
+        for (int i = 0; i < N; ++i) rank[i] += m > best[i] || (m == best[i] && g < own[i]) ? 1 : 0;
+    }
+#pragma unroll
+    for (int i = 0; i < N; ++i) if (rank[i] >= r.keep) v[i] = -INFINITY;
+}
 
 // One wave: the experts of token t, lane l holding the logits of experts l + 64 i. Every expert's rank is the number of
 // logits before its own; rank j < top is choice j.
@@ -20,6 +56,14 @@ template <int N> __device__ __forceinline__ void choose(const ExpertRoute & r, i
         rank[i] = 0;
         largest = fmaxf(largest, v[i]);
     }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) largest = fmaxf(largest, __shfl_xor(largest, o, 64));
+    float sum = 0.0f;
+    if (r.over_all) {
+#pragma unroll
+        for (int i = 0; i < N; ++i) sum += expf(v[i] - largest);
+    }
+    if (r.groups > 1) keep_groups<N>(r, lane, v);
 #pragma unroll 8
     for (int o = 0; o < 64; ++o) {
 #pragma unroll
@@ -29,20 +73,18 @@ template <int N> __device__ __forceinline__ void choose(const ExpertRoute & r, i
             for (int i = 0; i < N; ++i) rank[i] += other > v[i] || (other == v[i] && (j < i || (j == i && o < lane))) ? 1 : 0;
         }
     }
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) largest = fmaxf(largest, __shfl_xor(largest, o, 64));
-    float p[N], sum = 0.0f;
+    float p[N];
 #pragma unroll
     for (int i = 0; i < N; ++i) {
         p[i] = rank[i] < r.top ? expf(v[i] - largest) : 0.0f;
-        sum += p[i];
+        if (!r.over_all) sum += p[i];
     }
     sum = wave_sum(sum);
 #pragma unroll
     for (int i = 0; i < N; ++i)
         if (rank[i] < r.top) {
             sel[rank[i]] = lane + 64 * i;
-            r.weight[(size_t)t * r.top + rank[i]] = p[i] / sum;
+            r.weight[(size_t)t * r.top + rank[i]] = p[i] / sum * r.scale;
         }
 }
 __device__ __forceinline__ void choose_any(const ExpertRoute & r, int t, int lane, int32_t * sel) {
@@ -108,7 +150,8 @@ int expert_max_tiles(int T, int top, int experts, int block) {
 
 void expert_route(hipStream_t s, const ExpertRoute & r, int T) {
     if (T <= 0) return;
-    if (r.experts > MAX_EXPERTS || r.top > MAX_TOP || r.top > r.experts) throw std::runtime_error("expert routing: too many experts");
+    if (r.experts > MAX_EXPERTS || r.top > MAX_TOP || r.top > r.experts || r.groups < 1 || r.experts % r.groups != 0 || r.keep < 1
+            || (r.groups > 1 && (int64_t)r.keep * (r.experts / r.groups) < r.top)) throw std::runtime_error("expert routing: unsupported sizes");
     if (T <= ONE_LAUNCH_TOKENS) {
         hipLaunchKernelGGL(k_expert_route, dim3(1), dim3(1024), 0, s, r, T);
     } else {

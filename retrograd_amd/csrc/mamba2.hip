@@ -1,65 +1,11 @@
-// The Mamba-2 mixer between its two projections: short causal convolution with SiLU over x, B and C, the state-space
-// recurrence per head, and the gated grouped RMS norm. Everything here is f32 in both arithmetics; only the rows that
+// The Mamba-2 mixer between its two projections: short causal convolution with SiLU over x, B and C (short_conv.hip), the
+// state-space recurrence per head, and the gated grouped RMS norm. Everything here is f32 in both arithmetics; only the rows that
 // leave for the output projection take the arithmetic's activation type.
 #include "stack_dev.hpp"
 
 namespace rk {
 
 namespace {
-
-__device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
-__device__ __forceinline__ float softplus_f(float z) { return fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); }
-
-constexpr int kConvTokens = 16;       // tokens of a run one workgroup convolves
-
-// xbc[t][c] = silu(bias + sum over the taps); inputs before the run come from the slot's current plane, and the run's
-// last taps - 1 inputs go to the other plane (the workgroups of a run read the one while the other is written).
-template <int TAPS>
-__global__ __launch_bounds__(256) void k_mamba_conv(MambaJob j) {
-    const MambaShape sh = j.sh;
-    const int C = sh.channels(), c = blockIdx.y * 256 + threadIdx.x, K = TAPS > 0 ? TAPS : sh.taps;
-    const SeqRun run = j.runs[blockIdx.z];
-    const int first = blockIdx.x * kConvTokens;
-    if (c >= C || first >= run.n) return;
-    const int plane = (run.flags >> 1) & 1;
-    const bool fresh = run.flags & 1;
-    const float * old_in = j.conv_state + (size_t)plane * j.conv_plane + (size_t)run.slot * (K - 1) * C;
-    float * new_in = j.conv_state + (size_t)(1 - plane) * j.conv_plane + (size_t)run.slot * (K - 1) * C;
-    const int off = sh.inner() + c;
-    auto input = [&](int i) -> float {          // input of the run's token i; i < 0: what the slot remembers
-        if (i >= 0) return j.proj[(size_t)j.run_tok[run.start + i] * j.ld + off];
-        return fresh ? 0.0f : old_in[(size_t)(i + K - 1) * C + c];
-    };
-    const float * w = j.conv_w + (size_t)c * K;
-    const float bias = j.conv_b[c];
-    const int last = min(first + kConvTokens, run.n);
-    if constexpr (TAPS > 0) {                   // the window and the taps in registers
-        float win[TAPS], tap[TAPS];
-#pragma unroll
-        for (int k = 0; k < TAPS; ++k) {
-            tap[k] = w[k];
-            win[k] = k > 0 ? input(first - TAPS + k) : 0.0f;
-        }
-        for (int i = first; i < last; ++i) {
-            const int t = j.run_tok[run.start + i];
-            float v = 0.0f;
-#pragma unroll
-            for (int k = 0; k + 1 < TAPS; ++k) win[k] = win[k + 1];
-            win[TAPS - 1] = j.proj[(size_t)t * j.ld + off];
-#pragma unroll
-            for (int k = 0; k < TAPS; ++k) v += tap[k] * win[k];
-            j.xbc[(size_t)t * C + c] = silu_f(v + bias);
-        }
-    } else {
-        for (int i = first; i < last; ++i) {
-            float v = 0.0f;
-            for (int k = 0; k < K; ++k) v += w[k] * input(i - (K - 1) + k);
-            j.xbc[(size_t)j.run_tok[run.start + i] * C + c] = silu_f(v + bias);
-        }
-    }
-    if (last == run.n)
-        for (int k = 0; k < K - 1; ++k) new_in[(size_t)k * C + c] = input(run.n - (K - 1) + k);
-}
 
 constexpr int kScanP = 64;            // columns of the state one workgroup holds
 constexpr int kScanTokens = 8;        // tokens staged at once
@@ -72,7 +18,7 @@ __global__ __launch_bounds__(256) void k_mamba_scan(MambaJob j) {
     const int N = sh.state, P = sh.vdim, C = sh.channels();
     const int h = blockIdx.x, g = h / (sh.heads / sh.groups);
     const int p = blockIdx.y * kScanP + (threadIdx.x & 63), q = threadIdx.x >> 6;
-    const SeqRun run = j.runs[blockIdx.z];
+    const SeqRun run = j.runs.runs[blockIdx.z];
     float * sB = sm, * sC = sB + kScanTokens * N, * part = sC + kScanTokens * N;      // part [tokens][4][64]
     __shared__ float s_dt[kScanTokens], s_decay[kScanTokens];
     const bool mine = p < P;
@@ -89,18 +35,18 @@ __global__ __launch_bounds__(256) void k_mamba_scan(MambaJob j) {
         __syncthreads();
         for (int i = threadIdx.x; i < cnt * N; i += 256) {
             const int tk = i / N, n = i % N;
-            const float * row = j.xbc + (size_t)j.run_tok[run.start + base + tk] * C + sh.inner() + g * N + n;
+            const float * row = j.xbc + (size_t)j.runs.tok[run.start + base + tk] * C + sh.inner() + g * N + n;
             sB[i] = row[0];
             sC[i] = row[(size_t)sh.groups * N];
         }
         if ((int)threadIdx.x < cnt) {
-            const float dt = softplus_f(j.proj[(size_t)j.run_tok[run.start + base + threadIdx.x] * j.ld + sh.inner() + C + h] + bias);
+            const float dt = softplus_f(j.proj[(size_t)j.runs.tok[run.start + base + threadIdx.x] * j.ld + sh.inner() + C + h] + bias);
             s_dt[threadIdx.x] = dt;
             s_decay[threadIdx.x] = expf(-a * dt);
         }
         __syncthreads();
         for (int tk = 0; tk < cnt; ++tk) {
-            const float x = mine ? j.xbc[(size_t)j.run_tok[run.start + base + tk] * C + h * P + p] : 0.0f;
+            const float x = mine ? j.xbc[(size_t)j.runs.tok[run.start + base + tk] * C + h * P + p] : 0.0f;
             const float dx = s_dt[tk] * x, dec = s_decay[tk];
             float y = 0.0f;
 #pragma unroll
@@ -119,7 +65,7 @@ __global__ __launch_bounds__(256) void k_mamba_scan(MambaJob j) {
             float y = 0.0f;
 #pragma unroll
             for (int i = 0; i < 4; ++i) y += part[(tk * 4 + i) * 64 + (threadIdx.x & 63)];
-            const int t = j.run_tok[run.start + base + tk];
+            const int t = j.runs.tok[run.start + base + tk];
             j.y[(size_t)t * sh.inner() + h * P + p] = y + D * j.xbc[(size_t)t * C + h * P + p];
         }
     }
@@ -147,7 +93,7 @@ __global__ __launch_bounds__(256) void k_mamba_chunks(MambaJob j) {
     const MambaShape sh = j.sh;
     const int N = sh.state, Np = (N + 15) / 16 * 16, P = sh.vdim, C = sh.channels(), LB = Np + 4;
     const int h = blockIdx.x, g = h / (sh.heads / sh.groups), p0 = blockIdx.y * kChunkP;
-    const SeqRun run = j.runs[blockIdx.z];
+    const SeqRun run = j.runs.runs[blockIdx.z];
     const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, r16 = lane & 15, kg = lane >> 4;
     float * sB = sm, * sC = sB + kChunk * LB, * sX = sC + kChunk * LB, * sM = sX + kChunk * 36, * sS = sM + kChunk * 68;
     __shared__ double s_l[kChunk];
@@ -171,7 +117,7 @@ __global__ __launch_bounds__(256) void k_mamba_chunks(MambaJob j) {
     f4 nB[VEC ? RB : 1], nC[VEC ? RB : 1], nX[VEC ? RX : 1];
     float n_dt = 0.0f;
     int n_tok = 0;
-    auto token = [&](int base, int tk) { return j.run_tok[run.start + min(base + tk, run.n - 1)]; };
+    auto token = [&](int base, int tk) { return j.runs.tok[run.start + min(base + tk, run.n - 1)]; };
     auto fetch = [&](int base) {                // of the chunk at base into registers; nothing past the run's end is used
         if (w == 0) {
             n_tok = token(base, lane);
@@ -374,31 +320,31 @@ __global__ __launch_bounds__(256) void k_mamba_gate_norm(MambaJob j) {
 }  // namespace
 
 void mamba_mix(hipStream_t s, int arith, const MambaJob & j, int T) {
-    if (j.n_runs <= 0 || T <= 0) return;
+    if (j.runs.n <= 0 || T <= 0) return;
     const MambaShape & sh = j.sh;
     if (sh.state > 512) throw std::runtime_error("mamba2: at most 512 state rows per head");
-    const dim3 conv((unsigned)((j.max_run + kConvTokens - 1) / kConvTokens), (unsigned)((sh.channels() + 255) / 256), (unsigned)j.n_runs);
-    switch (sh.taps) {
-        case 2: hipLaunchKernelGGL(k_mamba_conv<2>, conv, dim3(256), 0, s, j); break;
-        case 3: hipLaunchKernelGGL(k_mamba_conv<3>, conv, dim3(256), 0, s, j); break;
-        case 4: hipLaunchKernelGGL(k_mamba_conv<4>, conv, dim3(256), 0, s, j); break;
-        default: hipLaunchKernelGGL(k_mamba_conv<0>, conv, dim3(256), 0, s, j);
-    }
-    check_launch("mamba_conv");
-    if (j.max_run >= kChunk / 2 && sh.state <= kChunkN) {
+    ShortConv conv;
+    conv.runs = j.runs;
+    conv.channels = sh.channels(); conv.taps = sh.taps;
+    conv.in = j.proj + sh.inner(); conv.ld = j.ld;
+    conv.w = j.conv_w; conv.b = j.conv_b;
+    conv.state = j.conv_state; conv.plane = j.conv_plane;
+    conv.out = j.xbc;
+    short_conv(s, conv);
+    if (j.runs.longest >= kChunk / 2 && sh.state <= kChunkN) {
         const int Np = (sh.state + 15) / 16 * 16;
         const size_t lds = ((size_t)2 * kChunk * (Np + 4) + kChunk * 36 + kChunk * 68 + (size_t)Np * 36) * 4;
         constexpr int most = (2 * kChunk * (kChunkN + 4) + kChunk * 36 + kChunk * 68 + kChunkN * 36) * 4;
         static const bool allowed = hipFuncSetAttribute((const void *)k_mamba_chunks<true>, hipFuncAttributeMaxDynamicSharedMemorySize, most) == hipSuccess
                                  && hipFuncSetAttribute((const void *)k_mamba_chunks<false>, hipFuncAttributeMaxDynamicSharedMemorySize, most) == hipSuccess;
         if (!allowed) throw std::runtime_error("mamba2: a chunk does not fit the LDS");
-        const dim3 grid((unsigned)sh.heads, (unsigned)((sh.vdim + kChunkP - 1) / kChunkP), (unsigned)j.n_runs);
+        const dim3 grid((unsigned)sh.heads, (unsigned)((sh.vdim + kChunkP - 1) / kChunkP), (unsigned)j.runs.n);
         // every row starts at a multiple of four floats
         if (sh.vdim % 4 == 0 && sh.state % 4 == 0) hipLaunchKernelGGL(k_mamba_chunks<true>, grid, dim3(256), lds, s, j);
         else hipLaunchKernelGGL(k_mamba_chunks<false>, grid, dim3(256), lds, s, j);
         check_launch("mamba_chunks");
     } else {
-        const dim3 grid((unsigned)sh.heads, (unsigned)((sh.vdim + kScanP - 1) / kScanP), (unsigned)j.n_runs);
+        const dim3 grid((unsigned)sh.heads, (unsigned)((sh.vdim + kScanP - 1) / kScanP), (unsigned)j.runs.n);
         const size_t lds = (size_t)(2 * kScanTokens * sh.state + kScanTokens * 256) * 4;
         const int npt = (sh.state + 3) / 4;
         if (npt <= 8) hipLaunchKernelGGL(k_mamba_scan<8>, grid, dim3(256), lds, s, j);

@@ -28,19 +28,36 @@ inline const GgufArch * find_gguf_arch(const std::string & name) {
 // What an architecture fixes about its layers. Parallel layers: x <- x + scale1 * mixer(n(x)) + scale2 * ff(n(x)), one
 // norm for both; otherwise x <- x + mixer(n1(x)), then x <- x + ff(n2(x)). The norm's kind and whether its weights are
 // stored as differences from one; the activations (DenseOut kinds) of the feed-forward and of experts; element-wise
-// layer scales or none; what positions of grouped attention a mask of some size leaves.
+// layer scales or none; whether a dense feed-forward has biases, a shared expert a gate per token, and the head its own matrix.
+// Grouped attention: what positions a mask of some size leaves; whether the values are the keys before rotation or a
+// projection of their own, with biases on all three and queries and keys normed over all their heads; how a head's columns
+// pair up for rotation (i with i + dims / 2, or neighbours) and what stretching the rotation means.
 enum class Mask { WINDOW, CHUNK };
-struct StackArch { const char * name; int norm; bool norm_around_one; bool parallel; int ff_act, expert_act; bool layer_scale; Mask mask; };
+enum class Stretch { RAMP, BANDS };
+enum class Pairs { HALVES, NEIGHBOURS };
+struct StackArch {
+    const char * name;
+    int norm;
+    bool norm_around_one, parallel;
+    int ff_act, expert_act;
+    bool layer_scale, ff_bias, shared_gate, own_head;
+    Mask mask;
+    bool keys_are_values;
+    Pairs pairs;
+    Stretch stretch;
+    bool route_over_all;         // an expert's weight is the softmax over all experts, not over the chosen ones
+};
 inline const StackArch * find_stack_arch(const std::string & name) {
     static const StackArch known[] = {
-        {"Dibosun", rk::NORM_LAYER, false, true, rk::OUT_ACT_RELU2, -1, true, Mask::WINDOW},
-        {"Pomisun", rk::NORM_RMS, true, false, rk::OUT_ACT_GEGLU, rk::OUT_ACT_SWIGLU, false, Mask::CHUNK},
+        {"Dibosun", rk::NORM_LAYER, false, true, rk::OUT_ACT_RELU2, -1, true, false, true, false, Mask::WINDOW, true, Pairs::HALVES, Stretch::RAMP, false},
+        {"Pomisun", rk::NORM_RMS, true, false, rk::OUT_ACT_GEGLU, rk::OUT_ACT_SWIGLU, false, false, true, false, Mask::CHUNK, true, Pairs::HALVES, Stretch::RAMP, false},
+        {"Vifanex", rk::NORM_RMS, false, false, rk::OUT_ACT_CLAMPED, rk::OUT_ACT_CLAMPED, false, true, false, true, Mask::WINDOW, false, Pairs::NEIGHBOURS, Stretch::BANDS, true},
     };
     for (const StackArch & a : known) if (name == a.name) return &a;
     return nullptr;
 }
 
-enum class Mixer { LATENT_ATTENTION, MAMBA2, ATTENTION };
+enum class Mixer { LATENT_ATTENTION, MAMBA2, ATTENTION, CHANNEL_DELTA };
 
 struct LatentSpec {
     int heads = 0, dim = 0, vdim = 0, q_rank = 0, kv_rank = 0;
@@ -49,13 +66,15 @@ struct LatentSpec {
     float scale = 1.0f;
 };
 
-// Rotary positions on the first `dims` columns of a head, optionally stretched (YaRN): frequencies that turn fewer than
-// `slow` times within the original length are divided by the factor, those above `fast` kept, a ramp in between.
+// Rotary positions on the first `dims` columns of a head, optionally stretched: frequencies that turn fewer than `slow` times
+// within the original length are divided by the factor, those above `fast` kept. In between a ramp over the index of the
+// pair, which also lengthens the rotated vectors (RAMP, as in YaRN), or one over the number of turns (BANDS, as in Llama 3.1).
 struct RotarySpec {
     int dims = 0;
     double base = 10000.0, factor = 1.0, original = 0.0, fast = 0.0, slow = 0.0;      // original 0: not stretched
+    Stretch stretch = Stretch::RAMP;
     bool operator==(const RotarySpec & o) const {
-        return dims == o.dims && base == o.base && factor == o.factor && original == o.original && fast == o.fast && slow == o.slow;
+        return dims == o.dims && stretch == o.stretch && base == o.base && factor == o.factor && original == o.original && fast == o.fast && slow == o.slow;
     }
     // Radians per position of the dims / 2 pairs.
     std::vector<double> frequencies() const {
@@ -67,36 +86,56 @@ struct RotarySpec {
         for (size_t i = 0; i < f.size(); ++i) {
             f[i] = std::pow(base, -2.0 * (double)i / dims);
             if (original <= 0.0) continue;
+            if (stretch == Stretch::BANDS) {
+                const double turns = original * f[i] / (2.0 * pi);
+                const double keep = turns > fast ? 1.0 : turns < slow ? 0.0 : fast > slow ? (turns - slow) / (fast - slow) : 1.0;
+                f[i] = keep * f[i] + (1.0 - keep) * f[i] / factor;
+                continue;
+            }
             const double ramp = std::min(std::max(((double)i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
             f[i] = f[i] / factor * ramp + f[i] * (1.0 - ramp);
         }
         return f;
     }
-    double magnitude() const { return original > 0.0 ? 0.1 * std::log(factor) + 1.0 : 1.0; }      // of cosines and sines
+    double magnitude() const { return original > 0.0 && stretch == Stretch::RAMP ? 0.1 * std::log(factor) + 1.0 : 1.0; }      // of cosines and sines
 };
 
-// Grouped attention whose values are its keys before rotation.
+// Grouped attention. Layers that mix their values take a share of those of the first such layer (of the same token).
 struct AttentionSpec {
-    int heads = 0, kv_heads = 0, dim = 0;
+    int heads = 0, kv_heads = 0, dim = 0, vdim = 0;
+    bool v_mix = false, v_first = false;
+    rk::PairFrags frags() const { return dim == vdim ? rk::PairFrags{rk::cache_frags(dim), rk::cache_frags(dim)} : rk::pair_frags(dim, vdim); }
     int window = 0, chunk = 0;   // positions seen: the last `window`, or those of the same chunk (0: no bound)
     float scale = 1.0f, softcap = 0.0f;
     RotarySpec rot;
 };
 
-// Experts of a feed-forward: every token takes `top` of them, and the shared one (ff 0: none) behind a gate per token.
-struct MoeSpec { int experts = 0, top = 0, ff = 0, shared_ff = 0; };
+// Experts of a feed-forward: every token takes `top` of them, out of the `keep` best of `groups` groups of neighbours, and
+// the shared one (ff 0: none). The limits are those of clamped activations.
+struct MoeSpec {
+    int experts = 0, top = 0, ff = 0, shared_ff = 0, groups = 1, keep = 1;
+    float limit = 0.0f, shared_limit = 0.0f, scale = 1.0f;
+};
 
 struct LayerSpec {
     Mixer mixer = Mixer::LATENT_ATTENTION;
     LatentSpec latent;
     rk::MambaShape mamba;
     AttentionSpec attention;
+    rk::DeltaShape delta;
     int ff = 0;                  // of a dense feed-forward; 0 and no experts: no feed-forward
+    float ff_limit = 0.0f;
     MoeSpec moe;
     bool has_ff() const { return ff > 0 || moe.experts > 0; }
-    // Columns a mixer hands to its output projection (a head of grouped attention padded as its cache rows are).
+    bool recurrent() const { return mixer == Mixer::MAMBA2 || mixer == Mixer::CHANNEL_DELTA; }
+    // Columns a mixer hands to its output projection (a head of grouped attention padded as its cached values are).
     int mix_width() const {
-        return mixer == Mixer::MAMBA2 ? mamba.inner() : mixer == Mixer::ATTENTION ? attention.heads * 32 * rk::cache_frags(attention.dim) : latent.heads * latent.vdim;
+        switch (mixer) {
+            case Mixer::MAMBA2: return mamba.inner();
+            case Mixer::CHANNEL_DELTA: return delta.inner();
+            case Mixer::ATTENTION: return attention.heads * 32 * attention.frags().v;
+            default: return latent.heads * latent.vdim;
+        }
     }
 };
 
@@ -107,10 +146,12 @@ struct StackConfig {
     const StackArch * arch = nullptr;
     int width = 0, vocab = 0;
     float eps = 0.0f;
+    float embedding_scale = 1.0f, logit_softcap = 0.0f;      // 0: none
+    int streams = 0;             // residual streams of hyper-connections (0: a plain residual sum)
     std::vector<LayerSpec> layers;
     std::vector<LayerRun> runs;
     bool recurrent() const {
-        for (const LayerSpec & l : layers) if (l.mixer == Mixer::MAMBA2) return true;
+        for (const LayerSpec & l : layers) if (l.recurrent()) return true;
         return false;
     }
 
@@ -133,6 +174,12 @@ struct StackConfig {
         c.width = size(v, "width");
         c.vocab = size(v, "vocab");
         c.eps = (float)number(need(v, "norm"), "eps");
+        if (present(v, "embedding") && present(need(v, "embedding"), "scale")) c.embedding_scale = (float)number(need(v, "embedding"), "scale");
+        if (present(v, "logit_softcap")) c.logit_softcap = (float)number(v, "logit_softcap");
+        if (!(c.logit_softcap >= 0.0f)) throw std::runtime_error("config.json: 'logit_softcap' must not be negative");
+        if (present(v, "streams")) c.streams = size(v, "streams");
+        if (c.streams > rk::MAX_STREAMS || (c.streams > 0 && (c.arch->parallel || c.arch->norm != rk::NORM_RMS || present(v, "loop"))))
+            throw std::runtime_error("config.json: 'streams' of sequential layers over RMS norms, without a loop, " + std::to_string(rk::MAX_STREAMS) + " at most");
         for (const JsonValue & l : need(v, "layers").items) c.layers.push_back(layer(*c.arch, l, c.layers));
         const int n = (int)c.layers.size();
         if (n < 1 || n > 4096) throw std::runtime_error("config.json: 'layers' must list 1 to 4096 layers");
@@ -172,8 +219,15 @@ private:
         return m && m->kind != JsonValue::NUL;
     }
     static bool positive(double v) { return v > 0.0 && std::isfinite(v); }
-    static RotarySpec rotary(const JsonValue & v, int dim) {
+    static float limit(const StackArch & arch, int act, const JsonValue & v) {
+        if (act != rk::OUT_ACT_CLAMPED) return 0.0f;
+        const double l = number(v, "limit");
+        if (!(l > 0.0)) throw std::runtime_error("config.json: 'limit' must be positive");
+        return (float)l;
+    }
+    static RotarySpec rotary(const StackArch & arch, const JsonValue & v, int dim) {
         RotarySpec r;
+        r.stretch = arch.stretch;
         r.dims = size(v, "dims", 0);
         r.base = number(v, "base");
         if (r.dims > dim || r.dims % 2 != 0) throw std::runtime_error("config.json: 'rot.dims' must be even and within a head");
@@ -182,8 +236,8 @@ private:
             const JsonValue & s = need(v, "scaling");
             r.factor = number(s, "factor");
             r.original = number(s, "original");
-            r.fast = number(s, "fast");
-            r.slow = number(s, "slow");
+            r.fast = number(s, arch.stretch == Stretch::BANDS ? "high" : "fast");
+            r.slow = number(s, arch.stretch == Stretch::BANDS ? "low" : "slow");
             if (!positive(r.factor) || !positive(r.original) || !positive(r.fast) || !positive(r.slow))
                 throw std::runtime_error("config.json: 'rot.scaling' must hold positive numbers");
         }
@@ -231,10 +285,29 @@ private:
             if (present(m, "softcap")) a.softcap = (float)number(m, "softcap");
             if (present(m, "mask") && present(need(m, "mask"), "size")) (arch.mask == Mask::CHUNK ? a.chunk : a.window) = size(need(m, "mask"), "size");
             if (a.heads % a.kv_heads != 0) throw std::runtime_error("attention: heads must be a multiple of kv_heads");
-            if (size(m, "vdim") != a.dim) throw std::runtime_error("attention: the values are the keys, so vdim must be dim");
-            if (a.dim > 1024) throw std::runtime_error("attention: heads above 1024 columns are not supported");
+            a.vdim = size(m, "vdim");
+            if (arch.keys_are_values && a.vdim != a.dim) throw std::runtime_error("attention: the values are the keys, so vdim must be dim");
+            if (a.dim > 1024 || a.vdim > 1024) throw std::runtime_error("attention: heads above 1024 columns are not supported");
+            if (!arch.keys_are_values && present(m, "v_mix")) a.v_mix = need(m, "v_mix").b;
+            a.v_first = a.v_mix;
+            for (const LayerSpec & b : before)
+                if (b.mixer == Mixer::ATTENTION && b.attention.v_mix) {
+                    a.v_first = false;
+                    if (a.v_mix && b.attention.kv_heads * b.attention.vdim != a.kv_heads * a.vdim)
+                        throw std::runtime_error("attention: layers that mix their values must have equally many");
+                }
             if (!(a.softcap >= 0.0f)) throw std::runtime_error("attention: softcap must not be negative");
-            a.rot = rotary(need(m, "rot"), a.dim);
+            if (arch.keys_are_values || present(m, "rot")) a.rot = rotary(arch, need(m, "rot"), a.dim);
+        } else if (type == "channel_delta") {
+            l.mixer = Mixer::CHANNEL_DELTA;
+            rk::DeltaShape & s = l.delta;
+            s.heads = size(m, "heads");
+            s.kv_heads = size(m, "kv_heads");
+            s.dim = size(m, "dim");
+            s.vdim = size(m, "vdim");
+            s.taps = size(m, "conv");
+            if (s.heads % s.kv_heads != 0) throw std::runtime_error("channel_delta: heads must be a multiple of kv_heads");
+            if (s.dim > 512 || s.vdim > 4096) throw std::runtime_error("channel_delta: at most 512 key and 4096 value channels per head are supported");
         } else {
             throw std::runtime_error("config.json: unknown layer type '" + type + "'");
         }
@@ -243,12 +316,24 @@ private:
             const std::string kind = need(f, "kind").text;
             if (kind == "dense") {
                 l.ff = size(f, "ff");
+                l.ff_limit = limit(arch, arch.ff_act, f);
             } else if (kind == "moe" && arch.expert_act >= 0) {
                 const JsonValue & r = need(f, "router");
                 l.moe.experts = size(r, "experts");
                 l.moe.top = size(r, "top");
                 l.moe.ff = size(need(f, "expert"), "ff");
-                if (present(f, "shared")) l.moe.shared_ff = size(need(f, "shared"), "ff");
+                l.moe.limit = limit(arch, arch.expert_act, need(f, "expert"));
+                if (present(f, "shared")) {
+                    l.moe.shared_ff = size(need(f, "shared"), "ff");
+                    l.moe.shared_limit = limit(arch, arch.expert_act, need(f, "shared"));
+                }
+                if (present(r, "scale")) l.moe.scale = (float)number(r, "scale");
+                if (present(r, "groups")) {
+                    l.moe.groups = size(need(r, "groups"), "count");
+                    l.moe.keep = size(need(r, "groups"), "keep");
+                    if (l.moe.experts % l.moe.groups != 0 || l.moe.keep > l.moe.groups || l.moe.keep * (l.moe.experts / l.moe.groups) < l.moe.top)
+                        throw std::runtime_error("moe: 'groups' must be equal parts of the experts, of which those kept hold at least 'top'");
+                }
                 if (l.moe.top > l.moe.experts) throw std::runtime_error("moe: 'top' exceeds 'experts'");
                 if (l.moe.experts > rk::MAX_EXPERTS || l.moe.top > rk::MAX_TOP) throw std::runtime_error("moe: more experts than are supported");
             } else {

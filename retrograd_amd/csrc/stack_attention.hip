@@ -2,7 +2,8 @@
 // Latent: keys and values of every head are up-projections of one cached latent per token, so a query is absorbed into
 // the latent space first (q' = W_uk^T q) and every head attends over the same cached rows, which are keys and values at
 // once. The attended latents leave as activations for the value up-projection.
-// Grouped: a cache of keys and one of values, each with a part per key/value head, and optionally soft-capped scores.
+// Grouped: a cache of keys and one of values, each with a part per key/value head, of one width or of two, and optionally
+// soft-capped scores.
 // Either sees all earlier positions, a sliding window of them, or those of the token's own chunk.
 #include "stack_dev.hpp"
 
@@ -78,6 +79,91 @@ __global__ __launch_bounds__(256) void k_latent_norms(LatentNorms a) {
     }
 }
 
+template <int ARITH, typename EL> __device__ __forceinline__ void store_el8(EL * dst, const float (&v)[8]) {
+    if constexpr (ARITH == ARITH_16) {
+        union { __half h[8]; u4 w; } p;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) p.h[i] = sat_half(v[i]);
+        *(u4 *)dst = p.w;
+    } else {
+        *(f4 *)dst = f4{v[0], v[1], v[2], v[3]};
+        *(f4 *)(dst + 4) = f4{v[4], v[5], v[6], v[7]};
+    }
+}
+
+// One workgroup per token: the squares of all queries and all keys, then every head in groups of eight columns.
+template <int ARITH>
+__global__ __launch_bounds__(256) void k_head_rows(HeadRows a) {
+    using EL = typename std::conditional<ARITH == ARITH_16, __half, float>::type;
+    __shared__ float scratch[16];
+    const int t = blockIdx.x;
+    const float * row = a.proj + (size_t)t * a.ld;
+    auto squares = [&](const float * x, int n) {       // rows start at multiples of four columns
+        float q = 0.0f;
+        const int whole = n / 4 * 4;
+        for (int k = 4 * (int)threadIdx.x; k < whole; k += 1024) {
+            const f4 v = *(const f4 *)(x + k);
+            q += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+        }
+        for (int k = whole + (int)threadIdx.x; k < n; k += 256) q += x[k] * x[k];
+        return 1.0f / sqrtf(block_sum(q, scratch) / (float)n + a.eps);
+    };
+    const float inv_q = squares(row + a.q_col, a.H * a.dim), inv_k = squares(row + a.k_col, a.G * a.dim);
+    auto load = [](const float * x, int n, bool aligned, float (&o)[8]) {      // n columns are left
+        if (aligned && n >= 8) {
+            const f4 u = *(const f4 *)x, v = *(const f4 *)(x + 4);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) { o[i] = u[i]; o[4 + i] = v[i]; }
+        } else {
+#pragma unroll
+            for (int i = 0; i < 8; ++i) o[i] = i < n ? x[i] : 0.0f;
+        }
+    };
+    const int per_k = a.kf * 4, per_v = a.vf * 4;       // groups of a head
+    const bool even = a.dim % 4 == 0, even_v = a.vdim % 4 == 0;
+    const int cell = a.cell[t];
+    EL * k_page = (EL *)a.k_pool + (size_t)(cell / PAGE) * cache_page_elems(a.kf * a.G);
+    EL * v_page = (EL *)a.v_pool + (size_t)(cell / PAGE) * cache_page_elems(a.vf * a.G);
+    for (int i = threadIdx.x; i < (a.H + a.G) * per_k; i += 256) {
+        const int head = i / per_k, c = (i - head * per_k) * 8;
+        const bool query = head < a.H;
+        const int h = query ? head : head - a.H, left = a.dim - c;
+        float v[8], w[8];
+        load(row + (query ? a.q_col : a.k_col) + h * a.dim + c, left, even, v);
+        load((query ? a.q_w : a.k_w) + h * a.dim + c, left, even, w);
+        const float inv = query ? inv_q : inv_k;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] = v[e] * inv * w[e];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int pair = c / 2 + e;
+            if (pair >= a.pairs) continue;
+            const float2 cs = *(const float2 *)(a.table + 2 * ((size_t)t * a.pairs + pair));
+            const float x = v[2 * e], y = v[2 * e + 1];
+            v[2 * e] = x * cs.x - y * cs.y;
+            v[2 * e + 1] = y * cs.x + x * cs.y;
+        }
+        if (query) store_el8<ARITH>((EL *)a.q + ((size_t)t * a.H + h) * (a.kf * 32) + c, v);
+        else store_el8<ARITH>(k_page + cache_at(cell % PAGE, h * a.kf * 32 + c), v);
+    }
+    const float share = a.share ? *a.share : 0.0f;
+    for (int i = threadIdx.x; i < a.G * per_v; i += 256) {
+        const int h = i / per_v, c = (i - h * per_v) * 8, left = a.vdim - c;
+        float v[8];
+        load(row + a.v_col + h * a.vdim + c, left, even_v, v);
+        if (a.first) {
+            float * f = a.first + (size_t)t * a.G * a.vdim + h * a.vdim + c;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                if (e >= left) break;
+                if (a.share) v[e] = (1.0f - share) * v[e] + share * f[e];
+                else f[e] = v[e];
+            }
+        }
+        store_el8<ARITH>(v_page + cache_at(cell % PAGE, h * a.vf * 32 + c), v);
+    }
+}
+
 // First position a token at `pos` sees.
 __device__ __forceinline__ int low_key(const StackAttn & a, int kv_begin, int pos) {
     return max(kv_begin, a.chunk > 0 ? pos - pos % a.chunk : a.window > 0 ? pos - a.window + 1 : 0);
@@ -88,14 +174,15 @@ template <int ARITH>
 __global__ __launch_bounds__(256) void k_stack_attention_any(StackAttn a) {
     using EL = typename std::conditional<ARITH == ARITH_16, __half, float>::type;
     extern __shared__ float sm[];
-    const int R = a.kf * 32, HG = a.H / a.G, kv_head = blockIdx.y;
+    const int R = a.kf * 32, V = a.vf * 32, HG = a.H / a.G, kv_head = blockIdx.y;
     float * q = sm, * p = sm + R;             // [R], [256]
     __shared__ float scratch[16];
     const AttnBlock blk = a.blocks[blockIdx.x];
     const RowDesc row = a.rows[blk.row];
     const int n_cols = row.n * HG;
-    const size_t page_elems = cache_page_elems(a.kf * a.G), head_at = cache_page_elems(a.kf * kv_head);
-    const EL * keys = (const EL *)a.pool + head_at, * values = (const EL *)(a.v_pool ? a.v_pool : a.pool) + head_at;
+    const size_t page_elems = cache_page_elems(a.kf * a.G), v_page_elems = cache_page_elems(a.vf * a.G);
+    const EL * keys = (const EL *)a.pool + cache_page_elems(a.kf * kv_head);
+    const EL * values = (const EL *)(a.v_pool ? a.v_pool : a.pool) + cache_page_elems(a.vf * kv_head);
     constexpr float LOG2E = 1.4426950408889634f;
     for (int c = blk.col0; c < min(blk.col0 + a.block_cols, n_cols); ++c) {
         const int tok = c / HG, h = kv_head * HG + c % HG, t = row.tok_off + tok, pos = row.pos0 + tok;
@@ -141,12 +228,12 @@ __global__ __launch_bounds__(256) void k_stack_attention_any(StackAttn a) {
             for (int k = 0; k < n; ++k) {
                 const int kk = base + k;
                 const int pg = a.table[(size_t)row.slot * a.max_pages + kk / PAGE];
-                const EL * page = values + (size_t)pg * page_elems;
+                const EL * page = values + (size_t)pg * v_page_elems;
                 const float pk = p[k];
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
                     const int col = threadIdx.x + 256 * i;
-                    if (col < R) acc[i] += pk * el_float<EL>(page[cache_at(kk % PAGE, col)]);
+                    if (col < V) acc[i] += pk * el_float<EL>(page[cache_at(kk % PAGE, col)]);
                 }
             }
         }
@@ -154,8 +241,8 @@ __global__ __launch_bounds__(256) void k_stack_attention_any(StackAttn a) {
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int col = threadIdx.x + 256 * i;
-            if (col >= R) break;
-            const size_t at = frag_at(t, h * R + col, a.out_kf);
+            if (col >= V) break;
+            const size_t at = frag_at(t, h * V + col, a.out_kf);
             if constexpr (ARITH == ARITH_16) ((uint16_t *)a.out)[at] = bf16_bits(acc[i] * inv);
             else ((float *)a.out)[at] = acc[i] * inv;
         }
@@ -165,21 +252,22 @@ __global__ __launch_bounds__(256) void k_stack_attention_any(StackAttn a) {
 typedef __fp16 q4 __attribute__((ext_vector_type(4)));
 typedef __attribute__((address_space(3))) q4 lds_q4;
 
-// Matrix-core form over f16 cache rows of KF fragments (per head). A workgroup serves CT * WC * 16 query columns of one
+// Matrix-core form over f16 cache rows of KF fragments (per head; values of VF). A workgroup serves CT * WC * 16 query columns of one
 // key/value head (blockIdx.z); WC waves share a page (staged once into LDS, double buffered, by direct-to-LDS loads), WK
 // such groups take pages in turn and merge at the end. Scores S^T = K q^T and outputs O^T = V^T P^T read pages of one
 // layout: the second product's operand is its transpose, which the LDS transpose read delivers, so rows that are keys
 // and values at once (KV false) are staged once; KV: a page of keys, then the page of values. With several splits
 // (blockIdx.y) every one leaves an unnormalised partial result.
-template <int KF, int CT, int WC, int WK, bool KV>
+template <int KF, int VF, int CT, int WC, int WK, bool KV>
 __global__ __launch_bounds__(64 * WC * WK) __attribute__((amdgpu_waves_per_eu(2, 2)))
 void k_stack_attention(StackAttn a) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
     __shared__ float merge_ml[WC][CT][2][64];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int wc = wave % WC, wk = wave / WC, g = lane >> 4;
-    constexpr int AHEAD = KF >= 4 ? 6 : 2 * KF;
-    constexpr int kf = KF, head_bytes = KF * 2048, page_bytes = (KV ? 2 : 1) * head_bytes;      // of a staged page
+    static_assert(KV || KF == VF);
+    constexpr int AHEAD = KF >= 4 ? 6 : 2 * KF, AHEAD_V = VF >= 4 ? 6 : 2 * VF;
+    constexpr int kf = KF, head_bytes = KF * 2048, value_bytes = VF * 2048, page_bytes = head_bytes + (KV ? value_bytes : 0);      // of a staged page
     constexpr int PIECES = page_bytes / 1024;
     const AttnBlock blk = a.blocks[blockIdx.x];
     const RowDesc row = a.rows[blk.row];
@@ -203,7 +291,7 @@ void k_stack_attention(StackAttn a) {
         const int id = __builtin_amdgcn_readfirstlane(((const __attribute__((address_space(4))) int32_t *)table)[__builtin_amdgcn_readfirstlane(page)]);
         const size_t at = KV ? ((size_t)id * a.G + kv_head) * head_bytes : (size_t)id * head_bytes;
         const uint8_t * src = (const uint8_t *)a.pool + at;
-        const uint8_t * src_v = KV ? (const uint8_t *)a.v_pool + at - head_bytes : src;
+        const uint8_t * src_v = KV ? (const uint8_t *)a.v_pool + ((size_t)id * a.G + kv_head) * value_bytes - head_bytes : src;
         for (int ch = wc; ch < PIECES; ch += WC)
             lds_dma16((ch < 2 * kf ? src : src_v) + ch * 1024, (uint32_t)lane * 16, __builtin_amdgcn_readfirstlane(to + (uint32_t)(b * page_bytes + ch * 1024)));
     };
@@ -231,14 +319,14 @@ void k_stack_attention(StackAttn a) {
     constexpr float LOG2E = 1.4426950408889634f;
     const float cap_out = KV ? a.softcap * LOG2E : 0.0f;
     const float score_in = KV ? (a.softcap > 0.0f ? 2.0f * LOG2E * a.scale / a.softcap : a.scale * LOG2E) : 1.0f;
-    f4 acc[CT][2 * KF];
+    f4 acc[CT][2 * VF];
     float m[CT], l[CT];
 #pragma unroll
     for (int c = 0; c < CT; ++c) {
         m[c] = -INFINITY;
         l[c] = 0.0f;
 #pragma unroll
-        for (int d = 0; d < 2 * KF; ++d) acc[c][d] = f4{0, 0, 0, 0};
+        for (int d = 0; d < 2 * VF; ++d) acc[c][d] = f4{0, 0, 0, 0};
     }
     const int idx = lane & 15;
     const int tr_lane = ((((idx >> 1) & 1) * 16 + 4 * g + (idx >> 2)) * 8 + (idx & 1) * 4) * 2;       // bytes into a 1 KiB piece
@@ -321,7 +409,7 @@ void k_stack_attention(StackAttn a) {
                 const float f = exp2f(m[c] - base);
                 l[c] *= f;
 #pragma unroll
-                for (int d = 0; d < 2 * KF; ++d) acc[c][d] *= f;
+                for (int d = 0; d < 2 * VF; ++d) acc[c][d] *= f;
                 m[c] = m2;
             }
 #pragma unroll
@@ -334,7 +422,7 @@ void k_stack_attention(StackAttn a) {
                 }
         }
 #pragma unroll
-        for (int d = 0; d < 2 * KF; ++d) {
+        for (int d = 0; d < 2 * VF; ++d) {
             const uint8_t * v0 = cur + (KV ? head_bytes : 0) + (d >> 1) * 2048 + (d & 1) * 512 + tr_lane;
             union { q4 half[2]; h8 all; } v;
             v.half[0] = __builtin_amdgcn_ds_read_tr16_b64_v4f16((lds_q4 *)(v0));
@@ -342,13 +430,13 @@ void k_stack_attention(StackAttn a) {
 #pragma unroll
             for (int c = 0; c < CT; ++c) acc[c][d] = __builtin_amdgcn_mfma_f32_16x16x32_f16(v.all, p[c], acc[c][d], 0, 0, 0);
         }
-        __builtin_amdgcn_sched_group_barrier(0x100, 2 * AHEAD, 1);
+        __builtin_amdgcn_sched_group_barrier(0x100, 2 * AHEAD_V, 1);
 #pragma unroll
-        for (int i = 0; i < 2 * KF - AHEAD; ++i) {
+        for (int i = 0; i < 2 * VF - AHEAD_V; ++i) {
             __builtin_amdgcn_sched_group_barrier(0x008, CT, 1);
             __builtin_amdgcn_sched_group_barrier(0x100, 2, 1);
         }
-        __builtin_amdgcn_sched_group_barrier(0x008, AHEAD * CT, 1);
+        __builtin_amdgcn_sched_group_barrier(0x008, AHEAD_V * CT, 1);
     }
 #pragma unroll
     for (int c = 0; c < CT; ++c) {
@@ -358,12 +446,12 @@ void k_stack_attention(StackAttn a) {
     if constexpr (WK > 1) {       // the groups' results, one after the other, into the first group's
         static_assert(WK == 2 && CT == 1);
         __syncthreads();
-        f4 * park = (f4 *)lds + (size_t)wc * 2 * kf * 64;      // 2 KiB per fragment and wave: within the pages
+        f4 * park = (f4 *)lds + (size_t)wc * 2 * VF * 64;      // 2 KiB per fragment and wave: within the pages
         if (wk == 1) {
             merge_ml[wc][0][0][lane] = m[0];
             merge_ml[wc][0][1][lane] = l[0];
 #pragma unroll
-            for (int d = 0; d < 2 * KF; ++d) park[d * 64 + lane] = acc[0][d];
+            for (int d = 0; d < 2 * VF; ++d) park[d * 64 + lane] = acc[0][d];
         }
         __syncthreads();
         if (wk == 1) return;
@@ -373,7 +461,7 @@ void k_stack_attention(StackAttn a) {
         l[0] = l[0] * f0 + lo2 * f1;
         m[0] = m2;
 #pragma unroll
-        for (int d = 0; d < 2 * KF; ++d) acc[0][d] = acc[0][d] * f0 + park[d * 64 + lane] * f1;
+        for (int d = 0; d < 2 * VF; ++d) acc[0][d] = acc[0][d] * f0 + park[d * 64 + lane] * f1;
     }
 #pragma unroll
     for (int c = 0; c < CT; ++c) {
@@ -382,10 +470,10 @@ void k_stack_attention(StackAttn a) {
         if (a.splits > 1) {
             const size_t at = ((size_t)t * a.H + h) * a.splits + sp;
             if (g == 0) *(float2 *)(a.partial_ml + 2 * at) = make_float2(m[c], l[c]);
-            __half * o = (__half *)a.partial + at * (size_t)(kf * 32);
+            __half * o = (__half *)a.partial + at * (size_t)(VF * 32);
             const float inv = l[c] > 0.0f ? 1.0f / l[c] : 0.0f;      // a split may lie outside this column's window
 #pragma unroll
-            for (int d = 0; d < 2 * KF; ++d) {
+            for (int d = 0; d < 2 * VF; ++d) {
                 union { __half h[4]; uint2 u; } w;
 #pragma unroll
                 for (int i = 0; i < 4; ++i) w.h[i] = __float2half_rn(acc[c][d][i] * inv);
@@ -394,12 +482,12 @@ void k_stack_attention(StackAttn a) {
         } else {
             const float inv = 1.0f / l[c];
 #pragma unroll
-            for (int d = 0; d < 2 * KF; ++d) {
+            for (int d = 0; d < 2 * VF; ++d) {
                 const f4 v = acc[c][d] * inv;
                 uint2 u;
                 u.x = (uint32_t)bf16_bits(v[0]) | ((uint32_t)bf16_bits(v[1]) << 16);
                 u.y = (uint32_t)bf16_bits(v[2]) | ((uint32_t)bf16_bits(v[3]) << 16);
-                *(uint2 *)((uint16_t *)a.out + frag_at(t, h * kf * 32 + d * 16 + 4 * g, a.out_kf)) = u;
+                *(uint2 *)((uint16_t *)a.out + frag_at(t, h * VF * 32 + d * 16 + 4 * g, a.out_kf)) = u;
             }
         }
     }
@@ -408,7 +496,7 @@ void k_stack_attention(StackAttn a) {
 // Merges the splits of one query column (at most 32), each a mean in f16 with its maximum and sum: a wave per column,
 // lane i the weight of split i; eight latent columns per lane and pass, the splits' values requested four at a time.
 __global__ __launch_bounds__(64) void k_stack_combine(StackAttn a) {
-    const int R = a.kf * 32, t = blockIdx.x / a.H, h = blockIdx.x - t * a.H, lane = threadIdx.x;
+    const int R = a.vf * 32, t = blockIdx.x / a.H, h = blockIdx.x - t * a.H, lane = threadIdx.x;
     const __half * p = (const __half *)a.partial + (size_t)blockIdx.x * a.splits * R;
     const float * ml = a.partial_ml + (size_t)blockIdx.x * a.splits * 2;
     const float m = lane < a.splits ? ml[2 * lane] : -INFINITY, l = lane < a.splits ? ml[2 * lane + 1] : 0.0f;
@@ -467,39 +555,56 @@ void latent_norms(hipStream_t s, int arith, const LatentNorms & a, int T) {
     check_launch("latent_norms");
 }
 
+void head_rows(hipStream_t s, int arith, const HeadRows & a, int T) {
+    if (T <= 0) return;
+    if (arith == ARITH_16) hipLaunchKernelGGL(k_head_rows<ARITH_16>, dim3((unsigned)T), dim3(256), 0, s, a);
+    else hipLaunchKernelGGL(k_head_rows<ARITH_32>, dim3((unsigned)T), dim3(256), 0, s, a);
+    check_launch("head_rows");
+}
+
 namespace {
 // Widest cache rows (in fragments) of the matrix-core kernel: rows that are keys and values at once, and separate ones.
 constexpr int kMatrixKf = 16, kMatrixKfPair = 8;
-bool on_matrix_cores(int arith, int kf, bool pair) { return arith == ARITH_16 && kf <= (pair ? kMatrixKfPair : kMatrixKf); }
+// Widths of keys and values where they differ.
+constexpr PairFrags kPairs[] = {{3, 1}, {4, 2}, {2, 4}, {6, 4}, {8, 4}, {4, 8}};
+bool on_matrix_cores(int arith, int kf, int vf, bool pair) { return arith == ARITH_16 && std::max(kf, vf) <= (pair ? kMatrixKfPair : kMatrixKf); }
 
-template <int KF, int CT, int WC, int WK, bool KV> void launch_attention(hipStream_t s, const StackAttn & a) {
-    constexpr int lds = WK * 2 * (KV ? 2 : 1) * KF * 2048;
-    auto kernel = k_stack_attention<KF, CT, WC, WK, KV>;
+template <int KF, int VF, int CT, int WC, int WK, bool KV> void launch_attention(hipStream_t s, const StackAttn & a) {
+    constexpr int lds = WK * 2 * (KF + (KV ? VF : 0)) * 2048;
+    auto kernel = k_stack_attention<KF, VF, CT, WC, WK, KV>;
     static const bool allowed = hipFuncSetAttribute((const void *)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, lds) == hipSuccess;
     if (!allowed) throw std::runtime_error("attention: the page buffers do not fit the LDS");
     hipLaunchKernelGGL(kernel, dim3((unsigned)a.n_blocks, (unsigned)a.splits, (unsigned)a.G), dim3(64 * WC * WK), lds, s, a);
 }
-template <int KF, bool KV> void launch_columns(hipStream_t s, const StackAttn & a) {
+template <int KF, int VF, bool KV> void launch_columns(hipStream_t s, const StackAttn & a) {
     switch (a.block_cols) {
-        case 16: launch_attention<KF, 1, 1, 2, KV>(s, a); break;
-        case 32: launch_attention<KF, 1, 2, 2, KV>(s, a); break;
-        case 64: launch_attention<KF, 1, 4, 1, KV>(s, a); break;
+        case 16: launch_attention<KF, VF, 1, 1, 2, KV>(s, a); break;
+        case 32: launch_attention<KF, VF, 1, 2, 2, KV>(s, a); break;
+        case 64: launch_attention<KF, VF, 1, 4, 1, KV>(s, a); break;
         case 128:
-            if constexpr (KF <= 8) { launch_attention<KF, 2, 4, 1, KV>(s, a); break; }      // wider: the registers do not suffice
+            if constexpr (KF <= 8) { launch_attention<KF, VF, 2, 4, 1, KV>(s, a); break; }      // wider: the registers do not suffice
             [[fallthrough]];
         default: throw std::runtime_error("attention: no kernel for this many columns per block");
     }
 }
+template <int I = 0> void launch_pair(hipStream_t s, const StackAttn & a) {
+    if constexpr (I < (int)(sizeof(kPairs) / sizeof(kPairs[0]))) {
+        if (a.kf == kPairs[I].k && a.vf == kPairs[I].v) return launch_columns<kPairs[I].k, kPairs[I].v, true>(s, a);
+        launch_pair<I + 1>(s, a);
+    } else {
+        throw std::runtime_error("attention: no kernel for this pair of cache widths");
+    }
+}
 template <bool KV> void launch_width(hipStream_t s, const StackAttn & a) {
     switch (a.kf) {                   // the widths cache_frags() rounds to
-        case 1: return launch_columns<1, KV>(s, a);
-        case 2: return launch_columns<2, KV>(s, a);
-        case 3: return launch_columns<3, KV>(s, a);
-        case 4: return launch_columns<4, KV>(s, a);
-        case 6: return launch_columns<6, KV>(s, a);
-        case 8: return launch_columns<8, KV>(s, a);
-        case 12: if constexpr (!KV) return launch_columns<12, KV>(s, a); break;
-        case 16: if constexpr (!KV) return launch_columns<16, KV>(s, a); break;
+        case 1: return launch_columns<1, 1, KV>(s, a);
+        case 2: return launch_columns<2, 2, KV>(s, a);
+        case 3: return launch_columns<3, 3, KV>(s, a);
+        case 4: return launch_columns<4, 4, KV>(s, a);
+        case 6: return launch_columns<6, 6, KV>(s, a);
+        case 8: return launch_columns<8, 8, KV>(s, a);
+        case 12: if constexpr (!KV) return launch_columns<12, 12, KV>(s, a); break;
+        case 16: if constexpr (!KV) return launch_columns<16, 16, KV>(s, a); break;
         default: break;
     }
     throw std::runtime_error("attention: no kernel for this cache width");
@@ -512,26 +617,36 @@ int cache_frags(int kv_rank) {
     return kf;
 }
 
-int stack_block_cols(int arith, int cols_per_token, int kf, bool pair, int n_tokens, int n_rows) {
-    if (!on_matrix_cores(arith, kf, pair)) return 1;
+PairFrags pair_frags(int key_columns, int value_columns) {
+    const int k = frags_of(key_columns), v = frags_of(value_columns), both = std::max(k, v);
+    if (both > kMatrixKfPair) return {k, v};
+    PairFrags best = {cache_frags(both * 32), cache_frags(both * 32)};
+    for (const PairFrags & p : kPairs)
+        if (k <= p.k && v <= p.v && p.k + p.v < best.k + best.v) best = p;
+    return best;
+}
+
+int stack_block_cols(int arith, int cols_per_token, int kf, int vf, bool pair, int n_tokens, int n_rows) {
+    if (!on_matrix_cores(arith, kf, vf, pair)) return 1;
     if (n_tokens == n_rows) return cols_per_token <= 16 ? 16 : cols_per_token <= 32 ? 32 : 64;      // one token per row
-    return kf <= 8 && (int64_t)n_tokens * cols_per_token >= 256 * 128 ? 128 : 64;
+    return std::max(kf, vf) <= 8 && (int64_t)n_tokens * cols_per_token >= 256 * 128 ? 128 : 64;
 }
 
 int stack_splits(int arith, const StackAttn & a, int max_resident) {
-    if (!on_matrix_cores(arith, a.kf, a.v_pool)) return 1;
+    if (!on_matrix_cores(arith, a.kf, a.vf, a.v_pool)) return 1;
     const int reach = a.chunk > 0 ? a.chunk : a.window, keys = reach > 0 ? std::min(reach, max_resident) : max_resident;
     const int pages = (keys + PAGE - 1) / PAGE + 1, per = a.block_cols <= 32 ? 2 : 1;
     return std::max(1, std::min({256 / std::max(a.n_blocks * a.G, 1), pages / per, 32}));
 }
 
-size_t stack_partial_floats(int T, int H, int kf, int splits) { return splits > 1 ? (size_t)T * H * splits * (kf * 16 + 2) : 0; }
+size_t stack_partial_floats(int T, int H, int vf, int splits) { return splits > 1 ? (size_t)T * H * splits * (vf * 16 + 2) : 0; }
 
 void stack_attention(hipStream_t s, int arith, const StackAttn & a) {
     if (a.n_blocks <= 0) return;
-    if (a.kf * 32 > 1024) throw std::runtime_error("attention: cache rows of at most 1024 columns per head");
-    if (on_matrix_cores(arith, a.kf, a.v_pool)) {
-        if (a.v_pool) launch_width<true>(s, a);
+    if (std::max(a.kf, a.vf) * 32 > 1024) throw std::runtime_error("attention: cache rows of at most 1024 columns per head");
+    if (on_matrix_cores(arith, a.kf, a.vf, a.v_pool)) {
+        if (a.v_pool && a.kf != a.vf) launch_pair(s, a);
+        else if (a.v_pool) launch_width<true>(s, a);
         else launch_width<false>(s, a);
         check_launch("stack_attention");
         return;

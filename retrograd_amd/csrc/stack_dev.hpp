@@ -14,6 +14,10 @@ typedef __bf16 b8 __attribute__((ext_vector_type(8)));
 __device__ __forceinline__ uint16_t bf16_bits(float v) { return __builtin_bit_cast(uint16_t, (__bf16)v); }
 __device__ __forceinline__ float bf16_float(uint16_t b) { return __builtin_bit_cast(float, (uint32_t)b << 16); }
 
+__device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
+__device__ __forceinline__ float softplus_f(float z) { return fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); }
+
 // Element (row, k) of a buffer in fragment order with kf fragments per row tile.
 __device__ __forceinline__ size_t frag_at(int row, int k, int kf) {
     return ((size_t)(row >> 4) * kf + (k >> 5)) * 512 + ((((k >> 3) & 3) * 16 + (row & 15)) * 8) + (k & 7);

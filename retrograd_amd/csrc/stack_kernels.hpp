@@ -49,8 +49,10 @@ enum : int {
     OUT_ACT_SWIGLU,     // ... silu(gate) * up
     OUT_ROTARY,         // queries, keys and values of grouped attention (RotaryOut)
     OUT_EXPERT,         // f32 rows dst[choice * stride + token * ld + col] = weight * v of an expert product's pairs
+    OUT_ACT_CLAMPED,    // ... g * sigmoid(slope * g) * (u + 1) of g = min(gate, limit), u = up clamped to [-limit, limit]
+    OUT_F32_CAPPED,     // f32 rows dst[t * ld + col] = limit * tanh(v / limit)
 };
-constexpr bool out_is_glu(int kind) { return kind == OUT_ACT_GEGLU || kind == OUT_ACT_SWIGLU; }
+constexpr bool out_is_glu(int kind) { return kind == OUT_ACT_GEGLU || kind == OUT_ACT_SWIGLU || kind == OUT_ACT_CLAMPED; }
 
 // Rows of a product that are heads of kf * 32 columns, H of queries, then G of keys: rotated, the queries to rows
 // [t][H][kf * 32], the keys to their cells; the keys as projected are the values. The columns of a rotated pair are
@@ -66,6 +68,7 @@ struct DenseOut {
     void * dst = nullptr;
     int ld = 0, col0 = 0, col_batch = 0;
     float scale = 1.0f;
+    float limit = 0.0f, slope = 1.0f;          // of the clamped gated pair (its gate's sigmoid), of the soft cap
     const float * gate = nullptr;
     int ld_gate = 0;
     size_t stride = 0;
@@ -100,11 +103,13 @@ struct DenseJob {
     int n_a = 0;                // true rows of part a when there is a part b
     const float * token_gate = nullptr;
     int ld_token_gate = 0;
+    const float * bias = nullptr;              // [batch][tiles * 16], in the weight's row order, added to the product
     const ExpertGroups * groups = nullptr;
     bool gather = false;
 };
 // Runs the product over T tokens. Where `ws` (dense_workspace_floats() floats) is given and the output is OUT_RESIDUAL,
-// a decode-sized product may come back as K-slices for the next norm to add instead.
+// a decode-sized product may come back as K-slices for the next norm to add instead; without a dst it always does (one
+// slice or more, and ws holds at least T * n floats).
 size_t dense_workspace_floats();
 Slices dense(hipStream_t s, int arith, const DenseJob & job, int T, float * ws);
 
@@ -116,6 +121,24 @@ void norm_act(hipStream_t s, int arith, int kind, float * x, const float * w, in
               int n_rows, void * act, int act_kf, const Slices & add, const float * plus = nullptr, void * act_rows = nullptr);
 // x[t][:] += the slices, for a stream that is read elsewhere than in the next norm.
 void add_slices(hipStream_t s, float * x, int E, int T, const Slices & add);
+// x[copy][t] = scale * embed[tok[t]] for `copies` planes `stride` floats apart (bf16 rows of E).
+void embed_rows(hipStream_t s, const uint16_t * embed, const int32_t * tok, int E, float scale, int T, float * x, int copies, size_t stride);
+
+// Several residual streams x_1 .. x_n of [T][E] floats (hyper-connections). A sublayer reads u = sum_a in[a] x_a; what it
+// leaves, y, changes every stream at once: x_b <- sum_a mix[a][b] x_a + out[b] y. A sublayer's weights: in[n], out[n], mix[n][n].
+constexpr int MAX_STREAMS = 16;
+constexpr int stream_weights(int n) { return n * (n + 2); }
+struct Streams {
+    float * x = nullptr;
+    int n = 0;
+    size_t stride = 0;             // floats from one stream to the next
+};
+// First the streams take in the slices of y by the weights `done` of the sublayer that left them (null: nothing is due), then
+// act[i] = norm(u[rows[i]]) * w with u read by the weights `next` (null: u is the streams' plain sum). RMS norm; act_rows as in norm_act.
+void streams_norm_act(hipStream_t s, int arith, const Streams & x, const float * done, const Slices & y, const float * next,
+                      const float * w, int E, float eps, const int32_t * rows, int n_rows, void * act, int act_kf, void * act_rows = nullptr);
+// out[t] = the sum of the streams once they have taken in y, which they do not here.
+void streams_sum(hipStream_t s, const Streams & x, const float * done, const Slices & y, int E, int T, float * out);
 
 // ---- attention ---------------------------------------------------------------------------------------
 // A page of a cache: PAGE tokens x kf fragments of 32 columns, f16 or f32,
@@ -123,6 +146,9 @@ void add_slices(hipStream_t s, float * x, int E, int T, const Slices & add);
 // (several key/value heads: one head's fragments behind the other's). Fragments a head's row of `columns` columns is
 // stored in: the widths the attention kernel is compiled for, zero padded.
 int cache_frags(int columns);
+// ... of a head's key row and its value row where their widths differ.
+struct PairFrags { int k, v; };
+PairFrags pair_frags(int key_columns, int value_columns);
 constexpr size_t cache_page_elems(int kf) { return (size_t)kf * 32 * PAGE; }
 // Queries' latent: act_q = RMS norm of proj[t][0, q_rank) times q_w. With kv_w also the cached latent: RMS norm of
 // proj[t][kv_col, kv_col + kv_rank) times kv_w into cell[t] of the pool.
@@ -139,13 +165,33 @@ struct LatentNorms {
 };
 void latent_norms(hipStream_t s, int arith, const LatentNorms & a, int T);
 
+// Grouped attention's rows between the input product and the cache, where they cannot leave in the product's epilogue:
+// proj[t] holds H queries of dim columns from q_col on, G keys and G values (vdim columns) from k_col and v_col on. Queries and keys
+// are RMS normed over all their heads at once (q_w, k_w), then the first `pairs` pairs (2 i, 2 i + 1) of each head rotated:
+// queries to rows [t][H][kf * 32], keys to their cells. Values go to their cells mixed with those of the same token in
+// `first`, (1 - share) v + share first; without `share`, first (where given) receives them.
+struct HeadRows {
+    const float * proj = nullptr;
+    int ld = 0, H = 0, G = 0, dim = 0, vdim = 0, q_col = 0, k_col = 0, v_col = 0;
+    const float * q_w = nullptr, * k_w = nullptr;
+    float eps = 0.0f;
+    int pairs = 0;
+    const float * table = nullptr;             // [T][pairs][2]: cosine and sine
+    const float * share = nullptr;             // one value
+    float * first = nullptr;                   // [T][G * vdim]
+    void * q = nullptr, * k_pool = nullptr, * v_pool = nullptr;
+    int kf = 0, vf = 0;
+    const int32_t * cell = nullptr;
+};
+void head_rows(hipStream_t s, int arith, const HeadRows & a, int T);
+
 // Attention over paged caches: absorbed queries over latents (v_pool null, one head's worth of rows that are keys and
 // values at once), or grouped attention over keys and values of G heads. A block serves up to `block_cols` of the
 // T x (H / G) query columns (token-major) of one row of the step, for every key/value head.
 struct AttnBlock { int32_t row, col0; };         // row of the step, first of its n * (H / G) columns
 struct StackAttn {
     const void * q = nullptr;      // [T][H][kf * 32]; latents: already scaled by scale * log2(e)
-    int H = 0, G = 1, kf = 0;
+    int H = 0, G = 1, kf = 0, vf = 0;            // fragments of a head's keys and of its values (latents: the same)
     int window = 0, chunk = 0;     // positions seen: the last `window`, or those of the same chunk of positions (0: no bound)
     float scale = 1.0f, softcap = 0.0f;          // with v_pool: score = scale * q.k, then softcap * tanh(score / softcap)
     const RowDesc * rows = nullptr;
@@ -154,15 +200,15 @@ struct StackAttn {
     const int32_t * table = nullptr;
     int max_pages = 0;
     const void * pool = nullptr, * v_pool = nullptr;
-    void * partial = nullptr;      // several splits: [T * H][splits][kf * 32] means in f16 ...
+    void * partial = nullptr;      // several splits: [T * H][splits][vf * 32] means in f16 ...
     float * partial_ml = nullptr;  // ... and [T * H][splits][2] maxima and sums (stack_partial_floats() for both)
-    void * out = nullptr;          // activations: column h * kf * 32 + c
+    void * out = nullptr;          // activations: column h * vf * 32 + c
     int out_kf = 0;
 };
-int stack_block_cols(int arith, int cols_per_token, int kf, bool pair, int n_tokens, int n_rows);
+int stack_block_cols(int arith, int cols_per_token, int kf, int vf, bool pair, int n_tokens, int n_rows);
 // Workgroups that share a block's keys, given the longest resident span among the step's rows.
 int stack_splits(int arith, const StackAttn & a, int max_resident);
-size_t stack_partial_floats(int T, int H, int kf, int splits);
+size_t stack_partial_floats(int T, int H, int vf, int splits);
 void stack_attention(hipStream_t s, int arith, const StackAttn & a);
 void stack_combine(hipStream_t s, const StackAttn & a, int T);      // of several splits (nothing to do for one)
 
@@ -171,12 +217,17 @@ void stack_combine(hipStream_t s, const StackAttn & a, int T);      // of severa
 void rotary_table(hipStream_t s, const double * freq, int pairs, double magnitude, const int32_t * pos, int T, float * table);
 
 // ---- expert routing --------------------------------------------------------------------------------------
-// Per token the `top` experts of largest logit (ties to the lower index) and the softmax over the chosen logits; then
-// the pairs sorted by expert into slots, every expert from a multiple of 16 on, cut into tiles of `block` slots.
+// Per token the `top` experts of largest logit (ties to the lower index), with several groups of neighbouring experts among
+// those of the `keep` groups whose largest logit is largest. Their weights: `scale` times the softmax over the chosen logits,
+// or over all of them. Then the pairs sorted by expert into slots, every expert from a multiple of 16 on, cut into tiles of
+// `block` slots.
 constexpr int MAX_EXPERTS = 1024, MAX_TOP = 64;
 struct ExpertRoute {
     const float * logits = nullptr;            // [T][ld]
     int ld = 0, experts = 0, top = 0, block = 0;
+    int groups = 1, keep = 1;
+    bool over_all = false;
+    float scale = 1.0f;
     int32_t * sel = nullptr;                   // [T * top]
     float * weight = nullptr;                  // [T * top]
     int32_t * slot_pair = nullptr;             // [expert_slots()]
@@ -191,10 +242,30 @@ void expert_route(hipStream_t s, const ExpertRoute & r, int T);
 void stack_copy_page(hipStream_t s, void * pool, size_t page_bytes, int src, int dst);
 void stack_cells(hipStream_t s, void * pool, int kf, int elem, const int32_t * cells, int n, void * rows, bool gather);
 
-// ---- state-space mixer (Mamba-2) ------------------------------------------------------------------------
-// The tokens of one sequence in a step, in order: seg_tok[start .. start + n) are flat token indices.
+// ---- recurrent mixers ---------------------------------------------------------------------------------
+// The tokens of one sequence in a step, in order: run_tok[start .. start + n) are flat token indices.
 struct SeqRun { int32_t slot, start, n, flags; };      // flags bit 0: the sequence starts here (state is zero), bit 1: the
                                                        // plane of the slot's convolution inputs that holds the current ones
+struct SeqRuns {
+    const SeqRun * runs = nullptr;
+    int n = 0, longest = 0, shortest = 0;
+    const int32_t * tok = nullptr;
+};
+// Short causal convolution over time per channel, then SiLU: out[t][c] from the taps newest last, zeros before a sequence
+// starts. Runs of fewer than `least` tokens are left out.
+struct ShortConv {
+    SeqRuns runs;
+    int channels = 0, taps = 0, least = 0;
+    const float * in = nullptr;    // [T][ld], the channels side by side
+    int ld = 0;
+    const float * w = nullptr, * b = nullptr;            // [channels][taps]; bias per channel or none
+    float * state = nullptr;       // [2 planes][slots][taps - 1][channels]
+    size_t plane = 0;              // floats of a plane
+    float * out = nullptr;         // [T][channels]
+};
+void short_conv(hipStream_t s, const ShortConv & c);
+
+// ---- state-space mixer (Mamba-2) ------------------------------------------------------------------------
 struct MambaShape {
     int heads = 0, vdim = 0, state = 0, groups = 0, taps = 0, norm_groups = 0;
     constexpr int inner() const { return heads * vdim; }
@@ -207,9 +278,7 @@ struct MambaJob {
     int ld = 0;
     const float * conv_w = nullptr, * conv_b = nullptr, * dt_bias = nullptr, * A_log = nullptr, * D = nullptr, * norm_w = nullptr;
     float eps = 0.0f;
-    const SeqRun * runs = nullptr;
-    int n_runs = 0, max_run = 0;
-    const int32_t * run_tok = nullptr;
+    SeqRuns runs;
     float * conv_state = nullptr;  // [2 planes][slots][taps - 1][channels]
     size_t conv_plane = 0;         // floats of a plane
     float * state = nullptr;       // [slots][heads][state][vdim]
@@ -219,6 +288,41 @@ struct MambaJob {
     int out_kf = 0;
 };
 void mamba_mix(hipStream_t s, int arith, const MambaJob & j, int T);
+
+// ---- gated delta rule with a decay per key channel ----------------------------------------------------------
+// Per head a state S [dim][vdim]: S <- g * S (rows scaled), S <- S + k (beta (v - S^T k))^T, o = S^T q; q and k unit vectors
+// per key/value head (q also times dim^-1/2) and, like v, convolved and through SiLU before; g = exp(-exp(A_log) softplus(a + dt_bias))
+// per head and row, beta a sigmoid per head. The read-out: o / rms(o) * norm_w * sigmoid(gate).
+struct DeltaShape {
+    int heads = 0, kv_heads = 0, dim = 0, vdim = 0, taps = 0;
+    int decay_rank = 0, gate_rank = 0;         // inner widths of the projections of a and gate
+    constexpr int keys() const { return kv_heads * dim; }
+    constexpr int inner() const { return heads * vdim; }
+    constexpr int channels() const { return 2 * keys() + inner(); }       // q | k | v
+    constexpr int vpitch() const { return (vdim + 3) / 4 * 4; }            // of a row of the state
+    constexpr size_t state_floats() const { return (size_t)heads * dim * vpitch(); }
+};
+struct DeltaJob {
+    DeltaShape sh;
+    const float * proj = nullptr;  // [T][ld]: q | k | v | beta (heads)
+    int ld = 0;
+    const float * decay = nullptr, * gate = nullptr;     // [T][ld_low]: a (heads x dim), gate (heads x vdim)
+    int ld_low = 0;
+    const float * conv_w = nullptr, * A_log = nullptr, * dt_bias = nullptr, * norm_w = nullptr;
+    float eps = 0.0f, unit_eps = 0.0f;
+    SeqRuns runs;
+    float * conv_state = nullptr;  // as in ShortConv
+    size_t conv_plane = 0;
+    float * state = nullptr;       // [slots][heads][dim][vpitch]
+    float * qkv = nullptr;         // scratch [T][channels]
+    float * y = nullptr;           // scratch [T][inner]
+    float * chunks = nullptr;      // scratch, delta_chunk_floats()
+    void * out = nullptr;          // activations, inner wide
+    int out_kf = 0;
+};
+size_t delta_chunk_floats(const DeltaShape & sh, int T, int n_runs);
+void delta_mix(hipStream_t s, int arith, const DeltaJob & j, int T);
+
 void copy_floats(hipStream_t s, const float * src, float * dst, size_t n);
 
 }  // namespace rk

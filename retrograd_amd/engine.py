@@ -169,7 +169,7 @@ KERNEL_SYMBOLS = [
 ]
 PROFILE_CATEGORIES = ["pack", "embed", "norm", "qkv", "rope", "attention", "combine", "o_proj", "gate_up", "swiglu",
                       "down", "head", "sample", "absorb", "scan", "route", "experts_in",
-                      "experts_out", "shared"]
+                      "experts_out", "shared", "low_rank"]
 
 _lib = None
 _i32p, _f32p, _u8p = C.POINTER(C.c_int32), C.POINTER(C.c_float), C.POINTER(C.c_uint8)
