@@ -61,6 +61,85 @@ def pomisun(width, vocab, layers, eps=1e-5, loop=None):
     return out
 
 
+def banded_rotary(dims, base=10000.0, factor=None, original=64, high=4.0, low=1.0):
+    r = {"dims": dims, "base": base}
+    if factor is not None:
+        r["scaling"] = {"factor": factor, "original": original, "high": high, "low": low}
+    return r
+
+
+def clamped_mlp(ff, limit=1.5):
+    return {"kind": "dense", "ff": ff, "limit": limit}
+
+
+def clamped_moe(experts, top, ff, limit=1.5, shared=None, groups=None, scale=1.0):
+    """shared: (width, limit) of the shared expert; groups: (count, kept)."""
+    router = {"experts": experts, "top": top, "scale": scale}
+    if groups:
+        router["groups"] = dict(zip(("count", "keep"), groups))
+    out = {"kind": "moe", "router": router, "expert": {"ff": ff, "limit": limit}}
+    if shared:
+        out["shared"] = dict(zip(("ff", "limit"), shared))
+    return out
+
+
+def normed_attention_layer(heads, kv_heads, dim, vdim, window, rot, mlp, scale=None, v_mix=False):
+    """Grouped attention with values of its own, biases, and queries and keys normed over all their heads."""
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "mask": {"size": window} if window else None, "rot": rot,
+         "scale": dim ** -0.5 if scale is None else scale, "v_mix": v_mix}
+    return {"type": "attention", "mixer": m, "mlp": mlp}
+
+
+def channel_delta_layer(heads, kv_heads, dim, vdim, conv, mlp, decay_rank, gate_rank):
+    """The two inner widths are what the tensors get; the engine takes them from there."""
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": conv, "decay_rank": decay_rank, "gate_rank": gate_rank}
+    return {"type": "channel_delta", "mixer": m, "mlp": mlp}
+
+
+def vifanex(width, vocab, layers, streams=2, eps=1e-5, softcap=20.0, embedding_scale=1.0):
+    return {"architecture": "Vifanex", "width": width, "vocab": vocab, "norm": {"eps": eps}, "streams": streams, "layers": layers,
+            "logit_softcap": softcap, "embedding": {"scale": embedding_scale}}
+
+
+def _vifanex_shapes(cfg) -> dict:
+    E, s = cfg["width"], cfg["streams"]
+    out = {"embed": (cfg["vocab"], E)}
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, mlp = "l%d." % i, layer["mixer"], layer.get("mlp")
+        x, H, G, D, V = p + "mix.", m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        for q in (1, 2) if mlp else (1,):
+            out[p + "norm%d" % q] = (E,)
+            out.update({p + "hc%d.in" % q: (s,), p + "hc%d.out" % q: (s,), p + "hc%d.mix" % q: (s, s)})
+        if layer["type"] == "attention":
+            for name, n in (("q", H * D), ("k", G * D), ("v", G * V)):
+                out[x + name] = (n, E)
+                out[x + name + ".b"] = (n,)
+            out[x + "q.norm"], out[x + "k.norm"] = (H * D,), (G * D,)
+            if m["v_mix"]:
+                out[x + "vmix"] = ()
+        else:
+            for name, n in (("q", G * D), ("k", G * D), ("v", H * V)):
+                out[x + name] = (n, E)
+                out[x + name + ".conv"] = (n, m["conv"])
+            out.update({x + "b": (H, E), x + "A_log": (H,), x + "norm": (V,), x + "a1": (m["decay_rank"], E), x + "a2": (H * D, m["decay_rank"]),
+                        x + "dt_bias": (H * D,), x + "g1": (m["gate_rank"], E), x + "g2": (H * V, m["gate_rank"])})
+        out[x + "o"] = (E, H * V)
+        if not mlp:
+            continue
+        if mlp["kind"] == "dense":
+            out.update(_gated_shapes(p + "mlp.", mlp["ff"], E))
+            out.update({p + "mlp.gate.b": (mlp["ff"],), p + "mlp.up.b": (mlp["ff"],), p + "mlp.down.b": (E,)})
+            continue
+        out[p + "mlp.router"] = (mlp["router"]["experts"], E)
+        for e in range(mlp["router"]["experts"]):
+            out.update(_gated_shapes(p + "mlp.e%d." % e, mlp["expert"]["ff"], E))
+        if mlp.get("shared"):
+            out.update(_gated_shapes(p + "mlp.shared.", mlp["shared"]["ff"], E))
+    out["final.norm"] = (E,)
+    out["head"] = (cfg["vocab"], E)
+    return out
+
+
 def _gated_shapes(p, ff, E):
     return {p + "gate": (ff, E), p + "up": (ff, E), p + "down": (E, ff)}
 
@@ -68,6 +147,8 @@ def _gated_shapes(p, ff, E):
 def tensor_shapes(cfg) -> dict:
     E = cfg["width"]
     out = {"embed": (cfg["vocab"], E)}
+    if cfg["architecture"] == "Vifanex":
+        return _vifanex_shapes(cfg)
     if cfg["architecture"] == "Pomisun":
         for i, layer in enumerate(cfg["layers"]):
             p, m, mlp = "l%d." % i, layer["mixer"], layer.get("mlp")
@@ -127,6 +208,15 @@ def mean_and_std(name, shape, architecture="Dibosun"):
     leaf = name.rsplit(".", 1)[-1]
     if architecture == "Pomisun" and leaf.startswith("norm"):
         return -0.1, 0.2                     # stored as the difference from one
+    if architecture == "Vifanex":
+        if ".hc" in name:
+            return (0.8, 0.3) if leaf == "out" else (1.0 / shape[0], 0.3)
+        if leaf == "vmix":
+            return 0.5, 0.3
+        if len(shape) == 2 and leaf == "b":
+            return 0.0, shape[-1] ** -0.5
+        if leaf == "b":
+            return 0.0, 0.3
     if leaf == "router":
         return 0.0, 2.0 * shape[-1] ** -0.5
     if leaf == "dt_bias":
