@@ -248,11 +248,11 @@ def _header(items):
 def to_bf16(x) -> np.ndarray:
     """f32 -> bf16 bits, to nearest even."""
     b = np.ascontiguousarray(x, np.float32).view(np.uint32).astype(np.uint64)
-    return ((b + 0x7FFF + ((b >> 16) & 1)) >> 16).astype(np.uint16)
+    return ((b + 0x7FFF + ((b >> 16) & 1)) >> 16).astype(np.uint16).reshape(np.shape(x))
 
 
 def from_bf16(b) -> np.ndarray:
-    return (np.asarray(b, np.uint32) << 16).view(np.float32)
+    return (np.atleast_1d(np.asarray(b, np.uint32)) << 16).view(np.float32).reshape(np.shape(b))
 
 
 def random_tensors(cfg, seed) -> dict:
