@@ -1,5 +1,5 @@
-"""Prefill and decode of layer-stack models at sizes that resemble a real model's layers, beside the closest GGUF models
-of the same width, feed-forward width and depth: what `bench.py --model dibosun` and `--model pomisun` run. Weights are random
+"""Prefill and decode of layer-stack models at sizes that resemble a real model's layers, beside the closest other models of
+the same width, feed-forward width and depth: what `bench.py --model dibosun`, `--model pomisun` and `--model vifanex` run. Weights are random
 (seeded), prompts random token ids. Every kernel category is also priced against its roofline, the larger of its
 algorithmic bytes over 8 TB/s and its products' flops over 2.5 PFLOP/s (a product counted once, however a model's
 arithmetic splits its operands; the scan's flops over the 157 TFLOP/s of f32)."""
@@ -37,6 +37,16 @@ def pomisun_config(size):
     E, F, H, D = SIZES[size][:4]
     layer = lambda mlp: Y.attention_layer(H, max(H // 4, 1), D, CHUNK, Y.rotary(D, 1e6, factor=8.0, original=8192), mlp, softcap=30.0)
     return Y.pomisun(E, VOCAB, [layer(Y.dense_mlp(F)), layer(Y.moe_mlp(*EXPERTS[size]))] * 4)
+
+
+def vifanex_config(size):
+    from . import synth_stack as Y
+    E, F, H, D = SIZES[size][:4]
+    n, top, fe, fs = EXPERTS[size]
+    dense, moe = Y.clamped_mlp(F, 7.0), Y.clamped_moe(n, top, fe, 7.0, shared=(fs, 7.0), groups=(8, 4), scale=2.5)
+    att = lambda mlp: Y.normed_attention_layer(H, max(H // 4, 1), D, D, WINDOW, Y.banded_rotary(D, 1e6, factor=8.0, original=8192), mlp, v_mix=True)
+    rec = lambda mlp: Y.channel_delta_layer(H, H, D, D, 4, mlp, 128, 128)
+    return Y.vifanex(E, VOCAB, [att(dense), rec(moe), att(moe), rec(dense)] * 2, streams=4, softcap=30.0)
 
 
 def qwen3moe_shape(size):
@@ -119,6 +129,45 @@ def pomisun_work(cfg, rows, ctx, n_out):
         n, top, F, S = mlp["router"]["experts"], mlp["router"]["top"], mlp["expert"]["ff"], mlp["shared"]["ff"]
         used = chosen_experts(n, top, T)
         add("shared", 2 * (n + 1 + 3 * S) * E + T * (2 * E + 4 * (n + 1) + 4 * S + 8 * E), 2 * T * E * (n + 1 + 3 * S))
+        add("route", T * (4 * n + 8 * top))
+        add("experts_in", 4 * used * F * E + T * 2 * E + T * top * 2 * F, 4 * T * top * E * F)
+        add("experts_out", 2 * used * F * E + T * top * (2 * F + 4 * E), 2 * T * top * E * F)
+    add("head", 2 * cfg["vocab"] * E + n_out * (2 * E + 4 * cfg["vocab"]), 2 * n_out * E * cfg["vocab"])
+    return w
+
+
+def vifanex_work(cfg, rows, ctx, n_out):
+    E, T, s = cfg["width"], rows, cfg["streams"]
+    w = {}
+
+    def add(k, by, fl=0.0, f32=0.0):
+        a = w.setdefault(k, [0.0, 0.0, 0.0])
+        a[0] += by
+        a[1] += fl
+        a[2] += f32
+    for layer in cfg["layers"]:
+        m, mlp = layer["mixer"], layer["mlp"]
+        H, G, D, V = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        add("norm", 2 * T * E * (8 * s + 4 + 2))                 # every stream read and written, what is added, the activations
+        if layer["type"] == "attention":
+            n = (H + G) * D + G * V
+            add("qkv", 2 * n * E + T * (2 * E + 4 * n), 2 * T * n * E)
+            add("rope", T * (4 + 2) * n)
+            add("attention", ctx[1] * 2 * G * (D + V) + T * H * 2 * (D + V), 2 * T * H * ctx[0] * (D + V))
+        else:
+            n, ra, rg = 2 * G * D + H * V + H, m["decay_rank"], m["gate_rank"]
+            add("qkv", 2 * (n + ra + rg) * E + T * (2 * E + 4 * n + 2 * (ra + rg)), 2 * T * (n + ra + rg) * E)
+            add("low_rank", 2 * H * (D * ra + V * rg) + T * (2 * (ra + rg) + 4 * H * (D + V)), 2 * T * H * (D * ra + V * rg))
+            add("scan", 8 * H * D * V * ctx[2] + T * (4 * n + 4 * H * (D + V) + 2 * H * V), 0, 6 * T * H * D * V)
+        add("o_proj", 2 * E * H * V + T * (2 * H * V + 4 * E), 2 * T * E * H * V)
+        if mlp["kind"] == "dense":
+            F = mlp["ff"]
+            add("gate_up", 4 * F * E + T * (2 * E + 2 * F), 4 * T * E * F)
+            add("down", 2 * E * F + T * (2 * F + 4 * E), 2 * T * E * F)
+            continue
+        n, top, F, S = mlp["router"]["experts"], mlp["router"]["top"], mlp["expert"]["ff"], mlp["shared"]["ff"]
+        used = chosen_experts(n, top, T)
+        add("shared", 2 * (n + 3 * S) * E + T * (2 * E + 4 * n + 4 * S + 4 * E), 2 * T * E * (n + 3 * S))
         add("route", T * (4 * n + 8 * top))
         add("experts_in", 4 * used * F * E + T * 2 * E + T * top * 2 * F, 4 * T * top * E * F)
         add("experts_out", 2 * used * F * E + T * top * (2 * F + 4 * E), 2 * T * top * E * F)
@@ -236,31 +285,34 @@ def main(args) -> int:
     if not torch.cuda.is_available():
         print("this benchmark needs an MI355X: no HIP device is visible", file=sys.stderr)
         return 2
-    causal = lambda p: p + 1
-    design, closest = {
-        "dibosun": ((dibosun_config, dibosun_work, lambda p: np.minimum(p + 1, WINDOW)), [("llama", llama_shape, llama_work)]),
-        "pomisun": ((pomisun_config, pomisun_work, lambda p: p % CHUNK + 1),
-                    [("llama", llama_shape, llama_work), ("qwen3moe", qwen3moe_shape, qwen3moe_work)]),
-    }[args.model]
+    causal, windowed, chunked = lambda p: p + 1, lambda p: np.minimum(p + 1, WINDOW), lambda p: p % CHUNK + 1
+    stacks = {"dibosun": (dibosun_config, dibosun_work, windowed), "pomisun": (pomisun_config, pomisun_work, chunked), "vifanex": (vifanex_config, vifanex_work, windowed)}
+    ggufs = {"llama": (llama_shape, llama_work), "qwen3moe": (qwen3moe_shape, qwen3moe_work)}
+    closest = {"dibosun": ["llama"], "pomisun": ["llama", "qwen3moe"], "vifanex": ["pomisun", "dibosun"]}[args.model]
     steps = min(args.steps, 16)
-    result = {"metric": "prefill and decode throughput, %s beside GGUF models (Q4_K, MXFP4 experts) of equal width, feed-forward and depth" % args.model.capitalize(),
+    result = {"metric": "prefill and decode throughput, %s beside other models (GGUF ones in Q4_K, MXFP4 experts) of equal width, feed-forward and depth" % args.model.capitalize(),
               "data": "synthetic", "context": CONTEXT, "vocab": VOCAB, "layers": 8, "sizes": {}}
     for size in args.stack_sizes.split(","):
-        cfg = design[0](size)
-        folder = Path(args.model_dir) / ("retro-bench-%s-%s" % (args.model, size))
-        if not (folder / "done").exists():
-            Y.write_random_checkpoint(folder, cfg, args.seed)
-            (folder / "done").write_text("")
-        print("[bench]", args.model, size, file=sys.stderr, flush=True)
-        entry = {args.model: measure(folder, E, VOCAB, lambda *a: design[1](cfg, *a), design[2], 4096, (512, 4096), steps)}
-        for name, shape_of, work in [] if args.no_closest_model else closest:
-            shape = shape_of(size)
-            path = Path(args.model_dir) / ("retro-bench-%s.gguf" % shape.name)
-            if not path.exists():
-                synth.write_model(path.with_suffix(".tmp"), shape, seed=args.seed, device="cuda")
-                os.replace(path.with_suffix(".tmp"), path)
+        entry = {}
+        for name in [args.model] + ([] if args.no_closest_model else closest):
             print("[bench]", name, size, file=sys.stderr, flush=True)
-            entry[name] = measure(path, E, VOCAB, lambda *a: work(shape, *a), causal, 4096, (512, 4096), steps)
+            if name in stacks:
+                config_of, work, keys = stacks[name]
+                cfg = config_of(size)
+                path = Path(args.model_dir) / ("retro-bench-%s-%s" % (name, size))
+                if not (path / "done").exists():
+                    Y.write_random_checkpoint(path, cfg, args.seed)
+                    (path / "done").write_text("")
+                work_of = lambda *a: work(cfg, *a)
+            else:
+                shape_of, work = ggufs[name]
+                shape, keys = shape_of(size), causal
+                path = Path(args.model_dir) / ("retro-bench-%s.gguf" % shape.name)
+                if not path.exists():
+                    synth.write_model(path.with_suffix(".tmp"), shape, seed=args.seed, device="cuda")
+                    os.replace(path.with_suffix(".tmp"), path)
+                work_of = lambda *a: work(shape, *a)
+            entry[name] = measure(path, E, VOCAB, work_of, keys, 4096, (512, 4096), steps)
         result["sizes"][size] = entry
     print(json.dumps(result), flush=True)
     return 0
