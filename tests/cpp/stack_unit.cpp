@@ -18,7 +18,19 @@ int main(int argc, char ** argv) {
                 for (const retro::LayerRun & r : c.runs) std::printf(" %s%d", r.add_embedding ? "+" : "", r.layer);
                 std::printf("\n");
             }
+            if (c.streams > 0) std::printf("streams %d embedding_scale %g logit_softcap %g\n", c.streams, (double)c.embedding_scale, (double)c.logit_softcap);
             for (const retro::LayerSpec & l : c.layers) {
+                if (c.streams > 0) {
+                    const retro::MoeSpec & e = l.moe;
+                    std::printf("limits %g %g %g groups %d keep %d scale %g vdim %d v_mix %d v_first %d\n", (double)l.ff_limit, (double)e.limit, (double)e.shared_limit,
+                                e.groups, e.keep, (double)e.scale, l.attention.vdim, l.attention.v_mix, l.attention.v_first);
+                }
+                if (l.mixer == retro::Mixer::CHANNEL_DELTA) {
+                    const rk::DeltaShape & d = l.delta;
+                    std::printf("channel_delta heads %d kv_heads %d dim %d vdim %d taps %d ff %d experts %d top %d of %d shared %d\n", d.heads, d.kv_heads, d.dim, d.vdim,
+                                d.taps, l.ff, l.moe.experts, l.moe.top, l.moe.ff, l.moe.shared_ff);
+                    continue;
+                }
                 if (l.mixer == retro::Mixer::ATTENTION) {
                     const retro::AttentionSpec & g = l.attention;
                     std::printf("attention heads %d kv_heads %d dim %d window %d chunk %d scale %g softcap %g ff %d experts %d top %d of %d shared %d\n", g.heads, g.kv_heads,

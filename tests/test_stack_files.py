@@ -136,6 +136,101 @@ def test_the_plain_pomisun_statements_against_closed_forms():
     assert np.allclose(PP.rms_norm_around_one(np.array([[3.0, 4.0]]), np.array([0.0, 1.0]), 0.0), [[3 / 12.5 ** 0.5, 8 / 12.5 ** 0.5]])
 
 
+VIFANEX = Y.vifanex(44, 30, [
+    Y.normed_attention_layer(heads=6, kv_heads=2, dim=10, vdim=12, window=9, rot=Y.banded_rotary(6, 1000.0, factor=3.0, original=30, high=2.5, low=0.5), mlp=Y.clamped_mlp(13, 0.75), scale=0.5),
+    Y.channel_delta_layer(heads=6, kv_heads=3, dim=7, vdim=5, conv=2, mlp=Y.clamped_moe(6, 2, 7, 1.25, shared=(11, 3.0), groups=(3, 2), scale=2.5), decay_rank=3, gate_rank=4),
+    Y.normed_attention_layer(heads=4, kv_heads=4, dim=8, vdim=6, window=None, rot=Y.banded_rotary(8, 50.0), mlp=None, v_mix=True),
+    Y.normed_attention_layer(heads=3, kv_heads=1, dim=16, vdim=24, window=3, rot=Y.banded_rotary(16, 50.0, factor=8.0, original=1000), mlp=Y.clamped_moe(4, 4, 3), v_mix=True)],
+    streams=5, softcap=7.5, embedding_scale=1.5)
+
+
+def test_every_field_of_a_vifanex_configuration(reader, tmp_path):
+    import plain_vifanex as PV
+
+    Y.write_checkpoint(tmp_path, VIFANEX, Y.random_tensors(VIFANEX, 1))
+    lines = reader(tmp_path, "config").splitlines()
+    assert lines[:2] == ["Vifanex width 44 vocab 30 eps 1e-05", "streams 5 embedding_scale 1.5 logit_softcap 7.5"]
+    assert [l for l in lines[2:] if not l.startswith("rotary")] == [
+        "limits 0.75 0 0 groups 1 keep 1 scale 1 vdim 12 v_mix 0 v_first 0",
+        "attention heads 6 kv_heads 2 dim 10 window 9 chunk 0 scale 0.5 softcap 0 ff 13 experts 0 top 0 of 0 shared 0",
+        "limits 0 1.25 3 groups 3 keep 2 scale 2.5 vdim 0 v_mix 0 v_first 0",
+        "channel_delta heads 6 kv_heads 3 dim 7 vdim 5 taps 2 ff 0 experts 6 top 2 of 7 shared 11",
+        "limits 0 0 0 groups 1 keep 1 scale 1 vdim 6 v_mix 1 v_first 1",
+        "attention heads 4 kv_heads 4 dim 8 window 0 chunk 0 scale 0.353553 softcap 0 ff 0 experts 0 top 0 of 0 shared 0",
+        "limits 0 1.5 0 groups 1 keep 1 scale 1 vdim 24 v_mix 1 v_first 0",
+        "attention heads 3 kv_heads 1 dim 16 window 3 chunk 0 scale 0.25 softcap 0 ff 0 experts 4 top 4 of 3 shared 0"]
+    rotary = [l.split() for l in lines if l.startswith("rotary")]
+    for words, layer in zip(rotary, [l for l in VIFANEX["layers"] if l["type"] == "attention"]):
+        assert words[3] == "1" and np.allclose([float(w) for w in words[4:]], PV.banded_frequencies(layer["mixer"]["rot"]), rtol=1e-13)
+    assert reader(tmp_path, "l1.mlp.e5.down").endswith("l1.mlp.e5.down BF16\n")
+    assert reader(tmp_path, "l2.mix.vmix").endswith("l2.mix.vmix BF16\n")
+    assert reader(tmp_path, "l2.hc2.in").endswith("l2.hc2.in missing\n")
+
+
+@pytest.mark.parametrize("edit, message", [
+    (lambda c: c.update(streams=17), "'streams'"),
+    (lambda c: c.update(loop={"start": 0, "stop": 1, "times": 2}), "'streams'"),
+    (lambda c: c.update(logit_softcap=-1), "logit_softcap"),
+    (lambda c: c["layers"][1]["mixer"].update(kv_heads=4), "multiple of kv_heads"),
+    (lambda c: c["layers"][1]["mixer"].update(dim=513), "512 key"),
+    (lambda c: c["layers"][1]["mixer"].pop("conv"), "lacks 'conv'"),
+    (lambda c: c["layers"][0]["mlp"].pop("limit"), "lacks 'limit'"),
+    (lambda c: c["layers"][1]["mlp"]["expert"].update(limit=0), "'limit' must be positive"),
+    (lambda c: c["layers"][1]["mlp"]["shared"].update(limit=-2), "'limit' must be positive"),
+    (lambda c: c["layers"][1]["mlp"]["router"]["groups"].update(count=4), "equal parts"),
+    (lambda c: c["layers"][1]["mlp"]["router"]["groups"].update(keep=4), "equal parts"),
+    (lambda c: c["layers"][1]["mlp"]["router"].update(top=5), "equal parts"),
+    (lambda c: c["layers"][3]["mixer"].update(vdim=23), "equally many"),
+    (lambda c: c["layers"][0]["mixer"]["rot"]["scaling"].pop("high"), "lacks 'high'"),
+])
+def test_refused_vifanex_configurations(reader, tmp_path, edit, message):
+    cfg = copy.deepcopy(VIFANEX)
+    edit(cfg)
+    (tmp_path / "config.json").write_text(json.dumps(cfg))
+    out = reader(tmp_path, "config")
+    assert out.startswith("refused: ") and message in out, out
+
+
+def test_the_plain_vifanex_statements_against_closed_forms():
+    import plain_vifanex as PV
+
+    rng = np.random.default_rng(0)
+    # neighbouring columns turn, the rest stays; scores depend on the distance alone
+    x = np.zeros((1, 1, 6))
+    x[..., 2], x[..., 5] = 1, 3
+    assert np.allclose(PV.rotate_neighbours(x, [3], Y.banded_rotary(4, 100.0))[0, 0], [0, 0, np.cos(0.3), np.sin(0.3), 0, 3])
+    # frequencies: kept, in between (half way of the turns), divided
+    rot = lambda turns: {"dims": 2, "base": 10.0, "scaling": {"factor": 4.0, "original": 2 * np.pi * turns, "high": 3.0, "low": 1.0}}
+    assert np.allclose([PV.banded_frequencies(rot(t))[0] for t in (9, 3, 2, 1, 0.5)], [1, 1, 0.625, 0.25, 0.25])
+    # one token: o = beta (k . q) v; the same unit key written again with beta 1 replaces what it held; strong decay forgets
+    q, k, v = rng.standard_normal((3, 1, 4)), np.zeros((3, 1, 4)), rng.standard_normal((3, 1, 2))
+    k[:, :, 1] = 1
+    one, half = np.ones((3, 1)), np.full((3, 1), 0.5)
+    o = PV.channel_delta_scan(q, k, v, one, np.ones((3, 1, 4)))
+    assert np.allclose(o[:, 0], q[:, 0, 1:2] * v[:, 0])
+    o = PV.channel_delta_scan(q, k, v, half, np.zeros((3, 1, 4)))
+    assert np.allclose(o[:, 0], 0.5 * q[:, 0, 1:2] * v[:, 0])
+    g = np.ones((3, 1, 4))
+    g[:, :, 1] = 0.5                                                 # only the key's own channel decays
+    held = 0.5 * v[0, 0]
+    held = 0.5 * held + 0.5 * (v[1, 0] - 0.5 * held)
+    assert np.allclose(PV.channel_delta_scan(q, k, v, half, g)[1, 0], q[1, 0, 1] * held)
+    # gated pair: below the limits g sigmoid(1.702 g) (u + 1), beyond them clamped (the gate from above only)
+    eye = np.eye(1)
+    y = lambda g, u, limit: PV.clamped_ff(np.array([[1.0]]), g * eye, u * eye, eye, limit)[0, 0]
+    gate = lambda g: g / (1 + np.exp(-1.702 * g))
+    assert np.allclose([y(0.5, 0.25, 2), y(9, 0, 2), y(-9, 0, 2), y(1, -9, 2), y(1, 9, 2)], [gate(0.5) * 1.25, gate(2.0), gate(-9.0), -gate(1.0), gate(1.0) * 3])
+    # groups: the best expert's group is kept although the second-best expert is elsewhere; weights over all experts
+    z = np.array([[5.0, 0.0, 4.0, 3.0]])
+    sel, w = PV.choose_experts(z, {"experts": 4, "top": 2, "scale": 2.0, "groups": {"count": 2, "keep": 1}})
+    assert sorted(sel[0].tolist()) == [0, 1] and np.allclose(np.sort(w[0]), np.sort(2 * np.exp([5.0, 0.0]) / np.exp(z).sum()))
+    # streams: mix is [from, to]
+    xs = rng.standard_normal((2, 1, 3))
+    mix = np.array([[0.0, 1.0], [0.0, 0.0]])
+    out = PV.streams_out(xs, np.ones((1, 3)), {"mix": mix, "out": np.array([0.0, 2.0])})
+    assert np.allclose(out[0], 0) and np.allclose(out[1], xs[0] + 2)
+
+
 @pytest.mark.parametrize("edit, message", [
     (lambda c: c.update(architecture="Other"), "unsupported model architecture: Other"),
     (lambda c: c.pop("width"), "lacks 'width'"),
