@@ -1,5 +1,5 @@
-// The gated delta rule with a decay per key channel, between its projections (stack_kernels.hpp: DeltaJob). Everything here is
-// f32 in both arithmetics; only the rows that leave for the output projection take the arithmetic's activation type.
+// Recurrent mixers with a matrix state - the gated delta rule with a decay per key channel or per head, and linear attention with
+// a forget gate - between their projections (stack_kernels.hpp: DeltaJob). Everything here is f32 in both arithmetics; only the rows that leave for the output projection take the arithmetic's activation type.
 // Short runs (decoding above all) take one launch from the projections' rows to those activations: a workgroup per run and
 // head convolves its channels, walks the tokens with the state in registers and norms and gates the read-outs. Long runs are
 // worked on in chunks of 64 tokens: everything inside a chunk that does not need the state, for all chunks at once; then the
@@ -21,19 +21,33 @@ constexpr int kScanRows = 16;         // most rows of the state a thread of the 
 
 int pad16(int n) { return (n + 15) / 16 * 16; }
 
-__device__ __forceinline__ float log_decay(const DeltaJob & j, int t, int h, int d, float rate) {
-    const int c = h * j.sh.dim + d;
+// c: the head's channel, or the head where it has one decay.
+__device__ __forceinline__ float log_decay(const DeltaJob & j, int t, int c, float rate) {
     return -rate * softplus_f(j.decay[(size_t)t * j.ld_low + c] + j.dt_bias[c]);
 }
+
+// The forget gate of a channel: g = lower + (1 - lower) sigmoid(z), and 1 - g, each without cancellation.
+struct Forget {
+    float keep, write;
+    __device__ __forceinline__ Forget(float z, float lower) : keep(lower + (1.0f - lower) * sigmoid_f(z)), write((1.0f - lower) * sigmoid_f(-z)) {}
+    __device__ __forceinline__ float log_keep() const { return write < 0.5f ? log1pf(-write) : logf(fmaxf(keep, 1e-37f)); }
+};
 
 // Eight columns c .. c + 7 of a head's read-out o, of which the first `left` are real.
 template <int ARITH>
 __device__ __forceinline__ void store_read_out(const DeltaJob & j, int t, int h, int c, int left, const float (&o)[8], float inv) {
-    const float * gate = j.gate + (size_t)t * j.ld_low + h * j.sh.vdim + c;
     const int col = h * j.sh.vdim + c;
     float v[8];
 #pragma unroll
-    for (int i = 0; i < 8; ++i) v[i] = i < left ? o[i] * inv * j.norm_w[c + i] * sigmoid_f(gate[i]) : 0.0f;
+    for (int i = 0; i < 8; ++i) v[i] = i < left ? o[i] * inv * j.norm_w[c + i] : 0.0f;
+    if (j.sh.gate != GATE_NONE) {
+        const float * gate = j.gate + (size_t)t * j.ld_low + col;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            const float z = i < left ? gate[i] : 0.0f, s = sigmoid_f(z);
+            v[i] *= j.sh.gate == GATE_SILU ? z * s : s;
+        }
+    }
     if (left >= 8 && col % 8 == 0) {
         store_frag8<ARITH>(j.out, j.out_kf, t, col, v);
     } else {
@@ -49,7 +63,7 @@ __device__ __forceinline__ void store_read_out(const DeltaJob & j, int t, int h,
 
 // Runs of fewer than `below` tokens. Thread (rg, cg) holds rows rg, rg + RG, ... of four columns of the state; wider heads
 // take several blocks of columns per token. The decayed state is multiplied with k and q in one pass: with u = beta (v - S^T k)
-// the read-out after the write is S^T q + (k . q) u.
+// the read-out after the write is S^T q + (k . q) u (forget rule: u = v).
 template <int ARITH, int CG, int NPT>
 __global__ __launch_bounds__(256) void k_delta_scan(DeltaJob j, int below) {
     constexpr int RG = 256 / CG;
@@ -84,19 +98,31 @@ __global__ __launch_bounds__(256) void k_delta_scan(DeltaJob j, int below) {
         return fresh ? 0.0f : old_in[(size_t)(i + K - 1) * C + c];
     };
     auto channel = [&](int i) { return i < D ? kv * D + i : i < 2 * D ? KC + kv * D + i - D : 2 * KC + h * V + i - 2 * D; };
-    const float rate = expf(j.A_log[h]);
+    const bool forget = sh.rule == RULE_FORGET;
+    const float rate = forget ? 0.0f : expf(j.A_log[h]);
     if (tid < VP - V) sv[V + tid] = 0.0f;
     int parity = 0;
     for (int i = 0; i < run.n; ++i) {
         const int t = j.runs.tok[run.start + i];
-        for (int a = tid; a < 2 * D + V; a += 256) {
-            const int c = channel(a);
-            float x = 0.0f;
-            for (int k = 0; k < K; ++k) x += j.conv_w[(size_t)c * K + k] * input(i - (K - 1) + k, c);
-            x = silu_f(x);
-            (a < D ? sq[a] : a < 2 * D ? sk[a - D] : sv[a - 2 * D]) = x;
+        if (forget) {
+            const float * row = j.proj + (size_t)t * j.ld;
+            for (int d = tid; d < D; d += 256) {
+                const Forget f(row[KC + h * D + d], j.lower[h * D + d]);
+                sq[d] = silu_f(row[h * D + d]);
+                sk[d] = f.write;
+                sg[d] = f.keep;
+            }
+            for (int c = tid; c < V; c += 256) sv[c] = row[2 * KC + h * V + c];
+        } else {
+            for (int a = tid; a < 2 * D + V; a += 256) {
+                const int c = channel(a);
+                float x = 0.0f;
+                for (int k = 0; k < K; ++k) x += j.conv_w[(size_t)c * K + k] * input(i - (K - 1) + k, c);
+                x = silu_f(x);
+                (a < D ? sq[a] : a < 2 * D ? sk[a - D] : sv[a - 2 * D]) = x;
+            }
+            for (int d = tid; d < D; d += 256) sg[d] = expf(log_decay(j, t, sh.rule == RULE_DELTA_HEADS ? h : h * D + d, rate));
         }
-        for (int d = tid; d < D; d += 256) sg[d] = expf(log_decay(j, t, h, d, rate));
         __syncthreads();
         if (wave < 3) {                                 // the squares of q and k, and their product
             const float * a = wave == 1 ? sk : sq, * b = wave == 0 ? sq : sk;
@@ -104,11 +130,11 @@ __global__ __launch_bounds__(256) void k_delta_scan(DeltaJob j, int below) {
             for (int d = lane; d < D; d += 64) x += a[d] * b[d];
             x = wave_sum(x);
             if (lane == 0) s_stat[wave] = x;
-        } else if (lane == 0) {
+        } else if (lane == 0 && !forget) {
             s_stat[3] = sigmoid_f(j.proj[(size_t)t * j.ld + C + h]);
         }
         __syncthreads();
-        const float inv_q = 1.0f / sqrtf((s_stat[0] + j.unit_eps) * (float)D), inv_k = 1.0f / sqrtf(s_stat[1] + j.unit_eps);
+        const float inv_q = forget ? 1.0f : 1.0f / sqrtf((s_stat[0] + j.unit_eps) * (float)D), inv_k = forget ? 1.0f : 1.0f / sqrtf(s_stat[1] + j.unit_eps);
         const float kq = s_stat[2] * inv_q * inv_k, beta = s_stat[3];
         for (int cb = 0; cb < n_blocks; ++cb) {
             const int c = cb * 4 * CG + 4 * cg;
@@ -139,7 +165,7 @@ __global__ __launch_bounds__(256) void k_delta_scan(DeltaJob j, int below) {
             read = red[parity][0][1][cg] + red[parity][1][1][cg] + red[parity][2][1][cg] + red[parity][3][1][cg];
             parity ^= 1;
             f4 u = {0, 0, 0, 0};
-            if (c < VP) u = beta * (*(const f4 *)(sv + c) - held * inv_k);
+            if (c < VP) u = forget ? *(const f4 *)(sv + c) : beta * (*(const f4 *)(sv + c) - held * inv_k);
             if (rg == 0 && c < VP) *(f4 *)(so + c) = read * inv_q + kq * u;
             const f4 w = u * inv_k;
 #pragma unroll
@@ -201,8 +227,15 @@ __device__ __forceinline__ float row_scan(float v) {
 // exponentiated as sums over a stretch of tokens, so nothing grows: inside a block pair by pair, between blocks from the
 // start of the one and to the end of the other. (1 + L)^-1 is applied by blocks of 16, whose own inverses are formed first.
 // Tokens past the run's end count as k = q = beta = 0 without decay, which changes nothing.
-template <int DT>
+// A decay per head comes out of the sums: products of k and q on the matrix instruction, then the factor of each pair, from sums in
+// double since differences of them are exponentiated. Under the forget rule u is v, and there is no L, W or U.
+template <int DT, int RULE> constexpr int chunk_lds_floats() {
+    constexpr int Dp = 16 * DT, rows = kChunk * (Dp + 4), pairs = kChunk * (kChunk + 4);
+    return rows + (RULE == RULE_DELTA_HEADS ? 0 : rows + 4 * Dp) + pairs + (RULE == RULE_FORGET ? 0 : pairs + kChunk * 20);
+}
+template <int DT, int RULE>
 __global__ __launch_bounds__(256) void k_delta_chunk(DeltaJob j, Chunks out) {
+    constexpr bool HEADS = RULE == RULE_DELTA_HEADS, FORGET = RULE == RULE_FORGET;
     constexpr int Dp = 16 * DT, LD = Dp + 4, LA = kChunk + 4;
     extern __shared__ __attribute__((aligned(16))) float sm[];
     const DeltaShape sh = j.sh;
@@ -212,21 +245,45 @@ __global__ __launch_bounds__(256) void k_delta_chunk(DeltaJob j, Chunks out) {
     const int cnt = min(kChunk, run.n - base);
     const int D = sh.dim, V = sh.vdim, C = sh.channels(), KC = sh.keys(), kv = h / (sh.heads / sh.kv_heads);
     const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, r16 = lane & 15, kg = lane >> 4;
-    float * sK = sm, * sP = sK + kChunk * LD, * sL = sP + kChunk * LD, * sA = sL + kChunk * LA, * sT = sA + kChunk * LA, * sInv = sT + 4 * Dp;
+    float * sK = sm, * sA = sK + kChunk * LD, * sP = sA + kChunk * LA, * sT = HEADS ? sP : sP + kChunk * LD;
+    float * sL = HEADS ? sT : sT + 4 * Dp, * sInv = sL + kChunk * LA;
     __shared__ float s_beta[kChunk];
     __shared__ int s_tok[kChunk];
     const int me = 16 * w + r16;                       // this lane's token
     const bool in = me < cnt;
     const int t = j.runs.tok[run.start + base + min(me, cnt - 1)];
-    const float beta = in ? sigmoid_f(j.proj[(size_t)t * j.ld + C + h]) : 0.0f;
-    if (kg == 0) {
+    const float beta = in && !FORGET ? sigmoid_f(j.proj[(size_t)t * j.ld + C + h]) : 0.0f;
+    if (!FORGET && kg == 0) {
         s_beta[me] = beta;
         s_tok[me] = t;
     }
-    f4 q[DT], k[DT], p[DT];
-    {
+    // a decay per head: lane s of every wave has the sum up to token s
+    double l_sum = 0.0;
+    if constexpr (HEADS) {
+        l_sum = lane < cnt ? (double)log_decay(j, j.runs.tok[run.start + base + lane], h, expf(j.A_log[h])) : 0.0;
+#pragma unroll
+        for (int o = 1; o < 64; o <<= 1) {
+            const double up = __shfl_up(l_sum, o, 64);
+            if (lane >= o) l_sum += up;
+        }
+    }
+    f4 q[DT], k[DT], p[HEADS ? 1 : DT];
+    if constexpr (FORGET) {
+        const float * row = j.proj + (size_t)t * j.ld + h * D;
+#pragma unroll
+        for (int e = 0; e < DT; ++e)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int d = 16 * e + 4 * kg + i;
+                const bool real = in && d < D;
+                const Forget f(real ? row[KC + d] : 0.0f, real ? j.lower[h * D + d] : 1.0f);
+                q[e][i] = real ? silu_f(row[d]) : 0.0f;
+                k[e][i] = f.write;
+                p[e][i] = real ? f.log_keep() : 0.0f;
+            }
+    } else {
         const float * row = j.qkv + (size_t)t * C + kv * D;
-        const float rate = expf(j.A_log[h]);
+        const float rate = HEADS ? 0.0f : expf(j.A_log[h]);
         float qq = 0.0f, kk = 0.0f;
 #pragma unroll
         for (int e = 0; e < DT; ++e)
@@ -236,7 +293,7 @@ __global__ __launch_bounds__(256) void k_delta_chunk(DeltaJob j, Chunks out) {
                 const bool real = in && d < D;
                 q[e][i] = real ? row[d] : 0.0f;
                 k[e][i] = real ? row[KC + d] : 0.0f;
-                p[e][i] = real ? log_decay(j, t, h, d, rate) : 0.0f;
+                if constexpr (!HEADS) p[e][i] = real ? log_decay(j, t, h * D + d, rate) : 0.0f;
                 qq += q[e][i] * q[e][i];
                 kk += k[e][i] * k[e][i];
             }
@@ -249,46 +306,78 @@ __global__ __launch_bounds__(256) void k_delta_chunk(DeltaJob j, Chunks out) {
         for (int e = 0; e < DT; ++e) {
             q[e] *= fq;
             k[e] *= fk;
+        }
+    }
+#pragma unroll
+    for (int e = 0; e < DT; ++e) {
+        *(f4 *)(sK + me * LD + 16 * e + 4 * kg) = k[e];
+        if constexpr (!HEADS) {
 #pragma unroll
             for (int i = 0; i < 4; ++i) p[e][i] = row_scan(p[e][i]);       // up to this token, from the start of the block
-            *(f4 *)(sK + me * LD + 16 * e + 4 * kg) = k[e];
             *(f4 *)(sP + me * LD + 16 * e + 4 * kg) = p[e];
             if (r16 == 15) *(f4 *)(sT + w * Dp + 16 * e + 4 * kg) = p[e];
         }
     }
     __syncthreads();
-    // the block with itself
-#pragma unroll 1
-    for (int s0 = 0; s0 < 16; s0 += 4) {
-        float kk[4] = {0, 0, 0, 0}, qk[4] = {0, 0, 0, 0};
+    if constexpr (HEADS) {
+        // the blocks up to this one
+        for (int b = 0; b <= w; ++b) {
+            f4 kk = {0, 0, 0, 0}, qk = {0, 0, 0, 0};
 #pragma unroll
-        for (int e = 0; e < DT; ++e)
-#pragma unroll
-            for (int s = 0; s < 4; ++s) {
-                const f4 ks = *(const f4 *)(sK + (16 * w + s0 + s) * LD + 16 * e + 4 * kg), ps = *(const f4 *)(sP + (16 * w + s0 + s) * LD + 16 * e + 4 * kg);
+            for (int e = 0; e < DT; ++e) {
+                const f4 x = *(const f4 *)(sK + (16 * b + r16) * LD + 16 * e + 4 * kg);
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
-                    const float x = ks[i] * __expf(fminf(p[e][i] - ps[i], 0.0f));       // later tokens are left out below
-                    kk[s] += k[e][i] * x;
-                    qk[s] += q[e][i] * x;
+                    kk = __builtin_amdgcn_mfma_f32_16x16x4f32(k[e][i], x[i], kk, 0, 0, 0);
+                    qk = __builtin_amdgcn_mfma_f32_16x16x4f32(q[e][i], x[i], qk, 0, 0, 0);
                 }
             }
+            const int s = 16 * b + r16;
+            const double ls = __shfl(l_sum, s, 64);
 #pragma unroll
-        for (int s = 0; s < 4; ++s) {
-            kk[s] += __shfl_xor(kk[s], 16, 64);
-            kk[s] += __shfl_xor(kk[s], 32, 64);
-            qk[s] += __shfl_xor(qk[s], 16, 64);
-            qk[s] += __shfl_xor(qk[s], 32, 64);
+            for (int i = 0; i < 4; ++i) {
+                const int r = 16 * w + 4 * kg + i;
+                const float f = expf(fminf((float)(__shfl(l_sum, r, 64) - ls), 0.0f));
+                sL[r * LA + s] = s < r ? s_beta[r] * kk[i] * f : 0.0f;
+                sA[r * LA + s] = s <= r ? qk[i] * f : 0.0f;
+            }
         }
-        if (kg == 0) {
-            const int s = s0;
-            *(f4 *)(sL + me * LA + 16 * w + s) = f4{s < r16 ? beta * kk[0] : 0.0f, s + 1 < r16 ? beta * kk[1] : 0.0f, s + 2 < r16 ? beta * kk[2] : 0.0f, s + 3 < r16 ? beta * kk[3] : 0.0f};
-            *(f4 *)(sA + me * LA + 16 * w + s) = f4{s <= r16 ? qk[0] : 0.0f, s + 1 <= r16 ? qk[1] : 0.0f, s + 2 <= r16 ? qk[2] : 0.0f, s + 3 <= r16 ? qk[3] : 0.0f};
+    } else {
+        // the block with itself
+#pragma unroll 1
+        for (int s0 = 0; s0 < 16; s0 += 4) {
+            float kk[4] = {0, 0, 0, 0}, qk[4] = {0, 0, 0, 0};
+#pragma unroll
+            for (int e = 0; e < DT; ++e)
+#pragma unroll
+                for (int s = 0; s < 4; ++s) {
+                    const f4 ks = *(const f4 *)(sK + (16 * w + s0 + s) * LD + 16 * e + 4 * kg), ps = *(const f4 *)(sP + (16 * w + s0 + s) * LD + 16 * e + 4 * kg);
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) {
+                        const float x = ks[i] * __expf(fminf(p[e][i] - ps[i], 0.0f));       // later tokens are left out below
+                        if constexpr (!FORGET) kk[s] += k[e][i] * x;
+                        qk[s] += q[e][i] * x;
+                    }
+                }
+#pragma unroll
+            for (int s = 0; s < 4; ++s) {
+                if constexpr (!FORGET) {
+                    kk[s] += __shfl_xor(kk[s], 16, 64);
+                    kk[s] += __shfl_xor(kk[s], 32, 64);
+                }
+                qk[s] += __shfl_xor(qk[s], 16, 64);
+                qk[s] += __shfl_xor(qk[s], 32, 64);
+            }
+            if (kg == 0) {
+                const int s = s0;
+                if constexpr (!FORGET) *(f4 *)(sL + me * LA + 16 * w + s) = f4{s < r16 ? beta * kk[0] : 0.0f, s + 1 < r16 ? beta * kk[1] : 0.0f, s + 2 < r16 ? beta * kk[2] : 0.0f, s + 3 < r16 ? beta * kk[3] : 0.0f};
+                *(f4 *)(sA + me * LA + 16 * w + s) = f4{s <= r16 ? qk[0] : 0.0f, s + 1 <= r16 ? qk[1] : 0.0f, s + 2 <= r16 ? qk[2] : 0.0f, s + 3 <= r16 ? qk[3] : 0.0f};
+            }
         }
     }
     __syncthreads();
     // the block's own inverse, column r16 per lane
-    {
+    if constexpr (!FORGET) {
         float x[16];
 #pragma unroll
         for (int r = 0; r < 16; ++r) {
@@ -307,68 +396,84 @@ __global__ __launch_bounds__(256) void k_delta_chunk(DeltaJob j, Chunks out) {
     }
     // from the start of the chunk, to its end, and within the block; what other blocks need of this one
     const size_t at = out.row(h, run.start + base + me) * Dp;
-#pragma unroll
-    for (int e = 0; e < DT; ++e) {
-        const int c = 16 * e + 4 * kg;
-        f4 before = {0, 0, 0, 0}, after = {0, 0, 0, 0};
-        for (int b = 0; b < w; ++b) before += *(const f4 *)(sT + b * Dp + c);
-        for (int b = w + 1; b < 4; ++b) after += *(const f4 *)(sT + b * Dp + c);
-        const f4 own = *(const f4 *)(sT + w * Dp + c);
-        f4 ke, qe, kr, kl;
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const float from = __expf(p[e][i]), f = __expf(before[i]), r = __expf(own[i] - p[e][i]);
-            ke[i] = beta * k[e][i] * from * f;
-            qe[i] = q[e][i] * from * f;
-            kr[i] = k[e][i] * r;
-            kl[i] = kr[i] * __expf(after[i]);
-            k[e][i] *= from;
-            q[e][i] *= from;
-        }
-        *(f4 *)(sK + me * LD + c) = ke;
-        *(f4 *)(sP + me * LD + c) = kr;
-        if (in) {
-            *(f4 *)(out.q + at + c) = qe;
-            *(f4 *)(out.k + at + c) = kl;
-        }
-        if (w == 0 && r16 == 0) {
-            f4 l;
-#pragma unroll
-            for (int i = 0; i < 4; ++i) l[i] = __expf(own[i] + after[i]);
-            *(f4 *)(out.last_of(h, blockIdx.z, run.start, blockIdx.x) + c) = l;
-        }
-    }
-    __syncthreads();
-    // with the blocks before it
-    for (int b = 0; b < w; ++b) {
-        f4 kk = {0, 0, 0, 0}, qk = {0, 0, 0, 0};
+    if constexpr (HEADS) {
+        const double l = __shfl(l_sum, me, 64), end = __shfl(l_sum, 63, 64);
+        const float from = expf((float)l), to = expf((float)(end - l)), all = expf((float)end);
 #pragma unroll
         for (int e = 0; e < DT; ++e) {
             const int c = 16 * e + 4 * kg;
-            f4 x = *(const f4 *)(sP + (16 * b + r16) * LD + c);
-            if (b + 1 < w) {
-                f4 between = {0, 0, 0, 0};
-                for (int m = b + 1; m < w; ++m) between += *(const f4 *)(sT + m * Dp + c);
+            *(f4 *)(sK + me * LD + c) = k[e] * (beta * from);
+            if (in) {
+                *(f4 *)(out.q + at + c) = q[e] * from;
+                *(f4 *)(out.k + at + c) = k[e] * to;
+            }
+            if (w == 0 && r16 == 0) *(f4 *)(out.last_of(h, blockIdx.z, run.start, blockIdx.x) + c) = f4{all, all, all, all};
+        }
+        __syncthreads();
+    } else {
 #pragma unroll
-                for (int i = 0; i < 4; ++i) x[i] *= __expf(between[i]);
+        for (int e = 0; e < DT; ++e) {
+            const int c = 16 * e + 4 * kg;
+            f4 before = {0, 0, 0, 0}, after = {0, 0, 0, 0};
+            for (int b = 0; b < w; ++b) before += *(const f4 *)(sT + b * Dp + c);
+            for (int b = w + 1; b < 4; ++b) after += *(const f4 *)(sT + b * Dp + c);
+            const f4 own = *(const f4 *)(sT + w * Dp + c);
+            f4 ke, qe, kr, kl;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const float from = __expf(p[e][i]), f = __expf(before[i]), r = __expf(own[i] - p[e][i]);
+                ke[i] = beta * k[e][i] * from * f;
+                qe[i] = q[e][i] * from * f;
+                kr[i] = k[e][i] * r;
+                kl[i] = kr[i] * __expf(after[i]);
+                k[e][i] *= from;
+                q[e][i] *= from;
+            }
+            if constexpr (!FORGET) *(f4 *)(sK + me * LD + c) = ke;
+            *(f4 *)(sP + me * LD + c) = kr;
+            if (in) {
+                *(f4 *)(out.q + at + c) = qe;
+                *(f4 *)(out.k + at + c) = kl;
+            }
+            if (w == 0 && r16 == 0) {
+                f4 l;
+#pragma unroll
+                for (int i = 0; i < 4; ++i) l[i] = __expf(own[i] + after[i]);
+                *(f4 *)(out.last_of(h, blockIdx.z, run.start, blockIdx.x) + c) = l;
+            }
+        }
+        __syncthreads();
+        // with the blocks before it
+        for (int b = 0; b < w; ++b) {
+            f4 kk = {0, 0, 0, 0}, qk = {0, 0, 0, 0};
+#pragma unroll
+            for (int e = 0; e < DT; ++e) {
+                const int c = 16 * e + 4 * kg;
+                f4 x = *(const f4 *)(sP + (16 * b + r16) * LD + c);
+                if (b + 1 < w) {
+                    f4 between = {0, 0, 0, 0};
+                    for (int m = b + 1; m < w; ++m) between += *(const f4 *)(sT + m * Dp + c);
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) x[i] *= __expf(between[i]);
+                }
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    if constexpr (!FORGET) kk = __builtin_amdgcn_mfma_f32_16x16x4f32(k[e][i], x[i], kk, 0, 0, 0);
+                    qk = __builtin_amdgcn_mfma_f32_16x16x4f32(q[e][i], x[i], qk, 0, 0, 0);
+                }
             }
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
-                kk = __builtin_amdgcn_mfma_f32_16x16x4f32(k[e][i], x[i], kk, 0, 0, 0);
-                qk = __builtin_amdgcn_mfma_f32_16x16x4f32(q[e][i], x[i], qk, 0, 0, 0);
+                const int r = 16 * w + 4 * kg + i;
+                if constexpr (!FORGET) sL[r * LA + 16 * b + r16] = s_beta[r] * kk[i];
+                sA[r * LA + 16 * b + r16] = qk[i];
             }
         }
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int r = 16 * w + 4 * kg + i;
-            sL[r * LA + 16 * b + r16] = s_beta[r] * kk[i];
-            sA[r * LA + 16 * b + r16] = qk[i];
-        }
+        __syncthreads();
     }
-    __syncthreads();
     // W and U, a tile of 16 columns at a time: block i of the solution is T_ii (Y_i - sum over b < i of L_ib X_b); a product's
     // result (rows 4 kg + i in register i) is the next one's operand with its K in that order
-    const int n_tiles = DT + out.Vp / 16;
+    const int n_tiles = FORGET ? 0 : DT + out.Vp / 16;
     for (int n = w; n < n_tiles; n += 4) {
         f4 X[4];
         const int c = (n < DT ? n : n - DT) * 16 + r16;
@@ -409,7 +514,8 @@ __global__ __launch_bounds__(256) void k_delta_chunk(DeltaJob j, Chunks out) {
 
 // The chunks of a run one after the other, for kWalkCols columns of one head's state. Wave w owns token block w of a chunk
 // and rows w, w + 4 (in tiles of 16) of the state. The rows of the next chunk are requested as soon as a chunk's were used.
-template <int DT>
+// DELTA: u = U - W S; otherwise u = v, as projected.
+template <int DT, bool DELTA>
 __global__ __launch_bounds__(256) void k_delta_walk(DeltaJob j, Chunks in, int col_blocks) {
     constexpr int Dp = 16 * DT, NT = (DT + 3) / 4, LS = kWalkCols + 4;
     __shared__ __attribute__((aligned(16))) float sS[Dp * LS], sU[kChunk * LS];
@@ -432,26 +538,37 @@ __global__ __launch_bounds__(256) void k_delta_walk(DeltaJob j, Chunks in, int c
                 const int n = (w + 4 * d) * 16 + 4 * kg + i, p = c * 16 + r16;
                 S[d][c][i] = n < D && p0 + p < V && !(run.flags & 1) ? st[(size_t)n * VP + p] : 0.0f;
             }
-    f4 rw[DT], rq[DT], ra[4], ru[2], rk[NT][4], rl[NT];
+    f4 rw[DELTA ? DT : 1], rq[DT], ra[4], ru[2], rk[NT][4], rl[NT];
+    int v_tok[4];                                // tokens of the lane's values in the chunk that is fetched next
+    auto fetch_tokens = [&](int base) {
+        if constexpr (!DELTA)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) v_tok[i] = j.runs.tok[run.start + min(base + t0 + 4 * kg + i, run.n - 1)];
+    };
     auto fetch_first = [&](int base) {          // what the first products of the chunk at base read
         const int cnt = min(kChunk, run.n - base);
         const bool mine = t0 + r16 < cnt;
         const size_t at = in.row(h, run.start + base + min(t0 + r16, cnt - 1)) * Dp + 4 * kg;
 #pragma unroll
         for (int e = 0; e < DT; ++e) {
-            rw[e] = *(const f4 *)(in.w + at + 16 * e);
+            if constexpr (DELTA) rw[e] = *(const f4 *)(in.w + at + 16 * e);
             rq[e] = *(const f4 *)(in.q + at + 16 * e);
         }
         if (!mine)
 #pragma unroll
-            for (int e = 0; e < DT; ++e) rw[e] = rq[e] = f4{0, 0, 0, 0};
+            for (int e = 0; e < DT; ++e) {
+                rq[e] = f4{0, 0, 0, 0};
+                if constexpr (DELTA) rw[e] = f4{0, 0, 0, 0};
+            }
 #pragma unroll
         for (int c = 0; c < 2; ++c)
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int r = t0 + 4 * kg + i, p = p0 + c * 16 + r16;
-                ru[c][i] = r < cnt && p < in.Vp ? in.u[in.row(h, run.start + base + r) * in.Vp + p] : 0.0f;
+                if constexpr (DELTA) ru[c][i] = r < cnt && p < in.Vp ? in.u[in.row(h, run.start + base + r) * in.Vp + p] : 0.0f;
+                else ru[c][i] = r < cnt && p < V ? j.proj[(size_t)v_tok[i] * j.ld + 2 * sh.keys() + h * V + p] : 0.0f;
             }
+        fetch_tokens(base + kChunk);
     };
     auto fetch_second = [&](int base) {
         const int cnt = min(kChunk, run.n - base);
@@ -473,6 +590,7 @@ __global__ __launch_bounds__(256) void k_delta_walk(DeltaJob j, Chunks in, int c
                 }
         }
     };
+    fetch_tokens(0);
     fetch_first(0);
     fetch_second(0);
     for (int base = 0; base < run.n; base += kChunk) {
@@ -494,7 +612,7 @@ __global__ __launch_bounds__(256) void k_delta_walk(DeltaJob j, Chunks in, int c
 #pragma unroll
                 for (int c = 0; c < 2; ++c) {
                     const float s = sS[(16 * e + 4 * kg + i) * LS + c * 16 + r16];
-                    u[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(-rw[e][i], s, u[c], 0, 0, 0);
+                    if constexpr (DELTA) u[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(-rw[e][i], s, u[c], 0, 0, 0);
                     o[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(rq[e][i], s, o[c], 0, 0, 0);
                 }
         if (base + kChunk < run.n) fetch_first(base + kChunk);
@@ -607,18 +725,28 @@ Chunks chunks_of(const DeltaShape & sh, int T, int n_runs, float * base) {
     return c;
 }
 
-template <int DT> void launch_chunks(hipStream_t s, const DeltaJob & j, const Chunks & c) {
+template <int DT, int RULE> void launch_chunks(hipStream_t s, const DeltaJob & j, const Chunks & c) {
     const DeltaShape & sh = j.sh;
-    constexpr int Dp = 16 * DT;
-    constexpr int lds = (2 * kChunk * (Dp + 4) + 2 * kChunk * (kChunk + 4) + 4 * Dp + kChunk * 20) * 4;
-    static const bool allowed = hipFuncSetAttribute((const void *)k_delta_chunk<DT>, hipFuncAttributeMaxDynamicSharedMemorySize, lds) == hipSuccess;
-    if (!allowed) throw std::runtime_error("delta rule: a chunk does not fit the LDS");
+    constexpr int lds = chunk_lds_floats<DT, RULE>() * 4;
+    static const bool allowed = hipFuncSetAttribute((const void *)k_delta_chunk<DT, RULE>, hipFuncAttributeMaxDynamicSharedMemorySize, lds) == hipSuccess;
+    if (!allowed) throw std::runtime_error("matrix states: a chunk does not fit the LDS");
     const unsigned n_chunks = (unsigned)((j.runs.longest + kChunk - 1) / kChunk);
-    hipLaunchKernelGGL(k_delta_chunk<DT>, dim3(n_chunks, (unsigned)sh.heads, (unsigned)j.runs.n), dim3(256), lds, s, j, c);
+    hipLaunchKernelGGL((k_delta_chunk<DT, RULE>), dim3(n_chunks, (unsigned)sh.heads, (unsigned)j.runs.n), dim3(256), lds, s, j, c);
     check_launch("delta_chunk");
     const int blocks = (sh.vdim + kWalkCols - 1) / kWalkCols;
-    hipLaunchKernelGGL(k_delta_walk<DT>, dim3((unsigned)((sh.heads + 7) / 8 * 8 * blocks), (unsigned)j.runs.n), dim3(256), 0, s, j, c, blocks);
+    hipLaunchKernelGGL((k_delta_walk<DT, RULE != RULE_FORGET>), dim3((unsigned)((sh.heads + 7) / 8 * 8 * blocks), (unsigned)j.runs.n), dim3(256), 0, s, j, c, blocks);
     check_launch("delta_walk");
+}
+
+template <int RULE> void launch_chunks(hipStream_t s, const DeltaJob & j, const Chunks & c) {
+    switch (chunk_tiles(j.sh.dim)) {
+        case 1: launch_chunks<1, RULE>(s, j, c); break;
+        case 2: launch_chunks<2, RULE>(s, j, c); break;
+        case 3: launch_chunks<3, RULE>(s, j, c); break;
+        case 4: launch_chunks<4, RULE>(s, j, c); break;
+        case 6: launch_chunks<6, RULE>(s, j, c); break;
+        default: launch_chunks<8, RULE>(s, j, c); break;
+    }
 }
 
 template <int ARITH, int CG, int NPT> void launch_scan(hipStream_t s, const DeltaJob & j, int below) {
@@ -654,25 +782,24 @@ size_t delta_chunk_floats(const DeltaShape & sh, int T, int n_runs) {
 void delta_mix(hipStream_t s, int arith, const DeltaJob & j, int T) {
     if (j.runs.n <= 0 || T <= 0) return;
     const DeltaShape & sh = j.sh;
-    if (sh.dim > 32 * kScanRows || sh.vdim > 4096) throw std::runtime_error("delta rule: at most 512 key and 4096 value channels per head");
+    if (sh.dim > 32 * kScanRows || sh.vdim > 4096) throw std::runtime_error("matrix states: at most 512 key and 4096 value channels per head");
     const int least = in_chunks(sh) ? kLongRun : INT_MAX;
     if (j.runs.longest >= least) {
-        ShortConv conv;
-        conv.runs = j.runs;
-        conv.channels = sh.channels(); conv.taps = sh.taps; conv.least = least;
-        conv.in = j.proj; conv.ld = j.ld;
-        conv.w = j.conv_w;
-        conv.state = j.conv_state; conv.plane = j.conv_plane;
-        conv.out = j.qkv;
-        short_conv(s, conv);
+        if (sh.rule != RULE_FORGET) {
+            ShortConv conv;
+            conv.runs = j.runs;
+            conv.channels = sh.channels(); conv.taps = sh.taps; conv.least = least;
+            conv.in = j.proj; conv.ld = j.ld;
+            conv.w = j.conv_w;
+            conv.state = j.conv_state; conv.plane = j.conv_plane;
+            conv.out = j.qkv;
+            short_conv(s, conv);
+        }
         const Chunks c = chunks_of(sh, T, j.runs.n, j.chunks);
-        switch (chunk_tiles(sh.dim)) {
-            case 1: launch_chunks<1>(s, j, c); break;
-            case 2: launch_chunks<2>(s, j, c); break;
-            case 3: launch_chunks<3>(s, j, c); break;
-            case 4: launch_chunks<4>(s, j, c); break;
-            case 6: launch_chunks<6>(s, j, c); break;
-            default: launch_chunks<8>(s, j, c); break;
+        switch (sh.rule) {
+            case RULE_DELTA_CHANNELS: launch_chunks<RULE_DELTA_CHANNELS>(s, j, c); break;
+            case RULE_DELTA_HEADS: launch_chunks<RULE_DELTA_HEADS>(s, j, c); break;
+            default: launch_chunks<RULE_FORGET>(s, j, c); break;
         }
         int lanes = 1;
         while (lanes < 64 && 8 * lanes < sh.vdim) lanes *= 2;

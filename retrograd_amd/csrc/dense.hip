@@ -40,6 +40,22 @@ template <bool GROUPED> __device__ __forceinline__ int row_of(const DenseArgs & 
 template <int ARITH> __device__ __forceinline__ void store_rotary(const DenseOut & o, int t, int n, f4 v) {
     using EL = typename std::conditional<ARITH == ARITH_16, __half, float>::type;
     const RotaryOut & r = o.rot;
+    auto put = [](EL * dst, const f4 & u) {
+        if constexpr (ARITH == ARITH_16) {
+            union { __half h[4]; uint2 w; } p;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) p.h[i] = sat_half(u[i]);
+            *(uint2 *)dst = p.w;
+        } else {
+            *(f4 *)dst = u;
+        }
+    };
+    const int own = n - (r.H + r.G) * r.kf * 32;         // column of the values' own rows
+    if (own >= 0) {
+        const int cell = r.cell[t];
+        put((EL *)r.v_pool + (size_t)(cell / PAGE) * cache_page_elems(r.vf * r.G) + cache_at(cell % PAGE, own), v);
+        return;
+    }
     const int head = n / (r.kf * 32), c = n - head * r.kf * 32;
     f4 y = v;
 #pragma unroll
@@ -51,23 +67,13 @@ template <int ARITH> __device__ __forceinline__ void store_rotary(const DenseOut
             y[2 * i + 1] = v[2 * i + 1] * cs.x + v[2 * i] * cs.y;
         }
     }
-    auto put = [](EL * dst, const f4 & u) {
-        if constexpr (ARITH == ARITH_16) {
-            union { __half h[4]; uint2 w; } p;
-#pragma unroll
-            for (int i = 0; i < 4; ++i) p.h[i] = sat_half(u[i]);
-            *(uint2 *)dst = p.w;
-        } else {
-            *(f4 *)dst = u;
-        }
-    };
     if (head < r.H) {
         put((EL *)o.dst + ((size_t)t * r.H + head) * (r.kf * 32) + c, y);
     } else {
         const int cell = r.cell[t];
         const size_t at = (size_t)(cell / PAGE) * cache_page_elems(r.kf * r.G) + cache_at(cell % PAGE, (head - r.H) * r.kf * 32 + c);
         put((EL *)r.k_pool + at, y);
-        put((EL *)r.v_pool + at, v);
+        if (r.vf == 0) put((EL *)r.v_pool + at, v);
     }
 }
 
@@ -184,11 +190,16 @@ __device__ __forceinline__ void store_expert(const DenseArgs & A, int t, int n, 
     const int cnt = A.j.w.n - n;
     if (cnt <= 0) return;
     const int pair = A.groups.slot_pair[t], token = pair / A.groups.top, choice = pair - token * A.groups.top;
-    v *= A.groups.weight[pair];
+    if (!A.groups.weigh_input) v *= A.groups.weight[pair];
     float * y = (float *)o.dst + (size_t)choice * o.stride + (size_t)token * o.ld + n;
     if (cnt >= 4 && (o.ld & 3) == 0) *(f4 *)y = v;
     else
         for (int i = 0; i < 4 && i < cnt; ++i) y[i] = v[i];
+}
+
+// What an expert's input rows are multiplied with, for the pair in slot t.
+__device__ __forceinline__ float input_weight(const DenseArgs & A, int t) {
+    return A.groups.weigh_input ? A.groups.weight[A.groups.slot_pair[t]] : 1.0f;
 }
 
 // K-slice `ks` of rows n .. n + 3 of token t; `add`: to what is there.
@@ -380,7 +391,13 @@ __global__ __launch_bounds__(64 * KW * RW) void k_dense(DenseArgs A) {
             } else if (DUAL && A.partial) {
                 store_slice(A, ks, t, tile * 16 + 4 * (lane >> 4), acc[r][c], false);
             } else {
-                store_rows<KA, KB, ARITH>(j, t, GROUPED ? 0 : b, tile, lane >> 4, acc[r][c], acc[RT > 1 ? r ^ 1 : r][c]);
+                f4 v = acc[r][c], next = acc[RT > 1 ? r ^ 1 : r][c];
+                if constexpr (GROUPED) {
+                    const float f = input_weight(A, t);
+                    v *= f;
+                    next *= f;
+                }
+                store_rows<KA, KB, ARITH>(j, t, GROUPED ? 0 : b, tile, lane >> 4, v, next);
             }
         }
     }
@@ -520,7 +537,13 @@ __global__ __launch_bounds__(256, 2) void k_dense_lds(DenseArgs A, int n_tok_blo
                 } else if (DUAL && A.partial) {
                     store_slice(A, ks, t, tile * 16 + 4 * (lane >> 4), v, !first);
                 } else {
-                    store_rows<KA, KB, ARITH_16>(j, t, 0, tile, lane >> 4, v, acc[r ^ 1][c]);
+                    f4 next = acc[r ^ 1][c];
+                    if constexpr (GROUPED) {
+                        const float w = input_weight(A, t);
+                        v *= w;
+                        next *= w;
+                    }
+                    store_rows<KA, KB, ARITH_16>(j, t, 0, tile, lane >> 4, v, next);
                 }
             }
         }
@@ -696,6 +719,7 @@ Slices dense(hipStream_t s, int arith, const DenseJob & job, int T, float * ws) 
         else if (job.a.kind == OUT_F32 && job.b.kind == OUT_ACT_SWIGLU) out = run<OUT_F32, OUT_ACT_SWIGLU>(s, arith, A, ws);
         else if (job.a.kind == OUT_F32 && job.b.kind == OUT_ACT_CLAMPED) out = run<OUT_F32, OUT_ACT_CLAMPED>(s, arith, A, ws);
         else if (job.a.kind == OUT_F32 && job.b.kind == OUT_ACT) out = run<OUT_F32, OUT_ACT>(s, arith, A, ws);
+        else if (job.a.kind == OUT_ROTARY && job.b.kind == OUT_F32) out = run<OUT_ROTARY, OUT_F32>(s, arith, A, ws);
         else throw std::runtime_error("dense: this pair of outputs is not compiled");
     } else {
         switch (job.a.kind) {

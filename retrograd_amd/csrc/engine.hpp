@@ -88,17 +88,19 @@ struct LayerWeights {
 struct StackLayer {
     struct Matrix { rk::DenseWeight w; DevBuf buf; };
     LayerSpec spec;
-    DevBuf norm, norm2, scale_mix, scale_ff;
+    DevBuf norm, norm2, scale_mix, scale_ff;      // the scales of a product's two halves along K
+    DevBuf after[2], taps[2];               // of the mixer and the feed-forward: the norm behind it, the convolution of its input
     DevBuf hyper[2];                        // of the mixer and the feed-forward: what they read of the residual streams and write to them
     Matrix w_in, w_out, ff_in, ff_out;
-    DevBuf in_bias, ff_in_bias, ff_out_bias;
+    DevBuf in_bias, out_bias, ff_in_bias, ff_out_bias;
     int in_tiles = 0, in_rows = 0;          // row tiles and rows of w_in that belong to the mixer
     int route_tiles = 0;                    // row tiles of ff_in that belong to the router
-    int kv_col = 0, gate_col = 0;           // columns of the input product: the latent, the head gates
-    int k_col = 0, v_col = 0;               // ... of grouped attention's own keys and values
+    int kv_col = 0, gate_col = 0;           // columns of the input product: the latent, the gates
+    int k_col = 0, v_col = 0;               // ... grouped attention's keys and values
+    int decay_col = 0;                      // ... a decay per head
     DevBuf q_norm, kv_norm, v_share;
     Matrix uq, uk, uv;                      // queries from their latent; per head: absorption and value up-projection
-    DevBuf conv_w, conv_b, dt_bias, A_log, D, gate_norm;
+    DevBuf conv_w, conv_b, dt_bias, A_log, D, lower, gate_norm;
     Matrix low;                             // the delta rule's decays and gates from their inner widths (low_frags fragments each)
     int low_frags = 0;
     int rotary = -1;                        // index of the layer's rotary table
@@ -109,12 +111,19 @@ struct StackLayer {
 struct StackRun {
     int layer = 0, pool = 0;                // the run whose pools are attended to
     bool add_embedding = false;
-    float * conv_state = nullptr, * state = nullptr;       // the run's part of the recurrent state
-    size_t conv_slot = 0, state_slot = 0;   // floats per slot (a plane of the convolution inputs holds every slot)
+    float * conv_state = nullptr, * state = nullptr;       // the run's parts of the recurrent state
+    float * history[2] = {};                // inputs of the mixer and the feed-forward that their convolutions remember
+};
+
+// A part of the recurrent state: floats per slot at base[slot], or in two planes of which a slot's current one counts.
+struct StatePart {
+    float ** base;
+    size_t slot;
+    bool planes;
 };
 
 struct Slot {
-    int plane = 0;                  // recurrent models: the plane that holds the slot's convolution inputs
+    int plane = 0;                  // recurrent models: the plane that holds the slot's convolution inputs and last token
     int begin = 0, end = 0;         // resident positions [begin, end)
     std::vector<int32_t> pages;     // page id per page index (position / PAGE), -1 = none
 };
@@ -301,9 +310,10 @@ private:
     void build_stack();
     void forward_stack(int T, int n_out);
     void mix_latent(const StackLayer & L, const StackRun & run, int T);
-    void mix_mamba(const StackLayer & L, const StackRun & run, int T);
+    void mix_mamba(const StackLayer & L, const StackRun & run, int T, void * out);
     void mix_attention(const StackLayer & L, const StackRun & run, int T);
     void mix_delta(const StackLayer & L, const StackRun & run, int T);
+    rk::SublayerNorm around(float * x, const DevBuf * after, const rk::Slices & add) const;
     rk::SeqRuns step_runs() const;
     void attend(rk::StackAttn & at, int T);
     rk::Slices stack_feed_forward(const StackLayer & L, int T);
@@ -360,8 +370,12 @@ private:
     bool looped_ = false;
     size_t moe_ws_floats_ = 0;
     DevBuf recurrent_slab_;
+    std::vector<StatePart> state_parts_;
     size_t recurrent_slot_floats_ = 0, conv_plane_floats_ = 0;
+    DevBuf pair_embd_, embed_norm_;         // the embedding of neighbouring tokens; the norm of the sum
+    float * last_token_ = nullptr;          // of every slot, in two planes
     DevBuf st_h_, st_proj_, st_cq_, st_q_, st_qa_, st_ol_, st_mix_, st_ff_, st_out_, st_partial_, st_xbc_, st_y_;
+    DevBuf st_beside_, st_in_rows_;         // Mamba-2 beside attention; a sublayer's input rows before their convolution
     DevBuf st_first_, st_low_, st_decay_, st_chunks_;      // values of the first layer that mixes them; the delta rule's
     DevBuf st_embed_, st_rows_, st_route_, ex_sel_, ex_weight_, ex_slot_, ex_tiles_, ex_h_;
     int st_proj_ld_ = 0;

@@ -64,6 +64,21 @@ public:
         }
         upload(all, out);
     }
+    // Raw rows that are gathered.
+    void table(const std::string & name, int rows, int cols, DevBuf & out) {
+        const StTensor & t = file_.require(name, {rows, cols});
+        if (t.dtype != "BF16") throw std::runtime_error("tensor " + name + " must be BF16");
+        out.alloc(t.nbytes);
+        hip_check(hipMemcpy(out.ptr, t.data, t.nbytes, hipMemcpyHostToDevice), "hipMemcpy");
+    }
+    // Taps [channels][taps] of a convolution, tap by tap.
+    void taps(const std::string & name, int channels, int taps, DevBuf & out) {
+        const std::vector<float> v = floats(name, {channels, taps});
+        std::vector<float> w(v.size());
+        for (int c = 0; c < channels; ++c)
+            for (int j = 0; j < taps; ++j) w[(size_t)j * channels + c] = v[(size_t)c * taps + j];
+        upload(w, out);
+    }
     // Biases of a matrix's rows, each tensor at its rows' places.
     void biases(const StackLayer::Matrix & m, const std::vector<std::tuple<std::string, int, rk::PackMap>> & parts, DevBuf & out) {
         std::vector<float> all((size_t)m.w.batch * m.w.tiles * 16, 0.0f);
@@ -111,12 +126,20 @@ public:
     static rk::PackMap gate_row(int tile0 = 0) { return {tile0 * 16, 16, 32}; }
     static rk::PackMap up_row(int tile0 = 0) { return {tile0 * 16 + 16, 16, 32}; }
     static int gated_rows(int ff) { return 2 * up16(ff); }
-    // The rows of `heads` heads, every head from a multiple of `padded` rows on, the columns of a rotated pair (i and i + rotated / 2) side by side.
-    void heads(const std::string & name, int heads, int dim, int padded, int rotated, int cols, StackLayer::Matrix & m, int head0) {
+    // The rows of `heads` heads from row0 on, every head padded, the columns of a rotated pair (i and i + rotated / 2) side by side.
+    void heads(const std::string & name, int heads, int dim, int padded, int rotated, int cols, StackLayer::Matrix & m, int row0) {
         const uint16_t * src = raw(name, heads * dim, cols);
         for (int h = 0; h < heads; ++h)
             each_part(dim, rotated, [&](int from, int n, int to, int step) {
-                rk::dense_pack(stream_, src + ((size_t)h * dim + from) * cols, n, cols, cols, 1, m.buf.as<uint16_t>(), m.w.kf, {(head0 + h) * padded + to, 1, step}, 0);
+                rk::dense_pack(stream_, src + ((size_t)h * dim + from) * cols, n, cols, cols, 1, m.buf.as<uint16_t>(), m.w.kf, {row0 + h * padded + to, 1, step}, 0);
+            });
+    }
+    // ... and their biases.
+    void head_biases(const std::string & name, int heads, int dim, int padded, int rotated, int row0, std::vector<float> & all) {
+        const std::vector<float> v = floats(name, {heads * dim});
+        for (int h = 0; h < heads; ++h)
+            each_part(dim, rotated, [&](int from, int n, int to, int step) {
+                for (int i = 0; i < n; ++i) all[(size_t)(row0 + h * padded + to + i * step)] = v[(size_t)(h * dim + from + i)];
             });
     }
     // ... and the columns of a matrix that reads them.
@@ -160,19 +183,18 @@ void Engine::load_stack(const std::string & path) {
     hp_.eps = c.eps;
     const int E = c.width, KE = rk::frags_of(E);
 
-    const StTensor & emb = file.require("embed", {c.vocab, E});
-    if (emb.dtype != "BF16") throw std::runtime_error("tensor embed must be BF16");
+    ld.table("embed", c.vocab, E, tok_embd_.buf);
     tok_embd_.w.type = rk::WT_BF16;
     tok_embd_.w.K = E;
     tok_embd_.w.N = c.vocab;
-    tok_embd_.w.bytes = emb.nbytes;
-    tok_embd_.buf.alloc(emb.nbytes);
-    hip_check(hipMemcpy(tok_embd_.buf.ptr, emb.data, emb.nbytes, hipMemcpyHostToDevice), "hipMemcpy");
+    tok_embd_.w.bytes = tok_embd_.buf.bytes;
     tok_embd_.w.raw = tok_embd_.buf.as<uint8_t>();
+    if (c.arch->norm_after) ld.table("bigram", (int)c.pair_buckets + 1, E, pair_embd_);
     ld.shape(stack_head_, c.vocab, KE);
     ld.matrix(c.arch->own_head ? "head" : "embed", c.vocab, E, stack_head_);
     const float norm_plus = c.arch->norm_around_one ? 1.0f : 0.0f;
     ld.vector("final.norm", {E}, out_norm_, norm_plus);
+    if (c.arch->norm_after) ld.vector("embed.norm", {E}, embed_norm_);
 
     stack_layers_.resize(c.layers.size());
     for (size_t l = 0; l < c.layers.size(); ++l) {
@@ -182,13 +204,18 @@ void Engine::load_stack(const std::string & path) {
         const std::string p = "l" + std::to_string(l) + ".", m = p + "mix.";
         const bool parallel = c.arch->parallel;
         if (parallel && sp.moe.experts > 0) throw std::runtime_error("experts in parallel layers are not supported");
-        if (parallel && sp.mixer == Mixer::CHANNEL_DELTA) throw std::runtime_error("channel_delta in parallel layers is not supported");
+        if (parallel && sp.mixer == Mixer::DELTA) throw std::runtime_error("matrix states in parallel layers are not supported");
         for (int q = 0; q < (sp.has_ff() ? 2 : 1) && c.streams > 0; ++q) {
             const std::string hc = p + (q == 0 ? "hc1." : "hc2.");
             ld.vectors({{hc + "in", {c.streams}}, {hc + "out", {c.streams}}, {hc + "mix", {c.streams, c.streams}}}, L.hyper[q]);
         }
         ld.vector(p + "norm1", {E}, L.norm, norm_plus);
         if (!parallel && sp.has_ff()) ld.vector(p + "norm2", {E}, L.norm2, norm_plus);
+        for (int q = 0; q < (sp.has_ff() ? 2 : 1); ++q) {
+            const std::string n = std::to_string(q + 1);
+            if (c.arch->norm_after) ld.vector(p + "norm" + n + "b", {E}, L.after[q], norm_plus);
+            if (c.input_taps > 0) ld.taps(p + "canon" + n, E, c.input_taps, L.taps[q]);
+        }
         if (c.arch->layer_scale) {
             ld.vector(p + "ls1", {E}, L.scale_mix);
             if (sp.ff > 0) ld.vector(p + "ls2", {E}, L.scale_ff);
@@ -198,20 +225,30 @@ void Engine::load_stack(const std::string & path) {
         const AttentionSpec & ga = sp.attention;
         const rk::PairFrags head = ga.frags();
         rk::DeltaShape & ds = L.spec.delta;
-        const bool own_values = sp.mixer == Mixer::ATTENTION && !c.arch->keys_are_values;
+        const bool own_values = !c.arch->keys_are_values, in_place = c.arch->rows_in_place();
+        const int rotated = c.arch->pairs == Pairs::HALVES ? ga.rot.dims : 0;      // columns of a head whose pairs are brought together
         int beside = parallel ? sp.ff : 0;              // rows behind the mixer's that go elsewhere
         if (sp.mixer == Mixer::LATENT_ATTENTION) {
             const bool own = a.kv_from < 0;
             L.kv_col = up16(a.q_rank);
             L.gate_col = L.kv_col + (own ? up16(a.kv_rank) : 0);
             L.in_rows = L.gate_col + a.heads;
-        } else if (own_values) {
+        } else if (sp.grouped_attention() && in_place) {
+            L.k_col = ga.heads * head.k * 32;
+            L.v_col = L.k_col + ga.kv_heads * head.k * 32;
+            L.in_rows = L.v_col + (own_values ? ga.kv_heads * head.v * 32 : 0);
+            if (sp.mixer == Mixer::ATTENTION_MAMBA2) beside = sp.mamba.rows();
+        } else if (sp.grouped_attention()) {
             L.k_col = up16(ga.heads * ga.dim);
             L.v_col = L.k_col + up16(ga.kv_heads * ga.dim);
             L.in_rows = L.v_col + ga.kv_heads * ga.vdim;
-        } else if (sp.mixer == Mixer::ATTENTION) {
-            L.in_rows = (ga.heads + ga.kv_heads) * head.k * 32;
-        } else if (sp.mixer == Mixer::CHANNEL_DELTA) {
+        } else if (sp.mixer == Mixer::DELTA && ds.rule == rk::RULE_FORGET) {
+            L.in_rows = ds.channels();
+        } else if (sp.mixer == Mixer::DELTA && ds.rule == rk::RULE_DELTA_HEADS) {
+            L.decay_col = ds.channels() + ds.heads;
+            L.gate_col = L.decay_col + ds.heads;
+            L.in_rows = L.gate_col + ds.inner();
+        } else if (sp.mixer == Mixer::DELTA) {
             ds.decay_rank = ld.rows_of(m + "a1", E);
             ds.gate_rank = ld.rows_of(m + "g1", E);
             L.low_frags = std::max(rk::frags_of(ds.decay_rank), rk::frags_of(ds.gate_rank));
@@ -224,9 +261,22 @@ void Engine::load_stack(const std::string & path) {
         ld.shape(L.w_in, beside > 0 ? L.in_tiles * 16 + beside : L.in_rows, KE);
         if (parallel && beside > 0) ld.matrix(p + "mlp.up", beside, E, L.w_in, L.in_tiles * 16);
         const int mix = sp.mix_width(), KM = rk::frags_of(mix);
-        ld.shape(L.w_out, E, KM + (parallel && beside > 0 ? rk::frags_of(beside) : 0));
-        if (sp.mixer == Mixer::ATTENTION) ld.from_heads(m + "o", E, ga.heads, ga.vdim, head.v * 32, own_values ? 0 : ga.rot.dims, L.w_out);
+        const bool two = sp.mixer == Mixer::ATTENTION_MAMBA2;
+        const std::string am = m + (two ? "left." : ""), sm = m + (two ? "right." : "");      // attention's tensors, Mamba-2's
+        ld.shape(L.w_out, E, KM + rk::frags_of(parallel ? beside : sp.beside_width()));
+        if (sp.grouped_attention()) ld.from_heads(am + "o", E, ga.heads, ga.vdim, head.v * 32, own_values ? 0 : rotated, L.w_out);
         else ld.matrix(m + "o", E, mix, L.w_out);
+        if (two) {
+            ld.matrix(sm + "o", E, sp.beside_width(), L.w_out, 0, KM * 32);
+            Loader::upload(std::vector<float>((size_t)E, sp.left_scale), L.scale_mix);
+            Loader::upload(std::vector<float>((size_t)E, sp.right_scale), L.scale_ff);
+        }
+        if (sp.grouped_attention() && c.arch->out_bias) {
+            std::vector<float> b((size_t)L.w_out.w.tiles * 16, 0.0f);
+            ld.head_biases(am + "o.b", 1, E, 0, 0, 0, b);
+            for (float & x : b) x *= sp.left_scale;
+            Loader::upload(b, L.out_bias);
+        }
         if (parallel && beside > 0) ld.matrix(p + "mlp.down", E, beside, L.w_out, 0, KM * 32);
         if (!parallel && sp.ff > 0) {
             if (rk::out_is_glu(c.arch->ff_act)) {
@@ -290,8 +340,8 @@ void Engine::load_stack(const std::string & path) {
             const size_t uv_head = rk::frag_weight_elems(L.uv.w.tiles, L.uv.w.kf);
             for (int h = 0; h < a.heads; ++h)
                 rk::dense_pack(stream_, uv + (size_t)h * a.vdim * a.kv_rank, a.vdim, a.kv_rank, a.kv_rank, 1, L.uv.buf.as<uint16_t>() + h * uv_head, L.uv.w.kf, 0, 0);
-        } else if (sp.mixer == Mixer::ATTENTION) {
-            if (own_values) {
+        } else if (sp.grouped_attention()) {
+            if (!in_place) {
                 const int nq = ga.heads * ga.dim, nk = ga.kv_heads * ga.dim, nv = ga.kv_heads * ga.vdim;
                 ld.matrix(m + "q", nq, E, L.w_in);
                 ld.matrix(m + "k", nk, E, L.w_in, L.k_col);
@@ -301,8 +351,16 @@ void Engine::load_stack(const std::string & path) {
                 ld.vector(m + "k.norm", {nk}, L.kv_norm);
                 if (ga.v_mix && !ga.v_first) ld.vector(m + "vmix", {}, L.v_share);
             } else {
-                ld.heads(m + "q", ga.heads, ga.dim, head.k * 32, ga.rot.dims, E, L.w_in, 0);
-                ld.heads(m + "k", ga.kv_heads, ga.dim, head.k * 32, ga.rot.dims, E, L.w_in, ga.heads);
+                ld.heads(am + "q", ga.heads, ga.dim, head.k * 32, rotated, E, L.w_in, 0);
+                ld.heads(am + "k", ga.kv_heads, ga.dim, head.k * 32, rotated, E, L.w_in, L.k_col);
+                if (own_values) {
+                    ld.heads(am + "v", ga.kv_heads, ga.vdim, head.v * 32, 0, E, L.w_in, L.v_col);
+                    std::vector<float> b((size_t)L.w_in.w.tiles * 16, 0.0f);
+                    ld.head_biases(am + "q.b", ga.heads, ga.dim, head.k * 32, rotated, 0, b);
+                    ld.head_biases(am + "k.b", ga.kv_heads, ga.dim, head.k * 32, rotated, L.k_col, b);
+                    ld.head_biases(am + "v.b", ga.kv_heads, ga.vdim, head.v * 32, 0, L.v_col, b);
+                    Loader::upload(b, L.in_bias);
+                }
             }
             for (size_t r = 0; r < rotary_.size(); ++r) if (rotary_[r].spec == ga.rot) L.rotary = (int)r;
             if (L.rotary < 0) {
@@ -314,7 +372,27 @@ void Engine::load_stack(const std::string & path) {
                 t.freq.alloc(f.size() * sizeof(double));
                 if (!f.empty()) hip_check(hipMemcpy(t.freq.ptr, f.data(), t.freq.bytes, hipMemcpyHostToDevice), "hipMemcpy");
             }
-        } else if (sp.mixer == Mixer::CHANNEL_DELTA) {
+        } else if (sp.mixer == Mixer::DELTA && ds.rule == rk::RULE_FORGET) {
+            ld.matrix(m + "q", ds.keys(), E, L.w_in);
+            ld.matrix(m + "f", ds.keys(), E, L.w_in, ds.keys());
+            ld.matrix(m + "v", ds.inner(), E, L.w_in, 2 * ds.keys());
+            ld.biases(L.w_in, {{m + "f.b", ds.keys(), ds.keys()}}, L.in_bias);
+            const std::vector<float> lower = ld.floats(m + "lower", {ds.keys()});
+            for (float x : lower) if (!(x >= 0.0f && x <= 1.0f)) throw std::runtime_error("tensor " + m + "lower must lie between 0 and 1");
+            Loader::upload(lower, L.lower);
+            ld.vector(m + "norm", {ds.vdim}, L.gate_norm);
+        } else if (sp.mixer == Mixer::DELTA && ds.rule == rk::RULE_DELTA_HEADS) {
+            ld.matrix(m + "q", ds.keys(), E, L.w_in);
+            ld.matrix(m + "k", ds.keys(), E, L.w_in, ds.keys());
+            ld.matrix(m + "v", ds.inner(), E, L.w_in, 2 * ds.keys());
+            ld.matrix(m + "b", ds.heads, E, L.w_in, ds.channels());
+            ld.matrix(m + "a", ds.heads, E, L.w_in, L.decay_col);
+            ld.matrix(m + "g", ds.inner(), E, L.w_in, L.gate_col);
+            ld.vectors({{m + "q.conv", {ds.keys(), ds.taps}}, {m + "k.conv", {ds.keys(), ds.taps}}, {m + "v.conv", {ds.inner(), ds.taps}}}, L.conv_w);
+            ld.vector(m + "dt_bias", {ds.heads}, L.dt_bias);
+            ld.vector(m + "A_log", {ds.heads}, L.A_log);
+            ld.vector(m + "norm", {ds.vdim}, L.gate_norm);
+        } else if (sp.mixer == Mixer::DELTA) {
             const int at_a = L.in_tiles * 16, decays = ds.heads * ds.dim, gates = ds.inner();
             ld.matrix(m + "q", ds.keys(), E, L.w_in);
             ld.matrix(m + "k", ds.keys(), E, L.w_in, ds.keys());
@@ -329,15 +407,16 @@ void Engine::load_stack(const std::string & path) {
             ld.vector(m + "dt_bias", {decays}, L.dt_bias);
             ld.vector(m + "A_log", {ds.heads}, L.A_log);
             ld.vector(m + "norm", {ds.vdim}, L.gate_norm);
-        } else {
+        }
+        if (sp.state_space()) {
             const rk::MambaShape & s = sp.mamba;
-            ld.matrix(m + "in", s.rows(), E, L.w_in);
-            ld.vector(m + "conv", {s.channels(), s.taps}, L.conv_w);
-            ld.vector(m + "conv.b", {s.channels()}, L.conv_b);
-            ld.vector(m + "dt_bias", {s.heads}, L.dt_bias);
-            ld.vector(m + "A_log", {s.heads}, L.A_log);
-            ld.vector(m + "D", {s.heads}, L.D);
-            ld.vector(m + "norm", {s.inner()}, L.gate_norm);
+            ld.matrix(sm + "in", s.rows(), E, L.w_in, two ? L.in_tiles * 16 : 0);
+            ld.vector(sm + "conv", {s.channels(), s.taps}, L.conv_w);
+            ld.vector(sm + "conv.b", {s.channels()}, L.conv_b);
+            ld.vector(sm + "dt_bias", {s.heads}, L.dt_bias);
+            ld.vector(sm + "A_log", {s.heads}, L.A_log);
+            ld.vector(sm + "D", {s.heads}, L.D);
+            ld.vector(sm + "norm", {s.inner()}, L.gate_norm);
         }
     }
     ld.finish();
@@ -386,7 +465,7 @@ void Engine::build_stack() {
         if (sp.mixer == Mixer::LATENT_ATTENTION) {
             if (sp.latent.kv_from >= 0) R.pool = last[(size_t)sp.latent.kv_from];
             else pool(r, false, rk::cache_frags(sp.latent.kv_rank));
-        } else if (sp.mixer == Mixer::ATTENTION) {
+        } else if (sp.grouped_attention()) {
             const rk::PairFrags f = sp.attention.frags();
             for (int v = 0; v < 2; ++v) pool(r, v != 0, sp.attention.kv_heads * (v ? f.v : f.k));
         }
@@ -396,29 +475,39 @@ void Engine::build_stack() {
     for (size_t i = 0; i < pools.size(); ++i)
         if (pools[i].bytes) (i & 1 ? v_pool_ : k_pool_)[i / 2] = PoolView{(uint8_t *)kv_slab_.ptr + pools[i].at, pools[i].bytes};
 
-    // recurrent state: [run][slot] states, then two planes of [run][slot] convolution inputs
-    size_t states = 0;
+    // recurrent state: states [part][slot], then two planes of what convolutions and embeddings remember [part][slot], each
+    // part from a multiple of four floats on
+    auto part = [&](float * & base, size_t slot, bool planes) {
+        if (slot > 0) state_parts_.push_back({&base, slot, planes});
+    };
     for (StackRun & R : stack_runs_) {
         const LayerSpec & sp = c.layers[(size_t)R.layer];
-        if (!sp.recurrent()) continue;
         const rk::MambaShape & s = sp.mamba;
         const rk::DeltaShape & d = sp.delta;
-        const bool delta = sp.mixer == Mixer::CHANNEL_DELTA;
-        R.state_slot = delta ? d.state_floats() : (size_t)s.heads * s.state * s.vdim;
-        R.conv_slot = delta ? (size_t)(d.taps - 1) * d.channels() : (size_t)(s.taps - 1) * s.channels();
-        states += R.state_slot * n_slots;
-        conv_plane_floats_ += R.conv_slot * n_slots;
-        recurrent_slot_floats_ += R.state_slot + R.conv_slot;
+        if (sp.mixer == Mixer::DELTA) {
+            part(R.state, d.state_floats(), false);
+            part(R.conv_state, (size_t)(d.taps - 1) * d.channels(), true);
+        } else if (sp.state_space()) {
+            part(R.state, (size_t)s.heads * s.state * s.vdim, false);
+            part(R.conv_state, (size_t)(s.taps - 1) * s.channels(), true);
+        }
+        for (int q = 0; q < (sp.has_ff() ? 2 : 1) && c.input_taps > 0; ++q) part(R.history[q], (size_t)(c.input_taps - 1) * E, true);
+    }
+    if (c.arch->norm_after) part(last_token_, 1, true);
+    auto held = [&](const StatePart & p) { return (p.slot * n_slots + 3) / 4 * 4; };
+    size_t states = 0;
+    for (const StatePart & p : state_parts_) {
+        (p.planes ? conv_plane_floats_ : states) += held(p);
+        recurrent_slot_floats_ += p.slot;
     }
     recurrent_slab_.alloc((states + 2 * conv_plane_floats_) * 4);
     if (recurrent_slab_.ptr) {
         hip_check(hipMemsetAsync(recurrent_slab_.ptr, 0, recurrent_slab_.bytes, stream_), "hipMemsetAsync");
         float * st = recurrent_slab_.as<float>(), * cv = st + states;
-        for (StackRun & R : stack_runs_) {
-            R.state = st;
-            R.conv_state = cv;
-            st += R.state_slot * n_slots;
-            cv += R.conv_slot * n_slots;
+        for (const StatePart & p : state_parts_) {
+            float * & at = p.planes ? cv : st;
+            *p.base = at;
+            at += held(p);
         }
     }
 
@@ -433,7 +522,7 @@ void Engine::build_stack() {
         b.alloc(n);
         if (n) hip_check(hipMemsetAsync(b.ptr, 0, n, stream_), "hipMemsetAsync");
     };
-    size_t route = 0, pairs = 0, slots = 0, tiles = 0, expert_h = 0, first = 0, low = 0, decay = 0, chunks = 0;
+    size_t route = 0, pairs = 0, slots = 0, tiles = 0, expert_h = 0, first = 0, low = 0, decay = 0, chunks = 0, beside = 0;
     for (const StackLayer & L : stack_layers_) {
         const LayerSpec & sp = L.spec;
         mix = std::max(mix, rk::frag_elems(B, rk::frags_of(sp.mix_width())));
@@ -444,20 +533,24 @@ void Engine::build_stack() {
             q = std::max(q, rk::frag_elems(B, a.heads * rk::frags_of(a.dim)));
             qa = std::max(qa, (size_t)B * a.heads * 32 * rk::cache_frags(a.kv_rank));
             ol = std::max(ol, rk::frag_elems(B, a.heads * rk::cache_frags(a.kv_rank)));
-        } else if (sp.mixer == Mixer::ATTENTION) {
+        } else if (sp.grouped_attention()) {
             const AttentionSpec & a = sp.attention;
             qa = std::max(qa, (size_t)B * a.heads * 32 * a.frags().k);
             if (a.v_mix) first = std::max(first, (size_t)B * a.kv_heads * a.vdim);
-        } else if (sp.mixer == Mixer::CHANNEL_DELTA) {
+        } else if (sp.mixer == Mixer::DELTA) {
             const rk::DeltaShape & d = sp.delta;
             xbc = std::max(xbc, (size_t)B * d.channels());
             y = std::max(y, (size_t)B * d.inner());
-            low = std::max(low, rk::frag_elems(B, 2 * L.low_frags));
-            decay = std::max(decay, (size_t)B * 2 * up16(L.low.w.n));
+            if (d.rule == rk::RULE_DELTA_CHANNELS) {
+                low = std::max(low, rk::frag_elems(B, 2 * L.low_frags));
+                decay = std::max(decay, (size_t)B * 2 * up16(L.low.w.n));
+            }
             chunks = std::max(chunks, rk::delta_chunk_floats(d, B, n_slots));
-        } else {
+        }
+        if (sp.state_space()) {
             xbc = std::max(xbc, (size_t)B * sp.mamba.channels());
             y = std::max(y, (size_t)B * sp.mamba.inner());
+            if (sp.beside_width() > 0) beside = std::max(beside, rk::frag_elems(B, rk::frags_of(sp.beside_width())));
         }
         if (sp.moe.experts > 0) {
             const MoeSpec & e = sp.moe;
@@ -471,8 +564,8 @@ void Engine::build_stack() {
             moe_ws_floats_ = std::max(moe_ws_floats_, (size_t)B * E * e.top);
         }
     }
-    for (const StackLayer & L : stack_layers_)
-        if (L.spec.mixer != Mixer::ATTENTION || !c.arch->keys_are_values) st_proj_ld_ = std::max(st_proj_ld_, L.in_tiles * 16);      // grouped attention's rows go to their places at once
+    for (const StackLayer & L : stack_layers_)        // what of the input product does not go to its place at once
+        st_proj_ld_ = std::max(st_proj_ld_, !L.spec.grouped_attention() || !c.arch->rows_in_place() ? L.in_tiles * 16 : (L.w_in.w.tiles - L.in_tiles) * 16);
     for (RotaryTable & t : rotary_) t.table.alloc((size_t)B * t.spec.dims * 4);
     if (looped_) st_embed_.alloc((size_t)B * E * 4);
     if (route) zeroed(st_rows_, (size_t)B * rk::frags_of(E) * 32 * elem);
@@ -483,6 +576,8 @@ void Engine::build_stack() {
     if (tiles) ex_tiles_.alloc((tiles + 1) * 16);           // the count behind the tiles
     x_.alloc((size_t)B * E * 4 * std::max(c.streams, 1));
     st_first_.alloc(first * 4);
+    zeroed(st_beside_, beside * elem);
+    if (c.input_taps > 0) st_in_rows_.alloc((size_t)B * E * 4);
     zeroed(st_low_, low * elem);
     zeroed(st_decay_, decay * 4);
     st_chunks_.alloc(chunks * 4);
@@ -498,46 +593,32 @@ void Engine::build_stack() {
     zeroed(st_xbc_, xbc * 4);
     zeroed(st_y_, y * 4);
     zeroed(ex_h_, expert_h * elem);
-    mm_ws_.alloc((std::max(rk::dense_workspace_floats(), c.streams > 0 ? (size_t)B * E : 0) + moe_ws_floats_) * 4);
+    mm_ws_.alloc((std::max(rk::dense_workspace_floats(), c.streams > 0 || c.around() ? (size_t)B * E : 0) + moe_ws_floats_) * 4);
 }
 
 // ---- recurrent state of a slot --------------------------------------------------------------------
 
 void Engine::state_copy(int32_t src, int32_t dst) {
-    const Slot & a = slots_[(size_t)src];
-    Slot & b = slots_[(size_t)dst];
-    b.plane = 0;
-    for (const StackRun & L : stack_runs_) {
-        if (L.state_slot == 0) continue;
-        rk::copy_floats(stream_, L.state + src * L.state_slot, L.state + dst * L.state_slot, L.state_slot);
-        rk::copy_floats(stream_, L.conv_state + a.plane * conv_plane_floats_ + src * L.conv_slot, L.conv_state + dst * L.conv_slot, L.conv_slot);
-    }
+    const int plane = slots_[(size_t)src].plane;
+    slots_[(size_t)dst].plane = 0;
+    for (const StatePart & p : state_parts_)
+        rk::copy_floats(stream_, *p.base + (p.planes ? plane * conv_plane_floats_ : 0) + src * p.slot, *p.base + dst * p.slot, p.slot);
 }
 
 void Engine::state_pack(int32_t slot, float * out) {
     const int plane = slots_[(size_t)slot].plane;
-    auto get = [&](const float * src, size_t n) {
-        if (n) hip_check(hipMemcpyAsync(out, src, n * 4, hipMemcpyDeviceToHost, stream_), "hipMemcpyAsync");
-        out += n;
-    };
-    for (const StackRun & L : stack_runs_) {
-        if (L.state_slot == 0) continue;
-        get(L.state + slot * L.state_slot, L.state_slot);
-        get(L.conv_state + plane * conv_plane_floats_ + slot * L.conv_slot, L.conv_slot);
+    for (const StatePart & p : state_parts_) {
+        hip_check(hipMemcpyAsync(out, *p.base + (p.planes ? plane * conv_plane_floats_ : 0) + slot * p.slot, p.slot * 4, hipMemcpyDeviceToHost, stream_), "hipMemcpyAsync");
+        out += p.slot;
     }
     hip_check(hipStreamSynchronize(stream_), "seq_save");
 }
 
 void Engine::state_unpack(int32_t slot, const float * in) {
     slots_[(size_t)slot].plane = 0;
-    auto put = [&](float * dst, size_t n) {
-        if (n) hip_check(hipMemcpyAsync(dst, in, n * 4, hipMemcpyHostToDevice, stream_), "hipMemcpyAsync");
-        in += n;
-    };
-    for (const StackRun & L : stack_runs_) {
-        if (L.state_slot == 0) continue;
-        put(L.state + slot * L.state_slot, L.state_slot);
-        put(L.conv_state + slot * L.conv_slot, L.conv_slot);
+    for (const StatePart & p : state_parts_) {
+        hip_check(hipMemcpyAsync(*p.base + slot * p.slot, in, p.slot * 4, hipMemcpyHostToDevice, stream_), "hipMemcpyAsync");
+        in += p.slot;
     }
     hip_check(hipStreamSynchronize(stream_), "seq_load");
 }
@@ -556,8 +637,8 @@ void Engine::plan_stack(const std::vector<RowView> & rows, const std::vector<std
     int total = 0;
     for (const RowView & r : rows) total += (int)r.n;
     for (const LayerSpec & sp : stack_->layers) {
-        if (sp.recurrent()) continue;
-        const bool pair = sp.mixer == Mixer::ATTENTION;
+        if (!sp.attends()) continue;
+        const bool pair = sp.grouped_attention();
         const int H = pair ? sp.attention.heads / sp.attention.kv_heads : sp.latent.heads, R = rk::cache_frags(std::max(sp.latent.kv_rank, 1));
         const rk::PairFrags f = pair ? sp.attention.frags() : rk::PairFrags{R, R};
         const int cols = rk::stack_block_cols(arith_, H, f.k, f.v, pair, total, (int)rows.size());
@@ -579,7 +660,7 @@ void Engine::plan_stack(const std::vector<RowView> & rows, const std::vector<std
             Slot & s = slots_[(size_t)r.slot];
             const bool fresh = before[(size_t)r.slot].second <= before[(size_t)r.slot].first;
             plan_runs_.push_back({r.slot, 0, 0, (fresh ? 1 : 0) | (s.plane << 1)});
-            s.plane = 1 - s.plane;            // this step leaves the convolution inputs in the other plane
+            s.plane = 1 - s.plane;            // this step leaves what the next one remembers in the other plane
             toks.emplace_back();
         }
         for (uint32_t i = 0; i < r.n; ++i) toks[(size_t)k].push_back(at + (int32_t)i);
@@ -679,7 +760,7 @@ void Engine::mix_latent(const StackLayer & L, const StackRun & run, int T) {
     prof_end(PC_OPROJ, pt);
 }
 
-void Engine::mix_mamba(const StackLayer & L, const StackRun & run, int T) {
+void Engine::mix_mamba(const StackLayer & L, const StackRun & run, int T, void * out) {
     const size_t pt = prof_begin(PC_SCAN);
     rk::MambaJob j;
     j.sh = L.spec.mamba;
@@ -690,7 +771,7 @@ void Engine::mix_mamba(const StackLayer & L, const StackRun & run, int T) {
     j.runs = step_runs();
     j.conv_state = run.conv_state; j.conv_plane = conv_plane_floats_; j.state = run.state;
     j.xbc = st_xbc_.as<float>(); j.y = st_y_.as<float>();
-    j.out = st_mix_.ptr; j.out_kf = rk::frags_of(L.spec.mix_width());
+    j.out = out; j.out_kf = rk::frags_of(L.spec.mamba.inner());
     rk::mamba_mix(stream_, arith_, j, T);
     prof_end(PC_SCAN, pt);
 }
@@ -701,24 +782,29 @@ rk::SeqRuns Engine::step_runs() const {
     return r;
 }
 
-// The input product has left queries, keys, values and write strengths as f32 rows, the inner columns of decays and gates as
-// activations.
+// The input product has left queries, keys, values and write strengths as f32 rows, decays and gates behind them, or the inner
+// columns of decays and gates as activations.
 void Engine::mix_delta(const StackLayer & L, const StackRun & run, int T) {
     const rk::DeltaShape & sh = L.spec.delta;
-    const int half = up16(L.low.w.n);
-    size_t pt = prof_begin(PC_LOW_RANK);
-    rk::DenseJob low;
-    low.w = L.low.w;
-    low.x = {st_low_.ptr, 2 * L.low_frags, L.low_frags};
-    low.a.kind = rk::OUT_F32; low.a.dst = st_decay_.ptr; low.a.ld = 2 * half; low.a.col_batch = half;
-    rk::dense(stream_, arith_, low, T, nullptr);
-    prof_end(PC_LOW_RANK, pt);
-    pt = prof_begin(PC_SCAN);
     rk::DeltaJob j;
     j.sh = sh;
     j.proj = st_proj_.as<float>(); j.ld = st_proj_ld_;
-    j.decay = st_decay_.as<float>(); j.gate = j.decay + half; j.ld_low = 2 * half;
-    j.conv_w = L.conv_w.as<float>(); j.A_log = L.A_log.as<float>(); j.dt_bias = L.dt_bias.as<float>(); j.norm_w = L.gate_norm.as<float>();
+    if (sh.rule == rk::RULE_DELTA_CHANNELS) {
+        const size_t pt = prof_begin(PC_LOW_RANK);
+        const int half = up16(L.low.w.n);
+        rk::DenseJob low;
+        low.w = L.low.w;
+        low.x = {st_low_.ptr, 2 * L.low_frags, L.low_frags};
+        low.a.kind = rk::OUT_F32; low.a.dst = st_decay_.ptr; low.a.ld = 2 * half; low.a.col_batch = half;
+        rk::dense(stream_, arith_, low, T, nullptr);
+        j.decay = st_decay_.as<float>(); j.gate = j.decay + half; j.ld_low = 2 * half;
+        prof_end(PC_LOW_RANK, pt);
+    } else if (sh.rule == rk::RULE_DELTA_HEADS) {
+        j.decay = j.proj + L.decay_col; j.gate = j.proj + L.gate_col; j.ld_low = st_proj_ld_;
+    }
+    const size_t pt = prof_begin(PC_SCAN);
+    j.conv_w = L.conv_w.as<float>(); j.A_log = L.A_log.as<float>(); j.dt_bias = L.dt_bias.as<float>(); j.lower = L.lower.as<float>();
+    j.norm_w = L.gate_norm.as<float>();
     j.eps = stack_->eps; j.unit_eps = kUnitEps;
     j.runs = step_runs();
     j.conv_state = run.conv_state; j.conv_plane = conv_plane_floats_; j.state = run.state;
@@ -728,13 +814,13 @@ void Engine::mix_delta(const StackLayer & L, const StackRun & run, int T) {
     prof_end(PC_SCAN, pt);
 }
 
-// Grouped attention. Where the values are the keys the input product has already left queries, keys and values in their
-// places; own values come as f32 rows with queries and keys that are still to be normed.
+// Grouped attention. The input product has already left queries, keys and values in their places, unless queries and keys are
+// still to be normed: then all come as f32 rows.
 void Engine::mix_attention(const StackLayer & L, const StackRun & run, int T) {
     const AttentionSpec & a = L.spec.attention;
     const rk::PairFrags f = a.frags();
     void * keys = k_pool_[(size_t)run.pool].ptr, * values = v_pool_[(size_t)run.pool].ptr;
-    if (!stack_->arch->keys_are_values) {
+    if (!stack_->arch->rows_in_place()) {
         const size_t pt = prof_begin(PC_ROPE);
         const RotaryTable & t = rotary_[(size_t)L.rotary];
         rk::HeadRows r;
@@ -778,7 +864,7 @@ rk::Slices Engine::stack_feed_forward(const StackLayer & L, int T) {
     out.w = L.ff_out.w;
     out.x = {st_ff_.ptr, KF, 0};
     out.kf1 = KF;
-    out.a.kind = rk::OUT_RESIDUAL; out.a.dst = c.streams > 0 ? nullptr : x_.ptr; out.a.ld = E;
+    out.a.kind = rk::OUT_RESIDUAL; out.a.dst = c.streams > 0 || c.around() ? nullptr : x_.ptr; out.a.ld = E;
     out.bias = L.ff_out_bias.as<float>();
     const rk::Slices left = rk::dense(stream_, arith_, out, T, ws);
     prof_end(PC_DOWN, pt);
@@ -807,7 +893,7 @@ rk::Slices Engine::stack_experts(const StackLayer & L, int T) {
     rk::ExpertRoute r;
     r.logits = route; r.ld = ld; r.experts = e.experts; r.top = e.top;
     r.block = rk::expert_block(arith_, T, e.top, e.experts);
-    r.groups = e.groups; r.keep = e.keep; r.over_all = c.arch->route_over_all; r.scale = e.scale;
+    r.groups = e.groups; r.keep = e.keep; r.score = c.arch->score; r.scale = e.scale;
     r.sel = ex_sel_.as<int32_t>(); r.weight = ex_weight_.as<float>(); r.slot_pair = ex_slot_.as<int32_t>();
     r.tiles = ex_tiles_.as<int32_t>();
     r.n_tiles = r.tiles + (ex_tiles_.bytes / 16 - 1) * 4;
@@ -816,6 +902,7 @@ rk::Slices Engine::stack_experts(const StackLayer & L, int T) {
     rk::ExpertGroups g;
     g.tiles = r.tiles; g.n_tiles = r.n_tiles; g.block = r.block; g.max_tiles = rk::expert_max_tiles(T, e.top, e.experts, r.block);
     g.slot_pair = r.slot_pair; g.weight = r.weight; g.top = e.top; g.pairs = T * e.top;
+    g.weigh_input = c.arch->weigh_input;
     pt = prof_begin(PC_EXPERTS_IN);
     rk::DenseJob up;
     up.w = L.experts_in.w;
@@ -833,7 +920,7 @@ rk::Slices Engine::stack_experts(const StackLayer & L, int T) {
         out.w = L.ff_out.w;
         out.x = {st_ff_.ptr, KS, 0};
         out.kf1 = KS;
-        out.a.kind = rk::OUT_RESIDUAL; out.a.dst = c.streams > 0 ? nullptr : x_.ptr; out.a.ld = E;
+        out.a.kind = rk::OUT_RESIDUAL; out.a.dst = c.streams > 0 || c.around() ? nullptr : x_.ptr; out.a.ld = E;
         if (c.arch->shared_gate) { out.token_gate = route + e.experts; out.ld_token_gate = ld; }
         left = rk::dense(stream_, arith_, out, T, ws);
         prof_end(PC_SHARED, pt);
@@ -854,25 +941,68 @@ rk::Slices Engine::stack_experts(const StackLayer & L, int T) {
     return left;
 }
 
+// The norm of a sublayer's output into the stream x.
+rk::SublayerNorm Engine::around(float * x, const DevBuf * after, const rk::Slices & add) const {
+    rk::SublayerNorm n;
+    n.x = x; n.E = stack_->width; n.groups = stack_->norm_groups; n.eps = stack_->eps;
+    n.mult = stack_->residual_mult;
+    n.add = add;
+    n.after = after ? after->as<float>() : nullptr;
+    return n;
+}
+
 void Engine::forward_stack(int T, int n_out) {
     const StackConfig & c = *stack_;
     const int E = c.width, KE = rk::frags_of(E);
     float * x = x_.as<float>(), * ws = mm_ws_.as<float>();
     rk::Slices pending;                         // what the stream, or the streams by the weights `due`, have yet to take in
     const float * due = nullptr;
+    const DevBuf * due_norm = nullptr;          // the norm that `pending` goes through
     rk::Streams streams;
     streams.x = x; streams.n = c.streams; streams.stride = (size_t)cfg_.n_batch * E;
-    // the norm before a sublayer, which reads the streams by its weights `hyper`
-    auto norm = [&](const DevBuf & w, const DevBuf * hyper, const int32_t * rows, int n, void * act, const float * plus, void * act_rows) {
-        const size_t pt = prof_begin(rows ? PC_HEAD : PC_NORM);
-        if (c.streams > 0)
-            rk::streams_norm_act(stream_, arith_, streams, due, pending, hyper ? hyper->as<float>() : nullptr, w.as<float>(), E, c.eps, rows, n, act, KE, act_rows);
-        else
-            rk::norm_act(stream_, arith_, c.arch->norm, x, w.as<float>(), E, c.eps, rows, n, act, KE, pending, plus, act_rows);
-        prof_end(rows ? PC_HEAD : PC_NORM, pt);
+    // the norm before a sublayer: the mixer (0) or the feed-forward (1) of a run
+    auto norm = [&](const StackLayer & L, const StackRun & run, int q, const float * plus, void * act_rows) {
+        const size_t pt = prof_begin(PC_NORM);
+        const float * w = (q ? L.norm2 : L.norm).as<float>();
+        if (c.around()) {
+            rk::SublayerNorm n = around(x, due_norm, pending);
+            n.w = w;
+            n.act = st_h_.ptr; n.act_kf = KE; n.act_rows = act_rows;
+            if (c.input_taps > 0) {
+                n.taps = L.taps[q].as<float>(); n.n_taps = c.input_taps;
+                n.history = run.history[q]; n.plane = conv_plane_floats_;
+                n.runs = step_runs();
+                n.h = st_in_rows_.as<float>();
+            }
+            rk::sublayer_norm(stream_, arith_, n, T);
+        } else if (c.streams > 0) {
+            rk::streams_norm_act(stream_, arith_, streams, due, pending, L.hyper[q].as<float>(), w, E, c.eps, nullptr, T, st_h_.ptr, KE, act_rows);
+        } else {
+            rk::norm_act(stream_, arith_, c.arch->norm, x, w, E, c.eps, nullptr, T, st_h_.ptr, KE, pending, plus, act_rows);
+        }
+        prof_end(PC_NORM, pt);
+    };
+    // what the sublayer q of L has left
+    auto leave = [&](const StackLayer & L, int q, const rk::Slices & y) {
+        pending = y;
+        due = L.hyper[q].as<float>();
+        due_norm = c.arch->norm_after ? &L.after[q] : nullptr;
     };
     size_t pt = prof_begin(PC_EMBED);
-    rk::embed_rows(stream_, (const uint16_t *)tok_embd_.w.raw, pk_.tok, E, c.embedding_scale, T, x, std::max(c.streams, 1), streams.stride);
+    if (c.arch->norm_after) {
+        rk::PairEmbedding e;
+        e.embed = (const uint16_t *)tok_embd_.w.raw; e.pairs = pair_embd_.as<uint16_t>();
+        e.tok = pk_.tok; e.scale = c.embedding_scale;
+        e.buckets = c.pair_buckets; e.mul_prev = c.pair_mul_prev; e.mul_cur = c.pair_mul_cur;
+        e.w = embed_norm_.as<float>();
+        e.E = E; e.groups = c.norm_groups; e.eps = c.eps;
+        e.runs = step_runs();
+        e.last = last_token_; e.plane = conv_plane_floats_;
+        e.x = x;
+        rk::embed_pairs(stream_, e, T);
+    } else {
+        rk::embed_rows(stream_, (const uint16_t *)tok_embd_.w.raw, pk_.tok, E, c.embedding_scale, T, x, std::max(c.streams, 1), streams.stride);
+    }
     if (looped_) rk::copy_floats(stream_, x, st_embed_.as<float>(), (size_t)T * E);
     for (RotaryTable & t : rotary_)
         rk::rotary_table(stream_, t.freq.as<double>(), t.spec.dims / 2, t.spec.magnitude(), pk_.pos, T, t.table.as<float>());
@@ -886,7 +1016,7 @@ void Engine::forward_stack(int T, int n_out) {
         const StackLayer & L = stack_layers_[(size_t)run.layer];
         const LayerSpec & sp = L.spec;
         const bool beside = c.arch->parallel && sp.ff > 0;
-        norm(L.norm, &L.hyper[0], nullptr, T, st_h_.ptr, run.add_embedding ? st_embed_.as<float>() : nullptr, nullptr);
+        norm(L, run, 0, run.add_embedding ? st_embed_.as<float>() : nullptr, nullptr);
         pt = prof_begin(PC_QKV);
         rk::DenseJob in;
         in.w = L.w_in.w;
@@ -894,18 +1024,20 @@ void Engine::forward_stack(int T, int n_out) {
         in.split_tile = L.in_tiles;
         in.n_a = L.in_rows;
         in.bias = L.in_bias.as<float>();
-        if (sp.mixer == Mixer::ATTENTION && c.arch->keys_are_values) {
+        if (sp.grouped_attention() && c.arch->rows_in_place()) {
             const AttentionSpec & a = sp.attention;
             const RotaryTable & t = rotary_[(size_t)L.rotary];
             in.a.kind = rk::OUT_ROTARY; in.a.dst = st_qa_.ptr;
-            in.a.rot.H = a.heads; in.a.rot.G = a.kv_heads; in.a.rot.kf = a.frags().k; in.a.rot.pairs = t.spec.dims / 2;
+            in.a.rot.H = a.heads; in.a.rot.G = a.kv_heads; in.a.rot.kf = a.frags().k; in.a.rot.vf = c.arch->keys_are_values ? 0 : a.frags().v; in.a.rot.pairs = t.spec.dims / 2;
             in.a.rot.table = t.table.as<float>();
             in.a.rot.k_pool = k_pool_[(size_t)run.pool].ptr; in.a.rot.v_pool = v_pool_[(size_t)run.pool].ptr;
             in.a.rot.cell = pk_.cell;
         } else {
             in.a.kind = rk::OUT_F32; in.a.dst = st_proj_.ptr; in.a.ld = st_proj_ld_;
         }
-        if (sp.mixer == Mixer::CHANNEL_DELTA) {
+        if (sp.mixer == Mixer::ATTENTION_MAMBA2) {
+            in.b.kind = rk::OUT_F32; in.b.dst = st_proj_.ptr; in.b.ld = st_proj_ld_;
+        } else if (sp.mixer == Mixer::DELTA) {
             in.b.kind = rk::OUT_ACT; in.b.dst = st_low_.ptr; in.b.ld = 2 * L.low_frags;
         } else {
             in.b.kind = c.arch->ff_act; in.b.dst = st_ff_.ptr; in.b.ld = rk::frags_of(std::max(sp.ff, 1));
@@ -913,9 +1045,9 @@ void Engine::forward_stack(int T, int n_out) {
         rk::dense(stream_, arith_, in, T, ws);
         prof_end(PC_QKV, pt);
         if (sp.mixer == Mixer::LATENT_ATTENTION) mix_latent(L, run, T);
-        else if (sp.mixer == Mixer::ATTENTION) mix_attention(L, run, T);
-        else if (sp.mixer == Mixer::CHANNEL_DELTA) mix_delta(L, run, T);
-        else mix_mamba(L, run, T);
+        else if (sp.mixer == Mixer::DELTA) mix_delta(L, run, T);
+        else if (sp.grouped_attention()) mix_attention(L, run, T);
+        if (sp.state_space()) mix_mamba(L, run, T, sp.mixer == Mixer::MAMBA2 ? st_mix_.ptr : st_beside_.ptr);
         const int out_cat = c.arch->parallel ? PC_DOWN : PC_OPROJ, KM = rk::frags_of(sp.mix_width());
         pt = prof_begin(out_cat);
         rk::DenseJob out;
@@ -926,15 +1058,17 @@ void Engine::forward_stack(int T, int n_out) {
         if (beside) {
             out.x2 = {st_ff_.ptr, rk::frags_of(sp.ff), 0};
             out.scale2 = L.scale_ff.as<float>();
+        } else if (sp.mixer == Mixer::ATTENTION_MAMBA2) {
+            out.x2 = {st_beside_.ptr, rk::frags_of(sp.beside_width()), 0};
+            out.scale2 = L.scale_ff.as<float>();
         }
-        out.a.kind = rk::OUT_RESIDUAL; out.a.dst = c.streams > 0 ? nullptr : x; out.a.ld = E;
-        pending = rk::dense(stream_, arith_, out, T, ws);
-        due = L.hyper[0].as<float>();
+        out.bias = L.out_bias.as<float>();
+        out.a.kind = rk::OUT_RESIDUAL; out.a.dst = c.streams > 0 || c.around() ? nullptr : x; out.a.ld = E;
+        leave(L, 0, rk::dense(stream_, arith_, out, T, ws));
         prof_end(out_cat, pt);
         if (!c.arch->parallel && sp.has_ff()) {
-            norm(L.norm2, &L.hyper[1], nullptr, T, st_h_.ptr, nullptr, sp.moe.experts > 0 ? st_rows_.ptr : nullptr);
-            pending = stack_feed_forward(L, T);
-            due = L.hyper[1].as<float>();
+            norm(L, run, 1, nullptr, sp.moe.experts > 0 ? st_rows_.ptr : nullptr);
+            leave(L, 1, stack_feed_forward(L, T));
         }
         if (keep_residual_) {
             float * kept = kept_residual_.as<float>() + r * (size_t)cfg_.n_batch * E;
@@ -942,13 +1076,26 @@ void Engine::forward_stack(int T, int n_out) {
                 rk::streams_sum(stream_, streams, due, pending, E, T, kept);
             } else {
                 rk::copy_floats(stream_, x, kept, (size_t)T * E);
-                rk::add_slices(stream_, kept, E, T, pending);
+                if (c.around()) rk::sublayer_norm(stream_, arith_, around(kept, due_norm, pending), T);
+                else rk::add_slices(stream_, kept, E, T, pending);
             }
         }
     }
     if (n_out > 0) {
         logits_.ensure((size_t)n_out * c.vocab * 4);
-        norm(out_norm_, nullptr, pk_.out_tok, n_out, st_out_.ptr, nullptr, nullptr);
+        pt = prof_begin(PC_HEAD);
+        if (c.around()) {
+            rk::SublayerNorm n = around(x, due_norm, pending);
+            n.w = out_norm_.as<float>();
+            n.rows = pk_.out_tok;
+            n.act = st_out_.ptr; n.act_kf = KE;
+            rk::sublayer_norm(stream_, arith_, n, n_out);
+        } else if (c.streams > 0) {
+            rk::streams_norm_act(stream_, arith_, streams, due, pending, nullptr, out_norm_.as<float>(), E, c.eps, pk_.out_tok, n_out, st_out_.ptr, KE);
+        } else {
+            rk::norm_act(stream_, arith_, c.arch->norm, x, out_norm_.as<float>(), E, c.eps, pk_.out_tok, n_out, st_out_.ptr, KE, pending);
+        }
+        prof_end(PC_HEAD, pt);
         pt = prof_begin(PC_HEAD);
         rk::DenseJob head;
         head.w = stack_head_.w;

@@ -1,6 +1,6 @@
 // Routing of mixture-of-experts feed-forwards of layer-stack models: the choice of experts per token and the order in
 // which the expert products (dense.hip) take the chosen pairs. Logits arrive in f32; the weights of a token are the
-// softmax over its chosen logits, or over all its logits.
+// softmax over its chosen logits, over all its logits, or each logit's own sigmoid.
 #include "stack_dev.hpp"
 
 namespace rk {
@@ -59,7 +59,7 @@ template <int N> __device__ __forceinline__ void choose(const ExpertRoute & r, i
 #pragma unroll
     for (int o = 32; o > 0; o >>= 1) largest = fmaxf(largest, __shfl_xor(largest, o, 64));
     float sum = 0.0f;
-    if (r.over_all) {
+    if (r.score == SCORE_OVER_ALL) {
 #pragma unroll
         for (int i = 0; i < N; ++i) sum += expf(v[i] - largest);
     }
@@ -77,14 +77,14 @@ template <int N> __device__ __forceinline__ void choose(const ExpertRoute & r, i
 #pragma unroll
     for (int i = 0; i < N; ++i) {
         p[i] = rank[i] < r.top ? expf(v[i] - largest) : 0.0f;
-        if (!r.over_all) sum += p[i];
+        if (r.score == SCORE_OVER_CHOSEN) sum += p[i];
     }
     sum = wave_sum(sum);
 #pragma unroll
     for (int i = 0; i < N; ++i)
         if (rank[i] < r.top) {
             sel[rank[i]] = lane + 64 * i;
-            r.weight[(size_t)t * r.top + rank[i]] = p[i] / sum * r.scale;
+            r.weight[(size_t)t * r.top + rank[i]] = (r.score == SCORE_SIGMOID ? sigmoid_f(v[i]) : p[i] / sum) * r.scale;
         }
 }
 __device__ __forceinline__ void choose_any(const ExpertRoute & r, int t, int lane, int32_t * sel) {

@@ -26,12 +26,14 @@ inline const GgufArch * find_gguf_arch(const std::string & name) {
 }
 
 // What an architecture fixes about its layers. Parallel layers: x <- x + scale1 * mixer(n(x)) + scale2 * ff(n(x)), one
-// norm for both; otherwise x <- x + mixer(n1(x)), then x <- x + ff(n2(x)). The norm's kind and whether its weights are
-// stored as differences from one; the activations (DenseOut kinds) of the feed-forward and of experts; element-wise
+// norm for both; otherwise x <- x + mixer(n1(x)), then x <- x + ff(n2(x)), and with norms after a
+// sublayer x <- x + mult * n1b(mixer(n1(x))), and so on. The norm's kind and whether its weights are stored as differences from
+// one; the activations (DenseOut kinds) of the feed-forward and of experts; element-wise
 // layer scales or none; whether a dense feed-forward has biases, a shared expert a gate per token, and the head its own matrix.
 // Grouped attention: what positions a mask of some size leaves; whether the values are the keys before rotation or a
-// projection of their own, with biases on all three and queries and keys normed over all their heads; how a head's columns
-// pair up for rotation (i with i + dims / 2, or neighbours) and what stretching the rotation means.
+// projection of their own, with biases on all three; how a head's columns pair up for rotation (i with i + dims / 2, or
+// neighbours) and what stretching the rotation means; whether queries and keys are normed over all their heads before it, and
+// whether the output has a bias too.
 enum class Mask { WINDOW, CHUNK };
 enum class Stretch { RAMP, BANDS };
 enum class Pairs { HALVES, NEIGHBOURS };
@@ -45,19 +47,27 @@ struct StackArch {
     bool keys_are_values;
     Pairs pairs;
     Stretch stretch;
-    bool route_over_all;         // an expert's weight is the softmax over all experts, not over the chosen ones
+    int score;                   // what an expert's weight is (rk::SCORE_*)
+    bool qk_norm, out_bias;
+    bool norm_after;             // norms after the sublayers, and of the embedding, to which one of two neighbouring tokens is added
+    bool weigh_input;            // an expert's weight multiplies what it reads
+    // Queries, keys and values leave the input product's epilogue for their places (norms over all heads need the whole row first).
+    bool rows_in_place() const { return keys_are_values || !qk_norm; }
 };
 inline const StackArch * find_stack_arch(const std::string & name) {
     static const StackArch known[] = {
-        {"Dibosun", rk::NORM_LAYER, false, true, rk::OUT_ACT_RELU2, -1, true, false, true, false, Mask::WINDOW, true, Pairs::HALVES, Stretch::RAMP, false},
-        {"Pomisun", rk::NORM_RMS, true, false, rk::OUT_ACT_GEGLU, rk::OUT_ACT_SWIGLU, false, false, true, false, Mask::CHUNK, true, Pairs::HALVES, Stretch::RAMP, false},
-        {"Vifanex", rk::NORM_RMS, false, false, rk::OUT_ACT_CLAMPED, rk::OUT_ACT_CLAMPED, false, true, false, true, Mask::WINDOW, false, Pairs::NEIGHBOURS, Stretch::BANDS, true},
+        {"Dibosun", rk::NORM_LAYER, false, true, rk::OUT_ACT_RELU2, -1, true, false, true, false, Mask::WINDOW, true, Pairs::HALVES, Stretch::RAMP, rk::SCORE_OVER_CHOSEN, false, false, false, false},
+        {"Pomisun", rk::NORM_RMS, true, false, rk::OUT_ACT_GEGLU, rk::OUT_ACT_SWIGLU, false, false, true, false, Mask::CHUNK, true, Pairs::HALVES, Stretch::RAMP, rk::SCORE_OVER_CHOSEN, false, false, false, false},
+        {"Vifanex", rk::NORM_RMS, false, false, rk::OUT_ACT_CLAMPED, rk::OUT_ACT_CLAMPED, false, true, false, true, Mask::WINDOW, false, Pairs::NEIGHBOURS, Stretch::BANDS, rk::SCORE_OVER_ALL, true, false, false, false},
+        {"Kilurax", rk::NORM_RMS, false, false, rk::OUT_ACT_SWIGLU, rk::OUT_ACT_SWIGLU, false, false, false, true, Mask::WINDOW, false, Pairs::HALVES, Stretch::RAMP, rk::SCORE_SIGMOID, false, true, true, true},
     };
     for (const StackArch & a : known) if (name == a.name) return &a;
     return nullptr;
 }
 
-enum class Mixer { LATENT_ATTENTION, MAMBA2, ATTENTION, CHANNEL_DELTA };
+// DELTA: every mixer with a matrix state and a rule of writing (its DeltaShape says which). ATTENTION_MAMBA2: both over one input,
+// their outputs scaled and added.
+enum class Mixer { LATENT_ATTENTION, MAMBA2, ATTENTION, DELTA, ATTENTION_MAMBA2 };
 
 struct LatentSpec {
     int heads = 0, dim = 0, vdim = 0, q_rank = 0, kv_rank = 0;
@@ -123,17 +133,24 @@ struct LayerSpec {
     rk::MambaShape mamba;
     AttentionSpec attention;
     rk::DeltaShape delta;
+    float left_scale = 1.0f, right_scale = 1.0f;      // of attention and Mamba-2 side by side
     int ff = 0;                  // of a dense feed-forward; 0 and no experts: no feed-forward
     float ff_limit = 0.0f;
     MoeSpec moe;
     bool has_ff() const { return ff > 0 || moe.experts > 0; }
-    bool recurrent() const { return mixer == Mixer::MAMBA2 || mixer == Mixer::CHANNEL_DELTA; }
-    // Columns a mixer hands to its output projection (a head of grouped attention padded as its cached values are).
+    bool grouped_attention() const { return mixer == Mixer::ATTENTION || mixer == Mixer::ATTENTION_MAMBA2; }
+    bool state_space() const { return mixer == Mixer::MAMBA2 || mixer == Mixer::ATTENTION_MAMBA2; }
+    bool attends() const { return mixer == Mixer::LATENT_ATTENTION || grouped_attention(); }
+    bool recurrent() const { return state_space() || mixer == Mixer::DELTA; }
+    // Columns a mixer hands to its output projection (a head of grouped attention padded as its cached values are), and those of
+    // Mamba-2 beside attention.
+    int beside_width() const { return mixer == Mixer::ATTENTION_MAMBA2 ? mamba.inner() : 0; }
     int mix_width() const {
         switch (mixer) {
             case Mixer::MAMBA2: return mamba.inner();
-            case Mixer::CHANNEL_DELTA: return delta.inner();
-            case Mixer::ATTENTION: return attention.heads * 32 * attention.frags().v;
+            case Mixer::DELTA: return delta.inner();
+            case Mixer::ATTENTION:
+            case Mixer::ATTENTION_MAMBA2: return attention.heads * 32 * attention.frags().v;
             default: return latent.heads * latent.vdim;
         }
     }
@@ -148,11 +165,17 @@ struct StackConfig {
     float eps = 0.0f;
     float embedding_scale = 1.0f, logit_softcap = 0.0f;      // 0: none
     int streams = 0;             // residual streams of hyper-connections (0: a plain residual sum)
+    int norm_groups = 1;         // equal parts of a row, normed each by its own
+    float residual_mult = 1.0f;  // of what a sublayer adds
+    int input_taps = 0;          // of the convolution over the tokens that every sublayer's input goes through (0: none)
+    int64_t pair_buckets = 0, pair_mul_prev = 0, pair_mul_cur = 0;      // an embedding of every two neighbouring tokens 
+    // The sublayers' norms are k_sublayer_norm's.
+    bool around() const { return arch->norm_after || norm_groups > 1 || residual_mult != 1.0f || input_taps > 0; }
     std::vector<LayerSpec> layers;
     std::vector<LayerRun> runs;
     bool recurrent() const {
         for (const LayerSpec & l : layers) if (l.recurrent()) return true;
-        return false;
+        return input_taps > 0 || pair_buckets > 0;
     }
 
     static bool is_folder(const std::string & path) {
@@ -180,6 +203,19 @@ struct StackConfig {
         if (present(v, "streams")) c.streams = size(v, "streams");
         if (c.streams > rk::MAX_STREAMS || (c.streams > 0 && (c.arch->parallel || c.arch->norm != rk::NORM_RMS || present(v, "loop"))))
             throw std::runtime_error("config.json: 'streams' of sequential layers over RMS norms, without a loop, " + std::to_string(rk::MAX_STREAMS) + " at most");
+        const JsonValue & norm = need(v, "norm");
+        if (present(norm, "groups")) c.norm_groups = size(norm, "groups");
+        if (c.width % c.norm_groups != 0) throw std::runtime_error("config.json: 'width' must be a multiple of 'norm.groups'");
+        if (present(v, "residual_mult")) c.residual_mult = (float)number(v, "residual_mult");
+        if (present(v, "canon")) c.input_taps = size(need(v, "canon"), "taps");
+        if (c.arch->norm_after) {
+            const JsonValue & b = need(need(v, "embedding"), "bigram");
+            c.pair_buckets = size(b, "buckets");
+            c.pair_mul_prev = factor(b, "mul_prev") % c.pair_buckets;      // of residues the products fit 64 bits
+            c.pair_mul_cur = factor(b, "mul_cur") % c.pair_buckets;
+        }
+        if (c.around() && (c.arch->parallel || c.arch->norm != rk::NORM_RMS || c.streams > 0 || present(v, "loop")))
+            throw std::runtime_error("config.json: grouped norms, 'residual_mult' and 'canon' need sequential layers over RMS norms, without streams or a loop");
         for (const JsonValue & l : need(v, "layers").items) c.layers.push_back(layer(*c.arch, l, c.layers));
         const int n = (int)c.layers.size();
         if (n < 1 || n > 4096) throw std::runtime_error("config.json: 'layers' must list 1 to 4096 layers");
@@ -214,6 +250,11 @@ private:
         if (n < lo || n > (1 << 24) || n != (double)(int)n) throw std::runtime_error(std::string("config.json: '") + key + "' is no size");
         return (int)n;
     }
+    static int64_t factor(const JsonValue & v, const char * key) {
+        const double n = number(v, key);
+        if (!(n >= 0.0) || n > 9007199254740992.0 || n != std::floor(n)) throw std::runtime_error(std::string("config.json: '") + key + "' is no whole number");
+        return (int64_t)n;
+    }
     static bool present(const JsonValue & v, const char * key) {
         const JsonValue * m = v.get(key);
         return m && m->kind != JsonValue::NUL;
@@ -243,6 +284,57 @@ private:
         }
         return r;
     }
+    static rk::MambaShape mamba2(const JsonValue & m) {
+        rk::MambaShape s;
+        s.heads = size(m, "heads");
+        s.vdim = size(m, "vdim");
+        s.state = size(m, "state");
+        s.groups = size(m, "groups");
+        s.taps = size(m, "conv");
+        s.norm_groups = size(m, "norm_groups");
+        if (s.heads % s.groups != 0) throw std::runtime_error("mamba2: heads must be a multiple of groups");
+        if (s.inner() % s.norm_groups != 0) throw std::runtime_error("mamba2: heads * vdim must be a multiple of norm_groups");
+        if (s.state > 512) throw std::runtime_error("mamba2: a state above 512 rows is not supported");
+        return s;
+    }
+    static AttentionSpec attention(const StackArch & arch, const JsonValue & m, const std::vector<LayerSpec> & before) {
+        AttentionSpec a;
+        a.heads = size(m, "heads");
+        a.kv_heads = size(m, "kv_heads");
+        a.dim = size(m, "dim");
+        a.scale = (float)number(m, "scale");
+        if (present(m, "softcap")) a.softcap = (float)number(m, "softcap");
+        if (present(m, "mask") && present(need(m, "mask"), "size")) (arch.mask == Mask::CHUNK ? a.chunk : a.window) = size(need(m, "mask"), "size");
+        if (a.heads % a.kv_heads != 0) throw std::runtime_error("attention: heads must be a multiple of kv_heads");
+        a.vdim = size(m, "vdim");
+        if (arch.keys_are_values && a.vdim != a.dim) throw std::runtime_error("attention: the values are the keys, so vdim must be dim");
+        if (a.dim > 1024 || a.vdim > 1024) throw std::runtime_error("attention: heads above 1024 columns are not supported");
+        if (!arch.rows_in_place() && present(m, "v_mix")) a.v_mix = need(m, "v_mix").b;
+        a.v_first = a.v_mix;
+        for (const LayerSpec & b : before)
+            if (b.mixer == Mixer::ATTENTION && b.attention.v_mix) {
+                a.v_first = false;
+                if (a.v_mix && b.attention.kv_heads * b.attention.vdim != a.kv_heads * a.vdim)
+                    throw std::runtime_error("attention: layers that mix their values must have equally many");
+            }
+        if (!(a.softcap >= 0.0f)) throw std::runtime_error("attention: softcap must not be negative");
+        if (arch.keys_are_values || present(m, "rot")) a.rot = rotary(arch, need(m, "rot"), a.dim);
+        return a;
+    }
+    static rk::DeltaShape delta(const JsonValue & m, const std::string & type) {
+        rk::DeltaShape s;
+        s.heads = size(m, "heads");
+        s.kv_heads = size(m, "kv_heads");
+        s.dim = size(m, "dim");
+        s.vdim = size(m, "vdim");
+        s.taps = size(m, "conv");
+        if (s.heads % s.kv_heads != 0) throw std::runtime_error(type + ": heads must be a multiple of kv_heads");
+        state_limits(s, type);
+        return s;
+    }
+    static void state_limits(const rk::DeltaShape & s, const std::string & type) {
+        if (s.dim > 512 || s.vdim > 4096) throw std::runtime_error(type + ": at most 512 key and 4096 value channels per head are supported");
+    }
     static LayerSpec layer(const StackArch & arch, const JsonValue & v, const std::vector<LayerSpec> & before) {
         LayerSpec l;
         const std::string type = need(v, "type").text;
@@ -265,49 +357,34 @@ private:
             if (a.kv_rank > 1024) throw std::runtime_error("latent attention: kv_rank above 1024 is not supported");
         } else if (type == "mamba2") {
             l.mixer = Mixer::MAMBA2;
-            rk::MambaShape & s = l.mamba;
-            s.heads = size(m, "heads");
-            s.vdim = size(m, "vdim");
-            s.state = size(m, "state");
-            s.groups = size(m, "groups");
-            s.taps = size(m, "conv");
-            s.norm_groups = size(m, "norm_groups");
-            if (s.heads % s.groups != 0) throw std::runtime_error("mamba2: heads must be a multiple of groups");
-            if (s.inner() % s.norm_groups != 0) throw std::runtime_error("mamba2: heads * vdim must be a multiple of norm_groups");
-            if (s.state > 512) throw std::runtime_error("mamba2: a state above 512 rows is not supported");
+            l.mamba = mamba2(m);
         } else if (type == "attention") {
             l.mixer = Mixer::ATTENTION;
-            AttentionSpec & a = l.attention;
-            a.heads = size(m, "heads");
-            a.kv_heads = size(m, "kv_heads");
-            a.dim = size(m, "dim");
-            a.scale = (float)number(m, "scale");
-            if (present(m, "softcap")) a.softcap = (float)number(m, "softcap");
-            if (present(m, "mask") && present(need(m, "mask"), "size")) (arch.mask == Mask::CHUNK ? a.chunk : a.window) = size(need(m, "mask"), "size");
-            if (a.heads % a.kv_heads != 0) throw std::runtime_error("attention: heads must be a multiple of kv_heads");
-            a.vdim = size(m, "vdim");
-            if (arch.keys_are_values && a.vdim != a.dim) throw std::runtime_error("attention: the values are the keys, so vdim must be dim");
-            if (a.dim > 1024 || a.vdim > 1024) throw std::runtime_error("attention: heads above 1024 columns are not supported");
-            if (!arch.keys_are_values && present(m, "v_mix")) a.v_mix = need(m, "v_mix").b;
-            a.v_first = a.v_mix;
-            for (const LayerSpec & b : before)
-                if (b.mixer == Mixer::ATTENTION && b.attention.v_mix) {
-                    a.v_first = false;
-                    if (a.v_mix && b.attention.kv_heads * b.attention.vdim != a.kv_heads * a.vdim)
-                        throw std::runtime_error("attention: layers that mix their values must have equally many");
-                }
-            if (!(a.softcap >= 0.0f)) throw std::runtime_error("attention: softcap must not be negative");
-            if (arch.keys_are_values || present(m, "rot")) a.rot = rotary(arch, need(m, "rot"), a.dim);
-        } else if (type == "channel_delta") {
-            l.mixer = Mixer::CHANNEL_DELTA;
+            l.attention = attention(arch, m, before);
+        } else if (type == "parallel") {
+            if (arch.keys_are_values || arch.qk_norm || arch.parallel) throw std::runtime_error("config.json: 'parallel' mixers are not supported for this architecture");
+            l.mixer = Mixer::ATTENTION_MAMBA2;
+            l.attention = attention(arch, need(m, "left"), before);
+            l.mamba = mamba2(need(m, "right"));
+            l.left_scale = (float)number(m, "left_scale");
+            l.right_scale = (float)number(m, "right_scale");
+        } else if (type == "hgrn2") {
+            l.mixer = Mixer::DELTA;
             rk::DeltaShape & s = l.delta;
-            s.heads = size(m, "heads");
-            s.kv_heads = size(m, "kv_heads");
+            s.rule = rk::RULE_FORGET;
+            s.gate = rk::GATE_NONE;
+            s.heads = s.kv_heads = size(m, "heads");
             s.dim = size(m, "dim");
             s.vdim = size(m, "vdim");
-            s.taps = size(m, "conv");
-            if (s.heads % s.kv_heads != 0) throw std::runtime_error("channel_delta: heads must be a multiple of kv_heads");
-            if (s.dim > 512 || s.vdim > 4096) throw std::runtime_error("channel_delta: at most 512 key and 4096 value channels per head are supported");
+            state_limits(s, type);
+        } else if (type == "delta") {
+            l.mixer = Mixer::DELTA;
+            l.delta = delta(m, type);
+            l.delta.rule = rk::RULE_DELTA_HEADS;
+            l.delta.gate = rk::GATE_SILU;
+        } else if (type == "channel_delta") {
+            l.mixer = Mixer::DELTA;
+            l.delta = delta(m, type);
         } else {
             throw std::runtime_error("config.json: unknown layer type '" + type + "'");
         }

@@ -1,6 +1,7 @@
 // Row norms of layer-stack models: the residual stream (completed with the slices the products before left), or what a
-// sublayer reads of several residual streams, through an RMS or layer norm into activations. Statistics in f32, two passes
-// over the row held in LDS. Also the rows that start a stream.
+// sublayer reads of several residual streams, through an RMS or layer norm into activations; norms in groups before and after
+// a sublayer with the convolution of what it reads. Statistics in f32, two passes over the row held in LDS. Also the rows that
+// start a stream.
 #include "stack_dev.hpp"
 
 #include <type_traits>
@@ -152,6 +153,246 @@ template <int N> __global__ void k_streams_sum(Streams x, const float * __restri
     }
 }
 
+// Norms in `groups` equal parts of a row of E columns held in LDS: its floats, then a factor per group and the partial sums.
+struct GroupNorm {
+    float * row, * inv, * part;
+    int E, groups, len;
+    float eps;
+    __device__ __forceinline__ GroupNorm(float * lds, int E, int groups, float eps)
+        : row(lds), inv(lds + (E + 3) / 4 * 4), part(inv + groups), E(E), groups(groups), len(E / groups), eps(eps) {}
+    // The factors of what the row holds. Waves share a group where there are fewer groups than waves.
+    __device__ __forceinline__ void factors() {
+        const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, waves = blockDim.x >> 6, per = max(1, waves / groups);
+        const bool even = len % (4 * per) == 0;
+        __syncthreads();
+        for (int i = wave; i < groups * per; i += waves) {
+            const int g = i / per, p = i - g * per, lo = g * len + (int)((int64_t)len * p / per), hi = g * len + (int)((int64_t)len * (p + 1) / per);
+            float q = 0.0f;
+            if (even) {
+                for (int k = lo + 4 * lane; k < hi; k += 256) {
+                    const f4 v = *(const f4 *)(row + k);
+                    q += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+                }
+            } else {
+                for (int k = lo + lane; k < hi; k += 64) q += row[k] * row[k];
+            }
+            q = wave_sum(q);
+            if (lane == 0) part[i] = q;
+        }
+        __syncthreads();
+        for (int g = threadIdx.x; g < groups; g += blockDim.x) {
+            float q = 0.0f;
+            for (int p = 0; p < per; ++p) q += part[g * per + p];
+            inv[g] = 1.0f / sqrtf(q / (float)len + eps);
+        }
+        __syncthreads();
+    }
+    static size_t bytes(int E, int groups) { return ((size_t)(E + 3) / 4 * 4 + groups + std::max(groups, 16)) * 4; }
+};
+
+// Where a sublayer's input goes: activations at once, f32 rows for the convolution that follows, or through the convolution
+// where every run is a single token (a workgroup per run).
+enum : int { NORM_TO_ACT = 0, NORM_TO_ROWS, NORM_CONVOLVED };
+
+template <int ARITH> __device__ __forceinline__ void store_input(const SublayerNorm & j, int row, int k, const float (&v)[8]) {
+    store_frag8<ARITH>(j.act, j.act_kf, row, k, v);
+    if (j.act_rows) store_act8_at<ARITH>(j.act_rows, (size_t)row * j.act_kf * 32 + k, v);
+}
+
+// W columns per thread and step, NV steps: the columns stay in registers between the two norms. A group is whole steps.
+template <int ARITH, int OUT, int W, int NV>
+__global__ __launch_bounds__(1024) void k_sublayer_norm(SublayerNorm j) {
+    typedef float vec __attribute__((ext_vector_type(W)));
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    GroupNorm norm(sm, j.E, j.groups, j.eps);
+    float * row = norm.row;
+    const int E = j.E, n_thr = blockDim.x;
+    SeqRun run = {};
+    if constexpr (OUT == NORM_CONVOLVED) run = j.runs.runs[blockIdx.x];
+    const int t = OUT == NORM_CONVOLVED ? j.runs.tok[run.start] : j.rows ? j.rows[blockIdx.x] : (int)blockIdx.x;
+    const int at = OUT == NORM_CONVOLVED ? t : (int)blockIdx.x;              // row of the activations
+    float * xr = j.x + (size_t)t * E;
+    vec x[NV];
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int k = W * ((int)threadIdx.x + n_thr * i);
+        if (k < E) x[i] = *(const vec *)(xr + k);
+    }
+    if (j.add.n > 0) {
+        vec y[NV];
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int k = W * ((int)threadIdx.x + n_thr * i);
+            y[i] = vec(0.0f);
+            if (k >= E) continue;
+            for (int base = 0; base < j.add.n; base += 8) {
+                const float * from = j.add.data + (size_t)base * j.add.stride + (size_t)t * E + k;
+                const int n = j.add.n - base;
+                vec d[8];
+#pragma unroll
+                for (int s = 0; s < 8; ++s) if (s < n) d[s] = *(const vec *)(from + (size_t)s * j.add.stride);
+#pragma unroll
+                for (int s = 0; s < 8; ++s) if (s < n) y[i] += d[s];
+            }
+            if (j.after) *(vec *)(row + k) = y[i];
+        }
+        if (j.after) norm.factors();
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int k = W * ((int)threadIdx.x + n_thr * i);
+            if (k >= E) continue;
+            if (j.after) y[i] = y[i] * norm.inv[k / norm.len] * *(const vec *)(j.after + k);
+            x[i] += j.mult * y[i];
+            if (!j.rows) *(vec *)(xr + k) = x[i];
+        }
+    }
+    if (!j.w) return;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int k = W * ((int)threadIdx.x + n_thr * i);
+        if (k < E) *(vec *)(row + k) = x[i];
+    }
+    norm.factors();
+    if constexpr (OUT == NORM_TO_ROWS) {
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int k = W * ((int)threadIdx.x + n_thr * i);
+            if (k < E) *(vec *)(j.h + (size_t)t * E + k) = x[i] * norm.inv[k / norm.len] * *(const vec *)(j.w + k);
+        }
+        return;
+    }
+    for (int k = 8 * (int)threadIdx.x; k < E; k += 8 * n_thr) {
+        float v[8];
+        int g = k / norm.len, next = (g + 1) * norm.len;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            if (k + i >= next) { ++g; next += norm.len; }
+            v[i] = k + i < E ? row[k + i] * norm.inv[g] * j.w[k + i] : 0.0f;
+        }
+        if constexpr (OUT == NORM_CONVOLVED) {
+            const int past = j.n_taps - 1, plane = (run.flags >> 1) & 1;
+            const bool fresh = run.flags & 1;
+            const float * old_in = j.history + (size_t)plane * j.plane + (size_t)run.slot * past * E;
+            float * new_in = j.history + (size_t)(1 - plane) * j.plane + (size_t)run.slot * past * E;
+            float h[8];
+#pragma unroll
+            for (int i = 0; i < 8; ++i) {
+                h[i] = v[i];
+                if (k + i < E) v[i] += j.taps[(size_t)past * E + k + i] * h[i];
+            }
+            for (int p = 0; p < past; ++p) {
+#pragma unroll
+                for (int i = 0; i < 8; ++i) {
+                    if (k + i >= E) break;
+                    const float o = fresh ? 0.0f : old_in[(size_t)p * E + k + i];
+                    v[i] += j.taps[(size_t)p * E + k + i] * o;
+                    if (p > 0) new_in[(size_t)(p - 1) * E + k + i] = o;
+                }
+            }
+            if (past > 0) {
+#pragma unroll
+                for (int i = 0; i < 8; ++i) if (k + i < E) new_in[(size_t)(past - 1) * E + k + i] = h[i];
+            }
+        }
+        store_input<ARITH>(j, at, k, v);
+    }
+}
+
+// The convolution over the rows k_sublayer_norm left: a thread takes eight columns of kRunTokens tokens of a run, with the
+// window and the taps in registers (TAPS 0: any number).
+constexpr int kRunTokens = 8;
+template <int ARITH, int TAPS>
+__global__ __launch_bounds__(256) void k_sublayer_conv(SublayerNorm j) {
+    const int E = j.E, K = TAPS > 0 ? TAPS : j.n_taps, groups = (E + 7) / 8;
+    const int item = blockIdx.x * 256 + threadIdx.x, k = item % groups * 8, first = item / groups * kRunTokens;
+    const SeqRun run = j.runs.runs[blockIdx.y];
+    if (first >= run.n) return;
+    const int plane = (run.flags >> 1) & 1, last = min(first + kRunTokens, run.n), left = E - k;
+    const bool even = E % 4 == 0;
+    const float * old_in = j.history + (size_t)plane * j.plane + (size_t)run.slot * (K - 1) * E;
+    float * new_in = j.history + (size_t)(1 - plane) * j.plane + (size_t)run.slot * (K - 1) * E;
+    auto load = [&](const float * p, float (&o)[8]) {
+        if (even && left >= 8) {
+            const f4 a = *(const f4 *)p, b = *(const f4 *)(p + 4);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) { o[e] = a[e]; o[4 + e] = b[e]; }
+        } else {
+#pragma unroll
+            for (int e = 0; e < 8; ++e) o[e] = e < left ? p[e] : 0.0f;
+        }
+    };
+    auto input = [&](int i, float (&o)[8]) {         // h of the run's token i; i < 0: what the slot remembers
+        if (i >= 0) return load(j.h + (size_t)j.runs.tok[run.start + i] * E + k, o);
+        if (!(run.flags & 1)) return load(old_in + (size_t)(i + K - 1) * E + k, o);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) o[e] = 0.0f;
+    };
+    if constexpr (TAPS > 0) {
+        float win[TAPS][8], tap[TAPS][8];
+#pragma unroll
+        for (int p = 0; p < TAPS; ++p) {
+            load(j.taps + (size_t)p * E + k, tap[p]);
+            if (p > 0) input(first - TAPS + p, win[p]);
+        }
+        for (int i = first; i < last; ++i) {
+            const int t = j.runs.tok[run.start + i];
+#pragma unroll
+            for (int p = 0; p + 1 < TAPS; ++p)
+#pragma unroll
+                for (int e = 0; e < 8; ++e) win[p][e] = win[p + 1][e];
+            load(j.h + (size_t)t * E + k, win[TAPS - 1]);
+            float v[8];
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                v[e] = win[TAPS - 1][e];
+#pragma unroll
+                for (int p = 0; p < TAPS; ++p) v[e] += tap[p][e] * win[p][e];
+            }
+            store_input<ARITH>(j, t, k, v);
+        }
+    } else {
+        for (int i = first; i < last; ++i) {
+            const int t = j.runs.tok[run.start + i];
+            float v[8], h[8], w[8];
+            load(j.h + (size_t)t * E + k, v);
+            for (int p = 0; p < K; ++p) {
+                input(i - (K - 1) + p, h);
+                load(j.taps + (size_t)p * E + k, w);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) v[e] += w[e] * h[e];
+            }
+            store_input<ARITH>(j, t, k, v);
+        }
+    }
+    if (last == run.n)
+        for (int p = 0; p < K - 1; ++p) {
+            float h[8];
+            input(run.n - (K - 1) + p, h);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) if (e < left) new_in[(size_t)p * E + k + e] = h[e];
+        }
+}
+
+// One workgroup per token of a run.
+__global__ __launch_bounds__(256) void k_embed_pairs(PairEmbedding j) {
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    const SeqRun run = j.runs.runs[blockIdx.y];
+    const int i = blockIdx.x;
+    if (i >= run.n) return;
+    GroupNorm norm(sm, j.E, j.groups, j.eps);
+    const int plane = (run.flags >> 1) & 1, t = j.runs.tok[run.start + i], tok = j.tok[t];
+    int64_t pair = j.buckets;
+    if (i > 0 || !(run.flags & 1)) {
+        const int before = i > 0 ? j.tok[j.runs.tok[run.start + i - 1]] : (int)j.last[(size_t)plane * j.plane + run.slot];
+        pair = (before * j.mul_prev + tok * j.mul_cur) % j.buckets;
+    }
+    const uint16_t * e = j.embed + (size_t)tok * j.E, * p = j.pairs + (size_t)pair * j.E;
+    for (int k = threadIdx.x; k < j.E; k += 256) norm.row[k] = bf16_float(e[k]) * j.scale + bf16_float(p[k]);
+    norm.factors();
+    for (int k = threadIdx.x; k < j.E; k += 256) j.x[(size_t)t * j.E + k] = norm.row[k] * norm.inv[k / norm.len] * j.w[k];
+    if (i == run.n - 1 && threadIdx.x == 0) j.last[(size_t)(1 - plane) * j.plane + run.slot] = (float)tok;      // exact: a vocabulary has at most 2^24 tokens
+}
+
 __global__ void k_embed_rows(const uint16_t * __restrict__ embed, const int32_t * __restrict__ tok, int E, float scale, size_t n,
                              float * __restrict__ x, int copies, size_t stride) {
     for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) {
@@ -217,6 +458,63 @@ void streams_sum(hipStream_t s, const Streams & x, const float * done, const Sli
     const size_t n = (size_t)T * E;
     hipLaunchKernelGGL(k_streams_sum<MAX_STREAMS>, dim3((unsigned)std::min<size_t>((n + 255) / 256, 4096)), dim3(256), 0, s, x, done, y, n, out);
     check_launch("streams_sum");
+}
+
+void sublayer_norm(hipStream_t s, int arith, const SublayerNorm & n, int n_rows) {
+    if (n_rows <= 0) return;
+    if (n.groups < 1 || n.E % n.groups != 0) throw std::runtime_error("norm: the row does not split into its groups");
+    const bool conv = n.taps && n.w;
+    const int out = !conv ? NORM_TO_ACT : n.runs.longest <= 1 ? NORM_CONVOLVED : NORM_TO_ROWS;
+    const bool vec = n.E % 4 == 0 && n.E / n.groups % 4 == 0;
+    const int width = vec ? 4 : 1;
+    int threads = n_rows <= 512 && n.E >= 2048 ? 1024 : 256;
+    if (n.E > 16 * width * threads) threads = 1024;
+    const int steps = (n.E + width * threads - 1) / (width * threads);
+    auto go = [&](auto kernel) {
+        hipLaunchKernelGGL(kernel, dim3((unsigned)(out == NORM_CONVOLVED ? n.runs.n : n_rows)), dim3((unsigned)threads), GroupNorm::bytes(n.E, n.groups), s, n);
+        check_launch("sublayer_norm");
+    };
+    auto step = [&](auto arithmetic, auto kind, auto w) {
+        constexpr int A = decltype(arithmetic)::value, O = decltype(kind)::value, W = decltype(w)::value;
+        if (steps <= 1) go(k_sublayer_norm<A, O, W, 1>);
+        else if (steps <= 2) go(k_sublayer_norm<A, O, W, 2>);
+        else if (steps <= 4) go(k_sublayer_norm<A, O, W, 4>);
+        else if (steps <= 16) go(k_sublayer_norm<A, O, W, 16>);
+        else throw std::runtime_error("norm: rows this wide are not supported");
+    };
+    auto columns = [&](auto arithmetic, auto kind) {
+        if (vec) step(arithmetic, kind, std::integral_constant<int, 4>());
+        else step(arithmetic, kind, std::integral_constant<int, 1>());
+    };
+    auto kinds = [&](auto arithmetic) {
+        if (out == NORM_TO_ACT) columns(arithmetic, std::integral_constant<int, NORM_TO_ACT>());
+        else if (out == NORM_TO_ROWS) columns(arithmetic, std::integral_constant<int, NORM_TO_ROWS>());
+        else columns(arithmetic, std::integral_constant<int, NORM_CONVOLVED>());
+    };
+    if (arith == ARITH_16) kinds(std::integral_constant<int, ARITH_16>());
+    else kinds(std::integral_constant<int, ARITH_32>());
+    if (out != NORM_TO_ROWS) return;
+    const int64_t items = (int64_t)((n.E + 7) / 8) * ((n.runs.longest + kRunTokens - 1) / kRunTokens);
+    const dim3 grid((unsigned)((items + 255) / 256), (unsigned)n.runs.n);
+    auto taps = [&](auto arithmetic) {
+        constexpr int A = decltype(arithmetic)::value;
+        switch (n.n_taps) {
+            case 2: hipLaunchKernelGGL((k_sublayer_conv<A, 2>), grid, dim3(256), 0, s, n); break;
+            case 3: hipLaunchKernelGGL((k_sublayer_conv<A, 3>), grid, dim3(256), 0, s, n); break;
+            case 4: hipLaunchKernelGGL((k_sublayer_conv<A, 4>), grid, dim3(256), 0, s, n); break;
+            default: hipLaunchKernelGGL((k_sublayer_conv<A, 0>), grid, dim3(256), 0, s, n);
+        }
+    };
+    if (arith == ARITH_16) taps(std::integral_constant<int, ARITH_16>());
+    else taps(std::integral_constant<int, ARITH_32>());
+    check_launch("sublayer_conv");
+}
+
+void embed_pairs(hipStream_t s, const PairEmbedding & e, int T) {
+    if (T <= 0 || e.runs.n <= 0) return;
+    if (e.groups < 1 || e.E % e.groups != 0 || e.buckets < 1) throw std::runtime_error("embedding: unsupported sizes");
+    hipLaunchKernelGGL(k_embed_pairs, dim3((unsigned)e.runs.longest, (unsigned)e.runs.n), dim3(256), GroupNorm::bytes(e.E, e.groups), s, e);
+    check_launch("embed_pairs");
 }
 
 void embed_rows(hipStream_t s, const uint16_t * embed, const int32_t * tok, int E, float scale, int T, float * x, int copies, size_t stride) {

@@ -55,10 +55,10 @@ enum : int {
 constexpr bool out_is_glu(int kind) { return kind == OUT_ACT_GEGLU || kind == OUT_ACT_SWIGLU || kind == OUT_ACT_CLAMPED; }
 
 // Rows of a product that are heads of kf * 32 columns, H of queries, then G of keys: rotated, the queries to rows
-// [t][H][kf * 32], the keys to their cells; the keys as projected are the values. The columns of a rotated pair are
-// neighbours (2 i, 2 i + 1).
+// [t][H][kf * 32], the keys to their cells. The values are the keys as projected (vf 0), or G heads of vf * 32 columns behind
+// them. The columns of a rotated pair are neighbours (2 i, 2 i + 1).
 struct RotaryOut {
-    int H = 0, G = 0, kf = 0, pairs = 0;       // rotated pairs of a head
+    int H = 0, G = 0, kf = 0, vf = 0, pairs = 0;      // rotated pairs of a head
     const float * table = nullptr;             // [T][pairs][2]: cosine and sine
     void * k_pool = nullptr, * v_pool = nullptr;
     const int32_t * cell = nullptr;
@@ -92,6 +92,7 @@ struct ExpertGroups {
     const int32_t * slot_pair = nullptr;       // the pair of a slot
     const float * weight = nullptr;            // of a pair
     int top = 0, pairs = 0;
+    bool weigh_input = false;                  // a pair's weight multiplies what its expert reads, not what it leaves
 };
 struct DenseJob {
     DenseWeight w;
@@ -112,6 +113,16 @@ struct DenseJob {
 // slice or more, and ws holds at least T * n floats).
 size_t dense_workspace_floats();
 Slices dense(hipStream_t s, int arith, const DenseJob & job, int T, float * ws);
+
+// ---- the tokens of a step by sequence ---------------------------------------------------------------
+// The tokens of one sequence in a step, in order: run_tok[start .. start + n) are flat token indices.
+struct SeqRun { int32_t slot, start, n, flags; };      // flags bit 0: the sequence starts here (state is zero), bit 1: the
+                                                       // plane of the slot's convolution inputs that holds the current ones
+struct SeqRuns {
+    const SeqRun * runs = nullptr;
+    int n = 0, longest = 0, shortest = 0;
+    const int32_t * tok = nullptr;
+};
 
 // ---- norms ----------------------------------------------------------------------------------------
 enum : int { NORM_RMS = 0, NORM_LAYER = 1 };
@@ -139,6 +150,46 @@ void streams_norm_act(hipStream_t s, int arith, const Streams & x, const float *
                       const float * w, int E, float eps, const int32_t * rows, int n_rows, void * act, int act_kf, void * act_rows = nullptr);
 // out[t] = the sum of the streams once they have taken in y, which they do not here.
 void streams_sum(hipStream_t s, const Streams & x, const float * done, const Slices & y, int E, int T, float * out);
+
+// Norms before and after each sublayer, RMS norms in `groups` equal consecutive parts of the row, each by its own root mean
+// square. First x[t] += mult * norm(slices) * after, written back (after null: no norm; no slices: x stays; rows: only
+// x[rows[i]] is read, and nothing written back). Then, with w, h[t] = norm(x[t]) * w goes to act, and with act_rows also to
+// plain rows. With taps it goes there as h_t + sum over j of taps[j] h_(t - n_taps + 1 + j), zeros before the sequence starts, a
+// causal convolution over the tokens of each run whose inputs from earlier steps lie in `history` as in ShortConv.
+struct SublayerNorm {
+    float * x = nullptr;
+    int E = 0, groups = 1;
+    float eps = 0.0f, mult = 1.0f;
+    Slices add;
+    const float * after = nullptr, * w = nullptr;
+    const int32_t * rows = nullptr;
+    void * act = nullptr, * act_rows = nullptr;
+    int act_kf = 0;
+    const float * taps = nullptr;  // [n_taps][E], the last row the current token's
+    int n_taps = 0;
+    float * history = nullptr;     // [2 planes][slots][n_taps - 1][E]
+    size_t plane = 0;
+    SeqRuns runs;
+    float * h = nullptr;           // scratch [T][E], for runs of more than one token
+};
+void sublayer_norm(hipStream_t s, int arith, const SublayerNorm & n, int n_rows);
+
+// x[t] = norm(scale * embed[tok[t]] + pairs[row]) * w, groups as above; row is (previous token * mul_prev + token * mul_cur) mod
+// buckets, and `buckets` for a sequence's first token. The last token of a run is left in `last` for the next step.
+struct PairEmbedding {
+    const uint16_t * embed = nullptr, * pairs = nullptr;      // bf16 rows of E
+    const int32_t * tok = nullptr;
+    float scale = 1.0f;
+    int64_t buckets = 0, mul_prev = 0, mul_cur = 0;
+    const float * w = nullptr;
+    int E = 0, groups = 1;
+    float eps = 0.0f;
+    SeqRuns runs;
+    float * last = nullptr;        // [2 planes][slots]
+    size_t plane = 0;
+    float * x = nullptr;
+};
+void embed_pairs(hipStream_t s, const PairEmbedding & e, int T);
 
 // ---- attention ---------------------------------------------------------------------------------------
 // A page of a cache: PAGE tokens x kf fragments of 32 columns, f16 or f32,
@@ -219,14 +270,15 @@ void rotary_table(hipStream_t s, const double * freq, int pairs, double magnitud
 // ---- expert routing --------------------------------------------------------------------------------------
 // Per token the `top` experts of largest logit (ties to the lower index), with several groups of neighbouring experts among
 // those of the `keep` groups whose largest logit is largest. Their weights: `scale` times the softmax over the chosen logits,
-// or over all of them. Then the pairs sorted by expert into slots, every expert from a multiple of 16 on, cut into tiles of
+// the softmax over all of them, or each logit's sigmoid. Then the pairs sorted by expert into slots, every expert from a multiple of 16 on, cut into tiles of
 // `block` slots.
 constexpr int MAX_EXPERTS = 1024, MAX_TOP = 64;
+enum : int { SCORE_OVER_CHOSEN = 0, SCORE_OVER_ALL, SCORE_SIGMOID };
 struct ExpertRoute {
     const float * logits = nullptr;            // [T][ld]
     int ld = 0, experts = 0, top = 0, block = 0;
     int groups = 1, keep = 1;
-    bool over_all = false;
+    int score = SCORE_OVER_CHOSEN;
     float scale = 1.0f;
     int32_t * sel = nullptr;                   // [T * top]
     float * weight = nullptr;                  // [T * top]
@@ -243,14 +295,6 @@ void stack_copy_page(hipStream_t s, void * pool, size_t page_bytes, int src, int
 void stack_cells(hipStream_t s, void * pool, int kf, int elem, const int32_t * cells, int n, void * rows, bool gather);
 
 // ---- recurrent mixers ---------------------------------------------------------------------------------
-// The tokens of one sequence in a step, in order: run_tok[start .. start + n) are flat token indices.
-struct SeqRun { int32_t slot, start, n, flags; };      // flags bit 0: the sequence starts here (state is zero), bit 1: the
-                                                       // plane of the slot's convolution inputs that holds the current ones
-struct SeqRuns {
-    const SeqRun * runs = nullptr;
-    int n = 0, longest = 0, shortest = 0;
-    const int32_t * tok = nullptr;
-};
 // Short causal convolution over time per channel, then SiLU: out[t][c] from the taps newest last, zeros before a sequence
 // starts. Runs of fewer than `least` tokens are left out.
 struct ShortConv {
@@ -289,16 +333,23 @@ struct MambaJob {
 };
 void mamba_mix(hipStream_t s, int arith, const MambaJob & j, int T);
 
-// ---- gated delta rule with a decay per key channel ----------------------------------------------------------
-// Per head a state S [dim][vdim]: S <- g * S (rows scaled), S <- S + k (beta (v - S^T k))^T, o = S^T q; q and k unit vectors
-// per key/value head (q also times dim^-1/2) and, like v, convolved and through SiLU before; g = exp(-exp(A_log) softplus(a + dt_bias))
-// per head and row, beta a sigmoid per head. The read-out: o / rms(o) * norm_w * sigmoid(gate).
+// ---- matrix states with a rule of writing: gated delta rules, linear attention with a forget gate -------------
+// Per head a state S [dim][vdim], decayed, written to and read out: S <- g * S (rows scaled), S <- S + k u^T, o = S^T q.
+// Delta rules: u = beta (v - S^T k); q and k unit vectors per key/value head (q also times dim^-1/2) and, like v, convolved and
+// through SiLU before; beta a sigmoid per head; g = exp(-exp(A_log) softplus(a + dt_bias)), a value per head and row of the state
+// (RULE_DELTA_CHANNELS) or one per head (RULE_DELTA_HEADS).
+// RULE_FORGET: what a row forgets is what it writes, g = lower + (1 - lower) sigmoid(z), k = 1 - g, u = v, q through SiLU; no
+// convolution.
+// The read-out of a head: o / rms(o) * norm_w, times the sigmoid or SiLU of a gate where there is one.
+enum : int { RULE_DELTA_CHANNELS = 0, RULE_DELTA_HEADS, RULE_FORGET };
+enum : int { GATE_NONE = 0, GATE_SIGMOID, GATE_SILU };
 struct DeltaShape {
-    int heads = 0, kv_heads = 0, dim = 0, vdim = 0, taps = 0;
-    int decay_rank = 0, gate_rank = 0;         // inner widths of the projections of a and gate
+    int rule = RULE_DELTA_CHANNELS, gate = GATE_SIGMOID;
+    int heads = 0, kv_heads = 0, dim = 0, vdim = 0, taps = 1;
+    int decay_rank = 0, gate_rank = 0;         // inner widths of the projections of a and gate, where they have one
     constexpr int keys() const { return kv_heads * dim; }
     constexpr int inner() const { return heads * vdim; }
-    constexpr int channels() const { return 2 * keys() + inner(); }       // q | k | v
+    constexpr int channels() const { return 2 * keys() + inner(); }       // q | k (forget rule: z) | v
     constexpr int vpitch() const { return (vdim + 3) / 4 * 4; }            // of a row of the state
     constexpr size_t state_floats() const { return (size_t)heads * dim * vpitch(); }
 };
@@ -306,9 +357,9 @@ struct DeltaJob {
     DeltaShape sh;
     const float * proj = nullptr;  // [T][ld]: q | k | v | beta (heads)
     int ld = 0;
-    const float * decay = nullptr, * gate = nullptr;     // [T][ld_low]: a (heads x dim), gate (heads x vdim)
+    const float * decay = nullptr, * gate = nullptr;     // [T][ld_low]: a (heads x dim, or heads), gate (heads x vdim)
     int ld_low = 0;
-    const float * conv_w = nullptr, * A_log = nullptr, * dt_bias = nullptr, * norm_w = nullptr;
+    const float * conv_w = nullptr, * A_log = nullptr, * dt_bias = nullptr, * lower = nullptr, * norm_w = nullptr;
     float eps = 0.0f, unit_eps = 0.0f;
     SeqRuns runs;
     float * conv_state = nullptr;  // as in ShortConv

@@ -19,15 +19,27 @@ int main(int argc, char ** argv) {
                 std::printf("\n");
             }
             if (c.streams > 0) std::printf("streams %d embedding_scale %g logit_softcap %g\n", c.streams, (double)c.embedding_scale, (double)c.logit_softcap);
+            if (c.around())
+                std::printf("embedding_scale %g buckets %lld factors %lld %lld norm groups %d residual %g taps %d\n", (double)c.embedding_scale, (long long)c.pair_buckets,
+                            (long long)c.pair_mul_prev, (long long)c.pair_mul_cur, c.norm_groups, (double)c.residual_mult, c.input_taps);
             for (const retro::LayerSpec & l : c.layers) {
                 if (c.streams > 0) {
                     const retro::MoeSpec & e = l.moe;
                     std::printf("limits %g %g %g groups %d keep %d scale %g vdim %d v_mix %d v_first %d\n", (double)l.ff_limit, (double)e.limit, (double)e.shared_limit,
                                 e.groups, e.keep, (double)e.scale, l.attention.vdim, l.attention.v_mix, l.attention.v_first);
                 }
-                if (l.mixer == retro::Mixer::CHANNEL_DELTA) {
+                if (l.mixer == retro::Mixer::ATTENTION_MAMBA2) {
+                    const retro::AttentionSpec & g = l.attention;
+                    const rk::MambaShape & s = l.mamba;
+                    std::printf("parallel heads %d kv_heads %d dim %d vdim %d rot %d base %g scale %g times %g, heads %d vdim %d state %d groups %d taps %d norm_groups %d times %g, "
+                                "ff %d experts %d top %d of %d shared %d\n", g.heads, g.kv_heads, g.dim, g.vdim, g.rot.dims, g.rot.base, (double)g.scale, (double)l.left_scale,
+                                s.heads, s.vdim, s.state, s.groups, s.taps, s.norm_groups, (double)l.right_scale, l.ff, l.moe.experts, l.moe.top, l.moe.ff, l.moe.shared_ff);
+                    continue;
+                }
+                if (l.mixer == retro::Mixer::DELTA) {
                     const rk::DeltaShape & d = l.delta;
-                    std::printf("channel_delta heads %d kv_heads %d dim %d vdim %d taps %d ff %d experts %d top %d of %d shared %d\n", d.heads, d.kv_heads, d.dim, d.vdim,
+                    const char * names[] = {"channel_delta", "delta", "hgrn2"};
+                    std::printf("%s heads %d kv_heads %d dim %d vdim %d taps %d ff %d experts %d top %d of %d shared %d\n", names[d.rule], d.heads, d.kv_heads, d.dim, d.vdim,
                                 d.taps, l.ff, l.moe.experts, l.moe.top, l.moe.ff, l.moe.shared_ff);
                     continue;
                 }
