@@ -101,6 +101,69 @@ def vifanex(width, vocab, layers, streams=2, eps=1e-5, softcap=20.0, embedding_s
             "logit_softcap": softcap, "embedding": {"scale": embedding_scale}}
 
 
+def parallel_mixer_layer(attention, mamba2, scales, rot, mlp, scale=None):
+    """Attention (heads, kv_heads, dim, vdim) and Mamba-2 (heads, vdim, state, groups, conv, norm_groups) over one input."""
+    left = dict(zip(("heads", "kv_heads", "dim", "vdim"), attention), rot=rot, scale=attention[2] ** -0.5 if scale is None else scale)
+    right = dict(zip(("heads", "vdim", "state", "groups", "conv", "norm_groups"), mamba2))
+    return {"type": "parallel", "mixer": {"left": left, "right": right, "left_scale": scales[0], "right_scale": scales[1]}, "mlp": mlp}
+
+
+def hgrn2_layer(heads, dim, vdim, mlp):
+    return {"type": "hgrn2", "mixer": {"heads": heads, "dim": dim, "vdim": vdim}, "mlp": mlp}
+
+
+def delta_layer(heads, kv_heads, dim, vdim, conv, mlp):
+    return {"type": "delta", "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": conv}, "mlp": mlp}
+
+
+def kilurax(width, vocab, layers, groups=2, taps=3, residual=0.7, eps=1e-5, embedding_scale=2.0, pairs=(97, 31, 5)):
+    """pairs: buckets and the two factors of the embedding of neighbouring tokens."""
+    return {"architecture": "Kilurax", "width": width, "vocab": vocab, "norm": {"eps": eps, "groups": groups}, "canon": {"taps": taps},
+            "residual_mult": residual, "embedding": {"scale": embedding_scale, "bigram": dict(zip(("buckets", "mul_prev", "mul_cur"), pairs))}, "layers": layers}
+
+
+def _kilurax_shapes(cfg) -> dict:
+    E = cfg["width"]
+    out = {"embed": (cfg["vocab"], E), "bigram": (cfg["embedding"]["bigram"]["buckets"] + 1, E), "embed.norm": (E,)}
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, mlp = "l%d." % i, layer["mixer"], layer.get("mlp")
+        x = p + "mix."
+        for q in ("1", "2") if mlp else ("1",):
+            out.update({p + "norm" + q: (E,), p + "norm" + q + "b": (E,), p + "canon" + q: (E, cfg["canon"]["taps"])})
+        if layer["type"] == "parallel":
+            a, s = m["left"], m["right"]
+            for name, n in (("q", a["heads"] * a["dim"]), ("k", a["kv_heads"] * a["dim"]), ("v", a["kv_heads"] * a["vdim"])):
+                out.update({x + "left." + name: (n, E), x + "left." + name + ".b": (n,)})
+            out.update({x + "left.o": (E, a["heads"] * a["vdim"]), x + "left.o.b": (E,)})
+            out.update(_mamba2_shapes(x + "right.", s, E))
+        elif layer["type"] == "hgrn2":
+            H, D, V = m["heads"], m["dim"], m["vdim"]
+            out.update({x + "q": (H * D, E), x + "f": (H * D, E), x + "f.b": (H * D,), x + "lower": (H * D,), x + "v": (H * V, E), x + "norm": (V,), x + "o": (E, H * V)})
+        else:
+            H, G, D, V = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+            for name, n in (("q", G * D), ("k", G * D), ("v", H * V)):
+                out.update({x + name: (n, E), x + name + ".conv": (n, m["conv"])})
+            out.update({x + "b": (H, E), x + "A_log": (H,), x + "norm": (V,), x + "a": (H, E), x + "dt_bias": (H,), x + "g": (H * V, E), x + "o": (E, H * V)})
+        if not mlp:
+            continue
+        out[p + "mlp.router"] = (mlp["router"]["experts"], E)
+        for e in range(mlp["router"]["experts"]):
+            out.update(_gated_shapes(p + "mlp.e%d." % e, mlp["expert"]["ff"], E))
+        if mlp.get("shared"):
+            out.update(_gated_shapes(p + "mlp.shared.", mlp["shared"]["ff"], E))
+    out["final.norm"] = (E,)
+    out["head"] = (cfg["vocab"], E)
+    return out
+
+
+def _mamba2_shapes(p, m, E):
+    inner, bc = m["heads"] * m["vdim"], 2 * m["groups"] * m["state"]
+    out = {p + "in": (2 * inner + bc + m["heads"], E), p + "conv": (inner + bc, m["conv"]), p + "conv.b": (inner + bc,)}
+    out.update({p + name: (m["heads"],) for name in ("dt_bias", "A_log", "D")})
+    out.update({p + "norm": (inner,), p + "o": (E, inner)})
+    return out
+
+
 def _vifanex_shapes(cfg) -> dict:
     E, s = cfg["width"], cfg["streams"]
     out = {"embed": (cfg["vocab"], E)}
@@ -149,6 +212,8 @@ def tensor_shapes(cfg) -> dict:
     out = {"embed": (cfg["vocab"], E)}
     if cfg["architecture"] == "Vifanex":
         return _vifanex_shapes(cfg)
+    if cfg["architecture"] == "Kilurax":
+        return _kilurax_shapes(cfg)
     if cfg["architecture"] == "Pomisun":
         for i, layer in enumerate(cfg["layers"]):
             p, m, mlp = "l%d." % i, layer["mixer"], layer.get("mlp")
@@ -186,14 +251,7 @@ def tensor_shapes(cfg) -> dict:
             out[p + "mix.g"] = (H, E)
             out[p + "mix.o"] = (E, H * m["vdim"])
         else:
-            inner, bc = m["heads"] * m["vdim"], 2 * m["groups"] * m["state"]
-            out[p + "mix.in"] = (2 * inner + bc + m["heads"], E)
-            out[p + "mix.conv"] = (inner + bc, m["conv"])
-            out[p + "mix.conv.b"] = (inner + bc,)
-            for name in ("dt_bias", "A_log", "D"):
-                out[p + "mix." + name] = (m["heads"],)
-            out[p + "mix.norm"] = (inner,)
-            out[p + "mix.o"] = (E, inner)
+            out.update(_mamba2_shapes(p + "mix.", m, E))
         out[p + "ls1"] = (E,)
         if layer.get("mlp"):
             out[p + "mlp.up"] = (layer["mlp"]["ff"], E)
@@ -216,6 +274,19 @@ def mean_and_std(name, shape, architecture="Dibosun"):
         if len(shape) == 2 and leaf == "b":
             return 0.0, shape[-1] ** -0.5
         if leaf == "b":
+            return 0.0, 0.3
+    if architecture == "Kilurax":
+        if leaf == "lower":
+            return 0.4, 0.3                  # clipped to what a lower bound may be
+        if name.endswith(".f.b"):
+            return 2.0, 1.5
+        if leaf.startswith("canon"):
+            return 0.0, 0.3
+        if leaf == "b" and len(shape) == 2:
+            return 0.0, shape[-1] ** -0.5
+        if name == "bigram":
+            return 0.0, 1.0
+        if leaf == "b" and ".left." in name:
             return 0.0, 0.3
     if leaf == "router":
         return 0.0, 2.0 * shape[-1] ** -0.5
@@ -261,7 +332,8 @@ def random_tensors(cfg, seed) -> dict:
     out = {}
     for name, shape in tensor_shapes(cfg).items():
         mean, std = mean_and_std(name, shape, cfg["architecture"])
-        out[name] = from_bf16(to_bf16(mean + std * rng.standard_normal(shape)))
+        v = mean + std * rng.standard_normal(shape)
+        out[name] = from_bf16(to_bf16(np.clip(v, 0.0, 1.0) if name.endswith(".lower") else v))
     return out
 
 
@@ -290,11 +362,12 @@ def write_random_checkpoint(folder, cfg, seed, device="cuda") -> Path:
         f.write(_header(shapes))
         for name, shape in shapes.items():
             mean, std = mean_and_std(name, shape, cfg["architecture"])
-            t = torch.empty(shape, device=device, dtype=torch.float32).normal_(mean, std, generator=gen).to(torch.bfloat16)
+            t = torch.empty(shape, device=device, dtype=torch.float32).normal_(mean, std, generator=gen)
+            t = (t.clamp_(0.0, 1.0) if name.endswith(".lower") else t).to(torch.bfloat16)
             f.write(t.view(torch.int16).cpu().numpy().tobytes())
     return folder
 
 
 def matrix_bytes(cfg) -> int:
     """Bytes of the matrices one step streams (the embedding counted once, as the output head)."""
-    return sum(2 * int(np.prod(s)) for n, s in tensor_shapes(cfg).items() if len(s) == 2 and not n.endswith(".conv"))
+    return sum(2 * int(np.prod(s)) for n, s in tensor_shapes(cfg).items() if len(s) == 2 and not n.endswith(".conv") and ".canon" not in n and n != "bigram")

@@ -2,13 +2,14 @@
 import numpy as np
 import pytest
 
+import plain_kilurax
 import plain_layers
 import plain_pomisun
 import plain_vifanex
 from retrograd_amd import engine as E
 from retrograd_amd import synth_stack as Y
 
-PLAIN = {"Dibosun": plain_layers, "Pomisun": plain_pomisun, "Vifanex": plain_vifanex}
+PLAIN = {"Dibosun": plain_layers, "Pomisun": plain_pomisun, "Vifanex": plain_vifanex, "Kilurax": plain_kilurax}
 
 LIMIT = {E.KV_F32: 3e-5, E.KV_F16: 0.035}
 KINDS = [pytest.param(E.KV_F32, id="f32"), pytest.param(E.KV_F16, id="bf16")]

@@ -231,6 +231,96 @@ def test_the_plain_vifanex_statements_against_closed_forms():
     assert np.allclose(out[0], 0) and np.allclose(out[1], xs[0] + 2)
 
 
+KILURAX = Y.kilurax(45, 30, [
+    Y.parallel_mixer_layer((6, 2, 10, 14), (4, 9, 12, 2, 3, 6), (0.75, -1.5), Y.rotary(6, 700.0), mlp=Y.moe_mlp(5, 2, 7, 11), scale=0.5),
+    Y.hgrn2_layer(heads=3, dim=7, vdim=5, mlp=None),
+    Y.delta_layer(heads=6, kv_heads=3, dim=8, vdim=4, conv=2, mlp=Y.moe_mlp(4, 1, 3))],
+    groups=5, taps=6, residual=0.3, embedding_scale=1.5, pairs=(23, 50, (1 << 41) + 5))
+
+
+def test_every_field_of_a_kilurax_configuration(reader, tmp_path):
+    Y.write_checkpoint(tmp_path, KILURAX, Y.random_tensors(KILURAX, 1))
+    assert reader(tmp_path, "config").splitlines() == [
+        "Kilurax width 45 vocab 30 eps 1e-05",
+        "embedding_scale 1.5 buckets 23 factors 4 %d norm groups 5 residual 0.3 taps 6" % (((1 << 41) + 5) % 23),
+        "parallel heads 6 kv_heads 2 dim 10 vdim 14 rot 6 base 700 scale 0.5 times 0.75, heads 4 vdim 9 state 12 groups 2 taps 3 norm_groups 6 times -1.5, ff 0 experts 5 top 2 of 7 shared 11",
+        "hgrn2 heads 3 kv_heads 3 dim 7 vdim 5 taps 1 ff 0 experts 0 top 0 of 0 shared 0",
+        "delta heads 6 kv_heads 3 dim 8 vdim 4 taps 2 ff 0 experts 4 top 1 of 3 shared 0"]
+    assert reader(tmp_path, "bigram").startswith("%d bytes" % sum(2 * int(np.prod(s)) for s in Y.tensor_shapes(KILURAX).values()))
+    assert reader(tmp_path, "l0.mix.right.conv.b").endswith("BF16\n") and reader(tmp_path, "l1.canon2").endswith("missing\n")
+
+
+@pytest.mark.parametrize("edit, message", [
+    (lambda c: c["norm"].update(groups=4), "multiple of 'norm.groups'"),
+    (lambda c: c["norm"].update(groups=0), "'groups' is no size"),
+    (lambda c: c["canon"].pop("taps"), "lacks 'taps'"),
+    (lambda c: c["embedding"].pop("bigram"), "lacks 'bigram'"),
+    (lambda c: c["embedding"]["bigram"].update(buckets=0), "'buckets' is no size"),
+    (lambda c: c["embedding"]["bigram"].update(mul_prev=1.5), "'mul_prev' is no whole number"),
+    (lambda c: c["embedding"]["bigram"].update(mul_cur=-1), "'mul_cur' is no whole number"),
+    (lambda c: c.update(streams=2), "without streams or a loop"),
+    (lambda c: c.update(loop={"start": 0, "stop": 1, "times": 2}), "without streams or a loop"),
+    (lambda c: c["layers"][0]["mixer"].pop("right_scale"), "lacks 'right_scale'"),
+    (lambda c: c["layers"][0]["mixer"].pop("left"), "lacks 'left'"),
+    (lambda c: c["layers"][0]["mixer"]["left"].update(kv_heads=4), "attention: heads must be a multiple of kv_heads"),
+    (lambda c: c["layers"][0]["mixer"]["right"].update(groups=3), "mamba2: heads must be a multiple of groups"),
+    (lambda c: c["layers"][0]["mixer"]["left"]["rot"].update(dims=12), "within a head"),
+    (lambda c: c["layers"][1]["mixer"].update(dim=513), "hgrn2: at most 512 key"),
+    (lambda c: c["layers"][2]["mixer"].update(kv_heads=4), "delta: heads must be a multiple of kv_heads"),
+    (lambda c: c["layers"][2]["mlp"]["router"].update(top=5), "exceeds 'experts'"),
+    (lambda c: c.update(architecture="Pomisun") or c["layers"].reverse(), "'parallel' mixers are not supported"),
+])
+def test_refused_kilurax_configurations(reader, tmp_path, edit, message):
+    cfg = copy.deepcopy(KILURAX)
+    edit(cfg)
+    (tmp_path / "config.json").write_text(json.dumps(cfg))
+    out = reader(tmp_path, "config")
+    assert out.startswith("refused: ") and message in out, out
+
+
+def test_the_plain_kilurax_statements_against_closed_forms():
+    import plain_kilurax as PK
+
+    rng = np.random.default_rng(0)
+    # every part of a row by its own length
+    assert np.allclose(PK.grouped_norm(np.array([[3.0, 4.0, 0.0, -2.0]]), np.array([1.0, 1.0, 1.0, 10.0]), 0.0, 2), [[3 / 12.5 ** 0.5, 4 / 12.5 ** 0.5, 0, -10 * 2 ** 0.5]])
+    # the first token's row lies behind the hashed ones; the previous token counts by its own factor
+    assert PK.bigram_rows([4, 2, 2], {"buckets": 7, "mul_prev": 10, "mul_cur": 3}) == [7, 46 % 7, 26 % 7]
+    # a sublayer reads its token and, here, half of the one two back
+    x = rng.standard_normal((5, 2))
+    y = PK.with_neighbours(x, np.array([[0.5, 0, 0], [0, 0, 1.0]]))
+    assert np.allclose(y[:2, 0], x[:2, 0]) and np.allclose(y[2:, 0], x[2:, 0] + 0.5 * x[:-2, 0]) and np.allclose(y[:, 1], 2 * x[:, 1])
+    # columns i and i + dims / 2 turn, the rest stays
+    x = np.zeros((4, 1, 6))
+    x[..., 1], x[..., 5] = 1, 3
+    assert np.allclose(PK.rotate_halves(x, Y.rotary(4, 100.0))[3, 0], [0, np.cos(0.3), 0, np.sin(0.3), 0, 3])
+    # a gate that keeps everything writes nothing; one that keeps nothing leaves the token's own value
+    q, v = rng.standard_normal((3, 1, 4)), rng.standard_normal((3, 1, 2))
+    assert np.allclose(PK.forget_scan(q, np.ones((3, 1, 4)), v), 0)
+    assert np.allclose(PK.forget_scan(q, np.zeros((3, 1, 4)), v), q.sum(-1, keepdims=True) * v)
+    f = np.ones((3, 1, 4))
+    f[:, :, 2] = 0.25
+    held = 0.75 * v[0, 0]
+    held = 0.25 * held + 0.75 * v[1, 0]
+    assert np.allclose(PK.forget_scan(q, f, v)[1, 0], q[1, 0, 2] * held)
+    assert np.allclose(PK.forget_gate(np.array([-800.0, 0.0, 800.0]), np.array([0.3, 0.3, 0.3])), [0.3, 0.65, 1.0])
+    # one token: o = beta (k . q) v; the same unit key written again with beta 1 replaces what it held; strong decay forgets
+    k, one, half = np.zeros((3, 1, 4)), np.ones((3, 1)), np.full((3, 1), 0.5)
+    k[:, :, 1] = 1
+    assert np.allclose(PK.delta_scan(q, k, v, one, one)[:, 0], q[:, 0, 1:2] * v[:, 0])
+    assert np.allclose(PK.delta_scan(q, k, v, half, 0 * one)[:, 0], 0.5 * q[:, 0, 1:2] * v[:, 0])
+    held = 0.5 * 0.5 * v[0, 0]
+    held = held + 0.5 * (v[1, 0] - held)
+    assert np.allclose(PK.delta_scan(q, k, v, half, half)[1, 0], q[1, 0, 1] * held)
+    assert np.allclose(PK.head_decay(np.array([0.0, -800.0]), 0.0, 0.0), [0.5, 1.0])
+    # scores are each logit's own sigmoid, and weigh what an expert reads: through a gated pair the output is not proportional
+    sel, s = PK.choose_experts(np.array([[0.0, 2.0, -1.0, 2.0]]), 3)
+    assert sel.tolist() == [[1, 3, 0]] and np.allclose(s, 1 / (1 + np.exp([[-2.0, -2.0, 0.0]])))
+    eye, h = np.eye(1), np.array([[3.0]])
+    y = PK.expert_ff(h, {"router": 0 * eye, "e0.gate": eye, "e0.up": eye, "e0.down": eye}, {"router": {"top": 1}})
+    assert np.allclose(y, 1.5 * 1.5 / (1 + np.exp(-1.5)))
+
+
 @pytest.mark.parametrize("edit, message", [
     (lambda c: c.update(architecture="Other"), "unsupported model architecture: Other"),
     (lambda c: c.pop("width"), "lacks 'width'"),
