@@ -75,8 +75,8 @@ def parse_args():
     ap.add_argument("--single-token-matvec", action="store_true",
                     help="with --one-sequence in the exact arithmetic: the matrix-vector kernel with f32 rows instead of the tile kernels "
                          "(what RETRO_GEMV_EXACT=1 selects)")
-    ap.add_argument("--model", default="llama", choices=["llama", "dibosun", "pomisun", "vifanex"],
-                    help="dibosun, pomisun, vifanex: prefill and decode of that layer-stack design at a few sizes, beside the closest other models "
+    ap.add_argument("--model", default="llama", choices=["llama", "dibosun", "pomisun", "vifanex", "kilurax"],
+                    help="dibosun, pomisun, vifanex, kilurax: prefill and decode of that layer-stack design at a few sizes, beside the closest other models "
                          "(another workload than the headline, with its own JSON line)")
     ap.add_argument("--stack-sizes", default="w2048,w4096", help="with a layer-stack --model: which sizes")
     ap.add_argument("--no-closest-model", action="store_true", help="with a layer-stack --model: only that design")

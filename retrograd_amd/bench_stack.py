@@ -1,5 +1,5 @@
 """Prefill and decode of layer-stack models at sizes that resemble a real model's layers, beside the closest other models of
-the same width, feed-forward width and depth: what `bench.py --model dibosun`, `--model pomisun` and `--model vifanex` run. Weights are random
+the same width, feed-forward width and depth: what `bench.py --model dibosun`, `--model pomisun`, `--model vifanex` and `--model kilurax` run. Weights are random
 (seeded), prompts random token ids. Every kernel category is also priced against its roofline, the larger of its
 algorithmic bytes over 8 TB/s and its products' flops over 2.5 PFLOP/s (a product counted once, however a model's
 arithmetic splits its operands; the scan's flops over the 157 TFLOP/s of f32)."""
@@ -47,6 +47,15 @@ def vifanex_config(size):
     att = lambda mlp: Y.normed_attention_layer(H, max(H // 4, 1), D, D, WINDOW, Y.banded_rotary(D, 1e6, factor=8.0, original=8192), mlp, v_mix=True)
     rec = lambda mlp: Y.channel_delta_layer(H, H, D, D, 4, mlp, 128, 128)
     return Y.vifanex(E, VOCAB, [att(dense), rec(moe), att(moe), rec(dense)] * 2, streams=4, softcap=30.0)
+
+
+def kilurax_config(size):
+    from . import synth_stack as Y
+    E, F, H, D, _, _, MH, G = SIZES[size]
+    moe = Y.moe_mlp(*EXPERTS[size])
+    two = Y.parallel_mixer_layer((H, max(H // 4, 1), D, D), (MH, 64, 128, G, 4, G), (0.6, 0.5), Y.rotary(D, 1e6), moe)
+    return Y.kilurax(E, VOCAB, [Y.delta_layer(H, H, D, D, 4, moe), two, Y.hgrn2_layer(H, D, D, moe), two] * 2, groups=4, taps=4,
+                     pairs=(65536, 40503, 1))
 
 
 def qwen3moe_shape(size):
@@ -175,6 +184,46 @@ def vifanex_work(cfg, rows, ctx, n_out):
     return w
 
 
+def kilurax_work(cfg, rows, ctx, n_out):
+    E, T = cfg["width"], rows
+    w = {}
+
+    def add(k, by, fl=0.0, f32=0.0):
+        a = w.setdefault(k, [0.0, 0.0, 0.0])
+        a[0] += by
+        a[1] += fl
+        a[2] += f32
+    for layer in cfg["layers"]:
+        m, mlp = layer["mixer"], layer["mlp"]
+        add("norm", 2 * T * E * (8 + 4 + 2))                     # the stream read and written, what is added, the activations
+        if layer["type"] == "parallel":
+            a, s = m["left"], m["right"]
+            H, G, D, V = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+            n_a, mix, bc = (H + G) * D + G * V, s["heads"] * s["vdim"], 2 * s["groups"] * s["state"]
+            n_s, state = 2 * mix + bc + s["heads"], s["heads"] * s["state"] * s["vdim"]
+            add("qkv", 2 * (n_a + n_s) * E + T * (2 * E + 2 * n_a + 4 * n_s), 2 * T * (n_a + n_s) * E)
+            add("attention", ctx[1] * 2 * G * (D + V) + T * H * 2 * (D + V), 2 * T * H * ctx[0] * (D + V))
+            add("scan", 8 * state * ctx[2] + T * (4 * (mix + bc) + 8 * mix + 2 * mix), 0, 4 * T * state)
+            n_o = H * V + mix
+        else:
+            H, D, V = m["heads"], m["dim"], m["vdim"]
+            G, per = m.get("kv_heads", H), 6 if layer["type"] == "delta" else 4
+            n = 2 * G * D + H * V + (2 * H + H * V if layer["type"] == "delta" else 0)
+            add("qkv", 2 * n * E + T * (2 * E + 4 * n), 2 * T * n * E)
+            add("scan", 8 * H * D * V * ctx[2] + T * (4 * n + 2 * H * V), 0, per * T * H * D * V)
+            n_o = H * V
+        add("o_proj", 2 * E * n_o + T * (2 * n_o + 4 * E), 2 * T * E * n_o)
+        n, top, F, S = mlp["router"]["experts"], mlp["router"]["top"], mlp["expert"]["ff"], mlp["shared"]["ff"]
+        used = chosen_experts(n, top, T)
+        add("shared", 2 * (n + 3 * S) * E + T * (2 * E + 4 * n + 4 * S + 4 * E), 2 * T * E * (n + 3 * S))
+        add("route", T * (4 * n + 8 * top))
+        add("experts_in", 4 * used * F * E + T * 2 * E + T * top * 2 * F, 4 * T * top * E * F)
+        add("experts_out", 2 * used * F * E + T * top * (2 * F + 4 * E), 2 * T * top * E * F)
+    add("embed", T * E * 8)
+    add("head", 2 * cfg["vocab"] * E + n_out * (2 * E + 4 * cfg["vocab"]), 2 * n_out * E * cfg["vocab"])
+    return w
+
+
 def qwen3moe_work(s, rows, ctx, n_out):
     from . import gguf_writer as gw
     w = llama_work(s, rows, ctx, n_out)
@@ -286,9 +335,10 @@ def main(args) -> int:
         print("this benchmark needs an MI355X: no HIP device is visible", file=sys.stderr)
         return 2
     causal, windowed, chunked = lambda p: p + 1, lambda p: np.minimum(p + 1, WINDOW), lambda p: p % CHUNK + 1
-    stacks = {"dibosun": (dibosun_config, dibosun_work, windowed), "pomisun": (pomisun_config, pomisun_work, chunked), "vifanex": (vifanex_config, vifanex_work, windowed)}
+    stacks = {"dibosun": (dibosun_config, dibosun_work, windowed), "pomisun": (pomisun_config, pomisun_work, chunked), "vifanex": (vifanex_config, vifanex_work, windowed),
+              "kilurax": (kilurax_config, kilurax_work, causal)}
     ggufs = {"llama": (llama_shape, llama_work), "qwen3moe": (qwen3moe_shape, qwen3moe_work)}
-    closest = {"dibosun": ["llama"], "pomisun": ["llama", "qwen3moe"], "vifanex": ["pomisun", "dibosun"]}[args.model]
+    closest = {"dibosun": ["llama"], "pomisun": ["llama", "qwen3moe"], "vifanex": ["pomisun", "dibosun"], "kilurax": ["vifanex", "pomisun", "dibosun"]}[args.model]
     steps = min(args.steps, 16)
     result = {"metric": "prefill and decode throughput, %s beside other models (GGUF ones in Q4_K, MXFP4 experts) of equal width, feed-forward and depth" % args.model.capitalize(),
               "data": "synthetic", "context": CONTEXT, "vocab": VOCAB, "layers": 8, "sizes": {}}

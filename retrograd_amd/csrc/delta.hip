@@ -16,7 +16,6 @@ namespace {
 constexpr int kChunk = 64;            // tokens of a chunk
 constexpr int kLongRun = 32;          // tokens from which a run is worked on in chunks
 constexpr int kChunkD = 128;          // most key channels of the chunk kernels
-constexpr int kWalkCols = 32;         // state columns a workgroup takes through the chunks
 constexpr int kScanRows = 16;         // most rows of the state a thread of the scan holds
 
 int pad16(int n) { return (n + 15) / 16 * 16; }
@@ -512,33 +511,33 @@ __global__ __launch_bounds__(256) void k_delta_chunk(DeltaJob j, Chunks out) {
     }
 }
 
-// The chunks of a run one after the other, for kWalkCols columns of one head's state. Wave w owns token block w of a chunk
+// The chunks of a run one after the other, for NC tiles of 16 columns of one head's state. Wave w owns token block w of a chunk
 // and rows w, w + 4 (in tiles of 16) of the state. The rows of the next chunk are requested as soon as a chunk's were used.
 // DELTA: u = U - W S; otherwise u = v, as projected.
-template <int DT, bool DELTA>
+template <int DT, bool DELTA, int NC>
 __global__ __launch_bounds__(256) void k_delta_walk(DeltaJob j, Chunks in, int col_blocks) {
-    constexpr int Dp = 16 * DT, NT = (DT + 3) / 4, LS = kWalkCols + 4;
+    constexpr int Dp = 16 * DT, NT = (DT + 3) / 4, LS = 16 * NC + 4;
     __shared__ __attribute__((aligned(16))) float sS[Dp * LS], sU[kChunk * LS];
     const DeltaShape sh = j.sh;
     const SeqRun run = j.runs.runs[blockIdx.y];
     if (run.n < kLongRun) return;
     // workgroup b runs on XCD b % 8: the column blocks of a head share its rows in one L2
-    const int group = (blockIdx.x >> 3) / col_blocks * 8 + (blockIdx.x & 7), p0 = (blockIdx.x >> 3) % col_blocks * kWalkCols, h = group;
+    const int group = (blockIdx.x >> 3) / col_blocks * 8 + (blockIdx.x & 7), p0 = (blockIdx.x >> 3) % col_blocks * 16 * NC, h = group;
     if (h >= sh.heads) return;
     const int D = sh.dim, V = sh.vdim, VP = sh.vpitch();
     const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, r16 = lane & 15, kg = lane >> 4, t0 = 16 * w;
     float * st = j.state + ((size_t)run.slot * sh.heads + h) * (size_t)D * VP + p0;
-    f4 S[NT][2];
+    f4 S[NT][NC];
 #pragma unroll
     for (int d = 0; d < NT; ++d)
 #pragma unroll
-        for (int c = 0; c < 2; ++c)
+        for (int c = 0; c < NC; ++c)
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int n = (w + 4 * d) * 16 + 4 * kg + i, p = c * 16 + r16;
                 S[d][c][i] = n < D && p0 + p < V && !(run.flags & 1) ? st[(size_t)n * VP + p] : 0.0f;
             }
-    f4 rw[DELTA ? DT : 1], rq[DT], ra[4], ru[2], rk[NT][4], rl[NT];
+    f4 rw[DELTA ? DT : 1], rq[DT], ra[4], ru[NC], rk[NT][4], rl[NT];
     int v_tok[4];                                // tokens of the lane's values in the chunk that is fetched next
     auto fetch_tokens = [&](int base) {
         if constexpr (!DELTA)
@@ -561,7 +560,7 @@ __global__ __launch_bounds__(256) void k_delta_walk(DeltaJob j, Chunks in, int c
                 if constexpr (DELTA) rw[e] = f4{0, 0, 0, 0};
             }
 #pragma unroll
-        for (int c = 0; c < 2; ++c)
+        for (int c = 0; c < NC; ++c)
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int r = t0 + 4 * kg + i, p = p0 + c * 16 + r16;
@@ -599,25 +598,30 @@ __global__ __launch_bounds__(256) void k_delta_walk(DeltaJob j, Chunks in, int c
         for (int d = 0; d < NT; ++d) {
             if (w + 4 * d >= DT) break;
 #pragma unroll
-            for (int c = 0; c < 2; ++c)
+            for (int c = 0; c < NC; ++c)
 #pragma unroll
                 for (int i = 0; i < 4; ++i) sS[((w + 4 * d) * 16 + 4 * kg + i) * LS + c * 16 + r16] = S[d][c][i];
         }
         __syncthreads();
-        f4 u[2] = {ru[0], ru[1]}, o[2] = {{0, 0, 0, 0}, {0, 0, 0, 0}};
+        f4 u[NC], o[NC];
+#pragma unroll
+        for (int c = 0; c < NC; ++c) {
+            u[c] = ru[c];
+            o[c] = f4{0, 0, 0, 0};
+        }
 #pragma unroll
         for (int e = 0; e < DT; ++e)
 #pragma unroll
             for (int i = 0; i < 4; ++i)
 #pragma unroll
-                for (int c = 0; c < 2; ++c) {
+                for (int c = 0; c < NC; ++c) {
                     const float s = sS[(16 * e + 4 * kg + i) * LS + c * 16 + r16];
                     if constexpr (DELTA) u[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(-rw[e][i], s, u[c], 0, 0, 0);
                     o[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(rq[e][i], s, o[c], 0, 0, 0);
                 }
         if (base + kChunk < run.n) fetch_first(base + kChunk);
 #pragma unroll
-        for (int c = 0; c < 2; ++c)
+        for (int c = 0; c < NC; ++c)
 #pragma unroll
             for (int i = 0; i < 4; ++i) sU[(t0 + 4 * kg + i) * LS + c * 16 + r16] = u[c][i];
         __syncthreads();
@@ -627,19 +631,19 @@ __global__ __launch_bounds__(256) void k_delta_walk(DeltaJob j, Chunks in, int c
 #pragma unroll
             for (int i = 0; i < 4; ++i)
 #pragma unroll
-                for (int c = 0; c < 2; ++c) o[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(ra[q][i], sU[(16 * q + 4 * kg + i) * LS + c * 16 + r16], o[c], 0, 0, 0);
+                for (int c = 0; c < NC; ++c) o[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(ra[q][i], sU[(16 * q + 4 * kg + i) * LS + c * 16 + r16], o[c], 0, 0, 0);
         }
 #pragma unroll
         for (int d = 0; d < NT; ++d) {
             if (w + 4 * d >= DT) break;
 #pragma unroll
-            for (int c = 0; c < 2; ++c) S[d][c] *= rl[d];
+            for (int c = 0; c < NC; ++c) S[d][c] *= rl[d];
 #pragma unroll
             for (int q = 0; q < 4; ++q)
 #pragma unroll
                 for (int i = 0; i < 4; ++i)
 #pragma unroll
-                    for (int c = 0; c < 2; ++c)
+                    for (int c = 0; c < NC; ++c)
                         S[d][c] = __builtin_amdgcn_mfma_f32_16x16x4f32(rk[d][q][i], sU[(16 * q + 4 * kg + i) * LS + c * 16 + r16], S[d][c], 0, 0, 0);
         }
         if (base + kChunk < run.n) fetch_second(base + kChunk);
@@ -649,7 +653,7 @@ __global__ __launch_bounds__(256) void k_delta_walk(DeltaJob j, Chunks in, int c
             if (r >= cnt) break;
             const int t = j.runs.tok[run.start + base + r];
 #pragma unroll
-            for (int c = 0; c < 2; ++c) {
+            for (int c = 0; c < NC; ++c) {
                 const int p = p0 + c * 16 + r16;
                 if (p < V) j.y[(size_t)t * sh.inner() + h * V + p] = o[c][i];
             }
@@ -658,7 +662,7 @@ __global__ __launch_bounds__(256) void k_delta_walk(DeltaJob j, Chunks in, int c
 #pragma unroll
     for (int d = 0; d < NT; ++d)
 #pragma unroll
-        for (int c = 0; c < 2; ++c)
+        for (int c = 0; c < NC; ++c)
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int n = (w + 4 * d) * 16 + 4 * kg + i, p = c * 16 + r16;
@@ -733,8 +737,12 @@ template <int DT, int RULE> void launch_chunks(hipStream_t s, const DeltaJob & j
     const unsigned n_chunks = (unsigned)((j.runs.longest + kChunk - 1) / kChunk);
     hipLaunchKernelGGL((k_delta_chunk<DT, RULE>), dim3(n_chunks, (unsigned)sh.heads, (unsigned)j.runs.n), dim3(256), lds, s, j, c);
     check_launch("delta_chunk");
-    const int blocks = (sh.vdim + kWalkCols - 1) / kWalkCols;
-    hipLaunchKernelGGL((k_delta_walk<DT, RULE != RULE_FORGET>), dim3((unsigned)((sh.heads + 7) / 8 * 8 * blocks), (unsigned)j.runs.n), dim3(256), 0, s, j, c, blocks);
+    // narrower blocks of columns while there are CUs for them: a chunk is a chain of products either way
+    const bool narrow = (int64_t)sh.heads * ((sh.vdim + 31) / 32) * j.runs.n <= 128;
+    const int blocks = narrow ? (sh.vdim + 15) / 16 : (sh.vdim + 31) / 32;
+    const dim3 grid((unsigned)((sh.heads + 7) / 8 * 8 * blocks), (unsigned)j.runs.n);
+    if (narrow) hipLaunchKernelGGL((k_delta_walk<DT, RULE != RULE_FORGET, 1>), grid, dim3(256), 0, s, j, c, blocks);
+    else hipLaunchKernelGGL((k_delta_walk<DT, RULE != RULE_FORGET, 2>), grid, dim3(256), 0, s, j, c, blocks);
     check_launch("delta_walk");
 }
 

@@ -194,123 +194,154 @@ struct GroupNorm {
 // where every run is a single token (a workgroup per run).
 enum : int { NORM_TO_ACT = 0, NORM_TO_ROWS, NORM_CONVOLVED };
 
-template <int ARITH> __device__ __forceinline__ void store_input(const SublayerNorm & j, int row, int k, const float (&v)[8]) {
-    store_frag8<ARITH>(j.act, j.act_kf, row, k, v);
-    if (j.act_rows) store_act8_at<ARITH>(j.act_rows, (size_t)row * j.act_kf * 32 + k, v);
+// W columns (1, or 4 from a multiple of 4) of a row as activations from element `at` on.
+template <int ARITH, typename VEC> __device__ __forceinline__ void store_columns(void * act, size_t at, const VEC & v) {
+    if constexpr (sizeof(VEC) == 4) {
+        if constexpr (ARITH == ARITH_16) ((uint16_t *)act)[at] = bf16_bits(v[0]);
+        else ((float *)act)[at] = v[0];
+    } else if constexpr (ARITH == ARITH_16) {
+        uint2 u;
+        u.x = (uint32_t)bf16_bits(v[0]) | ((uint32_t)bf16_bits(v[1]) << 16);
+        u.y = (uint32_t)bf16_bits(v[2]) | ((uint32_t)bf16_bits(v[3]) << 16);
+        *(uint2 *)((uint16_t *)act + at) = u;
+    } else {
+        *(VEC *)((float *)act + at) = v;
+    }
 }
 
-// W columns per thread and step, NV steps: the columns stay in registers between the two norms. A group is whole steps.
-template <int ARITH, int OUT, int W, int NV>
+// A thread holds W columns, NV times, from the reads to the writes; everything that does not hang on a norm is requested at
+// the start. WAVES: a group is whole steps of a wave, whose sums are all that goes through LDS.
+template <int ARITH, int OUT, int W, int NV, bool WAVES>
 __global__ __launch_bounds__(1024) void k_sublayer_norm(SublayerNorm j) {
     typedef float vec __attribute__((ext_vector_type(W)));
+    constexpr int PAST = NV <= 2 ? 3 : 0;         // inputs from earlier steps that are requested at the start
     extern __shared__ __attribute__((aligned(16))) float sm[];
     GroupNorm norm(sm, j.E, j.groups, j.eps);
-    float * row = norm.row;
-    const int E = j.E, n_thr = blockDim.x;
+    const int E = j.E, n_thr = blockDim.x, wave = threadIdx.x >> 6, waves = n_thr >> 6;
     SeqRun run = {};
     if constexpr (OUT == NORM_CONVOLVED) run = j.runs.runs[blockIdx.x];
     const int t = OUT == NORM_CONVOLVED ? j.runs.tok[run.start] : j.rows ? j.rows[blockIdx.x] : (int)blockIdx.x;
     const int at = OUT == NORM_CONVOLVED ? t : (int)blockIdx.x;              // row of the activations
+    const int past = OUT == NORM_CONVOLVED ? j.n_taps - 1 : 0, plane = (run.flags >> 1) & 1;
+    const bool fresh = run.flags & 1;
+    const float * old_in = nullptr;
+    float * new_in = nullptr;
+    if constexpr (OUT == NORM_CONVOLVED) {
+        old_in = j.history + (size_t)plane * j.plane + (size_t)run.slot * past * E;
+        new_in = j.history + (size_t)(1 - plane) * j.plane + (size_t)run.slot * past * E;
+    }
     float * xr = j.x + (size_t)t * E;
-    vec x[NV];
+    auto column = [&](int i) { return W * ((int)threadIdx.x + n_thr * i); };
+    auto remembered = [&](int p, int k) { return fresh ? vec(0.0f) : *(const vec *)(old_in + (size_t)p * E + k); };
+    vec x[NV], y[NV], w[NV], tap[NV], held[NV][PAST + 1], taps[NV][PAST + 1];
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-        const int k = W * ((int)threadIdx.x + n_thr * i);
-        if (k < E) x[i] = *(const vec *)(xr + k);
-    }
-    if (j.add.n > 0) {
-        vec y[NV];
+        const int k = column(i);
+        x[i] = y[i] = w[i] = vec(0.0f);
+        if (k >= E) continue;
+        x[i] = *(const vec *)(xr + k);
+        for (int base = 0; base < j.add.n; base += 8) {
+            const float * from = j.add.data + (size_t)base * j.add.stride + (size_t)t * E + k;
+            const int n = j.add.n - base;
+            vec d[8];
 #pragma unroll
-        for (int i = 0; i < NV; ++i) {
-            const int k = W * ((int)threadIdx.x + n_thr * i);
-            y[i] = vec(0.0f);
-            if (k >= E) continue;
-            for (int base = 0; base < j.add.n; base += 8) {
-                const float * from = j.add.data + (size_t)base * j.add.stride + (size_t)t * E + k;
-                const int n = j.add.n - base;
-                vec d[8];
+            for (int s = 0; s < 8; ++s) if (s < n) d[s] = *(const vec *)(from + (size_t)s * j.add.stride);
 #pragma unroll
-                for (int s = 0; s < 8; ++s) if (s < n) d[s] = *(const vec *)(from + (size_t)s * j.add.stride);
-#pragma unroll
-                for (int s = 0; s < 8; ++s) if (s < n) y[i] += d[s];
-            }
-            if (j.after) *(vec *)(row + k) = y[i];
+            for (int s = 0; s < 8; ++s) if (s < n) y[i] += d[s];
         }
-        if (j.after) norm.factors();
+        if (j.w) w[i] = *(const vec *)(j.w + k);
+        if constexpr (OUT == NORM_CONVOLVED) {
+            tap[i] = *(const vec *)(j.taps + (size_t)past * E + k);
+#pragma unroll
+            for (int p = 0; p < PAST; ++p)
+                if (p < past) {
+                    held[i][p] = remembered(p, k);
+                    taps[i][p] = *(const vec *)(j.taps + (size_t)p * E + k);
+                }
+        }
+    }
+    auto factors = [&](const vec (&v)[NV], int turn, float (&inv)[NV]) {
+        if constexpr (WAVES) {
+            float * part = sm + turn * NV * waves;
+#pragma unroll
+            for (int i = 0; i < NV; ++i) {
+                float q = 0.0f;
+#pragma unroll
+                for (int e = 0; e < W; ++e) q += v[i][e] * v[i][e];
+                q = wave_sum(q);
+                if ((threadIdx.x & 63) == 0) part[i * waves + wave] = q;
+            }
+            __syncthreads();
+            const int per = norm.len / (64 * W);
+#pragma unroll
+            for (int i = 0; i < NV; ++i) {
+                if (column(i) >= E) continue;
+                const int first = (i * waves + wave) / per * per;
+                float q = 0.0f;
+                for (int p = 0; p < per; ++p) q += part[first + p];
+                inv[i] = 1.0f / sqrtf(q / (float)norm.len + j.eps);
+            }
+        } else {
+#pragma unroll
+            for (int i = 0; i < NV; ++i) if (column(i) < E) *(vec *)(norm.row + column(i)) = v[i];
+            norm.factors();
+#pragma unroll
+            for (int i = 0; i < NV; ++i) if (column(i) < E) inv[i] = norm.inv[column(i) / norm.len];
+        }
+    };
+    float inv[NV];
+    if (j.add.n > 0) {
+        if (j.after) factors(y, 0, inv);
 #pragma unroll
         for (int i = 0; i < NV; ++i) {
-            const int k = W * ((int)threadIdx.x + n_thr * i);
+            const int k = column(i);
             if (k >= E) continue;
-            if (j.after) y[i] = y[i] * norm.inv[k / norm.len] * *(const vec *)(j.after + k);
+            if (j.after) y[i] = y[i] * inv[i] * *(const vec *)(j.after + k);
             x[i] += j.mult * y[i];
             if (!j.rows) *(vec *)(xr + k) = x[i];
         }
     }
     if (!j.w) return;
+    factors(x, 1, inv);
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-        const int k = W * ((int)threadIdx.x + n_thr * i);
-        if (k < E) *(vec *)(row + k) = x[i];
-    }
-    norm.factors();
-    if constexpr (OUT == NORM_TO_ROWS) {
-#pragma unroll
-        for (int i = 0; i < NV; ++i) {
-            const int k = W * ((int)threadIdx.x + n_thr * i);
-            if (k < E) *(vec *)(j.h + (size_t)t * E + k) = x[i] * norm.inv[k / norm.len] * *(const vec *)(j.w + k);
+        const int k = column(i);
+        if (k >= E) continue;
+        const vec h = x[i] * inv[i] * w[i];
+        if constexpr (OUT == NORM_TO_ROWS) {
+            *(vec *)(j.h + (size_t)t * E + k) = h;
+            continue;
         }
-        return;
-    }
-    for (int k = 8 * (int)threadIdx.x; k < E; k += 8 * n_thr) {
-        float v[8];
-        int g = k / norm.len, next = (g + 1) * norm.len;
-#pragma unroll
-        for (int i = 0; i < 8; ++i) {
-            if (k + i >= next) { ++g; next += norm.len; }
-            v[i] = k + i < E ? row[k + i] * norm.inv[g] * j.w[k + i] : 0.0f;
-        }
+        vec v = h;
         if constexpr (OUT == NORM_CONVOLVED) {
-            const int past = j.n_taps - 1, plane = (run.flags >> 1) & 1;
-            const bool fresh = run.flags & 1;
-            const float * old_in = j.history + (size_t)plane * j.plane + (size_t)run.slot * past * E;
-            float * new_in = j.history + (size_t)(1 - plane) * j.plane + (size_t)run.slot * past * E;
-            float h[8];
+            v += tap[i] * h;
+            auto take = [&](int p, const vec & o, const vec & f) {
+                v += f * o;
+                if (p > 0) *(vec *)(new_in + (size_t)(p - 1) * E + k) = o;
+            };
 #pragma unroll
-            for (int i = 0; i < 8; ++i) {
-                h[i] = v[i];
-                if (k + i < E) v[i] += j.taps[(size_t)past * E + k + i] * h[i];
-            }
-            for (int p = 0; p < past; ++p) {
-#pragma unroll
-                for (int i = 0; i < 8; ++i) {
-                    if (k + i >= E) break;
-                    const float o = fresh ? 0.0f : old_in[(size_t)p * E + k + i];
-                    v[i] += j.taps[(size_t)p * E + k + i] * o;
-                    if (p > 0) new_in[(size_t)(p - 1) * E + k + i] = o;
-                }
-            }
-            if (past > 0) {
-#pragma unroll
-                for (int i = 0; i < 8; ++i) if (k + i < E) new_in[(size_t)(past - 1) * E + k + i] = h[i];
-            }
+            for (int p = 0; p < PAST; ++p) if (p < past) take(p, held[i][p], taps[i][p]);
+            for (int p = PAST; p < past; ++p) take(p, remembered(p, k), *(const vec *)(j.taps + (size_t)p * E + k));
+            if (past > 0) *(vec *)(new_in + (size_t)(past - 1) * E + k) = h;
         }
-        store_input<ARITH>(j, at, k, v);
+        store_columns<ARITH>(j.act, frag_at(at, k, j.act_kf), v);
+        if (j.act_rows) store_columns<ARITH>(j.act_rows, (size_t)at * j.act_kf * 32 + k, v);
     }
 }
 
-// The convolution over the rows k_sublayer_norm left: a thread takes eight columns of kRunTokens tokens of a run, with the
-// window and the taps in registers (TAPS 0: any number).
-constexpr int kRunTokens = 8;
+// The convolution over the rows k_sublayer_norm left: a wave takes 16 tokens of a run and 32 columns, a lane eight columns of one
+// token, so that reads are whole cache lines and a wave's activations one fragment (TAPS 0: any number).
 template <int ARITH, int TAPS>
 __global__ __launch_bounds__(256) void k_sublayer_conv(SublayerNorm j) {
-    const int E = j.E, K = TAPS > 0 ? TAPS : j.n_taps, groups = (E + 7) / 8;
-    const int item = blockIdx.x * 256 + threadIdx.x, k = item % groups * 8, first = item / groups * kRunTokens;
-    const SeqRun run = j.runs.runs[blockIdx.y];
-    if (first >= run.n) return;
-    const int plane = (run.flags >> 1) & 1, last = min(first + kRunTokens, run.n), left = E - k;
+    const int E = j.E, K = TAPS > 0 ? TAPS : j.n_taps, lane = threadIdx.x & 63;
+    const int k = ((int)blockIdx.x * 4 + (threadIdx.x >> 6)) * 32 + 8 * (lane >> 4), i = blockIdx.y * 16 + (lane & 15), left = E - k;
+    const SeqRun run = j.runs.runs[blockIdx.z];
+    if (left <= 0 || i >= run.n) return;
+    const int plane = (run.flags >> 1) & 1;
     const bool even = E % 4 == 0;
-    const float * old_in = j.history + (size_t)plane * j.plane + (size_t)run.slot * (K - 1) * E;
-    float * new_in = j.history + (size_t)(1 - plane) * j.plane + (size_t)run.slot * (K - 1) * E;
+    const float * old_in = j.history + (size_t)plane * j.plane + (size_t)run.slot * (K - 1) * E + k;
+    float * new_in = j.history + (size_t)(1 - plane) * j.plane + (size_t)run.slot * (K - 1) * E + k;
+    const int32_t * tok = j.runs.tok + run.start;
     auto load = [&](const float * p, float (&o)[8]) {
         if (even && left >= 8) {
             const f4 a = *(const f4 *)p, b = *(const f4 *)(p + 4);
@@ -321,55 +352,38 @@ __global__ __launch_bounds__(256) void k_sublayer_conv(SublayerNorm j) {
             for (int e = 0; e < 8; ++e) o[e] = e < left ? p[e] : 0.0f;
         }
     };
-    auto input = [&](int i, float (&o)[8]) {         // h of the run's token i; i < 0: what the slot remembers
-        if (i >= 0) return load(j.h + (size_t)j.runs.tok[run.start + i] * E + k, o);
-        if (!(run.flags & 1)) return load(old_in + (size_t)(i + K - 1) * E + k, o);
+    auto input = [&](int at, float (&o)[8]) {        // of the run's token `at`; below 0: what the slot remembers
+        if (at >= 0) return load(j.h + (size_t)tok[at] * E + k, o);
+        if (!(run.flags & 1)) return load(old_in + (size_t)(at + K - 1) * E, o);
 #pragma unroll
         for (int e = 0; e < 8; ++e) o[e] = 0.0f;
     };
-    if constexpr (TAPS > 0) {
-        float win[TAPS][8], tap[TAPS][8];
+    auto remember = [&](int p, const float (&o)[8]) {
 #pragma unroll
-        for (int p = 0; p < TAPS; ++p) {
-            load(j.taps + (size_t)p * E + k, tap[p]);
-            if (p > 0) input(first - TAPS + p, win[p]);
-        }
-        for (int i = first; i < last; ++i) {
-            const int t = j.runs.tok[run.start + i];
+        for (int e = 0; e < 8; ++e) if (e < left) new_in[(size_t)p * E + e] = o[e];
+    };
+    const int t = tok[i];
+    float h[8], v[8];
+    load(j.h + (size_t)t * E + k, h);
 #pragma unroll
-            for (int p = 0; p + 1 < TAPS; ++p)
+    for (int e = 0; e < 8; ++e) v[e] = h[e];
+#pragma unroll TAPS > 0 ? TAPS : 1
+    for (int p = 0; p < K; ++p) {
+        float o[8], w[8];
+        input(i - (K - 1) + p, o);
+        load(j.taps + (size_t)p * E + k, w);
 #pragma unroll
-                for (int e = 0; e < 8; ++e) win[p][e] = win[p + 1][e];
-            load(j.h + (size_t)t * E + k, win[TAPS - 1]);
-            float v[8];
-#pragma unroll
-            for (int e = 0; e < 8; ++e) {
-                v[e] = win[TAPS - 1][e];
-#pragma unroll
-                for (int p = 0; p < TAPS; ++p) v[e] += tap[p][e] * win[p][e];
-            }
-            store_input<ARITH>(j, t, k, v);
-        }
-    } else {
-        for (int i = first; i < last; ++i) {
-            const int t = j.runs.tok[run.start + i];
-            float v[8], h[8], w[8];
-            load(j.h + (size_t)t * E + k, v);
-            for (int p = 0; p < K; ++p) {
-                input(i - (K - 1) + p, h);
-                load(j.taps + (size_t)p * E + k, w);
-#pragma unroll
-                for (int e = 0; e < 8; ++e) v[e] += w[e] * h[e];
-            }
-            store_input<ARITH>(j, t, k, v);
-        }
+        for (int e = 0; e < 8; ++e) v[e] += w[e] * o[e];
     }
-    if (last == run.n)
-        for (int p = 0; p < K - 1; ++p) {
-            float h[8];
-            input(run.n - (K - 1) + p, h);
-#pragma unroll
-            for (int e = 0; e < 8; ++e) if (e < left) new_in[(size_t)p * E + k + e] = h[e];
+    store_frag8<ARITH>(j.act, j.act_kf, t, k, v);
+    if (j.act_rows) store_act8_at<ARITH>(j.act_rows, (size_t)t * j.act_kf * 32 + k, v);
+    // the run's last inputs stay; a short run's first lane moves what is older
+    const int from = run.n - (K - 1);
+    if (i >= from) remember(i - from, h);
+    if (i == 0)
+        for (int p = 0; p < -from; ++p) {
+            input(from + p, h);
+            remember(p, h);
         }
 }
 
@@ -387,9 +401,25 @@ __global__ __launch_bounds__(256) void k_embed_pairs(PairEmbedding j) {
         pair = (before * j.mul_prev + tok * j.mul_cur) % j.buckets;
     }
     const uint16_t * e = j.embed + (size_t)tok * j.E, * p = j.pairs + (size_t)pair * j.E;
-    for (int k = threadIdx.x; k < j.E; k += 256) norm.row[k] = bf16_float(e[k]) * j.scale + bf16_float(p[k]);
+    float * x = j.x + (size_t)t * j.E;
+    if (j.E % 8 == 0) {
+        for (int k = 8 * (int)threadIdx.x; k < j.E; k += 8 * 256) {
+            const u4 a = *(const u4 *)(e + k), b = *(const u4 *)(p + k);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                norm.row[k + 2 * i] = bf16_float((uint16_t)a[i]) * j.scale + bf16_float((uint16_t)b[i]);
+                norm.row[k + 2 * i + 1] = bf16_float((uint16_t)(a[i] >> 16)) * j.scale + bf16_float((uint16_t)(b[i] >> 16));
+            }
+        }
+    } else {
+        for (int k = threadIdx.x; k < j.E; k += 256) norm.row[k] = bf16_float(e[k]) * j.scale + bf16_float(p[k]);
+    }
     norm.factors();
-    for (int k = threadIdx.x; k < j.E; k += 256) j.x[(size_t)t * j.E + k] = norm.row[k] * norm.inv[k / norm.len] * j.w[k];
+    if (norm.len % 4 == 0) {
+        for (int k = 4 * (int)threadIdx.x; k < j.E; k += 4 * 256) *(f4 *)(x + k) = *(const f4 *)(norm.row + k) * norm.inv[k / norm.len] * *(const f4 *)(j.w + k);
+    } else {
+        for (int k = threadIdx.x; k < j.E; k += 256) x[k] = norm.row[k] * norm.inv[k / norm.len] * j.w[k];
+    }
     if (i == run.n - 1 && threadIdx.x == 0) j.last[(size_t)(1 - plane) * j.plane + run.slot] = (float)tok;      // exact: a vocabulary has at most 2^24 tokens
 }
 
@@ -465,26 +495,29 @@ void sublayer_norm(hipStream_t s, int arith, const SublayerNorm & n, int n_rows)
     if (n.groups < 1 || n.E % n.groups != 0) throw std::runtime_error("norm: the row does not split into its groups");
     const bool conv = n.taps && n.w;
     const int out = !conv ? NORM_TO_ACT : n.runs.longest <= 1 ? NORM_CONVOLVED : NORM_TO_ROWS;
-    const bool vec = n.E % 4 == 0 && n.E / n.groups % 4 == 0;
-    const int width = vec ? 4 : 1;
-    int threads = n_rows <= 512 && n.E >= 2048 ? 1024 : 256;
+    const int len = n.E / n.groups, width = len % 4 == 0 ? 4 : 1;
+    const bool waves = len % 256 == 0;
+    // few rows: a column group per thread; many: fewer waves to wait for one another
+    int threads = n_rows <= 512 ? std::min(1024, (n.E / width + 63) / 64 * 64) : 256;
     if (n.E > 16 * width * threads) threads = 1024;
     const int steps = (n.E + width * threads - 1) / (width * threads);
     auto go = [&](auto kernel) {
         hipLaunchKernelGGL(kernel, dim3((unsigned)(out == NORM_CONVOLVED ? n.runs.n : n_rows)), dim3((unsigned)threads), GroupNorm::bytes(n.E, n.groups), s, n);
         check_launch("sublayer_norm");
     };
-    auto step = [&](auto arithmetic, auto kind, auto w) {
+    auto step = [&](auto arithmetic, auto kind, auto w, auto whole) {
         constexpr int A = decltype(arithmetic)::value, O = decltype(kind)::value, W = decltype(w)::value;
-        if (steps <= 1) go(k_sublayer_norm<A, O, W, 1>);
-        else if (steps <= 2) go(k_sublayer_norm<A, O, W, 2>);
-        else if (steps <= 4) go(k_sublayer_norm<A, O, W, 4>);
-        else if (steps <= 16) go(k_sublayer_norm<A, O, W, 16>);
+        constexpr bool V = decltype(whole)::value;
+        if (steps <= 1) go(k_sublayer_norm<A, O, W, 1, V>);
+        else if (steps <= 2) go(k_sublayer_norm<A, O, W, 2, V>);
+        else if (steps <= 4) go(k_sublayer_norm<A, O, W, 4, V>);
+        else if (steps <= 16) go(k_sublayer_norm<A, O, W, 16, V>);
         else throw std::runtime_error("norm: rows this wide are not supported");
     };
     auto columns = [&](auto arithmetic, auto kind) {
-        if (vec) step(arithmetic, kind, std::integral_constant<int, 4>());
-        else step(arithmetic, kind, std::integral_constant<int, 1>());
+        if (waves) step(arithmetic, kind, std::integral_constant<int, 4>(), std::true_type());
+        else if (width == 4) step(arithmetic, kind, std::integral_constant<int, 4>(), std::false_type());
+        else step(arithmetic, kind, std::integral_constant<int, 1>(), std::false_type());
     };
     auto kinds = [&](auto arithmetic) {
         if (out == NORM_TO_ACT) columns(arithmetic, std::integral_constant<int, NORM_TO_ACT>());
@@ -494,8 +527,7 @@ void sublayer_norm(hipStream_t s, int arith, const SublayerNorm & n, int n_rows)
     if (arith == ARITH_16) kinds(std::integral_constant<int, ARITH_16>());
     else kinds(std::integral_constant<int, ARITH_32>());
     if (out != NORM_TO_ROWS) return;
-    const int64_t items = (int64_t)((n.E + 7) / 8) * ((n.runs.longest + kRunTokens - 1) / kRunTokens);
-    const dim3 grid((unsigned)((items + 255) / 256), (unsigned)n.runs.n);
+    const dim3 grid((unsigned)((n.E + 127) / 128), (unsigned)((n.runs.longest + 15) / 16), (unsigned)n.runs.n);
     auto taps = [&](auto arithmetic) {
         constexpr int A = decltype(arithmetic)::value;
         switch (n.n_taps) {
