@@ -53,7 +53,7 @@ def kilurax_config(size):
     from . import synth_stack as Y
     E, F, H, D, _, _, MH, G = SIZES[size]
     moe = Y.moe_mlp(*EXPERTS[size])
-    two = Y.parallel_mixer_layer((H, max(H // 4, 1), D, D), (MH, 64, 128, G, 4, G), (0.6, 0.5), Y.rotary(D, 1e6), moe)
+    two = Y.parallel_mixer_layer((H, max(H // 4, 1), D, D), (MH, 64, 128, G, 4, G), (0.7, 0.4), Y.rotary(D, 1e6), moe)
     return Y.kilurax(E, VOCAB, [Y.delta_layer(H, H, D, D, 4, moe), two, Y.hgrn2_layer(H, D, D, moe), two] * 2, groups=4, taps=4,
                      pairs=(65536, 40503, 1))
 

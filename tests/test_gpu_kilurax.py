@@ -98,7 +98,7 @@ CONFIGS = {
         delta(heads=8, kv_heads=4, dim=128, vdim=128, conv=4, mlp=Y.moe_mlp(16, 4, 512, 544)),
         both((16, 4, 128, 128), (16, 64, 128, 4, 4, 4), (0.7, 0.6), Y.rotary(128, 1e5), mlp=Y.moe_mlp(12, 3, 160)),
         forget(heads=6, dim=96, vdim=200, mlp=Y.moe_mlp(12, 2, 160, 96)),
-        both((20, 20, 64, 80), (8, 32, 48, 1, 4, 1), (1.0, 1.0), Y.rotary(64, 1e4)),
+        both((20, 20, 72, 56), (8, 24, 40, 1, 4, 1), (1.0, 1.0), Y.rotary(72, 1e4)),
         forget(heads=4, dim=128, vdim=128), width=512, vocab=150, groups=4, taps=4, embedding_scale=2.0, pairs=(1009, 3, 17)),
 }
 BIG = ["all", "ones", "wide"]
@@ -254,7 +254,7 @@ def test_many_decoding_sequences(models, name, kv):
 
 
 @pytest.mark.parametrize("kv", KINDS)
-@pytest.mark.parametrize("dim, vdim", [(6, 30), (96, 20), (64, 80), (50, 100), (120, 40), (160, 128), (200, 66), (256, 256), (270, 90), (40, 300)])
+@pytest.mark.parametrize("dim, vdim", [(6, 30), (96, 20), (60, 90), (50, 100), (120, 40), (160, 128), (200, 66), (256, 256), (270, 90), (40, 300)])
 def test_key_and_value_widths(tmp_path, dim, vdim, kv):
     """Pairs of widths the attention kernels are compiled for, rounded up to and beyond them, with few, some and many query
     heads per key head: whole prompts, decoding one sequence (whose keys are shared out) and many."""
